@@ -8,7 +8,7 @@ from __future__ import annotations
 
 import json
 import os
-from dataclasses import dataclass, asdict, fields
+from dataclasses import dataclass, asdict, fields, replace
 from typing import Any, Mapping, Optional, Tuple
 
 
@@ -877,6 +877,208 @@ class PemuvikConfig:
                 if f.shared_ff is not None:
                     mlp["shared"] = {"ff": f.shared_ff}
             entries.append({"type": layer.kind, "mixer": mixer, "mlp": mlp})
+        out = {"architecture": self.architecture, "vocab": self.vocab, "width": self.width, "norm": {"eps": self.eps},
+               "layers": entries, "torch_dtype": self.dtype}
+        if self.eos_token_id is not None:
+            out["eos_token_id"] = list(self.eos_token_id)
+        return out
+
+
+# ---------------------------------------------------------------------------- Bamipel
+@dataclass(frozen=True)
+class QueryLatentAttentionConfig:
+    """Attention through a shared latent whose queries go through a latent of their own (q_rank entries): a head's query
+    has dim plain and rot_dim rotated entries, keys and values are made from a latent row of kv_rank entries and one rotated
+    key part per token; window None: every earlier position; an output gate of one number per head."""
+    heads: int
+    dim: int
+    rot_dim: int
+    vdim: int
+    q_rank: int
+    kv_rank: int
+    scale: float
+    window: Optional[int] = None
+    rot_base: float = 10000.0
+
+
+@dataclass(frozen=True)
+class WaveScalingConfig:
+    """Rotary frequencies by wavelength l: kept where l < original / high, divided by factor where l > original / low,
+    blended between."""
+    factor: float
+    low: float
+    high: float
+    original: float
+
+
+@dataclass(frozen=True)
+class HeadGateAttentionConfig:
+    """Grouped causal attention: the first rot_dims channels of every q and k head rotated (0: none), then every q and k
+    head divided by its root mean square; an output gate of one number per head."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    rot_dims: int = 0
+    rot_base: float = 10000.0
+    rot_scaling: Optional[WaveScalingConfig] = None
+
+
+@dataclass(frozen=True)
+class HeadDeltaConfig:
+    """The gated delta rule with one decay per head: `heads` value heads of vdim, kv_heads query/key heads of dim, short
+    convolutions of `conv` taps."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    conv: int
+
+
+@dataclass(frozen=True)
+class BamipelLayer:
+    kind: str                                    # "latent_attention" | "attention" | "delta"
+    mixer: Any                                   # QueryLatentAttentionConfig | HeadGateAttentionConfig | HeadDeltaConfig
+    ff: Optional[int]                            # the dense feed-forward's inner size, or None
+    weights_of: int                              # the entry whose tensors this one runs (itself where it has its own)
+
+
+@dataclass(frozen=True)
+class BamipelConfig:
+    """Bamipel: layers with a norm before and after each sublayer on a float32 residual stream; the mixer is, layer by
+    layer, a window attention through latents, a grouped attention or the gated delta rule; the feed-forward is dense
+    with the square of relu, or absent; a layer may run another layer's tensors again, with a cache of its own.
+    config.json gives every size and constant, layer by layer."""
+    vocab: int
+    width: int
+    eps: float
+    layers: Tuple[BamipelLayer, ...]
+    dtype: str = "bfloat16"
+    eos_token_id: Optional[Tuple[int, ...]] = None
+    architecture: str = "Bamipel"
+
+    @classmethod
+    def from_dict(cls, d: Mapping[str, Any]) -> "BamipelConfig":
+        where = "config.json"
+        entries = d.get("layers")
+        if not isinstance(entries, (list, tuple)) or not entries:
+            raise ConfigError(f"{where}: key 'layers' must be a list of layers")
+        layers = []
+        for i, entry in enumerate(entries):
+            at = f"{where}: layers[{i}]"
+            if not isinstance(entry, Mapping):
+                raise ConfigError(f"{at} must be an object")
+            kind = entry.get("type")
+            m = _section(entry, "mixer", at)
+            ma = at + ".mixer"
+            rot = m.get("rot")
+            dims, base, scaling = 0, 10000.0, None
+            if rot is not None:
+                dims = _whole(rot, "dims", ma + ".rot")
+                base = _require(rot, "base", float, ma + ".rot")
+                if rot.get("scaling") is not None:
+                    sa = ma + ".rot.scaling"
+                    scaling = WaveScalingConfig(*(_require(rot["scaling"], key, float, sa)
+                                                  for key in ("factor", "low", "high", "original")))
+            mixer: Any
+            if kind == "latent_attention":
+                mask = m.get("mask")
+                mixer = QueryLatentAttentionConfig(
+                    heads=_whole(m, "heads", ma), dim=_whole(m, "dim", ma), rot_dim=_whole(m, "rot_dim", ma),
+                    vdim=_whole(m, "vdim", ma), q_rank=_whole(m, "q_rank", ma), kv_rank=_whole(m, "kv_rank", ma),
+                    scale=_require(m, "scale", float, ma),
+                    window=None if mask is None else _whole(mask, "size", ma + ".mask"), rot_base=base)
+                if rot is None or dims != mixer.rot_dim or scaling is not None:
+                    raise ConfigError(f"{ma}: rot must be there without scaling and rot.dims equal rot_dim {mixer.rot_dim}, "
+                                      f"got {rot!r}")
+            elif kind == "attention":
+                mixer = HeadGateAttentionConfig(
+                    heads=_whole(m, "heads", ma), kv_heads=_whole(m, "kv_heads", ma), dim=_whole(m, "dim", ma),
+                    vdim=_whole(m, "vdim", ma), scale=_require(m, "scale", float, ma), rot_dims=dims, rot_base=base,
+                    rot_scaling=scaling)
+            elif kind == "delta":
+                mixer = HeadDeltaConfig(heads=_whole(m, "heads", ma), kv_heads=_whole(m, "kv_heads", ma),
+                                        dim=_whole(m, "dim", ma), vdim=_whole(m, "vdim", ma), conv=_whole(m, "conv", ma))
+            else:
+                raise ConfigError(f"{at}: type must be 'latent_attention', 'attention' or 'delta', got {kind!r}")
+            mlp = entry.get("mlp")
+            ff = None
+            if mlp is not None:
+                if not isinstance(mlp, Mapping) or mlp.get("kind", "dense") != "dense":
+                    raise ConfigError(f"{at}.mlp must be null or an object of kind 'dense', got {mlp!r}")
+                ff = _whole(mlp, "ff", at + ".mlp")
+            of = entry.get("weights_of")
+            layers.append(BamipelLayer(kind, mixer, ff, i if of is None else _count(entry, "weights_of", at)))
+        # (an entry may name one that has no tensors of its own either: it runs what that one runs)
+        for i, layer in enumerate(layers):
+            seen, j = {i}, layer.weights_of
+            while j < len(layers) and layers[j].weights_of != j and j not in seen:
+                seen.add(j)
+                j = layers[j].weights_of
+            layers[i] = replace(layer, weights_of=j)
+        norm = _section(d, "norm", where)
+        eos = d.get("eos_token_id")
+        eos = (eos,) if isinstance(eos, int) else tuple(int(x) for x in eos) if isinstance(eos, (list, tuple)) else None
+        cfg = cls(vocab=_whole(d, "vocab", where), width=_whole(d, "width", where),
+                  eps=_require(norm, "eps", float, where + ": norm"), layers=tuple(layers),
+                  dtype=canonical_dtype(d.get("dtype") or d.get("torch_dtype") or "bfloat16"), eos_token_id=eos,
+                  architecture=d.get("architecture") or (d.get("architectures") or ["Bamipel"])[0])
+        cfg.validate()
+        return cfg
+
+    def validate(self) -> None:
+        if not (self.eps > 0):
+            raise ConfigError(f"config.json: norm.eps must be positive, got {self.eps}")
+        for i, layer in enumerate(self.layers):
+            at = f"config.json: layers[{i}]"
+            m, j = layer.mixer, layer.weights_of
+            if j != i:
+                if not 0 <= j < len(self.layers) or self.layers[j].weights_of != j:
+                    raise ConfigError(f"{at}: weights_of names layer {j}, which must exist and have tensors of its own")
+                own = self.layers[j]
+                if (own.kind, own.mixer, own.ff) != (layer.kind, m, layer.ff):
+                    raise ConfigError(f"{at}: it differs from layer {j}, whose tensors it runs")
+            if layer.kind == "latent_attention":
+                if m.rot_dim % 2:
+                    raise ConfigError(f"{at}: rot_dim {m.rot_dim} must be even")
+            elif m.heads % m.kv_heads:
+                raise ConfigError(f"{at}: {m.heads} heads do not divide into {m.kv_heads} kv_heads")
+            if layer.kind == "delta":
+                continue
+            if not (m.scale > 0):
+                raise ConfigError(f"{at}: scale must be positive, got {m.scale}")
+            if not (m.rot_base > 0):
+                raise ConfigError(f"{at}: rot.base must be positive, got {m.rot_base}")
+            if layer.kind == "attention":
+                if m.rot_dims % 2 or m.rot_dims > m.dim:
+                    raise ConfigError(f"{at}: rot.dims {m.rot_dims} must be even and at most dim {m.dim}")
+                s = m.rot_scaling
+                if s is not None and not (s.factor > 0 and s.original > 0 and 0 < s.low <= s.high):
+                    raise ConfigError(f"{at}: rot.scaling needs positive numbers with low at most high, got {s}")
+
+    def to_dict(self) -> dict:
+        """The config.json that describes this configuration."""
+        entries = []
+        for i, layer in enumerate(self.layers):
+            m = layer.mixer
+            if layer.kind == "latent_attention":
+                mixer = {"heads": m.heads, "dim": m.dim, "rot_dim": m.rot_dim, "vdim": m.vdim, "q_rank": m.q_rank,
+                         "kv_rank": m.kv_rank, "scale": m.scale, "rot": {"dims": m.rot_dim, "base": m.rot_base}}
+                if m.window is not None:
+                    mixer["mask"] = {"size": m.window}
+            elif layer.kind == "attention":
+                mixer = {"heads": m.heads, "kv_heads": m.kv_heads, "dim": m.dim, "vdim": m.vdim, "scale": m.scale}
+                if m.rot_dims:
+                    mixer["rot"] = {"dims": m.rot_dims, "base": m.rot_base}
+                    if m.rot_scaling is not None:
+                        mixer["rot"]["scaling"] = asdict(m.rot_scaling)
+            else:
+                mixer = {"heads": m.heads, "kv_heads": m.kv_heads, "dim": m.dim, "vdim": m.vdim, "conv": m.conv}
+            entry = {"type": layer.kind, "mixer": mixer, "mlp": None if layer.ff is None else {"kind": "dense", "ff": layer.ff}}
+            if layer.weights_of != i:
+                entry["weights_of"] = layer.weights_of
+            entries.append(entry)
         out = {"architecture": self.architecture, "vocab": self.vocab, "width": self.width, "norm": {"eps": self.eps},
                "layers": entries, "torch_dtype": self.dtype}
         if self.eos_token_id is not None:

@@ -26,6 +26,10 @@ Options beyond the reference's attention, each a parameter:
     gate "sigmoid"                  the heads' outputs are multiplied, entry by entry, with sigmoid(x Wg^T)
                                     before the output projection; Wg [heads * v_head_dim, hidden] is packed
                                     below q, k and v into the one projection
+    gate "head_sigmoid"             one number per head: head h's output is multiplied by sigmoid(x Wg^T)_h, Wg
+                                    [heads, hidden]; the attention kernels apply it as they write their outputs
+    qk_norm_weight False            the per-head norms have no weight: every q and k head is divided by its root mean
+                                    square (the same before or after the rotation, which keeps a head's length)
     v_norm                          every value head is divided by its root mean square (eps inside the root, no
                                     weight) before it is cached
     v_mix (a name)                  the layers of a model that give the same name mix their values: the first of them
@@ -59,10 +63,10 @@ class Attention(Part):
     position_encoding (a name in the model's position encodings, or None), window (None or
     keys), scale (None: head_dim^-0.5), reads_shared_cache (bool: the run owns no cache, it
     projects q only and reads another run's keys and values), v_head_dim (None: head_dim),
-    qk_norm_scope ("head" | "projection"), q_temperature (None or {"coef", "every"}), sink (bool),
+    qk_norm_scope ("head" | "projection"), qk_norm_weight (bool, default True), q_temperature (None or {"coef", "every"}), sink (bool),
     chunk (None or positions), o_bias (bool), step_rotation (bool: rotate from the step's own table
     also where the per-head kernel could serve), softcap (None or a positive number), keep_first (positions),
-    sink_value (None or a number), gate (None or "sigmoid"), v_norm (bool), v_mix (None or a name shared by the layers
+    sink_value (None or a number), gate (None, "sigmoid" or "head_sigmoid"), v_norm (bool), v_mix (None or a name shared by the layers
     that mix), weights ("softmax" | "sigmoid"), and the names of the checkpoint tensors (q_name, ..., q_norm_name,
     k_norm_name, sink_name, g_name, v_mix_name, score_bias_name)."""
 
@@ -114,8 +118,13 @@ class Attention(Part):
         if self.keep_first < 0:
             raise ValueError(f"attention: keep_first {self.keep_first}")
         self.gate = p.get("gate")
-        if self.gate not in (None, "sigmoid"):
-            raise ValueError(f"attention: gate must be 'sigmoid' or absent, got {self.gate!r}")
+        if self.gate not in (None, "sigmoid", "head_sigmoid"):
+            raise ValueError(f"attention: gate must be 'sigmoid', 'head_sigmoid' or absent, got {self.gate!r}")
+        # columns of the gate in the packed projection
+        self.gate_rows = 0 if self.gate is None else self.heads if self.gate == "head_sigmoid" else self.heads * self.v_head_dim
+        self.qk_norm_weight = bool(p.get("qk_norm_weight", True))
+        if not self.qk_norm_weight and not (self.qk_norm and self.norm_scope == "head" and not self.shared):
+            raise ValueError("attention: norms without a weight are per-head norms of q and k")
         self.g_name = p.get("g_name", "g_proj")
         self.v_norm = bool(p.get("v_norm", False))
         self.v_mix = p.get("v_mix")
@@ -136,7 +145,7 @@ class Attention(Part):
         # and stores values of their own size; the per-head one rotates.  Each does what its model needs.
         self.row_prepare = self.norm_scope == "projection" or self.temp_coef != 0.0 or self.v_head_dim != self.head_dim \
             or bool(p.get("step_rotation", False)) or self.gate is not None or self.v_norm or bool(self.v_mix) \
-            or self.interleaved
+            or self.interleaved or not self.qk_norm_weight
         if self.row_prepare and self.position_encoding is not None and not hasattr(self.position_encoding, "step_table"):
             raise ValueError("attention: with whole-projection norms, a query temperature or values of their own "
                              "size the position encoding must offer step_table")
@@ -164,12 +173,14 @@ class Attention(Part):
             shards = ((self.q_name, 0, q), (self.k_name, q, kv), (self.v_name, q + kv, vv))
             rows = q + kv + vv
             if self.gate is not None:
-                shards += ((self.g_name, rows, self.heads * self.v_head_dim),)
-                rows += self.heads * self.v_head_dim
+                shards += ((self.g_name, rows, self.gate_rows),)
+                rows += self.gate_rows
+                if self.gate == "head_sigmoid":
+                    rows = (rows + 7) // 8 * 8          # (rows of the product in whole vectors, whatever the number of heads)
         d["qkv_proj.weight"] = ParamDecl((rows, h), sources=tuple(Source(f"{n}.weight", r, c) for n, r, c in shards))
         if self.bias:
             d["qkv_proj.bias"] = ParamDecl((rows,), sources=tuple(Source(f"{n}.bias", r, c) for n, r, c in shards))
-        if self.qk_norm:
+        if self.qk_norm and self.qk_norm_weight:
             whole = self.norm_scope == "projection"
             qn, kn = (q, kv) if whole else (self.head_dim, self.head_dim)
             d["q_norm.weight"] = ParamDecl((qn,), dtype="stored32", init="norm",
@@ -214,9 +225,9 @@ class Attention(Part):
         table = pe.rotary_table() if pe is not None and not self.row_prepare else None
         # (with a gate the row also holds the gate's columns, which outlive the preparation: a tensor, not partial sums)
         qkv = k.linear(x, w["qkv_proj.weight"], w.get("qkv_proj.bias"),
-                       deferred=self.gate is None and (self.row_prepare or pe is None or table is not None))
+                       deferred=self.gate != "sigmoid" and (self.row_prepare or pe is None or table is not None))
         gate = None
-        if self.gate is not None:
+        if self.gate == "sigmoid":
             qkv_width = (self.heads + self.kv_heads) * self.head_dim + self.kv_heads * self.v_head_dim
             gate, qkv = qkv[:, qkv_width:], qkv[:, :qkv_width]
         group = batch.groups[cache.group]
@@ -228,6 +239,11 @@ class Attention(Part):
             extra = {"rot_table": pe.step_table(batch)} if pe is not None else {}
             if self.qk_norm and self.norm_scope == "head":
                 extra["norm_per_head"] = True
+            if not self.qk_norm_weight:
+                extra["norm_unit"] = True
+            if self.gate == "head_sigmoid":
+                # the preparation also turns the row's gate columns into the heads' factors
+                extra["head_gate"] = head_gate = torch.empty((x.shape[0], self.heads), dtype=torch.float32, device=x.device)
             if self.interleaved:
                 extra["rot_interleaved"] = True
             if self.v_norm:
@@ -265,6 +281,8 @@ class Attention(Part):
         sinks = self._sinks()
         if self.weighting == "sigmoid":
             extra["sigmoid_bias"] = w["score_bias"]
+        if self.gate == "head_sigmoid":
+            extra["head_gate"] = head_gate
         if sinks is not None or self.v_head_dim != self.head_dim:
             o = k.paged_attention(q, self.heads, self.kv_heads, self.head_dim, cache.k, cache.v, batch, cache.group,
                                   self.scale, self.window, v_head_dim=self.v_head_dim, sinks=sinks, **extra)

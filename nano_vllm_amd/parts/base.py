@@ -25,7 +25,9 @@ class ParamDecl:
     # "model": the model's element type; "stored32": float32 if the checkpoint stores float32,
     # else the model's element type; "float32"; "int32" (integer tables)
     dtype: str = "model"
-    sources: Optional[Tuple[Source, ...]] = None     # None: one tensor of the parameter's own name
+    # None: one tensor of the parameter's own name.  Rows that no source fills are zero (a packed matrix whose
+    # product should have rows of a whole number of vectors).
+    sources: Optional[Tuple[Source, ...]] = None
     init: str = "normal"                             # random-weights mode: "normal" | "norm"
     # A size of -1 in `shape` is one that the checkpoint's tensor decides (a rank that no configuration
     # names); default_shape then says what random-weights mode draws.  Only for parameters of one source.

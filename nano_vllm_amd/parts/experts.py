@@ -50,7 +50,7 @@ class PlainMLP(Part):
                 f"{self.down_name}.weight": ParamDecl((self.hidden, self.inner))}
 
     def forward(self, x, batch=None):
-        z = self.kernels.act(self.kernels.linear(x, self.weights[f"{self.up_name}.weight"]), self.activation)
+        z = self.kernels.linear_act(x, self.weights[f"{self.up_name}.weight"], self.activation)
         return self.kernels.linear(z, self.weights[f"{self.down_name}.weight"], deferred=True)
 
 

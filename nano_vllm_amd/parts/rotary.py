@@ -14,6 +14,9 @@ The reference rotates the whole head (qwen3.py:49-54 passes rotary_dim = head_di
 smaller rotary_dim R the table is R wide and the first R channels of a head are rotated, in
 pairs (i, i + R/2), the others left as they are.
 With scaling_factor every frequency is divided by that constant (positions stretched linearly).
+With wave_scaling (factor, low, high, original) a frequency f is scaled by its wavelength l = 2 pi / f: kept where
+l < original / high, f / factor where l > original / low, and between the two the blend (1 - s) f / factor + s f
+with s = (original / l - low) / (high - low).
 A mixer whose model names no longest sequence asks for step_table(batch) instead of the table of all
 positions: the cosines and sines of the step's own tokens, [tokens, R], made once per step by a
 kernel that reads the positions on the device (so a captured step makes it anew at every replay) and
@@ -23,6 +26,7 @@ shared by all the layers that rotate alike.
 """
 from __future__ import annotations
 
+import math
 from typing import Mapping, Optional
 
 import torch
@@ -33,7 +37,7 @@ from .registry import register_part
 
 class RotaryNeox(Part):
     """params: head_dim, theta, max_position (rows of the table), rotary_dim (channels of a head
-    that are rotated; default all), scaling_factor (default 1)."""
+    that are rotated; default all), scaling_factor (default 1), wave_scaling (None or {factor, low, high, original})."""
 
     def __init__(self, params: Mapping, build: BuildContext):
         super().__init__(params, build)
@@ -53,17 +57,35 @@ class RotaryNeox(Part):
             raise ValueError(f"rotary_neox: the scaling factor must be positive, got {self.scaling_factor}")
         if self.scaling_factor != 1.0:
             inv_freq = inv_freq / self.scaling_factor
+        wave = params.get("wave_scaling")
+        self.wave_scaling = None if wave is None else tuple(float(wave[n]) for n in ("factor", "low", "high", "original"))
+        if self.wave_scaling is not None:
+            inv_freq = self._scaled_by_wavelength(*self.wave_scaling)
         self.inv_freq = inv_freq
         self._device = build.device
         self._table = None
         self._inv_freq_dev = None
+
+    def _scaled_by_wavelength(self, factor: float, low: float, high: float, original: float) -> torch.Tensor:
+        """The scaled frequencies, worked out in double and rounded once."""
+        out = []
+        for i in range(self.rotary_dim // 2):
+            f = self.theta ** (-2.0 * i / self.rotary_dim)
+            length = 2.0 * math.pi / f
+            if length > original / low:
+                f = f / factor
+            elif length >= original / high and high > low:
+                s = (original / length - low) / (high - low)
+                f = (1.0 - s) * f / factor + s * f
+            out.append(f / self.scaling_factor)
+        return torch.tensor(out, dtype=torch.float64).to(torch.float32)
 
     def step_table(self, batch) -> torch.Tensor:
         """float32 [tokens, rotary_dim]: cosines, then sines, of the step's tokens at their positions."""
         kept = getattr(batch, "step_cache", None)
         if kept is None:
             kept = batch.step_cache = {}
-        key = ("rotary_step", self.rotary_dim, self.theta, self.scaling_factor)
+        key = ("rotary_step", self.rotary_dim, self.theta, self.scaling_factor, self.wave_scaling)
         if key not in kept:
             if self._inv_freq_dev is None:
                 self._inv_freq_dev = self.inv_freq.to(self._device)

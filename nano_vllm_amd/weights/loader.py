@@ -115,8 +115,10 @@ def load_weights(model, folder: str) -> None:
                     if t.dtype in (torch.int64, torch.int32, torch.int16, torch.int8, torch.uint8) and decl.dtype != "int32":
                         wrong.append((name + f" (integer {t.dtype})", shape, slot.shape))
                         continue
-                    tensors[slot.param] = torch.empty(shape if slot.whole else decl.shape,
-                                                      dtype=_param_dtype(decl, t.dtype, model.dtype), device=model.device)
+                    # (rows of a packed parameter that no source fills stay zero)
+                    make = torch.empty if slot.whole or sum(s.rows for s in decl.sources) == decl.shape[0] else torch.zeros
+                    tensors[slot.param] = make(shape if slot.whole else decl.shape,
+                                               dtype=_param_dtype(decl, t.dtype, model.dtype), device=model.device)
                 dst = tensors[slot.param]
                 dst = dst if slot.whole else dst.narrow(0, slot.row, slot.rows)
                 dst.copy_(t.to(dst.dtype))

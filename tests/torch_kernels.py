@@ -314,13 +314,22 @@ class TorchKernels:
 
     def qk_rownorm_store(self, qkv, num_heads, num_kv_heads, head_dim, v_head_dim, q_weight, k_weight, eps,
                          positions, temp_coef, temp_every, slots, k_cache, v_cache, rot_table=None, norm_per_head=False,
-                         rot_interleaved=False, v_norm=False, v_first_in=None, v_mix=None, v_first_out=None):
+                         rot_interleaved=False, v_norm=False, v_first_in=None, v_mix=None, v_first_out=None, norm_unit=False,
+                         head_gate=None):
         """q and k normed over the whole projection, q times its position's temperature, both rotated by
         the rows of rot_table (one per token: cosines, then sines, for the first channels of a head),
         k and v stored."""
         T = qkv.shape[0]
         qd, kd = num_heads * head_dim, num_kv_heads * head_dim
         dt = qkv.dtype
+        if head_gate is not None:           # the row's columns behind v: a number per head
+            at = qd + kd + num_kv_heads * v_head_dim
+            head_gate.copy_(torch.sigmoid(qkv[:, at:at + num_heads].float()))
+            qkv = qkv[:, :at]
+        unit_q = unit_k = None
+        if norm_unit:
+            unit_q, unit_k = torch.ones(head_dim), torch.ones(head_dim)
+            q_weight, k_weight = unit_q.to(qkv.device), unit_k.to(qkv.device)
 
         def turn(x, heads):
             if rot_table is None:
@@ -375,6 +384,25 @@ class TorchKernels:
         out = x if out is None else out
         out.copy_(y)
         return out
+
+    def linear_act(self, x, weight, act):
+        return self.act(self.linear(x, weight), act)
+
+    def head_delta(self, proj, rates, heads, kv_heads, dim, vdim, taps, conv_w, dt_bias, a_log, norm_w, eps, conv_state,
+                   s_state, batch, out=None):
+        """The delta rule with one decay per head (all key channels alike) and a silu gate: proj [q | k | v | gate],
+        rates float [b | a]."""
+        C = 2 * kv_heads * dim + heads * vdim
+        decay_in = rates[:, heads:].float().repeat_interleave(dim, dim=1)
+        gate = proj[:, C:].float()
+        row = torch.cat((proj[:, :C].float(), rates[:, :heads].float()), dim=1)
+        y = self.channel_delta(row, decay_in, torch.full_like(gate, 1e4), heads, kv_heads, dim, vdim, taps, conv_w,
+                               dt_bias.repeat_interleave(dim), a_log, norm_w, eps, conv_state, s_state, batch)
+        y = (y * gate * torch.sigmoid(gate)).to(proj.dtype)
+        if out is not None:
+            out.copy_(y)
+            return out
+        return y
 
     def channel_delta(self, proj, decay_in, gate_in, heads, kv_heads, dim, vdim, taps, conv_w, dt_bias, a_log, norm_w,
                       eps, conv_state, s_state, batch, out=None):
@@ -502,7 +530,7 @@ class TorchKernels:
     # attention (attention.py:64-75): token by token through the block table
     def paged_attention(self, q, num_heads, num_kv_heads, head_dim, k_cache, v_cache, batch, group, scale,
                         window=None, out=None, v_head_dim=None, sinks=None, chunk=None, softcap=None, keep_first=0,
-                        sigmoid_bias=None):
+                        sigmoid_bias=None, head_gate=None):
         T = q.shape[0]
         D, G = head_dim, num_heads // num_kv_heads
         DV = v_head_dim or head_dim
@@ -535,7 +563,7 @@ class TorchKernels:
                     p = torch.softmax(torch.cat((s, sinks[h:h + 1].float())), dim=0)[:-1]
                 else:
                     p = torch.softmax(s, dim=0)
-                o[t, h * DV:(h + 1) * DV] = p @ vals[:, h // G]
+                o[t, h * DV:(h + 1) * DV] = (p @ vals[:, h // G]) * (1.0 if head_gate is None else head_gate[t, h].float())
         y = o.to(q.dtype)
         if out is not None:
             out.copy_(y)
@@ -543,40 +571,66 @@ class TorchKernels:
         return y
 
     # attention through a latent
-    def latent_prepare(self, proj, heads, dim, rot, rank, weight, eps, rot_table, slots, k_cache, v_cache):
-        T = proj.shape[0]
-        dt = proj.dtype
-        qd = heads * (dim + rot)
-        cos, sin = rot_table[:, : rot // 2], rot_table[:, rot // 2:]
-
-        def turn(x):                                    # [..., rot] with the tokens first
+    @staticmethod
+    def _latent_turn(x, rot_table, interleaved):        # [tokens, rot] or [tokens, heads, rot]
+        half = rot_table.shape[1] // 2
+        c, s = rot_table[:, :half], rot_table[:, half:]
+        if x.dim() == 3:
+            c, s = c[:, None], s[:, None]
+        if interleaved:
             a, b = x[..., 0::2], x[..., 1::2]
-            c, s = (cos, sin) if x.dim() == 2 else (cos[:, None], sin[:, None])
             return torch.stack((a * c - b * s, b * c + a * s), dim=-1).reshape(x.shape)
-        q = proj[:, :qd].float().reshape(T, heads, dim + rot)
-        q2 = torch.zeros((T, heads, rank + rot), dtype=dt, device=proj.device)
-        q2[:, :, rank:] = turn(q[:, :, dim:]).to(dt)
-        if k_cache is not None:
-            c = proj[:, qd:qd + rank].float()
-            c = (c * torch.rsqrt(c.pow(2).mean(-1, keepdim=True) + eps) * weight.float()).to(dt)
-            kr = turn(proj[:, qd + rank:].float()).to(dt)
-            page_size, vt = k_cache.shape[2], v_cache.shape[4]
-            s = slots.long()
-            ok = s >= 0
-            page, off = s[ok] // page_size, s[ok] % page_size
-            k_cache[page, 0, off, :] = torch.cat((c, kr), dim=-1)[ok]
-            v_cache[page, 0, off // vt, :, off % vt] = c[ok]
-        return q2.reshape(T, heads * (rank + rot))
+        a, b = x[..., :half], x[..., half:]
+        return torch.cat((a * c - b * s, b * c + a * s), dim=-1)
 
-    def latent_attention(self, q2, heads, rank, rot, k_cache, v_cache, batch, group, scale, sinks=None):
-        return self.paged_attention(q2, heads, 1, rank + rot, k_cache, v_cache, batch, group, scale, None, v_head_dim=rank,
+    def _latent_store(self, c, kr, rank, weight, eps, rot_table, slots, k_cache, v_cache, interleaved, dt):
+        c = c.float()
+        c = (c * torch.rsqrt(c.pow(2).mean(-1, keepdim=True) + eps) * weight.float()).to(dt)
+        kr = self._latent_turn(kr.float(), rot_table, interleaved).to(dt)
+        page_size, vt = k_cache.shape[2], v_cache.shape[4]
+        s = slots.long()
+        ok = s >= 0
+        page, off = s[ok] // page_size, s[ok] % page_size
+        k_cache[page, 0, off, :] = torch.cat((c, kr), dim=-1)[ok]
+        v_cache[page, 0, off // vt, :, off % vt] = c[ok]
+
+    def latent_prepare(self, proj, heads, dim, rot, rank, weight, eps, rot_table, slots, k_cache, v_cache, interleaved=True):
+        qd = heads * (dim + rot)
+        q2 = self.latent_queries(proj[:, :qd], heads, dim, rot, rank, rot_table, interleaved)[2]
+        if k_cache is not None:
+            self._latent_store(proj[:, qd:qd + rank], proj[:, qd + rank:], rank, weight, eps, rot_table, slots, k_cache, v_cache,
+                               interleaved, proj.dtype)
+        return q2
+
+    def latent_down(self, low, q_rank, rot, rank, gates, q_weight, weight, eps, rot_table, slots, k_cache, v_cache,
+                    interleaved=True):
+        cq = low[:, :q_rank].float()
+        cq = (cq * torch.rsqrt(cq.pow(2).mean(-1, keepdim=True) + eps) * q_weight.float()).to(low.dtype)
+        at = q_rank + rank + rot
+        if k_cache is not None:
+            self._latent_store(low[:, q_rank:q_rank + rank], low[:, q_rank + rank:at], rank, weight, eps, rot_table, slots,
+                               k_cache, v_cache, interleaved, low.dtype)
+        return cq, torch.sigmoid(low[:, at:at + gates].float()) if gates else None
+
+    def latent_queries(self, q, heads, dim, rot, rank, rot_table, interleaved=True):
+        T, dt = q.shape[0], q.dtype
+        x = q.float().reshape(T, heads, dim + rot)
+        q2 = torch.zeros((T, heads, rank + rot), dtype=dt, device=q.device)
+        q2[:, :, rank:] = self._latent_turn(x[:, :, dim:], rot_table, interleaved).to(dt)
+        return q, dim + rot, q2.reshape(T, heads * (rank + rot))
+
+    def latent_attention(self, q2, heads, rank, rot, k_cache, v_cache, batch, group, scale, sinks=None, window=None):
+        return self.paged_attention(q2, heads, 1, rank + rot, k_cache, v_cache, batch, group, scale, window, v_head_dim=rank,
                                     sinks=sinks)
 
-    def heads_linear(self, x, x_head, w, heads, n_out, k_in, transposed, y, y_head, y_offset=0):
+    def heads_linear(self, x, x_head, w, heads, n_out, k_in, transposed, y, y_head, y_offset=0, head_gate=None):
         wh = w.float().reshape(heads, k_in, n_out).transpose(1, 2) if transposed else w.float().reshape(heads, n_out, k_in)
         for h in range(heads):
             xh = x[:, h * x_head: h * x_head + k_in].float()
-            y[:, h * y_head + y_offset: h * y_head + y_offset + n_out] = (xh @ wh[h].T).to(y.dtype)
+            z = xh @ wh[h].T
+            if head_gate is not None:
+                z = z * head_gate[:, h:h + 1].float()
+            y[:, h * y_head + y_offset: h * y_head + y_offset + n_out] = z.to(y.dtype)
         return y
 
     # sampling (sampler.py:8-12), same counter-based noise as the kernel
