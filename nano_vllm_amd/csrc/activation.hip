@@ -82,6 +82,31 @@ NVA_EXPORT int NVA_NAME(nva_silu_mul)(const void* x, int64_t x_stride, void* out
 }
 
 // An activation without a gate: out[t, i] = act(x[t, i]); act by the codes of nva_gate_act (3: relu squared).
+// Eight entries a thread where rows and pointers allow.
+template <typename T>
+__global__ void __launch_bounds__(256)
+act8_kernel(const T* __restrict__ x, int64_t x_stride, T* __restrict__ out, int64_t out_stride, int64_t rows, int width8, int act) {
+    const int64_t idx = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
+    if (idx >= rows * width8) return;
+    const int64_t r = idx / width8;
+    const int i = (int)(idx % width8) * 8;
+    float v[8];
+    load8(x + r * x_stride + i, v);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) v[e] = nva_gate_act(act, v[e]);
+    store8(out + r * out_stride + i, v);
+}
+
+// The same from a product that was left as partial sums: out[t, i] = act(round(sum + bias)).
+template <typename T>
+__global__ void __launch_bounds__(256)
+act_of_partials_kernel(PartialInput part, T* __restrict__ out, int64_t out_stride, int width, int act) {
+    const int64_t r = blockIdx.y;
+    const int i = blockIdx.x * blockDim.x + threadIdx.x;
+    if (i >= width) return;
+    out[r * out_stride + i] = from_float<T>(nva_gate_act(act, partial_value<T>(part, r, width, i)));
+}
+
 template <typename T>
 __global__ void __launch_bounds__(256)
 act_kernel(const T* __restrict__ x, int64_t x_stride, T* __restrict__ out, int64_t out_stride, int64_t rows, int width, int act) {
@@ -98,9 +123,28 @@ NVA_EXPORT int NVA_NAME(nva_act)(const void* x, int64_t x_stride, void* out, int
     if (rows < 0 || width <= 0 || act < 0 || act > 3) return nva_fail("act: bad shape rows=%lld width=%d or activation %d", (long long)rows, width, act);
     const int64_t total = rows * width;
     if ((total + 255) / 256 > 0x7fffffff) return nva_fail("act: too many entries");
+    const size_t vb = 8 * sizeof(elem_t);
+    if (width % 8 == 0 && x_stride % 8 == 0 && out_stride % 8 == 0 && nva_aligned(x, vb) && nva_aligned(out, vb)) {
+        hipLaunchKernelGGL((act8_kernel<elem_t>), dim3((unsigned)((total / 8 + 255) / 256)), dim3(256), 0, stream,
+                           (const elem_t*)x, x_stride, (elem_t*)out, out_stride, rows, width / 8, act);
+        return nva_check_launch("act");
+    }
     hipLaunchKernelGGL((act_kernel<elem_t>), dim3((unsigned)((total + 255) / 256)), dim3(256), 0, stream, (const elem_t*)x,
                        x_stride, (elem_t*)out, out_stride, rows, width, act);
     return nva_check_launch("act");
+}
+
+// sums: float [splits][rows][width], with an optional bias of elements [width].
+NVA_EXPORT int NVA_NAME(nva_act_of_partials)(const float* sums, int splits, int64_t split_stride, const void* bias, void* out,
+                                             int64_t out_stride, int64_t rows, int width, int act, hipStream_t stream) {
+    if (rows == 0) return 0;
+    if (rows < 0 || rows > 65535 || width <= 0 || act < 0 || act > 3 || !sums || splits <= 0 || split_stride < rows * (int64_t)width ||
+        !out || out_stride < width)
+        return nva_fail("act_of_partials: bad shape rows=%lld width=%d splits=%d or activation %d", (long long)rows, width, splits, act);
+    const PartialInput part{sums, splits, split_stride, bias};
+    hipLaunchKernelGGL((act_of_partials_kernel<elem_t>), dim3((width + 255) / 256, (unsigned)rows), dim3(256), 0, stream, part,
+                       (elem_t*)out, out_stride, width, act);
+    return nva_check_launch("act_of_partials");
 }
 
 // A gate on finished outputs: out[t, i] = x[t, i] * sigmoid(g[t, i]), in float, rounded once (out may be x).

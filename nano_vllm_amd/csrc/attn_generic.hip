@@ -1,6 +1,6 @@
 // Causal attention of a step's tokens over the paged cache: the general kernel.
 //
-// It takes any head size up to 512, any number of heads and groups, any page size and an
+// It takes any head size up to 640, any number of heads and groups, any page size and an
 // optional window, in float arithmetic with an online softmax (scores, running maximum and
 // sum, and the output accumulator in float).  It is the attention of the 32-bit path and the
 // fallback of the bfloat16 path for shapes the matrix-core kernels refuse.
@@ -20,6 +20,7 @@
 // first, then the window.
 // sig_bias, float [Hq] or null (the per-token kernel): no softmax; a visible key weighs sigmoid(s_j + sig_bias_h) and the
 // weights are not normalised over the keys: o = sum_j sigmoid(s_j + b_h) v_j.  (No sink, no sharing of a token's keys.)
+// head_gate, float [tokens, Hq] or null: a head's output is multiplied by its token's number as it is written.
 //
 // Portions of prompts have a second kernel with the same arithmetic, operation for operation (the
 // results are the same bits): a workgroup takes 32 query rows of one request and one head, and the
@@ -29,7 +30,7 @@
 // a row's first visible key, and mask what lies before it).
 #include "common.h"
 
-#define ATT_MAX_D 512
+#define ATT_MAX_D 640
 #define ATT_ACC (ATT_MAX_D / NVA_WAVE)
 
 template <typename T>
@@ -40,7 +41,8 @@ paged_attention_generic_kernel(const T* __restrict__ q, int64_t q_stride, T* __r
                                const int32_t* __restrict__ token_seq, const int32_t* __restrict__ positions,
                                int num_q_heads, int num_kv_heads, int head_dim, int v_dim, int page_size, float scale,
                                int window, int chunk, int keep_first, float softcap, const float* __restrict__ sinks,
-                               const float* __restrict__ sig_bias, float* __restrict__ part, int32_t* error_flag) {
+                               const float* __restrict__ sig_bias, const float* __restrict__ head_gate,
+                               float* __restrict__ part, int32_t* error_flag) {
     __shared__ float q_s[ATT_MAX_D];
     __shared__ float p_s[NVA_WAVE];
     __shared__ int64_t v_off_s[NVA_WAVE];
@@ -175,7 +177,8 @@ paged_attention_generic_kernel(const T* __restrict__ q, int64_t q_stride, T* __r
         }
         return;
     }
-    const float inv = sig_bias ? 1.f : l_run > 0.f ? 1.f / l_run : 0.f;
+    float inv = sig_bias ? 1.f : l_run > 0.f ? 1.f / l_run : 0.f;
+    if (head_gate) inv *= head_gate[t * num_q_heads + h];
     T* orow = out + t * out_stride + (int64_t)h * v_dim;
 #pragma unroll
     for (int i = 0; i < ATT_ACC; ++i) {
@@ -188,7 +191,7 @@ paged_attention_generic_kernel(const T* __restrict__ q, int64_t q_stride, T* __r
 template <typename T>
 __global__ void __launch_bounds__(NVA_WAVE)
 paged_attention_merge_kernel(const float* __restrict__ part, int shares, T* __restrict__ out, int64_t out_stride,
-                             int num_q_heads, int v_dim) {
+                             int num_q_heads, int v_dim, const float* __restrict__ head_gate) {
     const int64_t t = blockIdx.x;
     const int h = blockIdx.y, lane = threadIdx.x;
     const float* mine = part + (t * num_q_heads + h) * shares * (int64_t)(2 + v_dim);
@@ -209,7 +212,8 @@ paged_attention_merge_kernel(const float* __restrict__ part, int shares, T* __re
             if (d < v_dim) acc[i] += p[2 + d] * f;
         }
     }
-    const float inv = l > 0.f ? 1.f / l : 0.f;
+    float inv = l > 0.f ? 1.f / l : 0.f;
+    if (head_gate) inv *= head_gate[t * num_q_heads + h];
     T* orow = out + t * out_stride + (int64_t)h * v_dim;
 #pragma unroll
     for (int i = 0; i < ATT_ACC; ++i) {
@@ -238,7 +242,7 @@ paged_attention_tiled_kernel(const T* __restrict__ q, int64_t q_stride, T* __res
                              const int32_t* __restrict__ cu_seqlens_q, const int32_t* __restrict__ kv_lens,
                              const int32_t* __restrict__ tiles, int num_q_heads, int num_kv_heads, int head_dim,
                              int v_dim, int page_size, float scale, int chunk, float softcap,
-                             const float* __restrict__ sinks, int32_t* error_flag) {
+                             const float* __restrict__ sinks, const float* __restrict__ head_gate, int32_t* error_flag) {
     extern __shared__ __attribute__((aligned(16))) float lds[];
     __shared__ int64_t k_off_s[NVA_WAVE], v_off_s[NVA_WAVE];       // of a chunk's keys; -1: the key has no page
     constexpr int ROWS_PER_WAVE = ATT_ROWS / ATT_TILED_WAVES;
@@ -443,7 +447,8 @@ paged_attention_tiled_kernel(const T* __restrict__ q, int64_t q_stride, T* __res
     for (int rr = 0; rr < ROWS_PER_WAVE; ++rr) {
         const int r = wave + ATT_TILED_WAVES * rr;
         if (r >= rows) continue;
-        const float inv = l_run[rr] > 0.f ? 1.f / l_run[rr] : 0.f;
+        float inv = l_run[rr] > 0.f ? 1.f / l_run[rr] : 0.f;
+        if (head_gate) inv *= head_gate[(int64_t)(q_begin + q0 + r) * num_q_heads + h];
         T* orow = out + (int64_t)(q_begin + q0 + r) * out_stride + (int64_t)h * v_dim;
 #pragma unroll
         for (int i = 0; i < ACC; ++i) {
@@ -460,7 +465,8 @@ NVA_EXPORT int NVA_NAME(nva_paged_attention_tiled)(
     const void* q, int64_t q_stride, void* out, int64_t out_stride, const void* k_cache, const void* v_cache,
     const int32_t* block_tables, int table_stride, const int32_t* cu_seqlens_q, const int32_t* kv_lens,
     const int32_t* tiles, int64_t num_tiles, int num_q_heads, int num_kv_heads, int head_dim, int v_dim,
-    int page_size, float scale, int chunk, float softcap, const float* sinks, int32_t* error_flag, hipStream_t stream) {
+    int page_size, float scale, int chunk, float softcap, const float* sinks, const float* head_gate, int32_t* error_flag,
+    hipStream_t stream) {
     if (num_tiles == 0) return 0;
     if (chunk < 0) return nva_fail("paged_attention_tiled: negative chunk");
     if (head_dim <= 0 || head_dim > ATT_TILED_MAX_D || v_dim <= 0 || v_dim > ATT_TILED_MAX_D) {
@@ -483,7 +489,7 @@ NVA_EXPORT int NVA_NAME(nva_paged_attention_tiled)(
     hipLaunchKernelGGL(kernel, grid, dim3(ATT_TILED_WAVES * NVA_WAVE), lds, stream, (const elem_t*)q, q_stride,
                        (elem_t*)out, out_stride, (const elem_t*)k_cache, (const elem_t*)v_cache, block_tables,
                        table_stride, cu_seqlens_q, kv_lens, tiles, num_q_heads, num_kv_heads, head_dim, v_dim,
-                       page_size, scale, chunk, softcap, sinks, error_flag);
+                       page_size, scale, chunk, softcap, sinks, head_gate, error_flag);
     return nva_check_launch("paged_attention_tiled");
 }
 
@@ -491,8 +497,8 @@ NVA_EXPORT int NVA_NAME(nva_paged_attention_generic)(
     const void* q, int64_t q_stride, void* out, int64_t out_stride, const void* k_cache, const void* v_cache,
     const int32_t* block_tables, int table_stride, const int32_t* token_seq, const int32_t* positions,
     int64_t tokens, int num_q_heads, int num_kv_heads, int head_dim, int v_dim, int page_size, float scale,
-    int window, int chunk, int keep_first, float softcap, const float* sinks, const float* sig_bias, float* part, int shares,
-    int32_t* error_flag, hipStream_t stream) {
+    int window, int chunk, int keep_first, float softcap, const float* sinks, const float* sig_bias, const float* head_gate, float* part,
+    int shares,    int32_t* error_flag, hipStream_t stream) {
     if (tokens == 0) return 0;
     if (tokens < 0 || tokens > 0x7fffffff) return nva_fail("paged_attention: bad token count %lld", (long long)tokens);
     if (shares < 1 || shares > 64 || (shares > 1 && !part))
@@ -508,11 +514,11 @@ NVA_EXPORT int NVA_NAME(nva_paged_attention_generic)(
     hipLaunchKernelGGL(paged_attention_generic_kernel<elem_t>, grid, dim3(NVA_WAVE), 0, stream, (const elem_t*)q,
                        q_stride, (elem_t*)out, out_stride, (const elem_t*)k_cache, (const elem_t*)v_cache,
                        block_tables, table_stride, token_seq, positions, num_q_heads, num_kv_heads, head_dim,
-                       v_dim, page_size, scale, window, chunk, keep_first, softcap, sinks, sig_bias,
+                       v_dim, page_size, scale, window, chunk, keep_first, softcap, sinks, sig_bias, head_gate,
                        shares > 1 ? part : nullptr, error_flag);
     if (shares > 1)
         hipLaunchKernelGGL(paged_attention_merge_kernel<elem_t>, dim3((unsigned)tokens, (unsigned)num_q_heads), dim3(NVA_WAVE), 0,
-                           stream, part, shares, (elem_t*)out, out_stride, num_q_heads, v_dim);
+                           stream, part, shares, (elem_t*)out, out_stride, num_q_heads, v_dim, head_gate);
     return nva_check_launch("paged_attention_generic");
 }
 

@@ -95,7 +95,8 @@ attn_prefill_kernel(const __bf16* __restrict__ q, int64_t q_stride, __bf16* __re
                     const int32_t* __restrict__ cu_seqlens_q, const int32_t* __restrict__ kv_lens,
                     const int32_t* __restrict__ tiles, int num_tiles, int paired, int num_q_heads, int num_kv_heads,
                     int page_size, float scale, int window, int key_chunk, int keep_first, float softcap,
-                    const float* __restrict__ sinks, const float* __restrict__ sig_bias, int32_t* error_flag) {
+                    const float* __restrict__ sinks, const float* __restrict__ sig_bias,
+                    const float* __restrict__ head_gate, int32_t* error_flag) {
     constexpr int DC = D / 16;            // 16-channel steps of the first product
     constexpr int MT = D / 32;            // 32-channel tiles of the output
     constexpr int KR = D / 8;             // 16-byte pieces of a K row (one key)
@@ -565,7 +566,8 @@ attn_prefill_kernel(const __bf16* __restrict__ q, int64_t q_stride, __bf16* __re
     // a sink: one more term exp(sink) in the denominator (a key without a value), in the units of the
     // running maximum; it joins once, after the tiles (and after the sets of waves have met)
     if (sinks) l_run += __builtin_amdgcn_exp2f(sinks[head] * 1.4426950408889634f - fmaxf(m_run, -1e30f) * c_exp);
-    const float inv = sig_bias ? 1.f : l_run > 0.f ? 1.f / l_run : 0.f;
+    float inv = sig_bias ? 1.f : l_run > 0.f ? 1.f / l_run : 0.f;
+    if (head_gate) inv *= head_gate[(int64_t)(q_begin + row) * num_q_heads + head];
     __bf16* orow = out + (int64_t)(q_begin + row) * out_stride + (int64_t)head * D;
 #pragma unroll
     for (int mt = 0; mt < MT; ++mt)
@@ -582,6 +584,7 @@ attn_prefill_kernel(const __bf16* __restrict__ q, int64_t q_stride, __bf16* __re
 // portions, ordered from the most visible keys to the fewest (the caller builds it once per step).
 // nva_attn_prefill_sets (-1, 1 or 2) fixes the sets of waves per workgroup for tests; -1 leaves the choice
 // to the launcher.
+// head_gate, float [tokens of the step, heads] or null: a head's output is multiplied by its token's number as it is written.
 // Refuses (non-zero code and a message) shapes this kernel does not take.
 static int forced_sets = -1;
 NVA_EXPORT void nva_attn_prefill_sets(int sets) { forced_sets = sets; }
@@ -591,7 +594,7 @@ NVA_EXPORT int nva_attn_prefill_bf16(const void* q, int64_t q_stride, void* out,
                                      int table_stride, const int32_t* cu_seqlens_q, const int32_t* kv_lens,
                                      const int32_t* tiles, int64_t num_tiles, int num_q_heads,
                                      int num_kv_heads, int head_dim, int page_size, float scale, int window, int chunk,
-                                     int keep_first, float softcap, const float* sinks, const float* sig_bias,
+                                     int keep_first, float softcap, const float* sinks, const float* sig_bias, const float* head_gate,
                                      int32_t* error_flag, hipStream_t stream) {
     if (num_tiles == 0) return 0;
     if (num_q_heads <= 0 || num_kv_heads <= 0 || num_q_heads % num_kv_heads)
@@ -635,7 +638,7 @@ NVA_EXPORT int nva_attn_prefill_bf16(const void* q, int64_t q_stride, void* out,
                        (const __bf16*)q, q_stride, (__bf16*)out, out_stride, (const __bf16*)k_cache,                 \
                        (const __bf16*)v_cache, block_tables, table_stride, cu_seqlens_q, kv_lens, tiles,             \
                        (int)num_tiles, SS == 1 && PF_WAVES_PER_SIMD(DD) == 2 && total <= 2 * cus ? (int)total : 0,   \
-                       num_q_heads, num_kv_heads, page_size, scale, window, chunk, keep_first, softcap, sinks, sig_bias, error_flag)
+                       num_q_heads, num_kv_heads, page_size, scale, window, chunk, keep_first, softcap, sinks, sig_bias, head_gate, error_flag)
 #define LAUNCH(DD)                                                                                                 \
     do {                                                                                                           \
         if (PF_WAVES_PER_SIMD(DD) == 2 && two_sets) LAUNCH_SETS(DD, PF_WAVES_PER_SIMD(DD));                         \

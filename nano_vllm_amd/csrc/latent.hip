@@ -7,22 +7,46 @@
 // row), the query of head h becomes [Wuk_h^T q_plain_h | q_turned_h], the attention runs with one key/value
 // head of C + R and C entries, and a head's output is Wuv_h applied to what the attention gives.
 //
+// Where the queries go through a latent of their own, what latent_prepare does is two kernels with the product
+// W_uq c_q between them:
+//   latent_down      row = [cq_raw (Q) | c_raw (C) | kr_raw (R) | g (one per head, or none)] of a token: cq and c normed by
+//                    weights of their own, kr rotated, the store as above, the gates' sigmoids as floats; the row may come as
+//                    the partial sums of a split product
+//   latent_queries   the turned part of every head's query rotated into place (and, from partial sums, its plain part
+//                    written out)
+// The rotation pairs neighbours (2i, 2i + 1), or (i, i + R/2) where `interleaved` is 0.  A window (window > 0): a query at
+// position p reads the keys of positions > p - window only.
+//
 //   latent_prepare   row = [q (H heads of [D plain | R turned]) | c_raw (C) | kr_raw (R)] of a token:
-//                    c = c_raw / sqrt(mean(c_raw^2) + eps) * w;  kr and every head's turned part rotated in pairs of
-//                    neighbours (2i, 2i + 1) by the token's row of the step's table (R/2 cosines, then R/2 sines);
+//                    c = c_raw / sqrt(mean(c_raw^2) + eps) * w;  kr and every head's turned part rotated in pairs
+//                    by the token's row of the step's table (R/2 cosines, then R/2 sines);
 //                    cache K <- [c | kr], cache V <- c at the token's slot; q2[t, h, C : C + R] <- the head's turned part.
 //                    Sums, scale and rotation float; each output rounded once to the element type.
 //   heads_linear     y[t, h, n] = sum_k W[h, n, k] x[t, h, k] for every head by itself, with strides for all three:
 //                    the plain parts of q into the latent's space (W read as [h, k, n]) and the attention's output
-//                    out of it.  A float sum over k in ascending order per output, rounded once.
+//                    out of it.  A float sum over k in ascending order per output (times the head's gate, where one is
+//                    given), rounded once.
 #include "common.h"
+
+// Entry d of a turned part whose raw entries raw(0) ... raw(rot - 1) are given, by a row of rot / 2 cosines and rot / 2 sines.
+template <typename F>
+__device__ __forceinline__ float latent_turned(F raw, const float* __restrict__ rot_row, int d, int rot, int interleaved) {
+    const int half = rot / 2;
+    if (interleaved) {
+        const float x = raw(d), y = raw(d ^ 1), c = rot_row[d >> 1], sn = rot_row[half + (d >> 1)];
+        return (d & 1) ? x * c + y * sn : x * c - y * sn;
+    }
+    const bool first = d < half;
+    const float x = raw(d), y = raw(first ? d + half : d - half), c = rot_row[first ? d : d - half], sn = rot_row[first ? half + d : d];
+    return first ? x * c - y * sn : x * c + y * sn;
+}
 
 template <typename T>
 __global__ void __launch_bounds__(256)
 latent_prepare_kernel(const T* __restrict__ proj, int64_t stride, int heads, int dim, int rot, int rank,
                       const void* __restrict__ weight, int w_is_f32, float eps, const float* __restrict__ rot_table,
                       T* __restrict__ q2, int64_t q2_stride, const int32_t* __restrict__ slots,
-                      T* __restrict__ k_cache, T* __restrict__ v_cache, int page_size) {
+                      T* __restrict__ k_cache, T* __restrict__ v_cache, int page_size, int interleaved) {
     __shared__ float scratch[16];
     const int64_t t = blockIdx.x;
     const int tid = threadIdx.x;
@@ -30,12 +54,9 @@ latent_prepare_kernel(const T* __restrict__ proj, int64_t stride, int heads, int
     const int qd = heads * (dim + rot);
     const int slot = slots ? slots[t] : -1;
     const float* rot_row = rot_table + t * (int64_t)rot;
-    const int half = rot / 2;
     // a turned entry d of a part that starts at `at` in the row
     auto turned = [&](int at, int d) -> float {
-        const float x = to_float(row[at + d]), y = to_float(row[at + (d ^ 1)]);
-        const float c = rot_row[d >> 1], sn = rot_row[half + (d >> 1)];
-        return (d & 1) ? x * c + y * sn : x * c - y * sn;
+        return latent_turned([&](int i) { return to_float(row[at + i]); }, rot_row, d, rot, interleaved);
     };
     for (int i = tid; i < heads * rot; i += blockDim.x) {
         const int h = i / rot, d = i % rot;
@@ -68,7 +89,7 @@ latent_prepare_kernel(const T* __restrict__ proj, int64_t stride, int heads, int
 NVA_EXPORT int NVA_NAME(nva_latent_prepare)(const void* proj, int64_t stride, int64_t tokens, int heads, int dim, int rot,
                                             int rank, const void* weight, int w_is_f32, float eps, const float* rot_table,
                                             void* q2, int64_t q2_stride, const int32_t* slots, void* k_cache,
-                                            void* v_cache, int page_size, hipStream_t stream) {
+                                            void* v_cache, int page_size, int interleaved, hipStream_t stream) {
     if (tokens == 0) return 0;
     if (tokens < 0 || tokens > 0x7fffffff) return nva_fail("latent_prepare: bad token count %lld", (long long)tokens);
     if (heads <= 0 || dim <= 0 || rot <= 0 || rot % 2 || rank <= 0)
@@ -80,8 +101,130 @@ NVA_EXPORT int NVA_NAME(nva_latent_prepare)(const void* proj, int64_t stride, in
         return nva_fail("latent_prepare: storing needs both caches, the slots and the page size");
     hipLaunchKernelGGL(latent_prepare_kernel<elem_t>, dim3((unsigned)tokens), dim3(256), 0, stream, (const elem_t*)proj,
                        stride, heads, dim, rot, rank, weight, w_is_f32, eps, rot_table, (elem_t*)q2, q2_stride, slots,
-                       (elem_t*)k_cache, (elem_t*)v_cache, page_size);
+                       (elem_t*)k_cache, (elem_t*)v_cache, page_size, interleaved ? 1 : 0);
     return nva_check_launch("latent_prepare");
+}
+
+// One workgroup a token; the row lies in LDS as floats.
+template <typename T>
+__global__ void __launch_bounds__(1024)
+latent_down_kernel(const T* __restrict__ low, int64_t stride, PartialInput part, int q_rank, int rank, int rot, int gates,
+                   const void* __restrict__ q_weight, const void* __restrict__ weight, int w_is_f32, float eps,
+                   const float* __restrict__ rot_table, T* __restrict__ cq, float* __restrict__ gate_out,
+                   const int32_t* __restrict__ slots, T* __restrict__ k_cache, T* __restrict__ v_cache, int page_size,
+                   int interleaved) {
+    extern __shared__ __attribute__((aligned(16))) float row_s[];
+    __shared__ float scratch[16];
+    const int64_t t = blockIdx.x;
+    const int tid = threadIdx.x;
+    const int width = q_rank + rank + rot + gates;
+    const int slot = slots ? slots[t] : -1;
+    float sq = 0.f, sc = 0.f;
+    for (int i = tid; i < width; i += blockDim.x) {
+        const float x = part.sums ? partial_value<T>(part, t, width, i) : to_float(low[t * stride + i]);
+        row_s[i] = x;
+        if (i < q_rank) sq += x * x; else if (i < q_rank + rank) sc += x * x;
+    }
+    sq = block_sum(sq, scratch);
+    sc = block_sum(sc, scratch);
+    const float q_scale = rsqrtf(sq / (float)q_rank + eps), c_scale = rsqrtf(sc / (float)rank + eps);
+    auto weight_of = [&](const void* w, int i) -> float {
+        return w_is_f32 ? static_cast<const float*>(w)[i] : to_float(static_cast<const T*>(w)[i]);
+    };
+    for (int i = tid; i < q_rank; i += blockDim.x) cq[t * q_rank + i] = from_float<T>(row_s[i] * q_scale * weight_of(q_weight, i));
+    for (int i = tid; i < gates; i += blockDim.x) gate_out[t * gates + i] = 1.f / (1.f + expf(-row_s[q_rank + rank + rot + i]));
+    if (slot < 0 || !k_cache) return;
+    const int page = slot / page_size, off = slot % page_size;
+    const int vt = nva_v_tile(page_size);
+    T* krow = k_cache + ((int64_t)page * page_size + off) * (rank + rot);
+    T* vpage = v_cache + (int64_t)page * rank * page_size;
+    for (int i = tid; i < rank; i += blockDim.x) {
+        const T c = from_float<T>(row_s[q_rank + i] * c_scale * weight_of(weight, i));
+        krow[i] = c;
+        vpage[nva_v_offset(off, i, rank, vt)] = c;
+    }
+    const float* rot_row = rot_table + t * (int64_t)rot;
+    for (int d = tid; d < rot; d += blockDim.x)
+        krow[rank + d] = from_float<T>(latent_turned([&](int i) { return row_s[q_rank + rank + i]; }, rot_row, d, rot, interleaved));
+}
+
+// low: elements [tokens, Q + C + R + gates] with rows `stride` apart, or (sums != null) partial sums
+// [splits][tokens][Q + C + R + gates].  q_weight [Q], weight [C] (both float or both elements); rot_table float [tokens, R];
+// cq [tokens, Q] elements; gate_out float [tokens, gates] (gates may be 0); the caches as for nva_latent_prepare.
+NVA_EXPORT int NVA_NAME(nva_latent_down)(const void* low, int64_t stride, const float* sums, int splits, int64_t split_stride,
+                                         int64_t tokens, int q_rank, int rank, int rot, int gates, const void* q_weight,
+                                         const void* weight, int w_is_f32, float eps, const float* rot_table, void* cq,
+                                         float* gate_out, const int32_t* slots, void* k_cache, void* v_cache, int page_size,
+                                         int interleaved, hipStream_t stream) {
+    if (tokens == 0) return 0;
+    if (tokens < 0 || tokens > 0x7fffffff) return nva_fail("latent_down: bad token count %lld", (long long)tokens);
+    const int64_t width = (int64_t)q_rank + rank + rot + gates;
+    if (q_rank <= 0 || rank <= 0 || rot <= 0 || rot % 2 || gates < 0 || width > 36 * 1024)
+        return nva_fail("latent_down: bad sizes q_rank=%d rank=%d rot=%d gates=%d", q_rank, rank, rot, gates);
+    if ((!sums && (!low || stride < width)) || (sums && (splits <= 0 || split_stride < tokens * width)) || !q_weight || !weight ||
+        !rot_table || !cq || (gates && !gate_out))
+        return nva_fail("latent_down: a tensor is missing or too narrow");
+    if ((k_cache || v_cache) && (!k_cache || !v_cache || !slots || page_size <= 0))
+        return nva_fail("latent_down: storing needs both caches, the slots and the page size");
+    auto kernel = latent_down_kernel<elem_t>;
+    const size_t lds = (size_t)width * sizeof(float);
+    static bool raised = false;
+    if (!raised && lds > 48 * 1024) {
+        if (hipFuncSetAttribute((const void*)kernel, hipFuncAttributeMaxDynamicSharedMemorySize, 150 * 1024) != hipSuccess)
+            return nva_fail("latent_down: cannot have %zu bytes of LDS", lds);
+        raised = true;
+    }
+    const PartialInput part{sums, splits, split_stride, nullptr};
+    const int threads = sums && tokens <= 64 && width >= 1024 ? 1024 : 256;
+    hipLaunchKernelGGL(kernel, dim3((unsigned)tokens), dim3(threads), lds, stream, (const elem_t*)low, stride, part, q_rank, rank,
+                       rot, gates, q_weight, weight, w_is_f32, eps, rot_table, (elem_t*)cq, gate_out, slots, (elem_t*)k_cache,
+                       (elem_t*)v_cache, page_size, interleaved ? 1 : 0);
+    return nva_check_launch("latent_down");
+}
+
+// A thread an entry: of all the queries' entries where they come as partial sums, of the turned ones where they are elements.
+template <typename T>
+__global__ void __launch_bounds__(256)
+latent_queries_kernel(const T* __restrict__ q, int64_t stride, PartialInput part, int heads, int dim, int rot, int rank,
+                      const float* __restrict__ rot_table, T* __restrict__ q2, T* __restrict__ q_plain, int interleaved) {
+    const int64_t t = blockIdx.y;
+    const int i = blockIdx.x * blockDim.x + threadIdx.x;
+    const int per = part.sums ? dim + rot : rot;
+    if (i >= heads * per) return;
+    const int h = i / per;
+    const int d = part.sums ? i % per - dim : i % per;                  // of the turned part; below 0: a plain entry
+    const int at = h * (dim + rot) + dim, width = heads * (dim + rot);
+    if (d < 0) {
+        q_plain[(t * heads + h) * dim + dim + d] = from_float<T>(partial_value<T>(part, t, width, at + d));
+        return;
+    }
+    const float v = latent_turned(
+        [&](int e) { return part.sums ? partial_value<T>(part, t, width, at + e) : to_float(q[t * stride + at + e]); },
+        rot_table + t * (int64_t)rot, d, rot, interleaved);
+    q2[(t * heads + h) * (int64_t)(rank + rot) + rank + d] = from_float<T>(v);
+}
+
+// q: elements [tokens, heads * (dim + rot)] with rows `stride` apart, or (sums != null) partial sums; q2 [tokens, heads *
+// (rank + rot)]: every head's last rot entries are written; q_plain [tokens, heads * dim], written from partial sums only.
+NVA_EXPORT int NVA_NAME(nva_latent_queries)(const void* q, int64_t stride, const float* sums, int splits, int64_t split_stride,
+                                            int64_t tokens, int heads, int dim, int rot, int rank, const float* rot_table,
+                                            void* q2, void* q_plain, int interleaved, hipStream_t stream) {
+    if (tokens == 0) return 0;
+    if (tokens < 0 || heads <= 0 || dim <= 0 || rot <= 0 || rot % 2 || rank <= 0 || (int64_t)heads * (dim + rot) > 0x3fffffff)
+        return nva_fail("latent_queries: bad sizes tokens=%lld heads=%d dim=%d rot=%d rank=%d", (long long)tokens, heads, dim, rot, rank);
+    const int64_t width = (int64_t)heads * (dim + rot);
+    if ((!sums && (!q || stride < width)) || (sums && (splits <= 0 || split_stride < tokens * width || !q_plain)) || !rot_table || !q2)
+        return nva_fail("latent_queries: a tensor is missing or too narrow");
+    const int per = sums ? dim + rot : rot;
+    for (int64_t t0 = 0; t0 < tokens; t0 += 65535) {
+        const unsigned n = (unsigned)(tokens - t0 < 65535 ? tokens - t0 : 65535);
+        const PartialInput part{sums ? sums + t0 * width : nullptr, splits, split_stride, nullptr};
+        hipLaunchKernelGGL(latent_queries_kernel<elem_t>, dim3((unsigned)((heads * per + 255) / 256), n), dim3(256), 0, stream,
+                           sums ? nullptr : (const elem_t*)q + t0 * stride, stride, part, heads, dim, rot, rank,
+                           rot_table + t0 * rot, (elem_t*)q2 + t0 * heads * (int64_t)(rank + rot),
+                           q_plain ? (elem_t*)q_plain + t0 * heads * (int64_t)dim : nullptr, interleaved ? 1 : 0);
+    }
+    return nva_check_launch("latent_queries");
 }
 
 #define HL_TOKENS 16        // tokens of a workgroup
@@ -92,7 +235,7 @@ template <typename T>
 __global__ void __launch_bounds__(256)
 heads_linear_kernel(const T* __restrict__ x, int64_t x_stride, int64_t x_head, const T* __restrict__ w, int64_t w_head,
                     int64_t w_n, int64_t w_k, T* __restrict__ y, int64_t y_stride, int64_t y_head, int64_t tokens,
-                    int n_out, int k_in) {
+                    int n_out, int k_in, const float* __restrict__ head_gate) {
     extern __shared__ __attribute__((aligned(16))) float x_s[];       // [HL_TOKENS][k_in]
     const int64_t t0 = (int64_t)blockIdx.x * HL_TOKENS;
     const int h = blockIdx.y;
@@ -125,15 +268,17 @@ heads_linear_kernel(const T* __restrict__ x, int64_t x_stride, int64_t x_head, c
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
         const int64_t t = t0 + wave * 4 + r;
-        if (t < tokens) y[t * y_stride + h * y_head + n] = from_float<T>(acc[r]);
+        if (t < tokens) y[t * y_stride + h * y_head + n] = from_float<T>(head_gate ? acc[r] * head_gate[t * gridDim.y + h] : acc[r]);
     }
 }
 
 // x: head h of token t starts at x + t * x_stride + h * x_head (k_in entries side by side); w: W[h, n, k] at
-// w + h * w_head + n * w_n + k * w_k; y: head h of token t at y + t * y_stride + h * y_head (n_out entries).
+// w + h * w_head + n * w_n + k * w_k; y: head h of token t at y + t * y_stride + h * y_head (n_out entries).  head_gate, float
+// [tokens, heads] or null: head h's outputs are multiplied by its token's number before they are rounded.
 NVA_EXPORT int NVA_NAME(nva_heads_linear)(const void* x, int64_t x_stride, int64_t x_head, const void* w, int64_t w_head,
                                           int64_t w_n, int64_t w_k, void* y, int64_t y_stride, int64_t y_head,
-                                          int64_t tokens, int heads, int n_out, int k_in, hipStream_t stream) {
+                                          int64_t tokens, int heads, int n_out, int k_in, const float* head_gate,
+                                          hipStream_t stream) {
     if (tokens == 0) return 0;
     if (tokens < 0 || tokens > 0x7fffffff || heads <= 0 || heads > 65535 || n_out <= 0 || k_in <= 0 || k_in > HL_MAX_K)
         return nva_fail("heads_linear: bad sizes tokens=%lld heads=%d outputs=%d inputs=%d (up to %d)", (long long)tokens,
@@ -150,7 +295,7 @@ NVA_EXPORT int NVA_NAME(nva_heads_linear)(const void* x, int64_t x_stride, int64
     const int64_t groups = (tokens + HL_TOKENS - 1) / HL_TOKENS;
     dim3 grid((unsigned)groups, (unsigned)heads, (unsigned)((n_out + NVA_WAVE - 1) / NVA_WAVE));
     hipLaunchKernelGGL(kernel, grid, dim3(256), lds, stream, (const elem_t*)x, x_stride, x_head, (const elem_t*)w, w_head,
-                       w_n, w_k, (elem_t*)y, y_stride, y_head, tokens, n_out, k_in);
+                       w_n, w_k, (elem_t*)y, y_stride, y_head, tokens, n_out, k_in, head_gate);
     return nva_check_launch("heads_linear");
 }
 
@@ -165,7 +310,8 @@ typedef __attribute__((ext_vector_type(4))) float hl_f32x4;
 
 __global__ void __launch_bounds__(NVA_WAVE)
 heads_linear_mfma_kernel(const __bf16* __restrict__ x, int64_t x_stride, int64_t x_head, const __bf16* __restrict__ w,
-                         __bf16* __restrict__ y, int64_t y_stride, int64_t y_head, int64_t tokens, int n_out, int k_in) {
+                         __bf16* __restrict__ y, int64_t y_stride, int64_t y_head, int64_t tokens, int n_out, int k_in,
+                         const float* __restrict__ head_gate) {
     const int64_t t0 = (int64_t)blockIdx.x * 16;
     const int h = blockIdx.y, n0 = blockIdx.z * 64;
     const int lane = threadIdx.x, col = lane & 15, g = lane >> 4;
@@ -196,12 +342,13 @@ heads_linear_mfma_kernel(const __bf16* __restrict__ x, int64_t x_stride, int64_t
     // acc[b][i] = y[token col][n0 + 16 b + 4 g + i]
     if (t >= tokens) return;
     __bf16* yr = y + t * y_stride + h * y_head;
+    const float gate = head_gate ? head_gate[t * gridDim.y + h] : 1.f;
 #pragma unroll
     for (int b = 0; b < 4; ++b)
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
             const int n = n0 + 16 * b + 4 * g + i;
-            if (n < n_out) yr[n] = (__bf16)acc[b][i];
+            if (n < n_out) yr[n] = (__bf16)(acc[b][i] * gate);
         }
 }
 
@@ -209,7 +356,7 @@ heads_linear_mfma_kernel(const __bf16* __restrict__ x, int64_t x_stride, int64_t
 // shapes it does not take: k_in a multiple of 8, x rows and heads at multiples of 8 elements, 16-byte aligned pointers.
 NVA_EXPORT int nva_heads_linear_mfma_bf16(const void* x, int64_t x_stride, int64_t x_head, const void* w, void* y,
                                           int64_t y_stride, int64_t y_head, int64_t tokens, int heads, int n_out, int k_in,
-                                          hipStream_t stream) {
+                                          const float* head_gate, hipStream_t stream) {
     if (tokens == 0) return 0;
     if (k_in % 8 || k_in <= 0 || x_stride % 8 || x_head % 8 || !nva_aligned(x, 16) || !nva_aligned(w, 16)) {
         nva_fail("heads_linear_mfma: rows that are not aligned for 16-byte loads (k_in %d)", k_in);
@@ -220,7 +367,7 @@ NVA_EXPORT int nva_heads_linear_mfma_bf16(const void* x, int64_t x_stride, int64
         return nva_fail("heads_linear_mfma: bad sizes tokens=%lld heads=%d outputs=%d", (long long)tokens, heads, n_out);
     dim3 grid((unsigned)((tokens + 15) / 16), (unsigned)heads, (unsigned)((n_out + 63) / 64));
     hipLaunchKernelGGL(heads_linear_mfma_kernel, grid, dim3(NVA_WAVE), 0, stream, (const __bf16*)x, x_stride, x_head,
-                       (const __bf16*)w, (__bf16*)y, y_stride, y_head, tokens, n_out, k_in);
+                       (const __bf16*)w, (__bf16*)y, y_stride, y_head, tokens, n_out, k_in, head_gate);
     return nva_check_launch("heads_linear_mfma");
 }
 
@@ -247,7 +394,7 @@ __global__ void __launch_bounds__(NVA_WAVE)
 latent_attn_kernel(const __bf16* __restrict__ q2, int64_t q_stride, __bf16* __restrict__ out, int64_t out_stride,
                    float* __restrict__ part, const __bf16* __restrict__ k_cache, const __bf16* __restrict__ v_cache,
                    const int32_t* __restrict__ block_tables, int table_stride, const int32_t* __restrict__ token_seq,
-                   const int32_t* __restrict__ positions, int heads, int rank, int rot, int page_size, float scale,
+                   const int32_t* __restrict__ positions, int heads, int rank, int rot, int page_size, float scale, int window,
                    const float* __restrict__ sinks, int32_t* error_flag) {
     constexpr int KS = (MAXC + LAT_MAX_ROT) / 32;      // steps of 32 channels of the first product, at most
     constexpr int CB = MAXC / 16;                      // blocks of 16 latent channels of the output, at most
@@ -262,9 +409,10 @@ latent_attn_kernel(const __bf16* __restrict__ q2, int64_t q_stride, __bf16* __re
     const int steps = (width + 31) / 32, blocks = rank / 16;
     const int pos = positions[t];
     const int32_t* table = block_tables + (int64_t)token_seq[t] * table_stride;
-    const int tiles = pos / LAT_TILE + 1;
-    const int per = (tiles + shares - 1) / shares;
-    const int tile_lo = share * per, tile_hi = min(tiles, tile_lo + per);
+    const int first = nva_first_key(pos, window, 0);
+    const int tile_0 = first / LAT_TILE, tiles = pos / LAT_TILE + 1;                      // of the keys it sees
+    const int per = (tiles - tile_0 + shares - 1) / shares;
+    const int tile_lo = tile_0 + share * per, tile_hi = min(tiles, tile_lo + per);
 
     lat_bf16x8 qf[KS];
     const __bf16* qrow = q2 + t * q_stride + (int64_t)(head_ok ? head : 0) * width;
@@ -329,7 +477,7 @@ latent_attn_kernel(const __bf16* __restrict__ q2, int64_t q_stride, __bf16* __re
         for (int i = 0; i < 8; ++i) {
             const int key = kb + (i < 4 ? 4 * g + i : 16 + 4 * g + i - 4);
             const float raw = (i < 4 ? sa[i] : sb[i - 4]) * scale;
-            s[i] = key <= pos && !no_page ? raw : -INFINITY;
+            s[i] = key <= pos && key >= first && !no_page ? raw : -INFINITY;
             m_new = fmaxf(m_new, s[i]);
         }
         m_new = nva_max_over_rows(m_new);
@@ -347,17 +495,19 @@ latent_attn_kernel(const __bf16* __restrict__ q2, int64_t q_stride, __bf16* __re
         l_run = l_run * alpha + psum;
         m_run = m_new;
         // ---- O^T += V^T P^T: channel 16 b + col, keys kb + 4 g .. + 3 and kb + 16 + 4 g .. + 3
-        const bool whole = kb + LAT_TILE - 1 <= pos && !no_page;
+        const bool whole = kb + LAT_TILE - 1 <= pos && kb >= first && !no_page;
 #pragma unroll
         for (int b = 0; b < CB; ++b) {
             if (b < blocks) {
                 lat_bf16x8 vf;
 #pragma unroll
                 for (int e = 0; e < 4; ++e) vf[e] = vlo[b][e], vf[4 + e] = vhi[b][e];
-                if (!whole) {              // what the cache holds beyond the token's own key may be anything
+                if (!whole) {              // what the cache holds beyond the token's own key, or before its window, may be anything
 #pragma unroll
-                    for (int e = 0; e < 8; ++e)
-                        if (no_page || kb + (e < 4 ? 4 * g + e : 16 + 4 * g + e - 4) > pos) vf[e] = (__bf16)0.f;
+                    for (int e = 0; e < 8; ++e) {
+                        const int key = kb + (e < 4 ? 4 * g + e : 16 + 4 * g + e - 4);
+                        if (no_page || key > pos || key < first) vf[e] = (__bf16)0.f;
+                    }
                 }
                 lat_f32x4 a = acc[b];
                 a[0] *= alpha; a[1] *= alpha; a[2] *= alpha; a[3] *= alpha;
@@ -402,7 +552,7 @@ latent_attn_quad_kernel(const __bf16* __restrict__ q2, int64_t q_stride, __bf16*
                         const __bf16* __restrict__ k_cache, const __bf16* __restrict__ v_cache,
                         const int32_t* __restrict__ block_tables, int table_stride, const int32_t* __restrict__ cu_seqlens_q,
                         const int32_t* __restrict__ kv_lens, const int32_t* __restrict__ row_tiles, int heads, int rank, int rot,
-                        int page_size, float scale, const float* __restrict__ sinks, int32_t* error_flag) {
+                        int page_size, float scale, int window, const float* __restrict__ sinks, int32_t* error_flag) {
     constexpr int KS = (MAXC + LAT_MAX_ROT) / 32, CB = MAXC / 16;
     constexpr int THREADS = WAVES * NVA_WAVE, PER_TILE = 32 / WAVES;   // tokens of a workgroup: WAVES; workgroups of a row tile
     constexpr int KP = (4 * (MAXC + LAT_MAX_ROT) + THREADS - 1) / THREADS, VP = (4 * MAXC + THREADS - 1) / THREADS;   // 16-byte pieces of a tile a thread moves, at most
@@ -422,6 +572,9 @@ latent_attn_quad_kernel(const __bf16* __restrict__ q2, int64_t q_stride, __bf16*
     const bool token_ok = row < q_len;
     const int pos = token_ok ? start + row : -1;
     const int64_t t = q_begin + (token_ok ? row : row0);
+    const int first = nva_first_key(pos, window, 0);
+    // the tiles that any token of the workgroup sees: the first token's window starts first
+    const int tile_0 = nva_first_key(start + row0, window, 0) / LAT_TILE;
     const int tiles = (start + min(row0 + WAVES - 1, q_len - 1)) / LAT_TILE + 1;
     const int head = blockIdx.z * 16 + col;
     const bool head_ok = head < heads;
@@ -490,14 +643,14 @@ latent_attn_quad_kernel(const __bf16* __restrict__ q2, int64_t q_stride, __bf16*
             }
         }
     };
-    ask(0);
-    for (int tile = 0; tile < tiles; ++tile) {
+    ask(tile_0);
+    for (int tile = tile_0; tile < tiles; ++tile) {
         const int kb = tile * LAT_TILE;
         put();
         no_page = no_page_next;
         __syncthreads();
         if (tile + 1 < tiles) ask(tile + 1);
-        if (kb <= pos) {                                    // (the same for the whole wave)
+        if (kb <= pos && kb + LAT_TILE > first) {           // (the same for the whole wave)
             lat_f32x4 sa = {0.f, 0.f, 0.f, 0.f}, sb = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
             for (int c = 0; c < KS; ++c) {
@@ -519,7 +672,7 @@ latent_attn_quad_kernel(const __bf16* __restrict__ q2, int64_t q_stride, __bf16*
             for (int i = 0; i < 8; ++i) {
                 const int key = kb + (i < 4 ? 4 * g + i : 16 + 4 * g + i - 4);
                 const float raw = (i < 4 ? sa[i] : sb[i - 4]) * scale;
-                s[i] = key <= pos && !no_page ? raw : -INFINITY;
+                s[i] = key <= pos && key >= first && !no_page ? raw : -INFINITY;
                 m_new = fmaxf(m_new, s[i]);
             }
             m_new = nva_max_over_rows(m_new);
@@ -536,7 +689,7 @@ latent_attn_quad_kernel(const __bf16* __restrict__ q2, int64_t q_stride, __bf16*
             const float alpha = __builtin_amdgcn_exp2f((fmaxf(m_run, -1e30f) - m_use) * log2e);
             l_run = l_run * alpha + psum;
             m_run = m_new;
-            const bool whole = kb + LAT_TILE - 1 <= pos && !no_page;
+            const bool whole = kb + LAT_TILE - 1 <= pos && kb >= first && !no_page;
 #pragma unroll
             for (int b = 0; b < CB; ++b) {
                 if (b < blocks) {
@@ -547,8 +700,10 @@ latent_attn_quad_kernel(const __bf16* __restrict__ q2, int64_t q_stride, __bf16*
                     for (int e = 0; e < 4; ++e) vf[e] = lo[e], vf[4 + e] = hi[e];
                     if (!whole) {
 #pragma unroll
-                        for (int e = 0; e < 8; ++e)
-                            if (no_page || kb + (e < 4 ? 4 * g + e : 16 + 4 * g + e - 4) > pos) vf[e] = (__bf16)0.f;
+                        for (int e = 0; e < 8; ++e) {
+                            const int key = kb + (e < 4 ? 4 * g + e : 16 + 4 * g + e - 4);
+                            if (no_page || key > pos || key < first) vf[e] = (__bf16)0.f;
+                        }
                     }
                     lat_f32x4 a = acc[b];
                     a[0] *= alpha; a[1] *= alpha; a[2] *= alpha; a[3] *= alpha;
@@ -618,7 +773,7 @@ NVA_EXPORT int nva_latent_attention_bf16(const void* q2, int64_t q_stride, void*
                                          int shares, const void* k_cache, const void* v_cache,
                                          const int32_t* block_tables, int table_stride, const int32_t* token_seq,
                                          const int32_t* positions, int64_t tokens, int heads, int rank, int rot,
-                                         int page_size, float scale, const float* sinks, int32_t* error_flag,
+                                         int page_size, float scale, int window, const float* sinks, int32_t* error_flag,
                                          hipStream_t stream) {
     if (tokens == 0) return 0;
     if (rank % 16 || rank <= 0 || rank > 512 || rot % 8 || rot <= 0 || rot > LAT_MAX_ROT || page_size % LAT_TILE || page_size <= 0) {
@@ -627,7 +782,7 @@ NVA_EXPORT int nva_latent_attention_bf16(const void* q2, int64_t q_stride, void*
         return 1;
     }
     if (tokens < 0 || tokens > 0x7fffffff || heads <= 0 || shares < 1 || shares > 65535 || (shares > 1 && !part) ||
-        table_stride <= 0 || !(scale > 0.f))
+        table_stride <= 0 || window < 0 || !(scale > 0.f))
         return nva_fail("latent_attention: bad sizes tokens=%lld heads=%d shares=%d", (long long)tokens, heads, shares);
     if (q_stride % 8 || out_stride % 4 || !nva_aligned(q2, 16) || !nva_aligned(out, 8) || !nva_aligned(k_cache, 16) ||
         !nva_aligned(v_cache, 8)) {
@@ -638,7 +793,7 @@ NVA_EXPORT int nva_latent_attention_bf16(const void* q2, int64_t q_stride, void*
 #define LAT_LAUNCH(MC)                                                                                               \
     hipLaunchKernelGGL(latent_attn_kernel<MC>, grid, dim3(NVA_WAVE), 0, stream, (const __bf16*)q2, q_stride,            \
                        (__bf16*)out, out_stride, part, (const __bf16*)k_cache, (const __bf16*)v_cache, block_tables,     \
-                       table_stride, token_seq, positions, heads, rank, rot, page_size, scale, sinks, error_flag)
+                       table_stride, token_seq, positions, heads, rank, rot, page_size, scale, window, sinks, error_flag)
     if (rank <= 128) LAT_LAUNCH(128);
     else if (rank <= 256) LAT_LAUNCH(256);
     else if (rank <= 384) LAT_LAUNCH(384);
@@ -658,14 +813,14 @@ NVA_EXPORT int nva_latent_attention_prefill_bf16(const void* q2, int64_t q_strid
                                                  const void* k_cache, const void* v_cache, const int32_t* block_tables,
                                                  int table_stride, const int32_t* cu_seqlens_q, const int32_t* kv_lens,
                                                  const int32_t* row_tiles, int64_t num_tiles, int heads, int rank, int rot,
-                                                 int page_size, float scale, const float* sinks, int32_t* error_flag,
+                                                 int page_size, float scale, int window, const float* sinks, int32_t* error_flag,
                                                  hipStream_t stream) {
     if (num_tiles == 0) return 0;
     if (rank % 16 || rank <= 0 || rank > 512 || rot % 8 || rot <= 0 || rot > LAT_MAX_ROT || page_size % LAT_TILE || page_size <= 0) {
         nva_fail("latent_attention_prefill: sizes it does not take (%d, %d, %d)", rank, rot, page_size);
         return 1;
     }
-    if (!row_tiles || num_tiles < 0 || num_tiles * 8 > 0x7fffffff || heads <= 0 || table_stride <= 0 || !(scale > 0.f))
+    if (!row_tiles || num_tiles < 0 || num_tiles * 8 > 0x7fffffff || heads <= 0 || table_stride <= 0 || window < 0 || !(scale > 0.f))
         return nva_fail("latent_attention_prefill: bad sizes tiles=%lld heads=%d", (long long)num_tiles, heads);
     if (q_stride % 8 || out_stride % 4 || !nva_aligned(q2, 16) || !nva_aligned(out, 8) || !nva_aligned(k_cache, 16) ||
         !nva_aligned(v_cache, 16)) {
@@ -686,7 +841,7 @@ NVA_EXPORT int nva_latent_attention_prefill_bf16(const void* q2, int64_t q_strid
         }                                                                                                            \
         hipLaunchKernelGGL(kernel, grid, dim3(WV * NVA_WAVE), lds, stream, (const __bf16*)q2, q_stride, (__bf16*)out,    \
                            out_stride, (const __bf16*)k_cache, (const __bf16*)v_cache, block_tables, table_stride,      \
-                           cu_seqlens_q, kv_lens, row_tiles, heads, rank, rot, page_size, scale, sinks, error_flag);    \
+                           cu_seqlens_q, kv_lens, row_tiles, heads, rank, rot, page_size, scale, window, sinks, error_flag);    \
     } while (0)
     if (rank <= 128) LAT_LAUNCH(128, 8);
     else if (rank <= 256) LAT_LAUNCH(256, 8);

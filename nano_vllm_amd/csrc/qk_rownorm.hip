@@ -23,6 +23,10 @@
 // v_first_out, float [tokens, Hkv * DV]: the values as they are after the norm are also written there, unrounded (the
 // first of the layers that mix values hands them to the later ones of the same step).  v_first_in with v_mix (one
 // float read on the device): v <- (1 - v_mix) v + v_mix v_first_in, after the norm, before the store.
+// norm_unit (with per_head, no weights): every q and k head is divided by its root mean square (eps inside the root); a
+// rotation keeps a head's length, so that is the same before it or after it.
+// gates > 0: the row has `gates` more columns behind v (and may have others behind those); gate_out, float [tokens, gates],
+// receives their sigmoids: the factors by which an attention kernel multiplies the heads' outputs.
 // One workgroup per token.
 #include "common.h"
 
@@ -36,7 +40,7 @@ qk_rownorm_store_kernel(const T* __restrict__ qkv, int64_t stride, PartialInput 
                         const int32_t* __restrict__ slots, T* __restrict__ k_cache, T* __restrict__ v_cache,
                         int page_size, int per_head, int rot_interleaved, int v_norm,
                         const float* __restrict__ v_first_in, const float* __restrict__ v_mix,
-                        float* __restrict__ v_first_out) {
+                        float* __restrict__ v_first_out, int norm_unit, int gates, float* __restrict__ gate_out, int row_width) {
     extern __shared__ __attribute__((aligned(16))) float row_s[];      // the token's row, as float; then a scale per head
     __shared__ float scratch[16];
     const int64_t t = blockIdx.x;
@@ -49,9 +53,13 @@ qk_rownorm_store_kernel(const T* __restrict__ qkv, int64_t stride, PartialInput 
 
     float sq = 0.f, sk = 0.f;
     for (int i = tid; i < width; i += blockDim.x) {
-        const float x = part.sums ? partial_value<T>(part, t, width, i) : to_float(qkv[t * stride + i]);
+        const float x = part.sums ? partial_value<T>(part, t, row_width, i) : to_float(qkv[t * stride + i]);
         row_s[i] = x;
         if (i < qd) sq += x * x; else if (i < qd + kd) sk += x * x;
+    }
+    for (int i = tid; i < gates; i += blockDim.x) {
+        const float x = part.sums ? partial_value<T>(part, t, row_width, width + i) : to_float(qkv[t * stride + width + i]);
+        gate_out[t * gates + i] = 1.f / (1.f + expf(-x));
     }
     float* const head_scale = row_s + width;                           // [num_heads + num_kv_heads], with per_head
     float* const v_scale = head_scale + (per_head ? num_heads + num_kv_heads : 0);      // [num_kv_heads], with v_norm
@@ -91,7 +99,7 @@ qk_rownorm_store_kernel(const T* __restrict__ qkv, int64_t stride, PartialInput 
     // entry i of a projection that starts at `at` in the row, scaled and weighted, then turned with its partner
     auto prepared = [&](int at, int i, float scale, const void* w) -> float {
         const int d = i % head_dim;
-        if (per_head && w) scale *= head_scale[(at + i) / head_dim];   // (at is a multiple of the head size)
+        if (per_head && (w || norm_unit)) scale *= head_scale[(at + i) / head_dim];   // (at is a multiple of the head size)
         const float x = row_s[at + i] * scale * weight_of(w, per_head ? d : i);
         if (!rot_row || d >= rot) return x;
         if (rot_interleaved) {
@@ -135,6 +143,7 @@ qk_rownorm_store_kernel(const T* __restrict__ qkv, int64_t stride, PartialInput 
 
 // qkv: [tokens, Hq * D + Hkv * D + Hkv * DV] with rows `stride` elements apart, or (sums != null) the float
 // partial sums [splits][tokens][width] of the projection with its bias, which are added up here.
+// row_width: the columns of a row of the projection, gate columns and padding included.
 // q_out: [tokens, Hq * D] with rows q_stride apart (it may be qkv itself: q is then rewritten in place).
 // q_weight [Hq * D], k_weight [Hkv * D] (per_head: both [D]): both or none.  positions are needed with a temperature.
 // rot_table: float [tokens, rot], a row per token of this call, or null.
@@ -147,7 +156,8 @@ NVA_EXPORT int NVA_NAME(nva_qk_rownorm_store)(const void* qkv, int64_t stride, c
                                               int temp_every, const float* rot_table, int rot, const int32_t* slots,
                                               void* k_cache, void* v_cache, int page_size, int per_head,
                                               int rot_interleaved, int v_norm, const float* v_first_in,
-                                              const float* v_mix, float* v_first_out, hipStream_t stream) {
+                                              const float* v_mix, float* v_first_out, int norm_unit, int gates,
+                                              float* gate_out, int64_t row_width, hipStream_t stream) {
     if (tokens == 0) return 0;
     if (tokens < 0 || tokens > 0x7fffffff) return nva_fail("qk_rownorm_store: bad token count %lld", (long long)tokens);
     if (num_heads <= 0 || num_kv_heads < 0 || head_dim <= 0 || v_dim <= 0)
@@ -155,9 +165,11 @@ NVA_EXPORT int NVA_NAME(nva_qk_rownorm_store)(const void* qkv, int64_t stride, c
                         head_dim, v_dim);
     const int64_t width = (int64_t)(num_heads + num_kv_heads) * head_dim + (int64_t)num_kv_heads * v_dim;
     if (width > 36 * 1024) return nva_fail("qk_rownorm_store: a row of %lld entries does not fit the LDS", (long long)width);
-    if (!sums && (!qkv || stride < width))
+    if (gates < 0 || (gates && !gate_out) || row_width < width + gates || row_width > 0x7fffffff || (norm_unit && (!per_head || q_weight || k_weight)))
+        return nva_fail("qk_rownorm_store: bad gate columns (%d of a row of %lld) or a weight with norms that have none", gates, (long long)row_width);
+    if (!sums && (!qkv || stride < row_width))
         return nva_fail("qk_rownorm_store: rows of %lld elements are %lld apart", (long long)width, (long long)stride);
-    if (sums && (splits <= 0 || split_stride < tokens * width)) return nva_fail("qk_rownorm_store: bad partial sums");
+    if (sums && (splits <= 0 || split_stride < tokens * row_width)) return nva_fail("qk_rownorm_store: bad partial sums");
     if (!q_out || q_stride < (int64_t)num_heads * head_dim) return nva_fail("qk_rownorm_store: no room for q");
     if (num_kv_heads && (q_weight == nullptr) != (k_weight == nullptr))
         return nva_fail("qk_rownorm_store: give both norm weights or none");
@@ -182,7 +194,7 @@ NVA_EXPORT int NVA_NAME(nva_qk_rownorm_store)(const void* qkv, int64_t stride, c
     hipLaunchKernelGGL(kernel, dim3((unsigned)tokens), dim3(threads), lds, stream, (const elem_t*)qkv, stride, part,
                        (elem_t*)q_out, q_stride, num_heads, num_kv_heads, head_dim, v_dim, q_weight, k_weight, w_is_f32, eps,
                        positions, temp_coef, temp_every, rot_table, rot_table ? rot : 0, slots, (elem_t*)k_cache, (elem_t*)v_cache, page_size,
-                       per_head ? 1 : 0, rot_interleaved ? 1 : 0, v_norm ? 1 : 0, v_first_in, v_mix, v_first_out);
+                       per_head ? 1 : 0, rot_interleaved ? 1 : 0, v_norm ? 1 : 0, v_first_in, v_mix, v_first_out, norm_unit ? 1 : 0, gates, gate_out, (int)row_width);
     return nva_check_launch("qk_rownorm_store");
 }
 

@@ -656,6 +656,20 @@ class HipKernels:
                      c_i32(self.PLAIN_ACTIVATIONS[act]), self._stream())
         return out
 
+    def linear_act(self, x: torch.Tensor, weight: torch.Tensor, act: str = "relu2") -> torch.Tensor:
+        """act(x @ weight.T), entry by entry; a product left as partial sums is added up by the activation's own pass."""
+        y = self.linear(x, weight, deferred=True)
+        if not isinstance(y, SplitSum):
+            y = _t(y)
+            return self.act(y, act, out=y)
+        if act not in self.PLAIN_ACTIVATIONS:
+            raise KernelError(f"act: unknown activation {act!r}; known: {sorted(self.PLAIN_ACTIVATIONS)}")
+        rows, width = y.shape
+        out = torch.empty((rows, width), dtype=y.dtype, device=y.device)
+        library.call("activation", "bf16", "nva_act_of_partials", _p(y.sums), c_i32(y.splits), c_i64(rows * width), _p(y.bias),
+                     _p(out), c_i64(width), c_i64(rows), c_i32(width), c_i32(self.PLAIN_ACTIVATIONS[act]), self._stream())
+        return out
+
     # ------------------------------------------------------------------ routed feed-forward
     ROUTINGS = {"sigmoid_groups": 0, "softmax_top": 1, "softmax_choice": 2}
 
@@ -1224,8 +1238,11 @@ class HipKernels:
                          v_cache: Optional[torch.Tensor], rot_table: Optional[torch.Tensor] = None,
                          norm_per_head: bool = False, rot_interleaved: bool = False, v_norm: bool = False,
                          v_first_in: Optional[torch.Tensor] = None, v_mix: Optional[torch.Tensor] = None,
-                         v_first_out: Optional[torch.Tensor] = None) -> torch.Tensor:
-        """rot_interleaved: the rotation pairs the neighbours (2i, 2i + 1).  v_norm: every value head divided by its root
+                         v_first_out: Optional[torch.Tensor] = None, norm_unit: bool = False,
+                         head_gate: Optional[torch.Tensor] = None) -> torch.Tensor:
+        """norm_unit (with norm_per_head, no weights): every q and k head is divided by its root mean square.
+        head_gate, float32 [tokens, heads]: receives the sigmoids of the row's columns behind v, one per head (the row
+        may be wider still).  rot_interleaved: the rotation pairs the neighbours (2i, 2i + 1).  v_norm: every value head divided by its root
         mean square (eps, no weight).  v_first_out, float32 [tokens, kv_heads * v_head_dim]: receives the values after the
         norm.  v_first_in (the same shape) with v_mix (float32, one number on the device): v <- (1 - v_mix) v + v_mix
         v_first_in before the store.
@@ -1243,8 +1260,14 @@ class HipKernels:
             qkv = _t(qkv)
             tokens, width, stride = _rows2d(qkv, "qkv")
         want = (num_heads + num_kv_heads) * head_dim + num_kv_heads * v_head_dim
-        if width != want:
-            raise KernelError(f"qkv width {width} is not heads * head_dim + kv_heads * (head_dim + v_head_dim) = {want}")
+        gates = 0 if head_gate is None else num_heads
+        if width != want and (not gates or width < want + gates):
+            raise KernelError(f"qkv width {width} is not heads * head_dim + kv_heads * (head_dim + v_head_dim) = {want}"
+                              + (f" and {gates} gate columns" if gates else ""))
+        if gates and (head_gate.dtype != torch.float32 or tuple(head_gate.shape) != (tokens, gates) or not head_gate.is_contiguous()):
+            raise KernelError(f"qk_rownorm_store: head_gate must be contiguous float32 [{tokens}, {gates}]")
+        if norm_unit and (not norm_per_head or q_weight is not None or k_weight is not None):
+            raise KernelError("qk_rownorm_store: norms without a weight are per-head norms, and take none")
         wf = 0
         for w, n in ((q_weight, num_heads * head_dim), (k_weight, num_kv_heads * head_dim)):
             if w is not None:
@@ -1287,9 +1310,9 @@ class HipKernels:
                      c_i32(num_heads), c_i32(num_kv_heads), c_i32(head_dim), c_i32(v_head_dim), _p(q_weight), _p(k_weight),
                      c_i32(wf), c_f32(eps), _p(positions), c_f32(float(temp_coef)), c_i32(int(temp_every) if temp_coef else 1),
                      _p(rot_table), c_i32(rot), _p(slots), _p(k_cache), _p(v_cache), c_i32(page_size),
-                     c_i32(1 if norm_per_head and q_weight is not None else 0), c_i32(1 if rot_interleaved else 0),
+                     c_i32(1 if norm_per_head and (q_weight is not None or norm_unit) else 0), c_i32(1 if rot_interleaved else 0),
                      c_i32(1 if v_norm else 0), _p(v_first_in), _p(v_mix) if v_first_in is not None else None,
-                     _p(v_first_out), self._stream())
+                     _p(v_first_out), c_i32(1 if norm_unit else 0), c_i32(gates), _p(head_gate), c_i64(width), self._stream())
         return q
 
     def sigmoid_mul(self, x: torch.Tensor, gate: torch.Tensor, out: Optional[torch.Tensor] = None) -> torch.Tensor:
@@ -1327,8 +1350,9 @@ class HipKernels:
                         window: Optional[int] = None, out: Optional[torch.Tensor] = None,
                         v_head_dim: Optional[int] = None, sinks: Optional[torch.Tensor] = None,
                         chunk: Optional[int] = None, softcap: Optional[float] = None, keep_first: int = 0,
-                        sigmoid_bias: Optional[torch.Tensor] = None) -> torch.Tensor:
-        """sigmoid_bias, float32 [heads]: no softmax; a visible key weighs sigmoid(score + sigmoid_bias[head]), and the
+                        sigmoid_bias: Optional[torch.Tensor] = None, head_gate: Optional[torch.Tensor] = None) -> torch.Tensor:
+        """head_gate, float32 [tokens, heads]: head h's output of a token is multiplied by its number as it is written.
+        sigmoid_bias, float32 [heads]: no softmax; a visible key weighs sigmoid(score + sigmoid_bias[head]), and the
         weights are not normalised over the keys.
         chunk: a query at position p reads the keys from floor(p / chunk) * chunk on only.
         softcap: a score s (after the scale) becomes softcap * tanh(s / softcap).  keep_first (with a window):
@@ -1374,12 +1398,15 @@ class HipKernels:
         if sigmoid_bias is not None and (sigmoid_bias.dtype != torch.float32 or sigmoid_bias.shape != (num_heads,) or
                                          not sigmoid_bias.is_contiguous() or sinks is not None):
             raise KernelError(f"attention: sigmoid_bias must be contiguous float32 [{num_heads}] and goes without sinks")
+        if head_gate is not None and (head_gate.dtype != torch.float32 or tuple(head_gate.shape) != (tokens, num_heads) or
+                                      not head_gate.is_contiguous()):
+            raise KernelError(f"attention: head_gate must be contiguous float32 [{tokens}, {num_heads}]")
         mfma = self.mfma_attention and q.dtype == torch.bfloat16 and 0.0 < scale < float("inf") and v_dim == head_dim
         if batch.num_decode > 0 and mfma and \
                 self._decode_kernel_takes(num_heads // num_kv_heads, head_dim, page_size, q, qs, out, os_):
             start = batch.num_decode
             self._attention_decode(q, qs, out, os_, k_cache, v_cache, tables, batch, start, num_heads, num_kv_heads,
-                                   head_dim, page_size, scale, window, sinks, chunk, keep, cap, sigmoid_bias)
+                                   head_dim, page_size, scale, window, sinks, chunk, keep, cap, sigmoid_bias, head_gate)
         if batch.num_decode < tokens and mfma and \
                 self._prefill_kernel_takes(head_dim, page_size, tables.shape[1], q, qs, out, os_):
             # portions of prompts: the matrix-core prefill kernel, one workgroup per 32 query rows
@@ -1388,7 +1415,7 @@ class HipKernels:
                          _p(v_cache), _p(tables), c_i32(tables.shape[1]), _p(batch.cu_seqlens_q), _p(batch.kv_lens),
                          _p(tiles), c_i64(tiles.shape[0]), c_i32(num_heads),
                          c_i32(num_kv_heads), c_i32(head_dim), c_i32(page_size), c_f32(scale), c_i32(window or 0),
-                         c_i32(chunk or 0), c_i32(keep), c_f32(cap), _p(sinks), _p(sigmoid_bias), _p(self.fault_flag),
+                         c_i32(chunk or 0), c_i32(keep), c_f32(cap), _p(sinks), _p(sigmoid_bias), _p(head_gate), _p(self.fault_flag),
                          self._stream())
             tokens = batch.num_decode            # what is left: the single tokens before the portions, if any
         if self.tiled_general_attention and start <= batch.num_decode < tokens and not window and sigmoid_bias is None and \
@@ -1400,7 +1427,7 @@ class HipKernels:
                          _p(k_cache), _p(v_cache), _p(tables), c_i32(tables.shape[1]), _p(batch.cu_seqlens_q),
                          _p(batch.kv_lens), _p(tiles), c_i64(tiles.shape[0]), c_i32(num_heads), c_i32(num_kv_heads),
                          c_i32(head_dim), c_i32(v_dim), c_i32(page_size), c_f32(scale), c_i32(chunk or 0), c_f32(cap),
-                         _p(sinks), _p(self.fault_flag), self._stream())
+                         _p(sinks), _p(head_gate), _p(self.fault_flag), self._stream())
             tokens = batch.num_decode            # what is left: the single tokens before the portions
         if start < tokens:
             n = tokens - start
@@ -1418,17 +1445,18 @@ class HipKernels:
                          _p(out[start:]), c_i64(os_), _p(k_cache), _p(v_cache), _p(tables), c_i32(tables.shape[1]),
                          _p(batch.token_seq[start:]), _p(batch.positions[start:]), c_i64(n), c_i32(num_heads),
                          c_i32(num_kv_heads), c_i32(head_dim), c_i32(v_dim), c_i32(page_size), c_f32(scale),
-                         c_i32(window or 0), c_i32(chunk or 0), c_i32(keep), c_f32(cap), _p(sinks), _p(sigmoid_bias), _p(part), c_i32(shares),
+                         c_i32(window or 0), c_i32(chunk or 0), c_i32(keep), c_f32(cap), _p(sinks), _p(sigmoid_bias),
+                         _p(None if head_gate is None else head_gate[start:]), _p(part), c_i32(shares),
                          _p(self.fault_flag), self._stream())
         return out
 
     # ------------------------------------------------------------------ attention through a latent
     def latent_prepare(self, proj: torch.Tensor, heads: int, dim: int, rot: int, rank: int, weight: torch.Tensor, eps: float,
                        rot_table: torch.Tensor, slots: Optional[torch.Tensor], k_cache: Optional[torch.Tensor],
-                       v_cache: Optional[torch.Tensor]) -> torch.Tensor:
+                       v_cache: Optional[torch.Tensor], interleaved: bool = True) -> torch.Tensor:
         """proj [tokens, heads * (dim + rot) + rank + rot]: per head [dim plain | rot turned] query entries, then the
         token's raw latent and its raw turned key part.  The latent is normed (weight, eps), the turned parts are
-        rotated in pairs of neighbours by rot_table (float32 [tokens, rot]: cosines, then sines); the cache's key row
+        rotated in pairs of neighbours (interleaved False: pairs (i, i + rot / 2)) by rot_table (float32 [tokens, rot]: cosines, then sines); the cache's key row
         of the token becomes [latent | turned key part], its value row the latent.  Returns q2 [tokens, heads *
         (rank + rot)] with every head's turned part in its last rot entries; the first rank are left for the caller."""
         proj = _t(proj)
@@ -1445,16 +1473,76 @@ class HipKernels:
         q2 = torch.empty((tokens, heads * (rank + rot)), dtype=proj.dtype, device=proj.device)
         library.call("latent", _suffix(proj), "nva_latent_prepare", _p(proj), c_i64(stride), c_i64(tokens), c_i32(heads),
                      c_i32(dim), c_i32(rot), c_i32(rank), _p(weight), c_i32(wf), c_f32(eps), _p(rot_table), _p(q2),
-                     c_i64(q2.shape[1]), _p(slots), _p(k_cache), _p(v_cache), c_i32(page_size), self._stream())
+                     c_i64(q2.shape[1]), _p(slots), _p(k_cache), _p(v_cache), c_i32(page_size), c_i32(1 if interleaved else 0),
+                     self._stream())
         return q2
 
+    def latent_down(self, low, q_rank: int, rot: int, rank: int, gates: int, q_weight: torch.Tensor, weight: torch.Tensor,
+                    eps: float, rot_table: torch.Tensor, slots: Optional[torch.Tensor], k_cache: Optional[torch.Tensor],
+                    v_cache: Optional[torch.Tensor], interleaved: bool = True):
+        """low [tokens, q_rank + rank + rot + gates] = [raw query latent | raw latent | raw turned key part | gates], or that
+        product left as partial sums.  The two latents are normed (q_weight, weight, eps), the turned key part is rotated
+        and the cache's rows of the token written as in latent_prepare.  Returns (the normed query latent [tokens,
+        q_rank], the sigmoids of the gate columns float32 [tokens, gates] or None)."""
+        partial = isinstance(low, SplitSum) and self.fuse_split_sums and low.bias is None
+        if partial:
+            (tokens, width), stride = low.shape, 0
+        else:
+            low = _t(low)
+            tokens, width, stride = _rows2d(low, "latent projection")
+        if width != q_rank + rank + rot + gates:
+            raise KernelError(f"latent_down: a row of {width} is not q_rank + rank + rot + gates")
+        if rot_table.dtype != torch.float32 or tuple(rot_table.shape) != (tokens, rot) or not rot_table.is_contiguous():
+            raise KernelError(f"latent_down: the rotation table must be contiguous float32 [{tokens}, {rot}]")
+        wf = self._norm_weight(weight, rank, low)
+        if self._norm_weight(q_weight, q_rank, low) != wf:
+            raise KernelError("latent_down: the two weights differ in type")
+        page_size = 0
+        if k_cache is not None:
+            page_size = self._check_cache(k_cache, v_cache, 1, rank + rot, low.dtype, rank)
+            _i32(slots, tokens, "slots")
+        cq = torch.empty((tokens, q_rank), dtype=low.dtype, device=low.device)
+        factors = torch.empty((tokens, gates), dtype=torch.float32, device=low.device) if gates else None
+        source = [None, c_i64(0), _p(low.sums), c_i32(low.splits), c_i64(tokens * width)] if partial else \
+            [_p(low), c_i64(stride), None, c_i32(0), c_i64(0)]
+        library.call("latent", "bf16" if partial else _suffix(low), "nva_latent_down", *source, c_i64(tokens), c_i32(q_rank),
+                     c_i32(rank), c_i32(rot), c_i32(gates), _p(q_weight), _p(weight), c_i32(wf), c_f32(eps), _p(rot_table), _p(cq),
+                     _p(factors), _p(slots), _p(k_cache), _p(v_cache), c_i32(page_size), c_i32(1 if interleaved else 0),
+                     self._stream())
+        return cq, factors
+
+    def latent_queries(self, q, heads: int, dim: int, rot: int, rank: int, rot_table: torch.Tensor, interleaved: bool = True):
+        """q [tokens, heads * (dim + rot)] = per head [dim plain | rot turned] query entries, or that product left as partial
+        sums.  Returns (rows that hold the plain parts, entries from one head's plain part to the next's in them, q2 [tokens,
+        heads * (rank + rot)] with every head's rotated part in its last rot entries; the first rank are left for the caller)."""
+        partial = isinstance(q, SplitSum) and self.fuse_split_sums and q.bias is None
+        if partial:
+            (tokens, width), stride = q.shape, 0
+        else:
+            q = _t(q)
+            tokens, width, stride = _rows2d(q, "latent queries")
+        if width != heads * (dim + rot):
+            raise KernelError(f"latent_queries: a row of {width} is not heads * (dim + rot)")
+        if rot_table.dtype != torch.float32 or tuple(rot_table.shape) != (tokens, rot) or not rot_table.is_contiguous():
+            raise KernelError(f"latent_queries: the rotation table must be contiguous float32 [{tokens}, {rot}]")
+        q2 = torch.empty((tokens, heads * (rank + rot)), dtype=q.dtype, device=q.device)
+        plain = torch.empty((tokens, heads * dim), dtype=q.dtype, device=q.device) if partial else None
+        source = [None, c_i64(0), _p(q.sums), c_i32(q.splits), c_i64(tokens * width)] if partial else \
+            [_p(q), c_i64(stride), None, c_i32(0), c_i64(0)]
+        library.call("latent", "bf16" if partial else _suffix(q), "nva_latent_queries", *source, c_i64(tokens), c_i32(heads),
+                     c_i32(dim), c_i32(rot), c_i32(rank), _p(rot_table), _p(q2), _p(plain), c_i32(1 if interleaved else 0),
+                     self._stream())
+        return (plain, dim, q2) if partial else (q, dim + rot, q2)
+
     def latent_attention(self, q2: torch.Tensor, heads: int, rank: int, rot: int, k_cache: torch.Tensor, v_cache: torch.Tensor,
-                         batch, group: int, scale: float, sinks: Optional[torch.Tensor] = None) -> torch.Tensor:
+                         batch, group: int, scale: float, sinks: Optional[torch.Tensor] = None,
+                         window: Optional[int] = None) -> torch.Tensor:
         """Causal softmax attention of heads that share one key/value head whose key rows are [latent | rotated part]
         (rank + rot entries) and whose value rows are the latent: q2 [tokens, heads * (rank + rot)] -> [tokens, heads *
         rank].  bfloat16 with a latent of a multiple of 16 runs on the matrix cores (a token's heads are the columns of
         the products, so a key row is fetched once for all of them; a token's keys are shared out among workgroups
-        where a step has few tokens); everything else runs the general attention kernel."""
+        where a step has few tokens); everything else runs the general attention kernel.  window: a query at position p
+        reads the keys of positions > p - window only."""
         q2 = _t(q2)
         tokens, width, qs = _rows2d(q2, "latent attention q")
         page_size = self._check_cache(k_cache, v_cache, 1, rank + rot, q2.dtype, rank)
@@ -1481,25 +1569,28 @@ class HipKernels:
                 library.call("latent", "bf16", "nva_latent_attention_prefill", _p(q2), c_i64(qs), _p(out), c_i64(out.shape[1]),
                              _p(k_cache), _p(v_cache), _p(tables), c_i32(tables.shape[1]), _p(batch.cu_seqlens_q),
                              _p(batch.kv_lens), _p(tiles), c_i64(tiles.shape[0]), c_i32(heads), c_i32(rank), c_i32(rot),
-                             c_i32(page_size), c_f32(scale), _p(sinks), _p(self.fault_flag), self._stream())
+                             c_i32(page_size), c_f32(scale), c_i32(window or 0), _p(sinks), _p(self.fault_flag), self._stream())
             if single > 0:
                 # few tokens with many keys: a token's tiles of 32 keys are shared out, four tiles a share or more, until
                 # about two waves a compute unit run; the number follows from the step's shape alone
                 blocks = (heads + 15) // 16
-                shares = max(1, min(64, ((batch.max_kv_len + 31) // 32) // 4, 512 // (single * blocks)))
+                reach = min(batch.max_kv_len, window + 31) if window else batch.max_kv_len
+                shares = max(1, min(64, ((reach + 31) // 32) // 4, 512 // (single * blocks)))
                 part = torch.empty(single * heads * shares * (2 + rank), dtype=torch.float32, device=q2.device) if shares > 1 else None
                 library.call("latent", "bf16", "nva_latent_attention", _p(q2), c_i64(qs), _p(out), c_i64(out.shape[1]), _p(part),
                              c_i32(shares), _p(k_cache), _p(v_cache), _p(tables), c_i32(tables.shape[1]), _p(batch.token_seq),
                              _p(batch.positions), c_i64(single), c_i32(heads), c_i32(rank), c_i32(rot), c_i32(page_size),
-                             c_f32(scale), _p(sinks), _p(self.fault_flag), self._stream())
+                             c_f32(scale), c_i32(window or 0), _p(sinks), _p(self.fault_flag), self._stream())
             return out
-        return self.paged_attention(q2, heads, 1, rank + rot, k_cache, v_cache, batch, group, scale, None, v_head_dim=rank,
+        return self.paged_attention(q2, heads, 1, rank + rot, k_cache, v_cache, batch, group, scale, window, v_head_dim=rank,
                                     sinks=sinks)
 
     def heads_linear(self, x: torch.Tensor, x_head: int, w: torch.Tensor, heads: int, n_out: int, k_in: int,
-                     transposed: bool, y: torch.Tensor, y_head: int, y_offset: int = 0) -> torch.Tensor:
+                     transposed: bool, y: torch.Tensor, y_head: int, y_offset: int = 0,
+                     head_gate: Optional[torch.Tensor] = None) -> torch.Tensor:
         """A product per head: y[t, h * y_head + y_offset + n] = sum_k W[h][n][k] x[t, h * x_head + k], n < n_out, k < k_in.
         w is contiguous [heads * n_out, k_in], or with transposed [heads * k_in, n_out] (W[h][n][k] = w[h * k_in + k, n]).
+        head_gate, float32 [tokens, heads]: head h's outputs of a token are multiplied by its number before they are rounded.
         x and y are 2-d with rows of any stride.  Float sums over k in ascending order, rounded once (bfloat16 with
         matrices that are not transposed: on the matrix cores, in the order of their steps of 32)."""
         x = _t(x)
@@ -1510,16 +1601,19 @@ class HipKernels:
             raise KernelError("heads_linear: the output or the matrices do not fit the input")
         if (heads - 1) * x_head + k_in > xw or (heads - 1) * y_head + y_offset + n_out > yw or x_head < 0 or y_head < 0:
             raise KernelError("heads_linear: the heads do not fit the rows")
+        if head_gate is not None and (head_gate.dtype != torch.float32 or tuple(head_gate.shape) != (tokens, heads) or
+                                      not head_gate.is_contiguous()):
+            raise KernelError(f"heads_linear: head_gate must be contiguous float32 [{tokens}, {heads}]")
         w_n, w_k = (1, n_out) if transposed else (k_in, 1)
         yv = y[:, y_offset:] if y_offset else y
         if x.dtype == torch.bfloat16 and not transposed and k_in % 8 == 0 and xs % 8 == 0 and x_head % 8 == 0 and \
                 x.data_ptr() % 16 == 0 and self.mfma_attention:
             library.call("latent", "bf16", "nva_heads_linear_mfma", _p(x), c_i64(xs), c_i64(x_head), _p(w), _p(yv), c_i64(ys),
-                         c_i64(y_head), c_i64(tokens), c_i32(heads), c_i32(n_out), c_i32(k_in), self._stream())
+                         c_i64(y_head), c_i64(tokens), c_i32(heads), c_i32(n_out), c_i32(k_in), _p(head_gate), self._stream())
             return y
         library.call("latent", _suffix(x), "nva_heads_linear", _p(x), c_i64(xs), c_i64(x_head), _p(w), c_i64(n_out * k_in),
                      c_i64(w_n), c_i64(w_k), _p(yv), c_i64(ys), c_i64(y_head), c_i64(tokens), c_i32(heads), c_i32(n_out),
-                     c_i32(k_in), self._stream())
+                     c_i32(k_in), _p(head_gate), self._stream())
         return y
 
     # ------------------------------------------------------------------ delta rule
@@ -1547,23 +1641,11 @@ class HipKernels:
         grows, gw, gs = _rows2d(gate_in, "delta-rule gate")
         if (grows, gw) != (tokens, vv) or gate_in.dtype != proj.dtype:
             raise KernelError("channel_delta: the gate's input does not match")
-        if s_state.dtype != torch.float32 or tuple(s_state.shape[1:]) != (heads, dim, vdim) or not s_state.is_contiguous():
-            raise KernelError(f"channel_delta: the state must be contiguous float32 [slots, {heads}, {dim}, {vdim}]")
-        if conv_state.dtype != torch.float32 or tuple(conv_state.shape) != (s_state.shape[0], channels, taps - 1) or \
-                not conv_state.is_contiguous():
-            raise KernelError(f"channel_delta: the kept inputs must be contiguous float32 [slots, {channels}, {taps - 1}]")
-        if tuple(conv_w.shape) != (channels, taps) or conv_w.dtype != proj.dtype or not conv_w.is_contiguous():
-            raise KernelError("channel_delta: the convolution's weights do not fit")
-        for v, n, what in ((dt_bias, hd, "dt_bias"), (a_log, heads, "a_log"), (norm_w, vdim, "norm_w")):
+        self._check_delta("channel_delta", proj, tokens, heads, dim, vdim, taps, channels, conv_w, norm_w, conv_state, s_state, batch)
+        for v, n, what in ((dt_bias, hd, "dt_bias"), (a_log, heads, "a_log")):
             if v.dtype != torch.float32 or tuple(v.shape) != (n,) or not v.is_contiguous():
                 raise KernelError(f"channel_delta: {what} must be contiguous float32 [{n}]")
         seqs = batch.num_seqs
-        _i32(batch.token_seq, tokens, "token_seq")
-        _i32(batch.cu_seqlens_q, seqs + 1, "cu_seqlens_q")
-        _i32(batch.seq_starts, seqs, "seq_starts")
-        _i32(batch.state_slots, seqs, "state_slots")
-        if sum(batch.q_lens) != tokens:
-            raise KernelError("channel_delta: the batch does not describe the projections' rows")
         if out is None:
             out = torch.empty((tokens, vv), dtype=proj.dtype, device=proj.device)
         orows, ow, os_ = _rows2d(out, "delta-rule output")
@@ -1577,6 +1659,58 @@ class HipKernels:
                      c_i32(heads), c_i32(kv_heads), c_i32(dim), c_i32(vdim), c_i32(taps), _p(conv_w), _p(dt_bias), _p(a_log),
                      _p(norm_w), c_f32(eps), self._stream())
         return out
+
+    def head_delta(self, proj: torch.Tensor, rates: torch.Tensor, heads: int, kv_heads: int, dim: int, vdim: int, taps: int,
+                   conv_w: torch.Tensor, dt_bias: torch.Tensor, a_log: torch.Tensor, norm_w: torch.Tensor, eps: float,
+                   conv_state: torch.Tensor, s_state: torch.Tensor, batch, out: Optional[torch.Tensor] = None) -> torch.Tensor:
+        """The gated delta rule with one decay per head over the step's tokens: proj [T, 2 G D + 2 H DV] = [q | k | v | gate],
+        rates float32 [T, 2 H] = [b | a].  As channel_delta, but the decay of a head is one number, exp(-exp(a_log) *
+        softplus(a + dt_bias)) with dt_bias and a_log float32 [H], and the gate is silu.  Returns [T, H DV] of proj's type."""
+        proj = _t(proj)
+        tokens, width, stride = _rows2d(proj, "delta-rule projections")
+        vv = heads * vdim
+        channels = 2 * kv_heads * dim + vv
+        if width != channels + vv:
+            raise KernelError(f"head_delta: projections of width {width}, expected {channels + vv}")
+        if rates.dtype != torch.float32 or tuple(rates.shape) != (tokens, 2 * heads) or not rates.is_contiguous():
+            raise KernelError(f"head_delta: the rates must be contiguous float32 [{tokens}, {2 * heads}]")
+        self._check_delta("head_delta", proj, tokens, heads, dim, vdim, taps, channels, conv_w, norm_w, conv_state, s_state, batch)
+        for v, what in ((dt_bias, "dt_bias"), (a_log, "a_log")):
+            if v.dtype != torch.float32 or tuple(v.shape) != (heads,) or not v.is_contiguous():
+                raise KernelError(f"head_delta: {what} must be contiguous float32 [{heads}]")
+        if out is None:
+            out = torch.empty((tokens, vv), dtype=proj.dtype, device=proj.device)
+        orows, ow, os_ = _rows2d(out, "delta-rule output")
+        if (orows, ow) != (tokens, vv) or out.dtype != proj.dtype:
+            raise KernelError("head_delta: output does not match")
+        dp = (dim + 3) // 4 * 4
+        scratch = torch.empty(tokens * (2 * kv_heads * dp + 2 * vv + 2 * heads), dtype=torch.float32, device=proj.device)
+        library.call("delta", _suffix(proj), "nva_head_delta", _p(proj), c_i64(stride), _p(rates), _p(scratch), _p(out), c_i64(os_),
+                     _p(s_state), _p(conv_state if taps > 1 else None), _p(batch.token_seq), _p(batch.cu_seqlens_q),
+                     _p(batch.seq_starts), _p(batch.state_slots), c_i64(batch.num_seqs), c_i64(tokens), c_i32(heads), c_i32(kv_heads),
+                     c_i32(dim), c_i32(vdim), c_i32(taps), _p(conv_w), _p(dt_bias), _p(a_log), _p(norm_w), c_f32(eps),
+                     self._stream())
+        return out
+
+    @staticmethod
+    def _check_delta(what, proj, tokens, heads, dim, vdim, taps, channels, conv_w, norm_w, conv_state, s_state, batch) -> None:
+        """The state, the convolution's weights, the norm's weight and the batch of a delta-rule layer."""
+        if s_state.dtype != torch.float32 or tuple(s_state.shape[1:]) != (heads, dim, vdim) or not s_state.is_contiguous():
+            raise KernelError(f"{what}: the state must be contiguous float32 [slots, {heads}, {dim}, {vdim}]")
+        if conv_state.dtype != torch.float32 or tuple(conv_state.shape) != (s_state.shape[0], channels, taps - 1) or \
+                not conv_state.is_contiguous():
+            raise KernelError(f"{what}: the kept inputs must be contiguous float32 [slots, {channels}, {taps - 1}]")
+        if tuple(conv_w.shape) != (channels, taps) or conv_w.dtype != proj.dtype or not conv_w.is_contiguous():
+            raise KernelError(f"{what}: the convolution's weights do not fit")
+        if norm_w.dtype != torch.float32 or tuple(norm_w.shape) != (vdim,) or not norm_w.is_contiguous():
+            raise KernelError(f"{what}: norm_w must be contiguous float32 [{vdim}]")
+        seqs = batch.num_seqs
+        _i32(batch.token_seq, tokens, "token_seq")
+        _i32(batch.cu_seqlens_q, seqs + 1, "cu_seqlens_q")
+        _i32(batch.seq_starts, seqs, "seq_starts")
+        _i32(batch.state_slots, seqs, "state_slots")
+        if sum(batch.q_lens) != tokens:
+            raise KernelError(f"{what}: the batch does not describe the projections' rows")
 
     # ------------------------------------------------------------------ state-space layer
     def state_space(self, proj: torch.Tensor, heads: int, vdim: int, n_state: int, groups: int, taps: int,
@@ -1783,7 +1917,8 @@ class HipKernels:
                                                                              out_stride)
 
     def _attention_decode(self, q, qs, out, os_, k_cache, v_cache, tables, batch, n, num_heads, num_kv_heads,
-                          head_dim, page_size, scale, window, sinks=None, chunk=None, keep=0, cap=0.0, sigmoid_bias=None):
+                          head_dim, page_size, scale, window, sinks=None, chunk=None, keep=0, cap=0.0, sigmoid_bias=None,
+                          head_gate=None):
         # The work is shared out on the device from the tokens' positions, once per step and (kv
         # heads, window): the first layer that asks makes the plan, the others find it on the batch.
         # The library says how large the partial results may get for this many tokens of at most
@@ -1811,7 +1946,8 @@ class HipKernels:
                          _p(scratch), _p(plan), _p(k_cache), _p(v_cache), _p(tables), c_i32(tables.shape[1]),
                          c_i64(t1 - t0), c_i32(num_heads),
                          c_i32(num_kv_heads), c_i32(head_dim), c_i32(page_size), c_f32(scale), c_f32(cap),
-                         c_i32(bound), c_i32(waves), _p(sinks), _p(sigmoid_bias), _p(self.fault_flag), self._stream())
+                         c_i32(bound), c_i32(waves), _p(sinks), _p(sigmoid_bias),
+                         _p(None if head_gate is None else head_gate[t0:t1]), _p(self.fault_flag), self._stream())
 
     # ------------------------------------------------------------------ sampling
     def sample(self, logits: torch.Tensor, temperatures: torch.Tensor, keys: torch.Tensor) -> torch.Tensor:
