@@ -42,6 +42,12 @@ size), beside Mafarax and Qwen3 at equal layer sizes.
 does the same for the Pemuvik design (layers of a window attention with sigmoid weights and a routed feed-forward,
 and of an attention through a shared latent and a dense feed-forward, in turn), beside Kirisun and Qwen3 at equal
 layer sizes.
+
+    python bench.py --design bamipel [--design-sizes 1024,2048,4096] [--layers 4]
+
+does the same for the Bamipel design (layers of a window attention through latents, of the gated delta rule, of a
+grouped attention and of the delta rule again, in turn, each with a dense feed-forward without a gate), beside Kirisun,
+Pemuvik and Qwen3 at equal layer sizes.
 """
 import argparse
 import json
@@ -73,7 +79,7 @@ def parse_args():
                     help="context of one more decode point at the default batch (0: none)")
     ap.add_argument("--serve-seqs", type=int, default=256,
                     help="requests of the reference's benchmark workload through LLM.generate (0: not run)")
-    ap.add_argument("--design", default=None, choices=["nozurax", "mafarax", "kirisun", "pemuvik"],
+    ap.add_argument("--design", default=None, choices=["nozurax", "mafarax", "kirisun", "pemuvik", "bamipel"],
                     help="measure this design beside Qwen3 at equal layer sizes instead of the default workload")
     ap.add_argument("--design-sizes", default="1024,2048,4096", help="model widths of the --design measurement")
     ap.add_argument("--design-alone", action="store_true", help="the --design measurement without the models beside it "
@@ -119,11 +125,25 @@ def pemuvik_config(width: int, layers: int, dtype: str) -> dict:
                     group_keep=2)
 
 
+def bamipel_config(width: int, layers: int, dtype: str) -> dict:
+    """A Bamipel model of the width's layer sizes: latent-attention layers (as many heads as the dense model has query heads,
+    128 plain and 64 rotated query entries a head, a query latent of 768, a key latent of 384, a window of 1024), delta-rule
+    layers (as many heads, a state of 128 x 128 a head, convolutions of 4 taps) and grouped-attention layers with the dense
+    model's heads, in the order latent, delta, grouped, delta; a feed-forward without a gate of 3/2 of the dense inner size
+    (as many weights as the dense model's gated one)."""
+    from nano_vllm_amd.models.shapes import _bamipel
+    heads, kv, dim, inner = DESIGN_SIZES[width]
+    return _bamipel(layers, width, heads, kv, dim, dim, 3 * inner // 2, DESIGN_VOCAB, window=1024, dtype=dtype)
+
+
 def design_configs(width: int, layers: int, dtype: str, design: str = "nozurax"):
     """config.json of a Nozurax model and of the Qwen3 model with the same layer sizes (and, for the Mafarax
     measurement, of the Mafarax model first)."""
     if design == "mafarax":
         return {"mafarax": mafarax_config(width, layers, dtype), **design_configs(width, layers, dtype)}
+    if design == "bamipel":
+        return {"bamipel": bamipel_config(width, layers, dtype), "kirisun": kirisun_config(width, layers, dtype),
+                "pemuvik": pemuvik_config(width, layers, dtype), "qwen3": design_configs(width, layers, dtype)["qwen3"]}
     if design == "pemuvik":
         return {"pemuvik": pemuvik_config(width, layers, dtype), "kirisun": kirisun_config(width, layers, dtype),
                 "qwen3": design_configs(width, layers, dtype)["qwen3"]}

@@ -1,7 +1,7 @@
 """Named config.json contents for runs with random weights (there is no checkpoint to read
 them from): two tiny test shapes and the Qwen3 dense sizes that the benchmarks use, three
 Nozurax shapes (a tiny one, and layers of the Qwen3 1.7B and 8B sizes), two Mafarax shapes (a tiny
-one, and layers of the Qwen3 1.7B sizes) and two Kirisun and two Pemuvik shapes of the same kind.  These are
+one, and layers of the Qwen3 1.7B sizes) and two Kirisun, two Pemuvik and two Bamipel shapes of the same kind.  These are
 inputs, as a model folder's config.json is; nothing in the model code reads them.
 
     python -m nano_vllm_amd.cli random-model --shape qwen3-8b --config-only --out DIR
@@ -109,7 +109,39 @@ def _pemuvik(layers, width, heads, kv_heads, dim, vdim, inner, vocab, window, ep
             "torch_dtype": dtype}
 
 
+def _bamipel(layers, width, heads, kv_heads, dim, vdim, inner, vocab, window, eps=1e-6, dtype="bfloat16", rot=None, scaling=None,
+             latent_heads=None, latent_dim=None, latent_rot=None, latent_vdim=None, q_rank=None, kv_rank=None, delta_heads=None,
+             delta_kv_heads=None, delta_dim=None, delta_vdim=None, conv=4, pattern=("latent_attention", "delta", "attention", "delta"),
+             again=None) -> dict:
+    """Layers that follow `pattern` in turn: the window attention through latents (as many heads as the grouped one has query
+    heads, a query latent of 6 and a key latent of 3 heads' size and a rotated part of half a head unless named), the gated
+    delta rule (as many value heads of the same size, as many query/key heads) and the grouped attention (the whole head
+    rotated), each with the dense layer of `inner`.  again {i: j}: layer i runs layer j's tensors."""
+    lh, ld, lv = latent_heads or heads, latent_dim or dim, latent_vdim or vdim
+    lr = latent_rot or max(2, dim // 2)
+    dh = delta_heads or heads
+    mixers = {
+        "latent_attention": {"heads": lh, "dim": ld, "rot_dim": lr, "vdim": lv, "q_rank": q_rank or 6 * dim, "kv_rank": kv_rank or 3 * dim,
+                             "scale": (ld + lr) ** -0.5, "mask": {"size": window}, "rot": {"dims": lr, "base": 1e4}},
+        "delta": {"heads": dh, "kv_heads": delta_kv_heads or dh, "dim": delta_dim or dim, "vdim": delta_vdim or vdim, "conv": conv},
+        "attention": {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "scale": dim ** -0.5,
+                      "rot": {"dims": rot or dim, "base": 5e5,
+                              "scaling": scaling or {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 8192}}},
+    }
+    out = []
+    for i in range(layers):
+        kind = pattern[i % len(pattern)]
+        out.append({"type": kind, "mixer": mixers[kind], "mlp": {"kind": "dense", "ff": inner}})
+        if again and i in again:
+            out[i]["weights_of"] = again[i]
+    return {"architecture": "Bamipel", "vocab": vocab, "width": width, "norm": {"eps": eps}, "layers": out, "torch_dtype": dtype}
+
+
 SHAPES: Dict[str, dict] = {
+    "bamipel-tiny": _bamipel(5, 64, 4, 2, 16, 24, 96, 256, window=12, eps=1e-5, dtype="float32", rot=8, latent_heads=2, latent_dim=12,
+                             latent_rot=4, latent_vdim=8, q_rank=28, kv_rank=20, delta_heads=4, delta_kv_heads=2, delta_dim=12,
+                             delta_vdim=8, conv=3, scaling={"factor": 4.0, "low": 1.0, "high": 4.0, "original": 64}, again={4: 0}),
+    "bamipel-1b": _bamipel(16, 2048, 16, 8, 128, 128, 9216, 32768, window=1024),
     "pemuvik-tiny": _pemuvik(4, 64, 4, 2, 16, 24, 96, 256, window=12, eps=1e-5, dtype="float32", rot=8, latent_heads=2, latent_dim=12,
                              latent_rot=4, latent_vdim=8, kv_rank=20, experts=6, top=2, identity=2, group_count=4, group_keep=2),
     "pemuvik-1b": _pemuvik(16, 2048, 16, 8, 128, 128, 6144, 32768, window=1024, experts=30, group_count=4, group_keep=2),

@@ -98,12 +98,12 @@ def head_gates(h, wg):
     return torch.sigmoid(h @ wg.T)
 
 
-def latent_parts(h, m, w, p, eps):
-    """Queries (plain and rotated parts), keys (plain per head, one rotated part) and values of every token."""
-    T, H, D, R, DV, C = h.shape[0], m["heads"], m["dim"], m["rot_dim"], m["vdim"], m["kv_rank"]
-    cq = unit_mean(h @ w[p + "dq"].T, eps) * w[p + "dq.norm"]
+def latent_parts(cq_raw, low, m, w, p, eps):
+    """From the two latents' projections: queries (plain and rotated parts), keys (plain per head, one rotated part) and
+    values of every token."""
+    T, H, D, R, DV, C = low.shape[0], m["heads"], m["dim"], m["rot_dim"], m["vdim"], m["kv_rank"]
+    cq = unit_mean(cq_raw, eps) * w[p + "dq.norm"]
     q = (cq @ w[p + "uq"].T).view(T, H, D + R)
-    low = h @ w[p + "dkv"].T
     c = unit_mean(low[:, :C], eps) * w[p + "dkv.norm"]
     k_turn = turn_halves(low[:, C:].reshape(T, 1, R), m["rot"])[:, 0]
     return (q[:, :, :D], turn_halves(q[:, :, D:], m["rot"]), (c @ w[p + "uk"].T).view(T, H, D), k_turn,
@@ -124,7 +124,7 @@ def latent_attend(q_plain, q_turn, k_plain, k_turn, v, scale, window, rows=None)
 
 def latent_attention(h, m, w, p, eps):
     window = m["mask"]["size"] if m.get("mask") else None
-    o = latent_attend(*latent_parts(h, m, w, p, eps), m["scale"], window)
+    o = latent_attend(*latent_parts(h @ w[p + "dq"].T, h @ w[p + "dkv"].T, m, w, p, eps), m["scale"], window)
     o = o * head_gates(h, w[p + "g"])[:, :, None]
     return o.reshape(h.shape[0], -1) @ w[p + "o"].T
 
@@ -172,30 +172,28 @@ def delta_step(S, q, k, v, beta, a):
     return S, S.T @ q
 
 
-def delta_inputs(h, m, w, p):
-    """Unit queries and keys [T, G, D], values [T, H, DV], write strengths and decays [T, H]."""
-    T, H, G, D, DV = h.shape[0], m["heads"], m["kv_heads"], m["dim"], m["vdim"]
-    q, k, v = (silu(causal_convolution(h @ w[p + n].T, w[p + n + ".conv"])) for n in ("q", "k", "v"))
+def delta_of_projections(q, k, v, gate, b, z, m, w, p, eps):
+    """The rule on the tokens' projections (z: the decays' input before dt_bias) -> [T, H * DV]."""
+    T, H, G, D, DV = q.shape[0], m["heads"], m["kv_heads"], m["dim"], m["vdim"]
+    q, k, v = (silu(causal_convolution(x, w[p + n + ".conv"])) for n, x in (("q", q), ("k", k), ("v", v)))
     q, k, v = q.view(T, G, D), k.view(T, G, D), v.view(T, H, DV)
     q = q / torch.sqrt(q.pow(2).sum(-1, keepdim=True) + 1e-6) * D ** -0.5
     k = k / torch.sqrt(k.pow(2).sum(-1, keepdim=True) + 1e-6)
-    beta = torch.sigmoid(h @ w[p + "b"].T)
-    z = h @ w[p + "a"].T + w[p + "dt_bias"]
-    a = torch.exp(-torch.exp(w[p + "A_log"]) * torch.log1p(torch.exp(-z.abs())).add(z.clamp(min=0)))
-    return q, k, v, beta, a
+    beta = torch.sigmoid(b)
+    z = z + w[p + "dt_bias"]
+    a = torch.exp(-torch.exp(w[p + "A_log"]) * (torch.log1p(torch.exp(-z.abs())) + z.clamp(min=0)))
+    o = torch.zeros(T, H, DV, dtype=v.dtype)
+    for head in range(H):
+        g = head // (H // G)
+        S = torch.zeros(D, DV, dtype=v.dtype)
+        for t in range(T):
+            S, o[t, head] = delta_step(S, q[t, g], k[t, g], v[t, head], beta[t, head], a[t, head])
+    return (unit_mean(o, eps) * w[p + "norm"] * silu(gate).view(T, H, DV)).reshape(T, -1)
 
 
 def delta_mixer(h, m, w, p, eps):
-    T, H, G, D, DV = h.shape[0], m["heads"], m["kv_heads"], m["dim"], m["vdim"]
-    q, k, v, beta, a = delta_inputs(h, m, w, p)
-    o = torch.zeros(T, H, DV, dtype=h.dtype)
-    for head in range(H):
-        g = head // (H // G)
-        S = torch.zeros(D, DV, dtype=h.dtype)
-        for t in range(T):
-            S, o[t, head] = delta_step(S, q[t, g], k[t, g], v[t, head], beta[t, head], a[t, head])
-    y = unit_mean(o, eps) * w[p + "norm"] * silu(h @ w[p + "g"].T).view(T, H, DV)
-    return y.reshape(T, -1) @ w[p + "o"].T
+    q, k, v, gate, b, z = (h @ w[p + n].T for n in ("q", "k", "v", "g", "b", "a"))
+    return delta_of_projections(q, k, v, gate, b, z, m, w, p, eps) @ w[p + "o"].T
 
 
 MIXERS = {"latent_attention": latent_attention, "attention": grouped_attention, "delta": delta_mixer}
