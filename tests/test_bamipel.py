@@ -309,7 +309,7 @@ def _lat(H_, D, R, DV, Q, C, window, base=1e3, scale=0.2):
     (_lat(2, 24, 16, 40, 24, 16, 33), 16, [50, 33], [17, 33]),
     (_lat(2, 64, 16, 32, 48, 176, 70), 64, [200], [37]),                            # key rows of more than 128 entries
     (_lat(2, 16, 32, 16, 40, 96, None), 64, [1, 200], [1, 150]),                    # no window; the first token of a sequence
-    (_lat(20, 32, 64, 32, 96, 384, 500), 64, [1500, 33, 700], [1, 1, 40]),          # shares of a token's window
+    (_lat(20, 32, 64, 32, 96, 384, 500, scale=0.05), 64, [1500, 33, 700], [1, 1, 40]),          # shares of a token's window
     (_lat(5, 24, 24, 40, 32, 80, 300), 32, [1000, 2, 640], [1, 1, 50]),             # a key row that ends inside a step of 32 channels
 ])
 def test_attention_through_latents_with_a_window(backend, dtype, m, page, lens, q_lens):
