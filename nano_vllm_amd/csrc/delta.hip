@@ -28,20 +28,50 @@
 //                     portion's tokens, the tokens' q, k, a and beta staged in LDS a batch at a time in two buffers,
 //                     v asked for a batch ahead
 //   delta_finish      one wave per (token, head): the norm and the gate
+//
+// With one decay per head two more ways run the same rule:
+//   delta_single      a request that brings one token: everything above for one (request, value head) in one workgroup
+//   delta_block_*     portions of many tokens, in blocks of 64 on the matrix cores (float products).  With G_i the sum of
+//                     the logarithms of the decays up to token i of a block, S_0 the state before the block, and
+//                     A_ij = beta_i exp(G_i - G_j) k_i.k_j for j < i, the writes of the block are
+//                         (I + A) u = beta v - beta exp(G) k^T S_0      (row i: beta_i v_i - beta_i exp(G_i) S_0^T k_i)
+//                     so u = U - W S_0 with (I + A) U = beta v and (I + A) W = beta exp(G) k, both by forward substitution
+//                     row by row; then o_i = exp(G_i) S_0^T q_i + sum over j <= i of P_ij u_j with P_ij = exp(G_i - G_j)
+//                     q_i.k_j, and the state behind the block is exp(G_63) S_0 + sum over j of exp(G_63 - G_j) k_j u_j^T.
+//     delta_block_prepare   the convolutions, unit norms, beta and log decays, 16 tokens of a head to a workgroup
+//     delta_block_solve     a workgroup per (block, head): A and P by products, U and W by substitution, a column a thread
+//     delta_block_scan      a workgroup per (portion, head, 16 columns of S): the blocks one after the other
 #include "common.h"
+
+typedef __attribute__((ext_vector_type(4))) float delta_f32x4;
 
 #define DELTA_MAX_TAPS 16
 #define DELTA_BATCH 8            // tokens whose q, k and a lie in LDS at a time
 #define DELTA_THREADS 256        // of the recurrence's workgroup: four waves
 #define DELTA_MAX_DIM 256        // key channels of a head at most
 #define DELTA_PREPARE_THREADS 128
+#define DELTA_BLOCK 64            // tokens of a block of the matrix-core form
+#define DELTA_SINGLE_THREADS 512
 
 // One workgroup per (token, unit); a unit is a query head, a key head, or a value head with its decays and beta.
 // Rows of qn, kn and decay are DP = dim rounded up to 4 floats apart, the padding zero.
-// HEAD: one decay per value head ([tokens, heads] of `decay`); decay_in is then rates.
+// Entry i of a token's rates [b | a], which may be left as partial sums of their product.
+struct DeltaRates {
+    const float* sums;               // [splits][tokens][2 heads]
+    int splits;
+    int64_t split_stride;
+};
+__device__ __forceinline__ float delta_rate(const DeltaRates& r, int64_t t, int heads, int i) {
+    float v = 0.f;
+    for (int s = 0; s < r.splits; ++s) v += r.sums[s * r.split_stride + t * (2 * heads) + i];
+    return v;
+}
+__device__ __forceinline__ float delta_softplus(float z) { return z > 20.f ? z : log1pf(expf(z)); }
+
+// HEAD: one decay per value head; `decay` [tokens, heads] then receives its logarithm.  t0: the first token of the launch.
 template <typename T, bool HEAD>
 __global__ void __launch_bounds__(DELTA_PREPARE_THREADS)
-delta_prepare_kernel(const T* __restrict__ proj, int64_t stride, const float* __restrict__ decay_in,
+delta_prepare_kernel(const T* __restrict__ proj, int64_t stride, const float* __restrict__ decay_in, DeltaRates rates, int64_t t0,
                      const T* __restrict__ conv_w, const float* __restrict__ dt_bias, const float* __restrict__ a_log,
                      const float* __restrict__ conv_state, const int32_t* __restrict__ token_seq,
                      const int32_t* __restrict__ cu_seqlens_q, const int32_t* __restrict__ seq_starts,
@@ -49,7 +79,7 @@ delta_prepare_kernel(const T* __restrict__ proj, int64_t stride, const float* __
                      float* __restrict__ qn, float* __restrict__ kn, float* __restrict__ vf, float* __restrict__ decay,
                      float* __restrict__ beta) {
     __shared__ float sum_s[16];
-    const int64_t t = blockIdx.x;
+    const int64_t t = t0 + blockIdx.x;
     const int unit = blockIdx.y;
     const int seq = token_seq[t];
     const int begin = cu_seqlens_q[seq];
@@ -98,9 +128,8 @@ delta_prepare_kernel(const T* __restrict__ proj, int64_t stride, const float* __
     const float rate = expf(a_log[h]);
     if (HEAD) {
         if (tid == 0) {
-            const float z = decay_in[t * (2 * heads) + heads + h] + dt_bias[h];
-            decay[t * heads + h] = expf(-rate * (z > 20.f ? z : log1pf(expf(z))));
-            beta[t * heads + h] = 1.f / (1.f + expf(-decay_in[t * (2 * heads) + h]));
+            decay[t * heads + h] = -rate * delta_softplus(delta_rate(rates, t, heads, heads + h) + dt_bias[h]);
+            beta[t * heads + h] = 1.f / (1.f + expf(-delta_rate(rates, t, heads, h)));
         }
         return;
     }
@@ -108,8 +137,7 @@ delta_prepare_kernel(const T* __restrict__ proj, int64_t stride, const float* __
         float a = 0.f;
         if (d < dim) {
             const float z = decay_in[t * (int64_t)(heads * dim) + h * dim + d] + dt_bias[h * dim + d];
-            const float step = z > 20.f ? z : log1pf(expf(z));
-            a = expf(-rate * step);
+            a = expf(-rate * delta_softplus(z));
         }
         decay[(t * heads + h) * dp + d] = a;
     }
@@ -209,7 +237,7 @@ delta_scan_kernel(const float* __restrict__ qn, const float* __restrict__ kn, co
             pre[i] = x;
         }
         pre_beta = tid < nb ? beta[(int64_t)(begin + t0 + tid) * heads + h] : 0.f;
-        if (HEAD) pre_decay = tid < nb ? decay[(int64_t)(begin + t0 + tid) * heads + h] : 0.f;
+        if (HEAD) pre_decay = tid < nb ? expf(decay[(int64_t)(begin + t0 + tid) * heads + h]) : 0.f;
     };
     auto put = [&](int buf) __attribute__((always_inline)) {
         float4* flat = &qka_s[buf][0][0][0];
@@ -316,8 +344,8 @@ template <typename T, bool SILU>
 __global__ void __launch_bounds__(NVA_WAVE)
 delta_finish_kernel(const float* __restrict__ o_raw, const T* __restrict__ gate, int64_t gate_stride,
                     const float* __restrict__ norm_w, float eps, T* __restrict__ out, int64_t out_stride, int heads,
-                    int vdim) {
-    const int64_t t = blockIdx.x;
+                    int vdim, int64_t t0) {
+    const int64_t t = t0 + blockIdx.x;
     const int h = blockIdx.y, lane = threadIdx.x;
     const float* o = o_raw + (t * heads + h) * (int64_t)vdim;
     float ss = 0.f;
@@ -331,59 +359,491 @@ delta_finish_kernel(const float* __restrict__ o_raw, const T* __restrict__ gate,
     }
 }
 
-// What both forms of the rule launch.  HEAD: decay_in is rates, float [tokens, 2 H], and the decays are one per head.
-template <bool HEAD>
-static int launch_delta(const char* what, const void* proj, int64_t stride, int64_t need, const float* decay_in, const void* gate_in,
-                        int64_t gate_stride, float* scratch, void* out, int64_t out_stride, float* s_state, float* conv_state,
-                        const int32_t* token_seq, const int32_t* cu_seqlens_q, const int32_t* seq_starts,
-                        const int32_t* state_slots, int64_t seqs, int64_t tokens, int heads, int kv_heads, int dim, int vdim,
-                        int taps, const void* conv_w, const float* dt_bias, const float* a_log, const float* norm_w, float eps,
-                        hipStream_t stream) {
-    if (tokens == 0) return 0;
-    if (tokens < 0 || tokens > 0x7fffffff || seqs <= 0 || seqs > 65535 * 32)
+// ---------------------------------------------------------------------------- single tokens, one decay per head
+// One workgroup per (request, value head) of the requests that bring one token; token t of the step is request t's.
+// Thread (r, c4) holds the columns 4 c4 .. + 3 of the rows r, r + RG, ... of S, CG = 512 / RG column groups (a power of
+// two).  The two sums over the rows run inside a thread, then over the RG threads of a column in order.  keep: the
+// workgroup also moves on the kept inputs of its channels (only where no other workgroup reads them: as many query/key
+// heads as value heads).
+template <typename T, int R>
+__global__ void __launch_bounds__(DELTA_SINGLE_THREADS)
+delta_single_kernel(const T* __restrict__ proj, int64_t stride, DeltaRates rates, const T* __restrict__ conv_w,
+                    const float* __restrict__ dt_bias, const float* __restrict__ a_log, const float* __restrict__ norm_w,
+                    float eps, float* __restrict__ s_state, float* __restrict__ conv_state,
+                    const int32_t* __restrict__ seq_starts, const int32_t* __restrict__ state_slots, int heads, int kv_heads,
+                    int dim, int vdim, int taps, int cg_log, int keep, T* __restrict__ out, int64_t out_stride) {
+    extern __shared__ __attribute__((aligned(16))) float single_s[];
+    __shared__ float scratch[16], sums_s[2];
+    const int CG = 1 << cg_log, RG = DELTA_SINGLE_THREADS >> cg_log;
+    const int vp = 4 * CG;                                              // columns, padded
+    float* const row_s = single_s;                                      // [2 dim + vdim]: q, k, v
+    float* const u_s = row_s + ((2 * dim + vdim + 3) & ~3);             // [vp]
+    float* const red_s = u_s + vp;                                      // [RG][vp]
+    const int64_t t = blockIdx.x;
+    const int h = blockIdx.y, tid = threadIdx.x;
+    const int g = h / (heads / kv_heads);
+    const int qk = kv_heads * dim, vv = heads * vdim, channels = 2 * qk + vv;
+    const int slot = state_slots[t];
+    const bool has_past = seq_starts[t] > 0;
+    const int c4 = tid & (CG - 1), r = tid >> cg_log;
+    const bool live = 4 * c4 < vdim;
+    float* S_g = s_state + ((int64_t)slot * heads + h) * dim * vdim + 4 * c4;
+    delta_f32x4 S[R];
+#pragma unroll
+    for (int i = 0; i < R; ++i) {
+        const int row = r + RG * i;
+        S[i] = delta_f32x4{0.f, 0.f, 0.f, 0.f};
+        if (has_past && live && row < dim) S[i] = *reinterpret_cast<const delta_f32x4*>(S_g + (int64_t)row * vdim);
+    }
+    const float gate_z = tid < vdim ? to_float(proj[t * stride + channels + h * vdim + tid]) : 0.f;
+    const float a = expf(-expf(a_log[h]) * delta_softplus(delta_rate(rates, t, heads, heads + h) + dt_bias[h]));
+    const float beta = 1.f / (1.f + expf(-delta_rate(rates, t, heads, h)));
+    for (int i = tid; i < 2 * dim + vdim; i += DELTA_SINGLE_THREADS) {
+        const int c = i < dim ? g * dim + i : i < 2 * dim ? qk + g * dim + (i - dim) : 2 * qk + h * vdim + (i - 2 * dim);
+        float* kept = conv_state + ((int64_t)slot * channels + c) * (taps - 1);
+        const float x = to_float(proj[t * stride + c]);
+        float sum = 0.f;
+        for (int j = 0; j < taps - 1; ++j) {
+            const float old = has_past ? kept[j] : 0.f;
+            sum += to_float(conv_w[(int64_t)c * taps + j]) * old;
+            if (keep && j > 0) kept[j - 1] = old;
+        }
+        if (keep && taps > 1) kept[taps - 2] = x;
+        sum += to_float(conv_w[(int64_t)c * taps + taps - 1]) * x;
+        row_s[i] = sum / (1.f + expf(-sum));
+    }
+    __syncthreads();
+    const int wave = tid / NVA_WAVE, lane = tid % NVA_WAVE;
+    if (wave < 2) {
+        float ss = 0.f;
+        for (int d = lane; d < dim; d += NVA_WAVE) ss += row_s[wave * dim + d] * row_s[wave * dim + d];
+        ss = wave_sum(ss);
+        if (lane == 0) sums_s[wave] = ss;
+    }
+    __syncthreads();
+    const float q_scale = (1.f / sqrtf(sums_s[0] + 1e-6f)) * (1.f / sqrtf((float)dim)), k_scale = 1.f / sqrtf(sums_s[1] + 1e-6f);
+    float kr[R], qr[R];
+    delta_f32x4 d = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int i = 0; i < R; ++i) {
+        const int row = r + RG * i;
+        kr[i] = row < dim ? row_s[dim + row] * k_scale : 0.f;
+        qr[i] = row < dim ? row_s[row] * q_scale : 0.f;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) d[e] += S[i][e] * kr[i];
+    }
+    *reinterpret_cast<delta_f32x4*>(&red_s[r * vp + 4 * c4]) = d;
+    __syncthreads();
+    if (tid < vp) {
+        float read = 0.f;
+        for (int i = 0; i < RG; ++i) read += red_s[i * vp + tid];
+        u_s[tid] = tid < vdim ? beta * (row_s[2 * dim + tid] - a * read) : 0.f;
+    }
+    __syncthreads();
+    const delta_f32x4 u = *reinterpret_cast<const delta_f32x4*>(&u_s[4 * c4]);
+    delta_f32x4 o = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int i = 0; i < R; ++i) {
+        const int row = r + RG * i;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+            S[i][e] = a * S[i][e] + kr[i] * u[e];
+            o[e] += S[i][e] * qr[i];
+        }
+        if (live && row < dim) *reinterpret_cast<delta_f32x4*>(S_g + (int64_t)row * vdim) = S[i];
+    }
+    *reinterpret_cast<delta_f32x4*>(&red_s[r * vp + 4 * c4]) = o;
+    __syncthreads();
+    float oc = 0.f;
+    if (tid < vdim)
+        for (int i = 0; i < RG; ++i) oc += red_s[i * vp + tid];
+    const float ss = block_sum(oc * oc, scratch);
+    const float scale = 1.f / sqrtf(ss / (float)vdim + eps);
+    if (tid < vdim)
+        out[t * out_stride + h * vdim + tid] = from_float<T>(oc * scale * norm_w[tid] * gate_z / (1.f + expf(-gate_z)));
+}
+
+// ---------------------------------------------------------------------------- portions in blocks, one decay per head
+// units: int32 [n][4] = (request, the block's first token counted through the step, its tokens, unused); a portion's blocks
+// side by side.  Scratch of block u and head h, each indexed by ub = u * heads + h: g_cum [ub][64], w [ub][64][DP],
+// u [ub][64][DV], p [ub][64][64], k_t [ub][DP][64]; tokens past a block's end are rows of zeros.
+template <typename T, int TAPS>
+__global__ void __launch_bounds__(DELTA_PREPARE_THREADS)
+delta_block_prepare_kernel(const T* __restrict__ proj, int64_t stride, DeltaRates rates, const T* __restrict__ conv_w,
+                           const float* __restrict__ dt_bias, const float* __restrict__ a_log,
+                           const float* __restrict__ conv_state, const int32_t* __restrict__ units,
+                           const int32_t* __restrict__ cu_seqlens_q, const int32_t* __restrict__ seq_starts,
+                           const int32_t* __restrict__ state_slots, int heads, int kv_heads, int dim, int vdim,
+                           float* __restrict__ qn, float* __restrict__ kn, float* __restrict__ vf, float* __restrict__ decay,
+                           float* __restrict__ beta) {
+    constexpr int N = 16;                                               // tokens of a workgroup
+    __shared__ float part_s[DELTA_PREPARE_THREADS / NVA_WAVE][N];
+    const int32_t* un = units + 4 * (blockIdx.x / (DELTA_BLOCK / N));
+    const int t0 = N * (blockIdx.x % (DELTA_BLOCK / N));
+    const int seq = un[0], n = un[2] - t0;
+    if (n <= 0) return;
+    const int nt = min(n, N);
+    const int64_t tok0 = un[1] + t0;
+    const int begin = cu_seqlens_q[seq], local0 = (int)tok0 - begin;
+    const bool has_past = seq_starts[seq] > 0;
+    const int slot = state_slots[seq];
+    const int qk = kv_heads * dim, vv = heads * vdim, channels = 2 * qk + vv;
+    const int dp = (dim + 3) & ~3;
+    const int unit = blockIdx.y, tid = threadIdx.x;
+    auto conv_silu = [&](int c, float* y) __attribute__((always_inline)) {
+        float w[TAPS], x[TAPS], in[N];
+#pragma unroll
+        for (int j = 0; j < TAPS; ++j) w[j] = to_float(conv_w[(int64_t)c * TAPS + j]);
+#pragma unroll
+        for (int i = 0; i < N; ++i) in[i] = to_float(proj[(tok0 + min(i, nt - 1)) * stride + c]);
+#pragma unroll
+        for (int j = 0; j < TAPS - 1; ++j) {
+            const int src = local0 - (TAPS - 1) + j;                    // < 0: before the portion
+            x[j] = 0.f;
+            if (src >= 0) x[j] = to_float(proj[(int64_t)(begin + src) * stride + c]);
+            else if (has_past) x[j] = conv_state[((int64_t)slot * channels + c) * (TAPS - 1) + (TAPS - 1 + src)];
+        }
+#pragma unroll
+        for (int i = 0; i < N; ++i) {
+            x[TAPS - 1] = in[i];
+            float sum = 0.f;
+#pragma unroll
+            for (int j = 0; j < TAPS; ++j) sum += w[j] * x[j];
+            y[i] = sum / (1.f + expf(-sum));
+#pragma unroll
+            for (int j = 0; j < TAPS - 1; ++j) x[j] = x[j + 1];
+        }
+    };
+    if (unit < 2 * kv_heads) {
+        constexpr int PER = (DELTA_MAX_DIM + DELTA_PREPARE_THREADS - 1) / DELTA_PREPARE_THREADS;
+        float y[PER][N], ss[N];
+#pragma unroll
+        for (int i = 0; i < N; ++i) ss[i] = 0.f;
+#pragma unroll
+        for (int p = 0; p < PER; ++p) {
+            const int d = p * DELTA_PREPARE_THREADS + tid;
+#pragma unroll
+            for (int i = 0; i < N; ++i) y[p][i] = 0.f;
+            if (d < dim) conv_silu(unit * dim + d, y[p]);
+#pragma unroll
+            for (int i = 0; i < N; ++i) ss[i] += y[p][i] * y[p][i];
+        }
+#pragma unroll
+        for (int i = 0; i < N; ++i) {
+            const float s = wave_sum(ss[i]);
+            if (tid % NVA_WAVE == 0) part_s[tid / NVA_WAVE][i] = s;
+        }
+        __syncthreads();
+        const bool is_q = unit < kv_heads;
+        float* dst = (is_q ? qn : kn) + (tok0 * kv_heads + (is_q ? unit : unit - kv_heads)) * dp;
+#pragma unroll
+        for (int i = 0; i < N; ++i) {
+            if (i >= nt) break;
+            float scale = 1.f / sqrtf(part_s[0][i] + part_s[1][i] + 1e-6f);
+            if (is_q) scale *= 1.f / sqrtf((float)dim);
+#pragma unroll
+            for (int p = 0; p < PER; ++p) {
+                const int d = p * DELTA_PREPARE_THREADS + tid;
+                if (d < dp) dst[(int64_t)i * kv_heads * dp + d] = y[p][i] * scale;      // (zeros in the padding)
+            }
+        }
+        return;
+    }
+    const int h = unit - 2 * kv_heads;
+    for (int d = tid; d < vdim; d += DELTA_PREPARE_THREADS) {
+        float y[N];
+        conv_silu(2 * qk + h * vdim + d, y);
+#pragma unroll
+        for (int i = 0; i < N; ++i)
+            if (i < nt) vf[(tok0 + i) * vv + h * vdim + d] = y[i];
+    }
+    if (tid < nt) {
+        decay[(tok0 + tid) * heads + h] = -expf(a_log[h]) * delta_softplus(delta_rate(rates, tok0 + tid, heads, heads + h) + dt_bias[h]);
+        beta[(tok0 + tid) * heads + h] = 1.f / (1.f + expf(-delta_rate(rates, tok0 + tid, heads, h)));
+    }
+}
+
+// KB: steps of 16 key channels (dim <= 16 KB).  Products by v_mfma_f32_16x16x4_f32: lane l holds row (or column) l % 16 and,
+// over the four instructions of a step of 16 channels, the channels 4 (l / 16) + j of both operands; results: row
+// 4 (l / 16) + i, column l % 16.
+template <int KB>
+__global__ void __launch_bounds__(256)
+delta_block_solve_kernel(const float* __restrict__ qn, const float* __restrict__ kn, const float* __restrict__ vf,
+                         const float* __restrict__ decay, const float* __restrict__ beta, const int32_t* __restrict__ units,
+                         int heads, int kv_heads, int dim, int vdim, float* __restrict__ g_cum, float* __restrict__ w_out,
+                         float* __restrict__ u_out, float* __restrict__ p_out, float* __restrict__ kt_out) {
+    __shared__ __attribute__((aligned(16))) float a_s[DELTA_BLOCK][DELTA_BLOCK + 4];
+    __shared__ float g_s[DELTA_BLOCK], b_s[DELTA_BLOCK], bg_s[DELTA_BLOCK], eg_s[DELTA_BLOCK];
+    const int h = blockIdx.x % heads;
+    const int64_t ub = blockIdx.x;
+    const int32_t* un = units + 4 * (blockIdx.x / heads);
+    const int64_t first = un[1];
+    const int n = un[2];
+    const int kvh = h / (heads / kv_heads);
+    const int dp = (dim + 3) & ~3, vv = heads * vdim;
+    const int tid = threadIdx.x, wave = tid / NVA_WAVE, lane = tid % NVA_WAVE, col = lane & 15, g = lane >> 4;
+    if (wave == 0) {
+        float sum = lane < n ? decay[(first + lane) * heads + h] : 0.f;
+#pragma unroll
+        for (int off = 1; off < NVA_WAVE; off <<= 1) {
+            const float up = __shfl_up(sum, off, NVA_WAVE);
+            if (lane >= off) sum += up;
+        }
+        const float be = lane < n ? beta[(first + lane) * heads + h] : 0.f;
+        g_s[lane] = sum;
+        b_s[lane] = be;
+        bg_s[lane] = be * expf(sum);
+        eg_s[lane] = expf(__shfl(sum, NVA_WAVE - 1, NVA_WAVE) - sum);
+        g_cum[ub * DELTA_BLOCK + lane] = sum;
+    }
+    __syncthreads();
+    // the ten blocks of 16 x 16 on and below the diagonal, of k k^T and of q k^T
+    for (int task = wave; task < 20; task += 4) {
+        const int pair = task >> 1;
+        const bool of_q = task & 1;
+        const int bi = pair < 1 ? 0 : pair < 3 ? 1 : pair < 6 ? 2 : 3, bj = pair - bi * (bi + 1) / 2;
+        const float* ar = (of_q ? qn : kn) + ((first + min(16 * bi + col, n - 1)) * kv_heads + kvh) * dp + 4 * g;
+        const float* br = kn + ((first + min(16 * bj + col, n - 1)) * kv_heads + kvh) * dp + 4 * g;
+        delta_f32x4 fa[KB], fb[KB];
+#pragma unroll
+        for (int s = 0; s < KB; ++s) {
+            fa[s] = fb[s] = delta_f32x4{0.f, 0.f, 0.f, 0.f};
+            if (16 * s + 4 * g < dp) {
+                fa[s] = *reinterpret_cast<const delta_f32x4*>(ar + 16 * s);
+                fb[s] = *reinterpret_cast<const delta_f32x4*>(br + 16 * s);
+            }
+        }
+        delta_f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int s = 0; s < KB; ++s)
+#pragma unroll
+            for (int j = 0; j < 4; ++j) acc = __builtin_amdgcn_mfma_f32_16x16x4f32(fa[s][j], fb[s][j], acc, 0, 0, 0);
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+            const int r = 16 * bi + 4 * g + i, c = 16 * bj + col;
+            const bool seen = r < n && (of_q ? c <= r : c < r);
+            const float v = seen ? expf(g_s[r] - g_s[c]) * acc[i] : 0.f;
+            if (of_q) p_out[(ub * DELTA_BLOCK + r) * DELTA_BLOCK + c] = v;
+            else a_s[r][c] = b_s[r] * v;
+        }
+    }
+    __syncthreads();
+    // forward substitution: a thread a column, of beta v (the first DV) and of beta exp(G) k (the DP behind them)
+    for (int base = 0; base < vdim + dp; base += 256) {
+        const int c = base + tid;
+        if (c >= vdim + dp) break;
+        const bool of_v = c < vdim;
+        const int d = of_v ? c : c - vdim;
+        const float* src = of_v ? vf + first * vv + h * vdim + d : kn + (first * kv_heads + kvh) * dp + d;
+        const int64_t step = of_v ? vv : (int64_t)kv_heads * dp;
+        float x[DELTA_BLOCK];
+#pragma unroll
+        for (int i = 0; i < DELTA_BLOCK; ++i) x[i] = src[min(i, n - 1) * step];
+        if (!of_v) {
+            float* kt = kt_out + (ub * dp + d) * DELTA_BLOCK;
+#pragma unroll
+            for (int i = 0; i < DELTA_BLOCK; i += 4) {
+                delta_f32x4 v;
+#pragma unroll
+                for (int e = 0; e < 4; ++e) v[e] = i + e < n ? x[i + e] * eg_s[i + e] : 0.f;
+                *reinterpret_cast<delta_f32x4*>(kt + i) = v;
+            }
+        }
+        const float* scale = of_v ? b_s : bg_s;                         // (zero past the block's end)
+#pragma unroll
+        for (int i = 0; i < DELTA_BLOCK; ++i) x[i] *= scale[i];
+#pragma unroll
+        for (int i = 1; i < DELTA_BLOCK; ++i) {
+            float s[4] = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (int j = 0; j + 4 <= i; j += 4) {
+                const delta_f32x4 a = *reinterpret_cast<const delta_f32x4*>(&a_s[i][j]);
+#pragma unroll
+                for (int e = 0; e < 4; ++e) s[e] += a[e] * x[j + e];
+            }
+#pragma unroll
+            for (int j = i / 4 * 4; j < i; ++j) s[j % 4] += a_s[i][j] * x[j];
+            x[i] -= (s[0] + s[1]) + (s[2] + s[3]);
+        }
+        float* dst = of_v ? u_out + ub * DELTA_BLOCK * vdim + d : w_out + ub * DELTA_BLOCK * dp + d;
+        const int width = of_v ? vdim : dp;
+#pragma unroll
+        for (int i = 0; i < DELTA_BLOCK; ++i) dst[(int64_t)i * width] = x[i];
+    }
+}
+
+// The workgroup's barrier, after this wave's own LDS traffic is done (loads on their way into registers are not waited for).
+__device__ __forceinline__ void delta_barrier() { asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory"); }
+
+// chains: int32 [n][4] = (a portion's first block, its blocks, its request, unused).  One workgroup of four waves per (head,
+// portion, 16 columns of S), heads fastest, so that the workgroups of a head meet in one die's L2.  The state's columns lie
+// in accumulators (wave w: the blocks w, w + 4, ... of 16 rows) and, transposed, in LDS for the products that read them.
+template <int KB>
+__global__ void __launch_bounds__(256)
+delta_block_scan_kernel(const float* __restrict__ qn, const float* __restrict__ g_cum, const float* __restrict__ w_in,
+                        const float* __restrict__ u_in, const float* __restrict__ p_in, const float* __restrict__ kt_in,
+                        float* __restrict__ o_raw, float* __restrict__ state, const int32_t* __restrict__ units,
+                        const int32_t* __restrict__ chains, int num_chains, const int32_t* __restrict__ seq_starts,
+                        const int32_t* __restrict__ state_slots, int heads, int kv_heads, int dim, int vdim) {
+    constexpr int NB = (KB + 3) / 4;
+    __shared__ __attribute__((aligned(16))) float s_s[16][16 * KB + 4];     // [column][row]
+    __shared__ __attribute__((aligned(16))) float u_s[16][DELTA_BLOCK + 4]; // [column][token]
+    const int h = blockIdx.x % heads, rest = blockIdx.x / heads;
+    const int32_t* ch = chains + 4 * (rest % num_chains);
+    const int unit0 = ch[0], blocks = ch[1], seq = ch[2];
+    const int tid = threadIdx.x, wave = tid / NVA_WAVE, lane = tid % NVA_WAVE, col = lane & 15, g = lane >> 4;
+    const int column = 16 * (rest / num_chains) + col;
+    const bool live = column < vdim;
+    const int kvh = h / (heads / kv_heads);
+    const int dp = (dim + 3) & ~3, vv = heads * vdim;
+    float* S_g = state + ((int64_t)state_slots[seq] * heads + h) * dim * vdim + column;
+    const bool has_past = seq_starts[seq] > 0;
+    delta_f32x4 S[NB];
+#pragma unroll
+    for (int b = 0; b < NB; ++b) {
+        const int kb = wave + 4 * b;
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+            const int row = 16 * kb + 4 * g + i;
+            S[b][i] = has_past && live && row < dim ? S_g[(int64_t)row * vdim] : 0.f;
+        }
+        if (kb < KB) *reinterpret_cast<delta_f32x4*>(&s_s[col][16 * kb + 4 * g]) = S[b];
+    }
+    delta_f32x4 wf[KB], qf[KB];
+    auto ask = [&](int blk) __attribute__((always_inline)) {
+        const int32_t* un = units + 4 * (unit0 + blk);
+        const int64_t ub = (int64_t)(unit0 + blk) * heads + h;
+        const float* wr = w_in + (ub * DELTA_BLOCK + 16 * wave + col) * dp + 4 * g;
+        const float* qr = qn + ((un[1] + min(16 * wave + col, un[2] - 1)) * (int64_t)kv_heads + kvh) * dp + 4 * g;
+#pragma unroll
+        for (int s = 0; s < KB; ++s) {
+            wf[s] = qf[s] = delta_f32x4{0.f, 0.f, 0.f, 0.f};
+            if (16 * s + 4 * g < dp) {
+                wf[s] = *reinterpret_cast<const delta_f32x4*>(wr + 16 * s);
+                qf[s] = *reinterpret_cast<const delta_f32x4*>(qr + 16 * s);
+            }
+        }
+    };
+    ask(0);
+    delta_barrier();
+    for (int blk = 0; blk < blocks; ++blk) {
+        const int64_t ub = (int64_t)(unit0 + blk) * heads + h;
+        const int64_t first = units[4 * (unit0 + blk) + 1];
+        const int n = units[4 * (unit0 + blk) + 2];
+        // what the second half reads is asked for before the first half's products
+        delta_f32x4 pf[4], kt[NB][4];
+        const float* pr = p_in + (ub * DELTA_BLOCK + 16 * wave + col) * DELTA_BLOCK + 4 * g;
+#pragma unroll
+        for (int s = 0; s < 4; ++s) {
+            pf[s] = delta_f32x4{0.f, 0.f, 0.f, 0.f};
+            if (s <= wave) pf[s] = *reinterpret_cast<const delta_f32x4*>(pr + 16 * s);
+        }
+#pragma unroll
+        for (int b = 0; b < NB; ++b) {
+            const int row = 16 * (wave + 4 * b) + col;
+#pragma unroll
+            for (int s = 0; s < 4; ++s) {
+                kt[b][s] = delta_f32x4{0.f, 0.f, 0.f, 0.f};
+                if (row < dp) kt[b][s] = *reinterpret_cast<const delta_f32x4*>(kt_in + (ub * dp + row) * DELTA_BLOCK + 16 * s + 4 * g);
+            }
+        }
+        const float* gr = g_cum + ub * DELTA_BLOCK;
+        const delta_f32x4 gi = *reinterpret_cast<const delta_f32x4*>(gr + 16 * wave + 4 * g);
+        const float g_end = gr[DELTA_BLOCK - 1];
+        delta_f32x4 u;
+#pragma unroll
+        for (int i = 0; i < 4; ++i) u[i] = live ? u_in[(ub * DELTA_BLOCK + 16 * wave + 4 * g + i) * vdim + column] : 0.f;
+        // W S and Q S of this wave's 16 tokens
+        delta_f32x4 x = {0.f, 0.f, 0.f, 0.f}, y = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int s = 0; s < KB; ++s) {
+            const delta_f32x4 sv = *reinterpret_cast<const delta_f32x4*>(&s_s[col][16 * s + 4 * g]);
+#pragma unroll
+            for (int j = 0; j < 4; ++j) {
+                x = __builtin_amdgcn_mfma_f32_16x16x4f32(wf[s][j], sv[j], x, 0, 0, 0);
+                y = __builtin_amdgcn_mfma_f32_16x16x4f32(qf[s][j], sv[j], y, 0, 0, 0);
+            }
+        }
+        if (blk + 1 < blocks) ask(blk + 1);
+#pragma unroll
+        for (int i = 0; i < 4; ++i) u[i] -= x[i], y[i] *= expf(gi[i]);
+        *reinterpret_cast<delta_f32x4*>(&u_s[col][16 * wave + 4 * g]) = u;
+        delta_barrier();                                                // the block's writes are in; the state is read
+        const float e_end = expf(g_end);
+#pragma unroll
+        for (int b = 0; b < NB; ++b)
+#pragma unroll
+            for (int i = 0; i < 4; ++i) S[b][i] *= e_end;
+#pragma unroll
+        for (int s = 0; s < 4; ++s) {
+            const delta_f32x4 uv = *reinterpret_cast<const delta_f32x4*>(&u_s[col][16 * s + 4 * g]);
+#pragma unroll
+            for (int j = 0; j < 4; ++j) {
+                if (s <= wave) y = __builtin_amdgcn_mfma_f32_16x16x4f32(pf[s][j], uv[j], y, 0, 0, 0);
+#pragma unroll
+                for (int b = 0; b < NB; ++b) S[b] = __builtin_amdgcn_mfma_f32_16x16x4f32(kt[b][s][j], uv[j], S[b], 0, 0, 0);
+            }
+        }
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+            const int row = 16 * wave + 4 * g + i;
+            if (live && row < n) o_raw[(first + row) * vv + h * vdim + column] = y[i];
+        }
+#pragma unroll
+        for (int b = 0; b < NB; ++b)
+            if (wave + 4 * b < KB) *reinterpret_cast<delta_f32x4*>(&s_s[col][16 * (wave + 4 * b) + 4 * g]) = S[b];
+        delta_barrier();                                                // the state is in; the block's writes are read
+    }
+    if (!live) return;
+#pragma unroll
+    for (int b = 0; b < NB; ++b)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+            const int row = 16 * (wave + 4 * b) + 4 * g + i;
+            if (row < dim) S_g[(int64_t)row * vdim] = S[b][i];
+        }
+}
+
+// What both forms of the rule check.
+static int check_delta(const char* what, const void* proj, int64_t stride, int64_t need, float* scratch, void* out,
+                       int64_t out_stride, float* s_state, float* conv_state, const int32_t* token_seq,
+                       const int32_t* cu_seqlens_q, const int32_t* seq_starts, const int32_t* state_slots, int64_t seqs,
+                       int64_t tokens, int heads, int kv_heads, int dim, int vdim, int taps, const void* conv_w,
+                       const float* dt_bias, const float* a_log, const float* norm_w) {
+    if (tokens < 0 || tokens > 0x7fffffff || seqs <= 0 || seqs > 65535)
         return nva_fail("%s: bad counts tokens=%lld requests=%lld", what, (long long)tokens, (long long)seqs);
     if (heads <= 0 || kv_heads <= 0 || heads % kv_heads || heads > 65535 || dim <= 0 || vdim <= 0)
         return nva_fail("%s: bad sizes heads=%d kv_heads=%d dim=%d vdim=%d", what, heads, kv_heads, dim, vdim);
     if (dim > DELTA_MAX_DIM) return nva_fail("%s: a head of %d key channels (up to %d)", what, dim, DELTA_MAX_DIM);
     if (taps < 1 || taps > DELTA_MAX_TAPS) return nva_fail("%s: %d taps (1 to %d)", what, taps, DELTA_MAX_TAPS);
-    const int qk = kv_heads * dim, vv = heads * vdim, channels = 2 * qk + vv;
-    if (!proj || stride < need || !decay_in || !gate_in || gate_stride < vv || !scratch || !out || out_stride < vv ||
-        !s_state || (taps > 1 && !conv_state) || !token_seq || !cu_seqlens_q || !seq_starts || !state_slots || !conv_w ||
-        !dt_bias || !a_log || !norm_w)
+    if (!proj || stride < need || !scratch || !out || out_stride < heads * (int64_t)vdim || !s_state || (taps > 1 && !conv_state) ||
+        !token_seq || !cu_seqlens_q || !seq_starts || !state_slots || !conv_w || !dt_bias || !a_log || !norm_w)
         return nva_fail("%s: a tensor is missing or too narrow", what);
     if (2 * (int64_t)kv_heads + heads > 65535) return nva_fail("%s: %d heads", what, heads);
-    // scratch: q, k (and the decays, where they are rows) in rows of dim rounded up to 4 floats, then v, the read-outs, beta
-    // and the decays, where they are one per head
-    const int dp = (dim + 3) & ~3;
-    float* qn = scratch;
-    float* kn = qn + tokens * kv_heads * dp;
-    float* rows = kn + tokens * kv_heads * dp;
-    float* vf = rows + (HEAD ? 0 : tokens * (int64_t)heads * dp);
-    float* o_raw = vf + tokens * vv;
-    float* beta = o_raw + tokens * vv;
-    float* decay = HEAD ? beta + tokens * heads : rows;
     if ((uintptr_t)scratch % 16) return nva_fail("%s: the scratch memory must be 16-byte aligned", what);
-    hipLaunchKernelGGL((delta_prepare_kernel<elem_t, HEAD>), dim3((unsigned)tokens, (unsigned)(2 * kv_heads + heads)),
-                       dim3(DELTA_PREPARE_THREADS), 0, stream, (const elem_t*)proj, stride, decay_in, (const elem_t*)conv_w, dt_bias,
-                       a_log, conv_state, token_seq, cu_seqlens_q, seq_starts, state_slots, heads, kv_heads, dim, vdim, taps, qn, kn,
-                       vf, decay, beta);
-    if (taps > 1) {
-        if (seqs > 65535) return nva_fail("%s: %lld requests a step", what, (long long)seqs);
+    return 0;
+}
+
+// The request's recurrence token by token, 16 lanes a column where a head has rows for them (twice the waves, half the sums
+// a lane), else 8.  The requests are the `seqs` from the pointers on.
+template <bool HEAD>
+static void launch_delta_scan(const float* qn, const float* kn, const float* vf, const float* decay, const float* beta, float* o_raw,
+                              float* s_state, const int32_t* cu_seqlens_q, const int32_t* seq_starts, const int32_t* state_slots,
+                              int64_t seqs, int heads, int kv_heads, int dim, int vdim, hipStream_t stream) {
+#define DELTA_SCAN(DM, LL)                                                                                                \
+    hipLaunchKernelGGL((delta_scan_kernel<DM, LL, HEAD>), dim3((unsigned)seqs, (unsigned)heads, (vdim + DELTA_THREADS / LL - 1) / (DELTA_THREADS / LL)), \
+                       dim3(DELTA_THREADS), 0, stream, qn, kn, vf, decay, beta, o_raw, s_state, cu_seqlens_q, seq_starts,   \
+                       state_slots, heads, kv_heads, dim, vdim)
+    if (dim <= 32) DELTA_SCAN(32, 8); else if (dim <= 64) DELTA_SCAN(64, 16); else if (dim <= 128) DELTA_SCAN(128, 16); else DELTA_SCAN(256, 16);
+#undef DELTA_SCAN
+}
+
+static void launch_delta_keep(const void* proj, int64_t stride, float* conv_state, const int32_t* cu_seqlens_q,
+                              const int32_t* seq_starts, const int32_t* state_slots, int64_t seqs, int channels, int taps,
+                              hipStream_t stream) {
+    if (taps > 1 && seqs > 0)
         hipLaunchKernelGGL(delta_keep_kernel<elem_t>, dim3((channels + 255) / 256, (unsigned)seqs), dim3(256), 0, stream,
                            (const elem_t*)proj, stride, conv_state, cu_seqlens_q, seq_starts, state_slots, channels, taps);
-    }
-    {
-        // 16 lanes a column where a head has rows for them (twice the waves, half the sums a lane), else 8
-#define DELTA_SCAN(DM, LL)                                                                                                \
-        hipLaunchKernelGGL((delta_scan_kernel<DM, LL, HEAD>), dim3((unsigned)seqs, (unsigned)heads, (vdim + DELTA_THREADS / LL - 1) / (DELTA_THREADS / LL)), \
-                           dim3(DELTA_THREADS), 0, stream, qn, kn, vf, decay, beta, o_raw, s_state, cu_seqlens_q, seq_starts,   \
-                           state_slots, heads, kv_heads, dim, vdim)
-        if (dim <= 32) DELTA_SCAN(32, 8); else if (dim <= 64) DELTA_SCAN(64, 16); else if (dim <= 128) DELTA_SCAN(128, 16); else DELTA_SCAN(256, 16);
-#undef DELTA_SCAN
-    }
-    hipLaunchKernelGGL((delta_finish_kernel<elem_t, HEAD>), dim3((unsigned)tokens, (unsigned)heads), dim3(NVA_WAVE), 0, stream, o_raw,
-                       (const elem_t*)gate_in, gate_stride, norm_w, eps, (elem_t*)out, out_stride, heads, vdim);
-    return nva_check_launch(what);
 }
 
 // proj: elements [tokens, 2 G D + H DV + H], rows `stride` apart.  decay_in: float [tokens, H D].  gate_in: elements
@@ -399,26 +859,148 @@ NVA_EXPORT int NVA_NAME(nva_channel_delta)(const void* proj, int64_t stride, con
                                            int kv_heads, int dim, int vdim, int taps, const void* conv_w,
                                            const float* dt_bias, const float* a_log, const float* norm_w, float eps,
                                            hipStream_t stream) {
-    return launch_delta<false>("channel_delta", proj, stride, 2 * (int64_t)kv_heads * dim + (int64_t)heads * (vdim + 1), decay_in,
-                               gate_in, gate_stride, scratch, out, out_stride, s_state, conv_state, token_seq, cu_seqlens_q,
-                               seq_starts, state_slots, seqs, tokens, heads, kv_heads, dim, vdim, taps, conv_w, dt_bias, a_log,
-                               norm_w, eps, stream);
+    if (tokens == 0) return 0;
+    const int qk = kv_heads * dim, vv = heads * vdim, channels = 2 * qk + vv;
+    const int bad = check_delta("channel_delta", proj, stride, channels + (int64_t)heads, scratch, out, out_stride, s_state, conv_state,
+                                token_seq, cu_seqlens_q, seq_starts, state_slots, seqs, tokens, heads, kv_heads, dim, vdim, taps, conv_w,
+                                dt_bias, a_log, norm_w);
+    if (bad) return bad;
+    if (!decay_in || !gate_in || gate_stride < vv) return nva_fail("channel_delta: a tensor is missing or too narrow");
+    // scratch: q, k and the decays in rows of dim rounded up to 4 floats, then v, the read-outs and beta
+    const int dp = (dim + 3) & ~3;
+    float* qn = scratch;
+    float* kn = qn + tokens * kv_heads * dp;
+    float* decay = kn + tokens * kv_heads * dp;
+    float* vf = decay + tokens * (int64_t)heads * dp;
+    float* o_raw = vf + tokens * vv;
+    float* beta = o_raw + tokens * vv;
+    hipLaunchKernelGGL((delta_prepare_kernel<elem_t, false>), dim3((unsigned)tokens, (unsigned)(2 * kv_heads + heads)),
+                       dim3(DELTA_PREPARE_THREADS), 0, stream, (const elem_t*)proj, stride, decay_in, DeltaRates{nullptr, 0, 0},
+                       (int64_t)0, (const elem_t*)conv_w, dt_bias, a_log, conv_state, token_seq, cu_seqlens_q, seq_starts, state_slots,
+                       heads, kv_heads, dim, vdim, taps, qn, kn, vf, decay, beta);
+    launch_delta_keep(proj, stride, conv_state, cu_seqlens_q, seq_starts, state_slots, seqs, channels, taps, stream);
+    launch_delta_scan<false>(qn, kn, vf, decay, beta, o_raw, s_state, cu_seqlens_q, seq_starts, state_slots, seqs, heads, kv_heads, dim,
+                             vdim, stream);
+    hipLaunchKernelGGL((delta_finish_kernel<elem_t, false>), dim3((unsigned)tokens, (unsigned)heads), dim3(NVA_WAVE), 0, stream, o_raw,
+                       (const elem_t*)gate_in, gate_stride, norm_w, eps, (elem_t*)out, out_stride, heads, vdim, (int64_t)0);
+    return nva_check_launch("channel_delta");
+}
+
+// The form for single tokens: how a head's columns are shared out, or -1 where it does not take the sizes.
+static int delta_single_groups(int dim, int vdim) {
+    if (vdim % 4 || vdim > DELTA_SINGLE_THREADS || dim > DELTA_MAX_DIM) return -1;
+    int cg = 0;
+    while ((4 << cg) < vdim) ++cg;
+    const int rg = DELTA_SINGLE_THREADS >> cg;
+    return rg >= 1 && (dim + rg - 1) / rg <= 16 ? cg : -1;
+}
+
+// Floats that nva_head_delta's block_scratch holds for n blocks of portions.
+NVA_EXPORT int64_t NVA_NAME(nva_head_delta_block_floats)(int64_t n, int heads, int dim, int vdim) {
+    const int64_t dp = (dim + 3) & ~3;
+    return n * heads * DELTA_BLOCK * (2 * dp + vdim + DELTA_BLOCK + 1);
 }
 
 // One decay per head.  proj: elements [tokens, 2 G D + 2 H DV] = [q | k | v | gate], rows `stride` apart.  rates: float
-// [tokens, 2 H] = [b | a].  dt_bias and a_log float [H].  scratch: float [tokens * (2 G DP + 2 H DV + 2 H)], 16-byte aligned.
-// Everything else as for nva_channel_delta.
-NVA_EXPORT int NVA_NAME(nva_head_delta)(const void* proj, int64_t stride, const float* rates, float* scratch, void* out,
-                                        int64_t out_stride, float* s_state, float* conv_state, const int32_t* token_seq,
-                                        const int32_t* cu_seqlens_q, const int32_t* seq_starts, const int32_t* state_slots,
-                                        int64_t seqs, int64_t tokens, int heads, int kv_heads, int dim, int vdim, int taps,
+// [rate_splits][tokens, 2 H] = [b | a], the splits rate_stride apart and added up here.  dt_bias and a_log float [H].  scratch:
+// float [tokens * (2 G DP + 2 H DV + 2 H)], 16-byte aligned.  The first `singles` requests bring one token each, which
+// single_kernel (1 or 0) may take in a kernel of its own.  units [n_units][4] and chains [n_chains][4] (see the kernels) with
+// block_scratch cover the other requests, which then run in blocks; n_units 0: token by token.  Everything else as for
+// nva_channel_delta.
+NVA_EXPORT int NVA_NAME(nva_head_delta)(const void* proj, int64_t stride, const float* rates, int rate_splits, int64_t rate_stride,
+                                        float* scratch, void* out, int64_t out_stride, float* s_state, float* conv_state,
+                                        const int32_t* token_seq, const int32_t* cu_seqlens_q, const int32_t* seq_starts,
+                                        const int32_t* state_slots, int64_t seqs, int64_t tokens, int64_t singles,
+                                        int single_kernel, int heads, int kv_heads, int dim, int vdim, int taps,
                                         const void* conv_w, const float* dt_bias, const float* a_log, const float* norm_w,
-                                        float eps, hipStream_t stream) {
-    const int64_t channels = 2 * (int64_t)kv_heads * dim + (int64_t)heads * vdim;
-    return launch_delta<true>("head_delta", proj, stride, channels + (int64_t)heads * vdim, rates,
-                              proj ? (const elem_t*)proj + channels : nullptr, stride, scratch, out, out_stride, s_state, conv_state,
-                              token_seq, cu_seqlens_q, seq_starts, state_slots, seqs, tokens, heads, kv_heads, dim, vdim, taps,
-                              conv_w, dt_bias, a_log, norm_w, eps, stream);
+                                        float eps, const int32_t* units, int64_t n_units, const int32_t* chains,
+                                        int64_t n_chains, float* block_scratch, hipStream_t stream) {
+    if (tokens == 0) return 0;
+    const int qk = kv_heads * dim, vv = heads * vdim, channels = 2 * qk + vv;
+    const int bad = check_delta("head_delta", proj, stride, channels + (int64_t)vv, scratch, out, out_stride, s_state, conv_state, token_seq,
+                                cu_seqlens_q, seq_starts, state_slots, seqs, tokens, heads, kv_heads, dim, vdim, taps, conv_w, dt_bias,
+                                a_log, norm_w);
+    if (bad) return bad;
+    if (!rates || rate_splits <= 0 || (rate_splits > 1 && rate_stride < tokens * 2 * heads) || singles < 0 || singles > seqs)
+        return nva_fail("head_delta: bad rates (%d splits) or %lld single tokens of %lld requests", rate_splits, (long long)singles, (long long)seqs);
+    if (n_units && (!units || !chains || n_chains <= 0 || !block_scratch || (uintptr_t)block_scratch % 16 || n_units < n_chains ||
+                    n_units * heads * (DELTA_BLOCK / 16) > 0x7fffffff || n_chains * heads * (int64_t)((vdim + 15) / 16) > 0x7fffffff))
+        return nva_fail("head_delta: bad blocks (%lld in %lld portions)", (long long)n_units, (long long)n_chains);
+    const DeltaRates rt{rates, rate_splits, rate_stride};
+    const elem_t* pr = (const elem_t*)proj;
+    const elem_t* cw = (const elem_t*)conv_w;
+    const int cg = single_kernel && singles ? delta_single_groups(dim, vdim) : -1;
+    if (cg >= 0) {
+        const int rg = DELTA_SINGLE_THREADS >> cg, rows = (dim + rg - 1) / rg, keep = heads == kv_heads ? 1 : 0;
+        const size_t lds = (size_t)(((2 * dim + vdim + 3) & ~3) + (4 << cg) + rg * (4 << cg)) * sizeof(float);
+#define DELTA_SINGLE(RR)                                                                                                  \
+        hipLaunchKernelGGL((delta_single_kernel<elem_t, RR>), dim3((unsigned)singles, (unsigned)heads), dim3(DELTA_SINGLE_THREADS),  \
+                           lds, stream, pr, stride, rt, cw, dt_bias, a_log, norm_w, eps, s_state, conv_state, seq_starts, state_slots, \
+                           heads, kv_heads, dim, vdim, taps, cg, keep, (elem_t*)out, out_stride)
+        if (rows <= 1) DELTA_SINGLE(1); else if (rows <= 2) DELTA_SINGLE(2); else if (rows <= 4) DELTA_SINGLE(4);
+        else if (rows <= 8) DELTA_SINGLE(8); else DELTA_SINGLE(16);
+#undef DELTA_SINGLE
+        if (!keep) launch_delta_keep(proj, stride, conv_state, cu_seqlens_q, seq_starts, state_slots, singles, channels, taps, stream);
+    }
+    // what is left: requests from first_seq on, whose tokens start at first (a single token a request before them)
+    const int64_t first = cg >= 0 ? singles : 0, left = tokens - first;
+    if (left <= 0) return nva_check_launch("head_delta");
+    const int dp = (dim + 3) & ~3;
+    float* qn = scratch;
+    float* kn = qn + tokens * kv_heads * dp;
+    float* vf = kn + tokens * kv_heads * dp;
+    float* o_raw = vf + tokens * vv;
+    float* beta = o_raw + tokens * vv;
+    float* decay = beta + tokens * heads;
+    const int64_t blocked_from = n_units ? singles : seqs;              // requests that run in blocks
+    const int64_t plain_tokens = n_units ? singles - first : left;      // tokens of [first, ...) that run one by one
+    const unsigned heads_y = (unsigned)(2 * kv_heads + heads);
+    auto prepare = [&](int64_t t0, int64_t count) {
+        if (count > 0)
+            hipLaunchKernelGGL((delta_prepare_kernel<elem_t, true>), dim3((unsigned)count, heads_y), dim3(DELTA_PREPARE_THREADS), 0, stream,
+                               pr, stride, (const float*)nullptr, rt, t0, cw, dt_bias, a_log, conv_state, token_seq, cu_seqlens_q,
+                               seq_starts, state_slots, heads, kv_heads, dim, vdim, taps, qn, kn, vf, decay, beta);
+    };
+    if (n_units && taps <= 4) {
+        prepare(first, plain_tokens);
+        const dim3 grid((unsigned)(n_units * (DELTA_BLOCK / 16)), heads_y);
+#define DELTA_BLOCK_PREPARE(TT)                                                                                           \
+        hipLaunchKernelGGL((delta_block_prepare_kernel<elem_t, TT>), grid, dim3(DELTA_PREPARE_THREADS), 0, stream, pr, stride, rt, cw, \
+                           dt_bias, a_log, conv_state, units, cu_seqlens_q, seq_starts, state_slots, heads, kv_heads, dim, vdim, qn, kn, \
+                           vf, decay, beta)
+        if (taps == 1) DELTA_BLOCK_PREPARE(1); else if (taps == 2) DELTA_BLOCK_PREPARE(2);
+        else if (taps == 3) DELTA_BLOCK_PREPARE(3); else DELTA_BLOCK_PREPARE(4);
+#undef DELTA_BLOCK_PREPARE
+    } else {
+        prepare(first, left);
+    }
+    launch_delta_keep(proj, stride, conv_state, cu_seqlens_q + first, seq_starts + first, state_slots + first, seqs - first, channels,
+                      taps, stream);
+    if (blocked_from > first)
+        launch_delta_scan<true>(qn, kn, vf, decay, beta, o_raw, s_state, cu_seqlens_q + first, seq_starts + first, state_slots + first,
+                                blocked_from - first, heads, kv_heads, dim, vdim, stream);
+    if (n_units) {
+        const int64_t rows = n_units * heads * DELTA_BLOCK;
+        float* w = block_scratch;
+        float* u = w + rows * dp;
+        float* p = u + rows * vdim;
+        float* kt = p + rows * DELTA_BLOCK;
+        float* gc = kt + rows * dp;
+        const unsigned slices = (unsigned)((vdim + 15) / 16);
+#define DELTA_BLOCKS(KK)                                                                                                  \
+        do {                                                                                                              \
+            hipLaunchKernelGGL((delta_block_solve_kernel<KK>), dim3((unsigned)(n_units * heads)), dim3(256), 0, stream, qn, kn, vf, decay, \
+                               beta, units, heads, kv_heads, dim, vdim, gc, w, u, p, kt);                                     \
+            hipLaunchKernelGGL((delta_block_scan_kernel<KK>), dim3((unsigned)(slices * n_chains * heads)), dim3(256), 0, stream, qn, gc, w,  \
+                               u, p, kt, o_raw, s_state, units, chains, (int)n_chains, seq_starts, state_slots, heads, kv_heads, dim,  \
+                               vdim);                                                                                     \
+        } while (0)
+        if (dim <= 32) DELTA_BLOCKS(2); else if (dim <= 64) DELTA_BLOCKS(4); else if (dim <= 128) DELTA_BLOCKS(8); else DELTA_BLOCKS(16);
+#undef DELTA_BLOCKS
+    }
+    hipLaunchKernelGGL((delta_finish_kernel<elem_t, true>), dim3((unsigned)left, (unsigned)heads), dim3(NVA_WAVE), 0, stream, o_raw,
+                       pr + channels, stride, norm_w, eps, (elem_t*)out, out_stride, heads, vdim, first);
+    return nva_check_launch("head_delta");
 }
 
 NVA_DEFINE_LAST_ERROR(nva_delta)

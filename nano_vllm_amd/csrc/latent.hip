@@ -301,55 +301,102 @@ NVA_EXPORT int NVA_NAME(nva_heads_linear)(const void* x, int64_t x_stride, int64
 
 #if defined(NVA_BF16)
 // ---------------------------------------------------------------------------- the product per head on the matrix cores
-// W [heads, n_out, k_in] with k side by side.  A wave takes 16 tokens of one head and 64 outputs: the rows of W are the
+// W [heads, n_out, k_in] with k side by side.  A wave takes 16 TB tokens of one head and 64 outputs: the rows of W are the
 // A operand and the tokens' rows the B operand of v_mfma_f32_16x16x32_bf16, both straight from global memory (a lane 16
-// bytes a load); a fragment of x serves four products.  The sum over k runs in the order of the steps of 32, whatever
-// the other tokens of the tile.
+// bytes a load); a fragment of x serves four products, a fragment of W TB of them.  The sum over k runs in the order of the
+// steps of 32, whatever the other tokens of the tile.  SPLIT > 1 (few tokens): the workgroup's waves share k out in runs of
+// steps and their sums meet in LDS, in the order of the waves.
 typedef __attribute__((ext_vector_type(8))) __bf16 hl_bf16x8;
+typedef __attribute__((ext_vector_type(4))) __bf16 hl_bf16x4;
 typedef __attribute__((ext_vector_type(4))) float hl_f32x4;
 
-__global__ void __launch_bounds__(NVA_WAVE)
+template <int TB, int SPLIT>
+__global__ void __launch_bounds__(SPLIT * NVA_WAVE)
 heads_linear_mfma_kernel(const __bf16* __restrict__ x, int64_t x_stride, int64_t x_head, const __bf16* __restrict__ w,
                          __bf16* __restrict__ y, int64_t y_stride, int64_t y_head, int64_t tokens, int n_out, int k_in,
-                         const float* __restrict__ head_gate) {
-    const int64_t t0 = (int64_t)blockIdx.x * 16;
+                         int wide_stores, const float* __restrict__ head_gate) {
+    __shared__ hl_f32x4 sums_s[SPLIT > 1 ? (SPLIT - 1) * TB * 4 * NVA_WAVE : 1];
+    const int64_t t0 = (int64_t)blockIdx.x * 16 * TB;
     const int h = blockIdx.y, n0 = blockIdx.z * 64;
-    const int lane = threadIdx.x, col = lane & 15, g = lane >> 4;
-    const int64_t t = t0 + col;
-    const __bf16* xr = x + (t < tokens ? t : tokens - 1) * x_stride + h * x_head + 8 * g;
+    const int wave = threadIdx.x / NVA_WAVE, lane = threadIdx.x % NVA_WAVE, col = lane & 15, g = lane >> 4;
+    const __bf16* xr[TB];
+#pragma unroll
+    for (int b = 0; b < TB; ++b) {
+        const int64_t t = t0 + 16 * b + col;
+        xr[b] = x + (t < tokens ? t : tokens - 1) * x_stride + h * x_head + 8 * g;
+    }
     const __bf16* wr[4];
 #pragma unroll
     for (int b = 0; b < 4; ++b) wr[b] = w + ((int64_t)h * n_out + min(n0 + 16 * b + col, n_out - 1)) * k_in + 8 * g;
-    hl_f32x4 acc[4];
+    hl_f32x4 acc[TB][4];
 #pragma unroll
-    for (int b = 0; b < 4; ++b) acc[b] = hl_f32x4{0.f, 0.f, 0.f, 0.f};
+    for (int i = 0; i < TB; ++i)
+#pragma unroll
+        for (int b = 0; b < 4; ++b) acc[i][b] = hl_f32x4{0.f, 0.f, 0.f, 0.f};
     const int k_last = k_in - 8;                    // k_in is a multiple of 8: a piece lies inside the row or outside
+    const int steps = (k_in + 31) / 32, per = (steps + SPLIT - 1) / SPLIT;
+    const int k_hi = SPLIT > 1 ? min(k_in, (wave + 1) * per * 32) : k_in;
 #pragma unroll 4
-    for (int k0 = 0; k0 < k_in; k0 += 32) {
+    for (int k0 = SPLIT > 1 ? wave * per * 32 : 0; k0 < k_hi; k0 += 32) {
         const bool inside = k0 + 8 * g <= k_last;
         const int at = inside ? k0 : -8 * g;        // (every load unconditional: a piece outside the row reads the row's first, and counts as zero)
-        hl_bf16x8 xf = *reinterpret_cast<const hl_bf16x8*>(xr + at);
-        hl_bf16x8 wf[4];
+        hl_bf16x8 xf[TB], wf[4];
+#pragma unroll
+        for (int b = 0; b < TB; ++b) xf[b] = *reinterpret_cast<const hl_bf16x8*>(xr[b] + at);
 #pragma unroll
         for (int b = 0; b < 4; ++b) wf[b] = *reinterpret_cast<const hl_bf16x8*>(wr[b] + at);
         if (!inside) {
 #pragma unroll
-            for (int e = 0; e < 8; ++e) xf[e] = (__bf16)0.f;
+            for (int i = 0; i < TB; ++i)
+#pragma unroll
+                for (int e = 0; e < 8; ++e) xf[i][e] = (__bf16)0.f;
         }
 #pragma unroll
-        for (int b = 0; b < 4; ++b) acc[b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf[b], xf, acc[b], 0, 0, 0);
+        for (int i = 0; i < TB; ++i)
+#pragma unroll
+            for (int b = 0; b < 4; ++b) acc[i][b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf[b], xf[i], acc[i][b], 0, 0, 0);
     }
-    // acc[b][i] = y[token col][n0 + 16 b + 4 g + i]
-    if (t >= tokens) return;
-    __bf16* yr = y + t * y_stride + h * y_head;
-    const float gate = head_gate ? head_gate[t * gridDim.y + h] : 1.f;
+    if (SPLIT > 1) {
+        if (wave > 0) {
 #pragma unroll
-    for (int b = 0; b < 4; ++b)
+            for (int i = 0; i < TB; ++i)
 #pragma unroll
-        for (int i = 0; i < 4; ++i) {
-            const int n = n0 + 16 * b + 4 * g + i;
-            if (n < n_out) yr[n] = (__bf16)(acc[b][i] * gate);
+                for (int b = 0; b < 4; ++b) sums_s[(((wave - 1) * TB + i) * 4 + b) * NVA_WAVE + lane] = acc[i][b];
         }
+        __syncthreads();
+        if (wave > 0) return;
+#pragma unroll
+        for (int v = 0; v < SPLIT - 1; ++v)
+#pragma unroll
+            for (int i = 0; i < TB; ++i)
+#pragma unroll
+                for (int b = 0; b < 4; ++b) {
+                    const hl_f32x4 o = sums_s[((v * TB + i) * 4 + b) * NVA_WAVE + lane];
+                    acc[i][b][0] += o[0]; acc[i][b][1] += o[1]; acc[i][b][2] += o[2]; acc[i][b][3] += o[3];
+                }
+    }
+    // acc[i][b][e] = y[token 16 i + col][n0 + 16 b + 4 g + e]
+#pragma unroll
+    for (int i = 0; i < TB; ++i) {
+        const int64_t t = t0 + 16 * i + col;
+        if (t >= tokens) continue;
+        __bf16* yr = y + t * y_stride + h * y_head;
+        const float gate = head_gate ? head_gate[t * gridDim.y + h] : 1.f;
+#pragma unroll
+        for (int b = 0; b < 4; ++b) {
+            const int n = n0 + 16 * b + 4 * g;
+            if (wide_stores) {                      // (n_out a multiple of 4: the four entries are inside or outside together)
+                hl_bf16x4 v;
+#pragma unroll
+                for (int e = 0; e < 4; ++e) v[e] = (__bf16)(acc[i][b][e] * gate);
+                if (n < n_out) *reinterpret_cast<hl_bf16x4*>(yr + n) = v;
+                continue;
+            }
+#pragma unroll
+            for (int e = 0; e < 4; ++e)
+                if (n + e < n_out) yr[n + e] = (__bf16)(acc[i][b][e] * gate);
+        }
+    }
 }
 
 // As nva_heads_linear with w_n = k_in, w_k = 1 (W [heads * n_out, k_in], contiguous).  Returns 1 (and a message) for
@@ -365,9 +412,16 @@ NVA_EXPORT int nva_heads_linear_mfma_bf16(const void* x, int64_t x_stride, int64
     if (tokens < 0 || tokens > 0x7fffffffLL * 16 || heads <= 0 || heads > 65535 || n_out <= 0 || (n_out + 63) / 64 > 65535 ||
         !x || !w || !y)
         return nva_fail("heads_linear_mfma: bad sizes tokens=%lld heads=%d outputs=%d", (long long)tokens, heads, n_out);
-    dim3 grid((unsigned)((tokens + 15) / 16), (unsigned)heads, (unsigned)((n_out + 63) / 64));
-    hipLaunchKernelGGL(heads_linear_mfma_kernel, grid, dim3(NVA_WAVE), 0, stream, (const __bf16*)x, x_stride, x_head,
-                       (const __bf16*)w, (__bf16*)y, y_stride, y_head, tokens, n_out, k_in, head_gate);
+    const int wide = n_out % 4 == 0 && y_stride % 4 == 0 && y_head % 4 == 0 && nva_aligned(y, 8) ? 1 : 0;
+    const int64_t blocks = (n_out + 63) / 64 * (int64_t)heads;
+#define HL_LAUNCH(TB, SP)                                                                                              \
+    hipLaunchKernelGGL((heads_linear_mfma_kernel<TB, SP>), dim3((unsigned)((tokens + 16 * TB - 1) / (16 * TB)), (unsigned)heads, \
+                       (unsigned)((n_out + 63) / 64)), dim3(SP * NVA_WAVE), 0, stream, (const __bf16*)x, x_stride, x_head,      \
+                       (const __bf16*)w, (__bf16*)y, y_stride, y_head, tokens, n_out, k_in, wide, head_gate)
+    if ((tokens + 63) / 64 * blocks >= 512) HL_LAUNCH(4, 1);            // waves enough with 64 tokens each
+    else if ((tokens + 15) / 16 * blocks < 512 && k_in >= 256) HL_LAUNCH(1, 4);
+    else HL_LAUNCH(1, 1);
+#undef HL_LAUNCH
     return nva_check_launch("heads_linear_mfma");
 }
 

@@ -330,7 +330,9 @@ NVA_EXPORT int NVA_NAME(nva_stream_scaled_norm)(const void* a, int64_t a_stride,
 //     r <- r + mult * u
 //     y = r / sqrt(mean(r^2) + eps) * w               rounded once, to the element type
 // All arithmetic in float; r float, in place.  One workgroup a row, which keeps its entries between the sums.
-template <typename T>
+// A thread keeps KEEP entries of the row between the passes, and everything it needs of them (addend, stream, both weights)
+// is asked for before the first sum; rows of more than KEEP entries a thread read the rest again.
+template <typename T, int KEEP>
 __global__ void __launch_bounds__(1024)
 stream_post_norm_kernel(const T* __restrict__ a, int64_t a_stride, PartialInput pa, const void* __restrict__ a_weight,
                         int aw_is_f32, float a_eps, float mult, float* residual, int64_t r_stride,
@@ -341,35 +343,66 @@ stream_post_norm_kernel(const T* __restrict__ a, int64_t a_stride, PartialInput 
     const T* ar = a ? a + row * a_stride : nullptr;
     float* rr = residual + row * r_stride;
     T* yr = y + row * y_stride;
-    constexpr int KEEP = 8;                       // entries a thread keeps between the passes
-    float kept[KEEP];
+    const int step = blockDim.x, tid = threadIdx.x;
+    auto vec = [](const void* v, int is_f32, int i) -> float {
+        return is_f32 ? static_cast<const float*>(v)[i] : to_float(static_cast<const T*>(v)[i]);
+    };
+    float kept[KEEP], r_k[KEEP], wa_k[KEEP], w_k[KEEP];
+#pragma unroll
+    for (int n = 0; n < KEEP; ++n) {
+        const int i = tid + n * step;
+        const bool in = i < width;
+        kept[n] = in && !pa.sums ? to_float(ar[i]) : 0.f;
+        r_k[n] = in ? rr[i] : 0.f;
+        wa_k[n] = in ? vec(a_weight, aw_is_f32, i) : 0.f;
+        w_k[n] = in ? vec(weight, w_is_f32, i) : 0.f;
+    }
+    if (pa.sums) {
+        // the splits' sums of all kept entries side by side, each in the order of the splits
+        const float* q = pa.sums + row * width + tid;
+#pragma unroll 4
+        for (int s = 0; s < pa.splits; ++s)
+#pragma unroll
+            for (int n = 0; n < KEEP; ++n)
+                if (tid + n * step < width) kept[n] += q[s * pa.split_stride + n * step];
+#pragma unroll
+        for (int n = 0; n < KEEP; ++n) {
+            const int i = tid + n * step;
+            if (pa.bias && i < width) kept[n] += to_float(static_cast<const T*>(pa.bias)[i]);
+            kept[n] = round_through<T>(kept[n]);
+        }
+    }
     float ss = 0.f;
-    int n = 0;
-    for (int i = threadIdx.x; i < width; i += blockDim.x, ++n) {
+#pragma unroll
+    for (int n = 0; n < KEEP; ++n) ss += kept[n] * kept[n];
+    for (int i = tid + KEEP * step; i < width; i += step) {
         const float v = pa.sums ? partial_value<T>(pa, row, width, i) : to_float(ar[i]);
-        if (n < KEEP) kept[n] = v;
         ss += v * v;
     }
     ss = block_sum(ss, scratch);
     const float a_scale = rsqrtf(ss / (float)width + a_eps) * mult;
     float ss2 = 0.f;
-    n = 0;
-    for (int i = threadIdx.x; i < width; i += blockDim.x, ++n) {
-        const float v = n < KEEP ? kept[n] : (pa.sums ? partial_value<T>(pa, row, width, i) : to_float(ar[i]));
-        const float wa = aw_is_f32 ? static_cast<const float*>(a_weight)[i] : to_float(static_cast<const T*>(a_weight)[i]);
-        const float s = rr[i] + v * a_scale * wa;
+#pragma unroll
+    for (int n = 0; n < KEEP; ++n) {
+        const int i = tid + n * step;
+        kept[n] = r_k[n] + kept[n] * a_scale * wa_k[n];
+        if (i < width) rr[i] = kept[n];
+        ss2 += kept[n] * kept[n];                                     // (entries outside the row are zero)
+    }
+    for (int i = tid + KEEP * step; i < width; i += step) {
+        const float v = pa.sums ? partial_value<T>(pa, row, width, i) : to_float(ar[i]);
+        const float s = rr[i] + v * a_scale * vec(a_weight, aw_is_f32, i);
         rr[i] = s;
-        if (n < KEEP) kept[n] = s;
         ss2 += s * s;
     }
     ss2 = block_sum(ss2, scratch);
     const float scale = rsqrtf(ss2 / (float)width + eps);
-    n = 0;
-    for (int i = threadIdx.x; i < width; i += blockDim.x, ++n) {
-        const float s = n < KEEP ? kept[n] : rr[i];
-        const float w = w_is_f32 ? static_cast<const float*>(weight)[i] : to_float(static_cast<const T*>(weight)[i]);
-        yr[i] = from_float<T>(s * scale * w);
+#pragma unroll
+    for (int n = 0; n < KEEP; ++n) {
+        const int i = tid + n * step;
+        if (i < width) yr[i] = from_float<T>(kept[n] * scale * w_k[n]);
     }
+    for (int i = tid + KEEP * step; i < width; i += step) yr[i] = from_float<T>(rr[i] * scale * vec(weight, w_is_f32, i));
 }
 
 // a: elements [rows, width], or (a_sums) partial sums [splits][rows][width] with an optional bias.
@@ -387,9 +420,13 @@ NVA_EXPORT int NVA_NAME(nva_stream_post_norm)(const void* a, int64_t a_stride, c
     const PartialInput pa{a_sums, a_splits, a_split_stride, a_bias};
     const int threads = a_sums && rows <= 64 && width >= 1024 ? 1024
                         : width >= 2048 ? 512 : width >= 1024 ? 256 : width >= 256 ? 128 : 64;
-    hipLaunchKernelGGL((stream_post_norm_kernel<elem_t>), dim3((unsigned)rows), dim3(threads), 0, stream,
-                       (const elem_t*)a, a_stride, pa, a_weight, aw_is_f32, a_eps, mult, residual, r_stride, weight, w_is_f32,
-                       (elem_t*)y, y_stride, width, eps);
+    const int per = (width + threads - 1) / threads;
+#define POST_NORM(KK)                                                                                                  \
+    hipLaunchKernelGGL((stream_post_norm_kernel<elem_t, KK>), dim3((unsigned)rows), dim3(threads), 0, stream,              \
+                       (const elem_t*)a, a_stride, pa, a_weight, aw_is_f32, a_eps, mult, residual, r_stride, weight, w_is_f32, \
+                       (elem_t*)y, y_stride, width, eps)
+    if (per <= 1) POST_NORM(1); else if (per <= 2) POST_NORM(2); else if (per <= 4) POST_NORM(4); else POST_NORM(8);
+#undef POST_NORM
     return nva_check_launch("stream_post_norm");
 }
 

@@ -62,11 +62,12 @@ def _i32(t: torch.Tensor, n: int, what: str):
 class SplitSum:
     """A bfloat16 product left as float partial sums [splits, rows, width] (+ bias) by the
     weight-streaming kernel, for the next kernel to add up while it reads them: the norms and
-    the q/k preparation take it in place of a tensor; anything else gets `tensor()`."""
+    the q/k preparation take it in place of a tensor; anything else gets `tensor()`.  float32: the product of
+    bfloat16 operands whose result is wanted as float, not rounded."""
 
-    def __init__(self, kernels, sums: torch.Tensor, splits: int, rows: int, width: int, bias):
+    def __init__(self, kernels, sums: torch.Tensor, splits: int, rows: int, width: int, bias, float32: bool = False):
         self.kernels, self.sums, self.splits, self.rows, self.width, self.bias = kernels, sums, splits, rows, width, bias
-        self.dtype = torch.bfloat16
+        self.dtype = torch.float32 if float32 else torch.bfloat16
         self.device = sums.device
         self.shape = (rows, width)
         self._tensor = None
@@ -75,7 +76,7 @@ class SplitSum:
         if self._tensor is None:
             out = torch.empty(self.shape, dtype=self.dtype, device=self.device)
             library.call("gemm_skinny", "bf16", "nva_linear_skinny_finish", _p(self.sums), c_i32(self.splits),
-                         _p(self.bias), _p(out), c_i64(self.width), c_i32(0), c_i32(0), c_i64(self.rows),
+                         _p(self.bias), _p(out), c_i64(self.width), c_i32(1 if self.dtype == torch.float32 else 0), c_i32(0), c_i64(self.rows),
                          c_i64(self.width), self.kernels._stream())
             self._tensor = out
         return self._tensor
@@ -148,6 +149,25 @@ def retention_blocks(q_lens, first_seq: int):
         for b in range(nb):
             units += [s - first_seq, b * bt, min(bt, n - b * bt), nb]
     return bt, units, chains
+
+
+DELTA_BLOCK = 64        # tokens of a block of the delta rule's matrix-core form
+
+
+def delta_blocks(q_lens, first_seq: int):
+    """The step's portions (the requests from `first_seq` on, which single tokens precede) in blocks of DELTA_BLOCK tokens:
+    (units, chains), units a flat list of (request, the block's first token counted through the step, its tokens, 0) and
+    chains one of (first unit, blocks, request, 0)."""
+    units, chains = [], []
+    token = sum(q_lens[:first_seq])
+    for s in range(first_seq, len(q_lens)):
+        n = q_lens[s]
+        nb = (n + DELTA_BLOCK - 1) // DELTA_BLOCK
+        chains += [len(units) // 4, nb, s, 0]
+        for b in range(nb):
+            units += [s, token + b * DELTA_BLOCK, min(DELTA_BLOCK, n - b * DELTA_BLOCK), 0]
+        token += n
+    return units, chains
 
 
 def state_space_blocks(q_lens, first_seq: int):
@@ -303,6 +323,12 @@ class HipKernels:
         self.tiled_general_attention = True
         # False: the general kernel walks all of a token's keys in one workgroup, however many
         self.shared_general_attention = True
+        # False: the delta rule with one decay per head runs portions token by token / single tokens as portions of one token;
+        # portions run in blocks where one of the step has more tokens than delta_block_min
+        self.latent_tiles_per_share = 0     # tiles of keys a share of a single token's latent attention has at least; 0: the rule
+        self.delta_blocks = True
+        self.delta_single_kernel = True
+        self.delta_block_min = DELTA_BLOCK
         # False: the state-space layer runs a portion's tokens one after the other, whatever its length
         self.state_space_blocks_side_by_side = True
         # how the recurrence holds a state of 65 to 128 rows: 0 two lanes a column (what serves), 1 a thread a column
@@ -657,13 +683,21 @@ class HipKernels:
         return out
 
     def linear_act(self, x: torch.Tensor, weight: torch.Tensor, act: str = "relu2") -> torch.Tensor:
-        """act(x @ weight.T), entry by entry; a product left as partial sums is added up by the activation's own pass."""
+        """act(x @ weight.T), entry by entry: in the product's epilogue where a wide weight meets few rows; a product left as
+        partial sums is added up by the activation's own pass."""
+        if act not in self.PLAIN_ACTIVATIONS:
+            raise KernelError(f"act: unknown activation {act!r}; known: {sorted(self.PLAIN_ACTIVATIONS)}")
+        x = _t(x)
+        m, k, xs = _rows2d(x, "linear input")
+        n, wk, ws = _rows2d(weight, "linear weight")
+        if x.dtype == torch.bfloat16 and weight.dtype == x.dtype and wk == k and self._skinny_takes(x, xs, weight, ws, k) and \
+                self._own_kernel(m, n, k) == "team":
+            out = torch.empty((m, n), dtype=x.dtype, device=x.device)
+            return self._linear_team(x, xs, weight, ws, None, out, n, 5 + self.PLAIN_ACTIVATIONS[act], m, n, k)
         y = self.linear(x, weight, deferred=True)
         if not isinstance(y, SplitSum):
             y = _t(y)
             return self.act(y, act, out=y)
-        if act not in self.PLAIN_ACTIVATIONS:
-            raise KernelError(f"act: unknown activation {act!r}; known: {sorted(self.PLAIN_ACTIVATIONS)}")
         rows, width = y.shape
         out = torch.empty((rows, width), dtype=y.dtype, device=y.device)
         library.call("activation", "bf16", "nva_act_of_partials", _p(y.sums), c_i32(y.splits), c_i64(rows * width), _p(y.bias),
@@ -773,7 +807,8 @@ class HipKernels:
         float kernel; bfloat16 inputs with many rows run the library product (also for a float
         result of more than 16 rows), with few rows the weight-streaming kernels.  deferred: the caller hands the result to a norm or to the q/k
         preparation only, so a product split over k may come back as a SplitSum, and a library
-        product as a PendingProduct."""
+        product as a PendingProduct; with out_float32 (the caller hands the result to the delta rule's kernels) only the
+        former, unrounded."""
         x = _t(x)
         m, k, xs = _rows2d(x, "linear input")
         n, wk, ws = _rows2d(weight, "linear weight")
@@ -811,6 +846,8 @@ class HipKernels:
             run = self._linear_medium if own == "medium" else self._linear_tile if own == "tile" else self._linear_skinny
             if deferred and own and not out_float32 and out is None and self.fuse_split_sums:
                 return run(x, xs, weight, ws, bias, None, 0, False, False, m, n, k, defer=True)
+            if deferred and own == "skinny" and out_float32 and out is None and self.fuse_split_sums:
+                return self._linear_skinny(x, xs, weight, ws, bias, None, 0, True, False, m, n, k, defer=True)
             if own or out_float32:
                 if out is None:
                     out = torch.empty((m, n), dtype=out_dtype, device=x.device)
@@ -970,7 +1007,7 @@ class HipKernels:
             splits = 1          # wide enough without a split of k: the gating happens in the product kernel
         if defer and splits == 1:
             defer = False
-            out = torch.empty((m, n), dtype=x.dtype, device=x.device)
+            out = torch.empty((m, n), dtype=torch.float32 if out_float32 else x.dtype, device=x.device)
             os_ = n
         direct = splits == 1 and bias is None
         scratch = None if direct else torch.empty(splits * m * n, dtype=torch.float32, device=x.device)
@@ -980,7 +1017,7 @@ class HipKernels:
                      c_i32(int(swiglu)), _p(scratch), c_i32(splits), c_i32(kw), c_i32(1 if defer else 0), c_i64(m), c_i64(n),
                      c_i64(k), ctypes.byref(used), self._stream())
         if defer:
-            return SplitSum(self, scratch, used.value, m, n, bias)
+            return SplitSum(self, scratch, used.value, m, n, bias, float32=bool(out_float32))
         return out
 
     def _medium_shape(self, m: int, blocks: int, k: int):
@@ -1105,7 +1142,7 @@ class HipKernels:
         return out
 
     def _linear_team(self, x, xs, weight, ws, bias, out, os_, mode, m, n, k):
-        """The kernel for wide weights and at most 16 rows.  mode: 0 elements, 1 float, 2 gated."""
+        """The kernel for wide weights and at most 16 rows.  mode: 0 elements, 1 float, 2 gated, 5 to 8 an activation."""
         library.call("gemm_team", "bf16", "nva_linear_team", _p(x), c_i64(xs), _p(weight), c_i64(ws), _p(bias), _p(out),
                      c_i64(os_), c_i32(mode), c_i64(m), c_i64(n), c_i64(k), c_i32(self.teams), self._stream())
         return out
@@ -1574,8 +1611,11 @@ class HipKernels:
                 # few tokens with many keys: a token's tiles of 32 keys are shared out, four tiles a share or more, until
                 # about two waves a compute unit run; the number follows from the step's shape alone
                 blocks = (heads + 15) // 16
+                # (two tiles a share where a window leaves so few keys that four would not give every compute unit a wave)
                 reach = min(batch.max_kv_len, window + 31) if window else batch.max_kv_len
-                shares = max(1, min(64, ((reach + 31) // 32) // 4, 512 // (single * blocks)))
+                tiles = (reach + 31) // 32
+                per_share = self.latent_tiles_per_share or (4 if (tiles // 4) * single * blocks >= self.cus else 2)
+                shares = max(1, min(64, tiles // per_share, 512 // (single * blocks)))
                 part = torch.empty(single * heads * shares * (2 + rank), dtype=torch.float32, device=q2.device) if shares > 1 else None
                 library.call("latent", "bf16", "nva_latent_attention", _p(q2), c_i64(qs), _p(out), c_i64(out.shape[1]), _p(part),
                              c_i32(shares), _p(k_cache), _p(v_cache), _p(tables), c_i32(tables.shape[1]), _p(batch.token_seq),
@@ -1664,16 +1704,25 @@ class HipKernels:
                    conv_w: torch.Tensor, dt_bias: torch.Tensor, a_log: torch.Tensor, norm_w: torch.Tensor, eps: float,
                    conv_state: torch.Tensor, s_state: torch.Tensor, batch, out: Optional[torch.Tensor] = None) -> torch.Tensor:
         """The gated delta rule with one decay per head over the step's tokens: proj [T, 2 G D + 2 H DV] = [q | k | v | gate],
-        rates float32 [T, 2 H] = [b | a].  As channel_delta, but the decay of a head is one number, exp(-exp(a_log) *
-        softplus(a + dt_bias)) with dt_bias and a_log float32 [H], and the gate is silu.  Returns [T, H DV] of proj's type."""
+        rates float32 [T, 2 H] = [b | a] (or that product left as partial sums).  As channel_delta, but the decay of a head is one number, exp(-exp(a_log) *
+        softplus(a + dt_bias)) with dt_bias and a_log float32 [H], and the gate is silu.  Returns [T, H DV] of proj's type.
+        Requests that bring one token run in a kernel of their own where it takes the sizes; where a portion of a prompt is
+        longer than a block of 64 tokens, the step's portions run in blocks on the matrix cores (float products), else
+        token by token."""
         proj = _t(proj)
         tokens, width, stride = _rows2d(proj, "delta-rule projections")
         vv = heads * vdim
         channels = 2 * kv_heads * dim + vv
         if width != channels + vv:
             raise KernelError(f"head_delta: projections of width {width}, expected {channels + vv}")
-        if rates.dtype != torch.float32 or tuple(rates.shape) != (tokens, 2 * heads) or not rates.is_contiguous():
-            raise KernelError(f"head_delta: the rates must be contiguous float32 [{tokens}, {2 * heads}]")
+        if rates.dtype != torch.float32 or tuple(rates.shape) != (tokens, 2 * heads):
+            raise KernelError(f"head_delta: the rates must be float32 [{tokens}, {2 * heads}]")
+        if isinstance(rates, SplitSum) and self.fuse_split_sums and rates.bias is None:
+            rate_sums, rate_splits = rates.sums, rates.splits
+        else:
+            rate_sums, rate_splits = _t(rates), 1
+            if not rate_sums.is_contiguous():
+                raise KernelError("head_delta: the rates must be contiguous")
         self._check_delta("head_delta", proj, tokens, heads, dim, vdim, taps, channels, conv_w, norm_w, conv_state, s_state, batch)
         for v, what in ((dt_bias, "dt_bias"), (a_log, "a_log")):
             if v.dtype != torch.float32 or tuple(v.shape) != (heads,) or not v.is_contiguous():
@@ -1683,13 +1732,35 @@ class HipKernels:
         orows, ow, os_ = _rows2d(out, "delta-rule output")
         if (orows, ow) != (tokens, vv) or out.dtype != proj.dtype:
             raise KernelError("head_delta: output does not match")
+        if any(n != 1 for n in batch.q_lens[:batch.num_decode]):
+            raise KernelError("head_delta: the first num_decode requests of a batch must bring one token each")
         dp = (dim + 3) // 4 * 4
         scratch = torch.empty(tokens * (2 * kv_heads * dp + 2 * vv + 2 * heads), dtype=torch.float32, device=proj.device)
-        library.call("delta", _suffix(proj), "nva_head_delta", _p(proj), c_i64(stride), _p(rates), _p(scratch), _p(out), c_i64(os_),
-                     _p(s_state), _p(conv_state if taps > 1 else None), _p(batch.token_seq), _p(batch.cu_seqlens_q),
-                     _p(batch.seq_starts), _p(batch.state_slots), c_i64(batch.num_seqs), c_i64(tokens), c_i32(heads), c_i32(kv_heads),
-                     c_i32(dim), c_i32(vdim), c_i32(taps), _p(conv_w), _p(dt_bias), _p(a_log), _p(norm_w), c_f32(eps),
-                     self._stream())
+        # the step's portions in blocks (the same cut for every layer of the step)
+        units = chains = block_scratch = None
+        n_units = n_chains = 0
+        first = batch.num_decode
+        if self.delta_blocks and max(batch.q_lens) > self.delta_block_min:
+            kept = getattr(batch, "step_cache", None)
+            if kept is None:
+                kept = batch.step_cache = {}
+            plan = kept.get(("delta_blocks", first))
+            if plan is None:
+                flat_units, flat_chains = delta_blocks(batch.q_lens, first)
+                both = torch.tensor(flat_units + flat_chains, dtype=torch.int32).to(proj.device, non_blocking=True)
+                plan = (len(flat_units) // 4, len(flat_chains) // 4, both[: len(flat_units)], both[len(flat_units):])
+                kept[("delta_blocks", first)] = plan
+            n_units, n_chains, units, chains = plan
+            need = getattr(library.load("delta", self.suffix), f"nva_head_delta_block_floats_{self.suffix}")
+            need.restype = ctypes.c_int64
+            block_scratch = torch.empty(int(need(c_i64(n_units), c_i32(heads), c_i32(dim), c_i32(vdim))), dtype=torch.float32,
+                                        device=proj.device)
+        library.call("delta", _suffix(proj), "nva_head_delta", _p(proj), c_i64(stride), _p(rate_sums), c_i32(rate_splits),
+                     c_i64(tokens * 2 * heads), _p(scratch), _p(out), c_i64(os_), _p(s_state), _p(conv_state if taps > 1 else None),
+                     _p(batch.token_seq), _p(batch.cu_seqlens_q), _p(batch.seq_starts), _p(batch.state_slots), c_i64(batch.num_seqs),
+                     c_i64(tokens), c_i64(first), c_i32(1 if self.delta_single_kernel else 0), c_i32(heads), c_i32(kv_heads), c_i32(dim),
+                     c_i32(vdim), c_i32(taps), _p(conv_w), _p(dt_bias), _p(a_log), _p(norm_w), c_f32(eps), _p(units), c_i64(n_units),
+                     _p(chains), c_i64(n_chains), _p(block_scratch), self._stream())
         return out
 
     @staticmethod

@@ -78,7 +78,7 @@ class HeadDelta(Part):
     def forward(self, x, batch, cache):
         k, w, n = self.kernels, self.weights, self.names
         proj = k.linear(x, w["proj.weight"])
-        rates = k.linear(x, w["rates.weight"], out_float32=True)
+        rates = k.linear(x, w["rates.weight"], out_float32=True, deferred=True)
         y = k.head_delta(proj, rates, self.heads, self.kv_heads, self.dim, self.vdim, self.taps, w["conv.weight"],
                          w[self.dt_bias_name], w[self.a_log_name], w[f"{self.norm_name}.weight"], self.eps,
                          cache.state["conv"], cache.state["s"], batch)

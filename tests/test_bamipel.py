@@ -216,7 +216,7 @@ def test_attention_multiplies_every_heads_output_by_its_gate(backend, dtype, hq,
 
 @pytest.mark.parametrize("backend", BACKENDS)
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("tokens,heads,n_out,k_in", [(1, 3, 20, 10), (37, 2, 7, 16), (16, 4, 64, 32), (70, 5, 130, 176)])
+@pytest.mark.parametrize("tokens,heads,n_out,k_in", [(1, 3, 20, 10), (37, 2, 7, 16), (16, 4, 64, 32), (70, 5, 130, 176), (8, 6, 128, 384), (600, 20, 128, 72)])
 def test_a_product_per_head_times_its_gate(backend, dtype, tokens, heads, n_out, k_in):
     k, dev = _kernels(backend, dtype)
     g = torch.Generator().manual_seed(tokens + n_out)
@@ -386,8 +386,25 @@ def test_preparations_add_up_a_products_partial_sums(tokens):
                                norm_unit=True, head_gate=gate)
         return q.clone(), gate, kc, vc
     both(mat((H_ + 4) * D + 8), prepare)
-    w = mat(320)
-    assert torch.equal(k.linear_act(x, w, "relu2"), k.act(k.linear(x, w), "relu2"))
+    for n in (320, 32 * k.cus):               # (a wide weight and few rows: the activation in the product's epilogue)
+        w = mat(n)
+        for act in ("relu2", "silu"):
+            assert torch.equal(k.linear_act(x, w, act), k.act(k.linear(x, w), act)), (n, act)
+
+    def rule(rates):
+        shape = (4, 4, 16, 8, 3)
+        wt = K.delta_weights(shape, 3, torch.bfloat16)
+        proj, _ = K.delta_inputs(shape, tokens, 4, torch.bfloat16)
+        states = K.new_states(dev, tokens, shape, 0.5)
+        out = k.head_delta(proj.to(dev), rates, 4, 4, 16, 8, 3, wt["conv"].to(dev), wt["dt_bias"].to(dev), wt["A_log"].to(dev),
+                           wt["norm"].to(dev), 1e-5, *states, K.state_batch(dev, [1] * tokens, [1] * tokens, list(range(tokens))))
+        return out, states[1]
+    if tokens <= 16:
+        split = k.linear(x, mat(8), out_float32=True, deferred=True)
+        assert isinstance(split, SplitSum) and split.dtype == torch.float32 and split.tensor().dtype == torch.float32
+        a, b = rule(split), rule(split.tensor())
+        for p, q in zip(a, b):
+            assert torch.allclose(p.float(), q.float(), rtol=1e-2, atol=1e-5)
 
 
 @pytest.mark.parametrize("backend", BACKENDS)
@@ -520,6 +537,76 @@ def test_an_impulse_shows_for_exactly_the_convolutions_taps(backend, dtype, taps
             pos += n
         seen = torch.cat(outs).float().cpu().abs().amax(-1) > 1e-4
         assert seen.nonzero().flatten().tolist() == list(range(at, at + taps)), portions
+
+
+@pytest.mark.parametrize("backend", BACKENDS)
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("shape", [(4, 2, 12, 8, 3), (2, 2, 64, 64, 4), (1, 1, 130, 20, 6), (3, 1, 30, 18, 1), (2, 1, 128, 128, 4)])
+def test_long_portions_beside_single_tokens(backend, dtype, shape):
+    """Portions of more than a block of 64 tokens (and of exactly one, one more, and a few tokens) beside single tokens,
+    from a start and from a state: outputs and states are the plain implementation's, whatever runs them."""
+    k, dev = _kernels(backend, dtype)
+    if backend == "cpu" and (dtype == torch.bfloat16 or shape[2] > 64):
+        pytest.skip("the stand-ins run one way only")
+    heads, kv_heads, dim, vdim, taps = shape
+    eps = 1e-5
+    w = K.delta_weights(shape, 41, dtype)
+    lens = {"a": 9, "b": 130, "c": 67, "d": 200, "e": 68}
+    inputs = {r: K.delta_inputs(shape, n, 50 + i, dtype) for i, (r, n) in enumerate(lens.items())}
+    want = {r: K.plain_delta(shape, w, inputs[r], eps) for r in lens}
+    slot = {"a": 2, "b": 0, "c": 4, "d": 1, "e": 3}
+    steps = [[("a", 0, 8), ("b", 0, 64), ("c", 0, 65), ("d", 0, 3)],
+             [("a", 8, 1), ("b", 64, 1), ("d", 3, 131), ("c", 65, 2), ("e", 0, 67)],
+             [("e", 67, 1), ("b", 65, 65), ("d", 134, 66)]]
+    found = {}
+    ways = [(True, True), (False, False)] if backend == "hip" else [(True, True)]
+    for blocks, single in ways:
+        if backend == "hip":
+            k.delta_blocks, k.delta_single_kernel = blocks, single
+        try:
+            states, got = K.new_states(dev, 6, shape), {r: [] for r in lens}
+            for step in steps:
+                part = tuple(torch.cat([inputs[r][i][s:s + n] for r, s, n in step]) for i in range(2))
+                out = K.run_delta(k, dev, shape, w, part, eps, states, [n for _, _, n in step], [s for _, s, _ in step], [slot[r] for r, _, _ in step])
+                row = 0
+                for r, s, n in step:
+                    got[r].append(out[row:row + n])
+                    row += n
+            for r in lens:
+                _close(torch.cat(got[r]), want[r], dtype, (r, blocks), 4e-2 if dtype == torch.bfloat16 else 1e-4)
+            assert torch.isnan(states[1][5]).all()
+            found[blocks] = states
+        finally:
+            if backend == "hip":
+                k.delta_blocks = k.delta_single_kernel = True
+    if backend == "hip":
+        # the states agree far below what bfloat16's outputs show (the inputs are the same numbers)
+        assert torch.equal(found[True][0][:5], found[False][0][:5])
+        _close(found[True][1][:5], found[False][1][:5].cpu(), torch.float32, "states")
+
+
+@pytest.mark.parametrize("backend", BACKENDS)
+def test_blocks_of_keys_that_are_nearly_one_direction(backend):
+    """Keys that all lie within a few degrees, full write strengths and next to no decay: every write cancels most of what
+    the ones before it left, which is where a block's triangular system is hardest."""
+    k, dev = _kernels(backend)
+    shape, T, eps = (2, 1, 32, 16, 1), 150, 1e-6
+    w = K.delta_weights(shape, 8, torch.float32)
+    w["A_log"][:] = -9.0
+    w["conv"][:] = 1.0
+    proj, rates = K.delta_inputs(shape, T, 9, torch.float32)
+    proj[:, 32:64] = 3.0 + 0.1 * proj[:, 32:64]
+    rates[:, :2] = 8.0
+    want = K.plain_delta(shape, w, (proj, rates), eps)
+    states = K.new_states(dev, 1, shape)
+    _close(K.run_delta(k, dev, shape, w, (proj, rates), eps, states, [T], [0], [0]), want, torch.float32, "one direction", 2e-4)
+
+
+def test_portions_are_cut_into_blocks():
+    from nano_vllm_amd.kernels.ops import delta_blocks
+    units, chains = delta_blocks([1, 1, 130, 2, 64], 2)
+    assert units == [2, 2, 64, 0, 2, 66, 64, 0, 2, 130, 2, 0, 3, 132, 2, 0, 4, 134, 64, 0]
+    assert chains == [0, 3, 2, 0, 3, 1, 3, 0, 4, 1, 4, 0]
 
 
 # ------------------------------------------------------------------------------ the model through the step function
