@@ -35,11 +35,12 @@
 //                     the logarithms of the decays up to token i of a block, S_0 the state before the block, and
 //                     A_ij = beta_i exp(G_i - G_j) k_i.k_j for j < i, the writes of the block are
 //                         (I + A) u = beta v - beta exp(G) k^T S_0      (row i: beta_i v_i - beta_i exp(G_i) S_0^T k_i)
-//                     so u = U - W S_0 with (I + A) U = beta v and (I + A) W = beta exp(G) k, both by forward substitution
-//                     row by row; then o_i = exp(G_i) S_0^T q_i + sum over j <= i of P_ij u_j with P_ij = exp(G_i - G_j)
+//                     so u = U - W S_0 with (I + A) U = beta v and (I + A) W = beta exp(G) k, both by forward
+//                     substitution; then o_i = exp(G_i) S_0^T q_i + sum over j <= i of P_ij u_j with P_ij = exp(G_i - G_j)
 //                     q_i.k_j, and the state behind the block is exp(G_63) S_0 + sum over j of exp(G_63 - G_j) k_j u_j^T.
 //     delta_block_prepare   the convolutions, unit norms, beta and log decays, 16 tokens of a head to a workgroup
-//     delta_block_solve     a workgroup per (block, head): A and P by products, U and W by substitution, a column a thread
+//     delta_block_solve     a workgroup per (block, head): A and P by products; U and W by substitution in blocks of 16 rows,
+//                           the diagonal blocks of I + A inverted row by row, everything else products
 //     delta_block_scan      a workgroup per (portion, head, 16 columns of S): the blocks one after the other
 #include "common.h"
 
@@ -573,6 +574,7 @@ delta_block_solve_kernel(const float* __restrict__ qn, const float* __restrict__
                          int heads, int kv_heads, int dim, int vdim, float* __restrict__ g_cum, float* __restrict__ w_out,
                          float* __restrict__ u_out, float* __restrict__ p_out, float* __restrict__ kt_out) {
     __shared__ __attribute__((aligned(16))) float a_s[DELTA_BLOCK][DELTA_BLOCK + 4];
+    __shared__ __attribute__((aligned(16))) float inv_s[4][16][20];
     __shared__ float g_s[DELTA_BLOCK], b_s[DELTA_BLOCK], bg_s[DELTA_BLOCK], eg_s[DELTA_BLOCK];
     const int h = blockIdx.x % heads;
     const int64_t ub = blockIdx.x;
@@ -628,47 +630,87 @@ delta_block_solve_kernel(const float* __restrict__ qn, const float* __restrict__
         }
     }
     __syncthreads();
-    // forward substitution: a thread a column, of beta v (the first DV) and of beta exp(G) k (the DP behind them)
-    for (int base = 0; base < vdim + dp; base += 256) {
-        const int c = base + tid;
-        if (c >= vdim + dp) break;
-        const bool of_v = c < vdim;
-        const int d = of_v ? c : c - vdim;
-        const float* src = of_v ? vf + first * vv + h * vdim + d : kn + (first * kv_heads + kvh) * dp + d;
+    // the inverses of the four diagonal blocks of I + A: wave w's of block w, a lane a column, row by row
+    {
+        float x[16];
+        const int b0 = 16 * wave;
+#pragma unroll
+        for (int i = 0; i < 16; ++i) {
+            float s[4] = {i == col ? 1.f : 0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (int j = 0; j < i; j += 4) {
+                const delta_f32x4 av = *reinterpret_cast<const delta_f32x4*>(&a_s[b0 + i][b0 + j]);
+#pragma unroll
+                for (int e = 0; e < 4; ++e)
+                    if (j + e < i) s[e] -= av[e] * x[j + e];
+            }
+            x[i] = (s[0] + s[1]) + (s[2] + s[3]);
+        }
+        if (g == 0) {
+#pragma unroll
+            for (int i = 0; i < 16; ++i) inv_s[wave][i][col] = x[i];
+        }
+    }
+    __syncthreads();
+    // Block rows of A (negated) and the inverses as left operands: row lane % 16, columns 4 (lane / 16) + j.  A result of a
+    // product (rows 4 (lane / 16) + i) is the right operand of the next as it stands.
+    delta_f32x4 af[6], inv[4];
+#pragma unroll
+    for (int bi = 0; bi < 4; ++bi) {
+        inv[bi] = *reinterpret_cast<const delta_f32x4*>(&inv_s[bi][col][4 * g]);
+#pragma unroll
+        for (int bj = 0; bj < bi; ++bj) {
+            const delta_f32x4 v = *reinterpret_cast<const delta_f32x4*>(&a_s[16 * bi + col][16 * bj + 4 * g]);
+            af[bi * (bi - 1) / 2 + bj] = delta_f32x4{-v[0], -v[1], -v[2], -v[3]};
+        }
+    }
+    // forward substitution by blocks of 16 rows: a wave 16 columns at a time, of beta v (the first DV) or of beta exp(G) k
+    const int v_blocks = (vdim + 15) / 16, blocks = v_blocks + (dp + 15) / 16;
+    for (int cb = wave; cb < blocks; cb += 4) {
+        const bool of_v = cb < v_blocks;
+        const int d = 16 * (of_v ? cb : cb - v_blocks) + col, width = of_v ? vdim : dp;
+        const bool live = d < width;
+        const float* src = of_v ? vf + first * vv + h * vdim : kn + (first * kv_heads + kvh) * dp;
         const int64_t step = of_v ? vv : (int64_t)kv_heads * dp;
-        float x[DELTA_BLOCK];
+        const float* scale = of_v ? b_s : bg_s;                         // (zero past the block's end)
+        delta_f32x4 x[4];
 #pragma unroll
-        for (int i = 0; i < DELTA_BLOCK; ++i) x[i] = src[min(i, n - 1) * step];
-        if (!of_v) {
-            float* kt = kt_out + (ub * dp + d) * DELTA_BLOCK;
+        for (int bi = 0; bi < 4; ++bi)
 #pragma unroll
-            for (int i = 0; i < DELTA_BLOCK; i += 4) {
+            for (int i = 0; i < 4; ++i) x[bi][i] = src[min(16 * bi + 4 * g + i, n - 1) * step + min(d, width - 1)];
+        if (!of_v && live) {
+#pragma unroll
+            for (int bi = 0; bi < 4; ++bi) {
                 delta_f32x4 v;
 #pragma unroll
-                for (int e = 0; e < 4; ++e) v[e] = i + e < n ? x[i + e] * eg_s[i + e] : 0.f;
-                *reinterpret_cast<delta_f32x4*>(kt + i) = v;
+                for (int i = 0; i < 4; ++i) {
+                    const int t = 16 * bi + 4 * g + i;
+                    v[i] = t < n ? x[bi][i] * eg_s[t] : 0.f;
+                }
+                *reinterpret_cast<delta_f32x4*>(kt_out + (ub * dp + d) * DELTA_BLOCK + 16 * bi + 4 * g) = v;
             }
         }
-        const float* scale = of_v ? b_s : bg_s;                         // (zero past the block's end)
 #pragma unroll
-        for (int i = 0; i < DELTA_BLOCK; ++i) x[i] *= scale[i];
+        for (int bi = 0; bi < 4; ++bi) {
+            delta_f32x4 r;
 #pragma unroll
-        for (int i = 1; i < DELTA_BLOCK; ++i) {
-            float s[4] = {0.f, 0.f, 0.f, 0.f};
+            for (int i = 0; i < 4; ++i) r[i] = x[bi][i] * scale[16 * bi + 4 * g + i];
 #pragma unroll
-            for (int j = 0; j + 4 <= i; j += 4) {
-                const delta_f32x4 a = *reinterpret_cast<const delta_f32x4*>(&a_s[i][j]);
+            for (int bj = 0; bj < bi; ++bj)
 #pragma unroll
-                for (int e = 0; e < 4; ++e) s[e] += a[e] * x[j + e];
-            }
+                for (int j = 0; j < 4; ++j) r = __builtin_amdgcn_mfma_f32_16x16x4f32(af[bi * (bi - 1) / 2 + bj][j], x[bj][j], r, 0, 0, 0);
+            delta_f32x4 y = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-            for (int j = i / 4 * 4; j < i; ++j) s[j % 4] += a_s[i][j] * x[j];
-            x[i] -= (s[0] + s[1]) + (s[2] + s[3]);
+            for (int j = 0; j < 4; ++j) y = __builtin_amdgcn_mfma_f32_16x16x4f32(inv[bi][j], r[j], y, 0, 0, 0);
+            x[bi] = y;
         }
         float* dst = of_v ? u_out + ub * DELTA_BLOCK * vdim + d : w_out + ub * DELTA_BLOCK * dp + d;
-        const int width = of_v ? vdim : dp;
+        if (live) {
 #pragma unroll
-        for (int i = 0; i < DELTA_BLOCK; ++i) dst[(int64_t)i * width] = x[i];
+            for (int bi = 0; bi < 4; ++bi)
+#pragma unroll
+                for (int i = 0; i < 4; ++i) dst[(int64_t)(16 * bi + 4 * g + i) * width] = x[bi][i];
+        }
     }
 }
 
@@ -709,50 +751,41 @@ delta_block_scan_kernel(const float* __restrict__ qn, const float* __restrict__ 
         }
         if (kb < KB) *reinterpret_cast<delta_f32x4*>(&s_s[col][16 * kb + 4 * g]) = S[b];
     }
-    delta_f32x4 wf[KB], qf[KB];
-    auto ask = [&](int blk) __attribute__((always_inline)) {
+    // A block's operands, asked for while the block before it is at work.
+    struct Operands {
+        delta_f32x4 wf[KB], qf[KB], pf[4], kt[NB][4], gi, u;
+        float g_end;
+        int first, n;
+    };
+    auto ask = [&](int blk, Operands& o) __attribute__((always_inline)) {
         const int32_t* un = units + 4 * (unit0 + blk);
         const int64_t ub = (int64_t)(unit0 + blk) * heads + h;
-        const float* wr = w_in + (ub * DELTA_BLOCK + 16 * wave + col) * dp + 4 * g;
-        const float* qr = qn + ((un[1] + min(16 * wave + col, un[2] - 1)) * (int64_t)kv_heads + kvh) * dp + 4 * g;
+        o.first = un[1], o.n = un[2];
+        const float* wr = w_in + (ub * DELTA_BLOCK + 16 * wave + col) * dp;
+        const float* qr = qn + ((o.first + min(16 * wave + col, o.n - 1)) * (int64_t)kv_heads + kvh) * dp;
+        const float* pr = p_in + (ub * DELTA_BLOCK + 16 * wave + col) * DELTA_BLOCK + 4 * g;
+        const float* gr = g_cum + ub * DELTA_BLOCK;
+        // (every load unconditional: what lies outside the row reads its first entries, and meets rows of zeros of the state)
 #pragma unroll
         for (int s = 0; s < KB; ++s) {
-            wf[s] = qf[s] = delta_f32x4{0.f, 0.f, 0.f, 0.f};
-            if (16 * s + 4 * g < dp) {
-                wf[s] = *reinterpret_cast<const delta_f32x4*>(wr + 16 * s);
-                qf[s] = *reinterpret_cast<const delta_f32x4*>(qr + 16 * s);
-            }
+            const int at = 16 * s + 4 * g < dp ? 16 * s + 4 * g : 0;
+            o.wf[s] = *reinterpret_cast<const delta_f32x4*>(wr + at);
+            o.qf[s] = *reinterpret_cast<const delta_f32x4*>(qr + at);
         }
-    };
-    ask(0);
-    delta_barrier();
-    for (int blk = 0; blk < blocks; ++blk) {
-        const int64_t ub = (int64_t)(unit0 + blk) * heads + h;
-        const int64_t first = units[4 * (unit0 + blk) + 1];
-        const int n = units[4 * (unit0 + blk) + 2];
-        // what the second half reads is asked for before the first half's products
-        delta_f32x4 pf[4], kt[NB][4];
-        const float* pr = p_in + (ub * DELTA_BLOCK + 16 * wave + col) * DELTA_BLOCK + 4 * g;
 #pragma unroll
-        for (int s = 0; s < 4; ++s) {
-            pf[s] = delta_f32x4{0.f, 0.f, 0.f, 0.f};
-            if (s <= wave) pf[s] = *reinterpret_cast<const delta_f32x4*>(pr + 16 * s);
-        }
+        for (int i = 0; i < 4; ++i) o.u[i] = u_in[(ub * DELTA_BLOCK + 16 * wave + 4 * g + i) * vdim + (live ? column : 0)];
+#pragma unroll
+        for (int s = 0; s < 4; ++s) o.pf[s] = *reinterpret_cast<const delta_f32x4*>(pr + 16 * (s <= wave ? s : 0));
 #pragma unroll
         for (int b = 0; b < NB; ++b) {
-            const int row = 16 * (wave + 4 * b) + col;
+            const int row = min(16 * (wave + 4 * b) + col, dp - 1);
 #pragma unroll
-            for (int s = 0; s < 4; ++s) {
-                kt[b][s] = delta_f32x4{0.f, 0.f, 0.f, 0.f};
-                if (row < dp) kt[b][s] = *reinterpret_cast<const delta_f32x4*>(kt_in + (ub * dp + row) * DELTA_BLOCK + 16 * s + 4 * g);
-            }
+            for (int s = 0; s < 4; ++s) o.kt[b][s] = *reinterpret_cast<const delta_f32x4*>(kt_in + (ub * dp + row) * DELTA_BLOCK + 16 * s + 4 * g);
         }
-        const float* gr = g_cum + ub * DELTA_BLOCK;
-        const delta_f32x4 gi = *reinterpret_cast<const delta_f32x4*>(gr + 16 * wave + 4 * g);
-        const float g_end = gr[DELTA_BLOCK - 1];
-        delta_f32x4 u;
-#pragma unroll
-        for (int i = 0; i < 4; ++i) u[i] = live ? u_in[(ub * DELTA_BLOCK + 16 * wave + 4 * g + i) * vdim + column] : 0.f;
+        o.gi = *reinterpret_cast<const delta_f32x4*>(gr + 16 * wave + 4 * g);
+        o.g_end = gr[DELTA_BLOCK - 1];
+    };
+    auto run = [&](const Operands& o) __attribute__((always_inline)) {
         // W S and Q S of this wave's 16 tokens
         delta_f32x4 x = {0.f, 0.f, 0.f, 0.f}, y = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
@@ -760,16 +793,16 @@ delta_block_scan_kernel(const float* __restrict__ qn, const float* __restrict__ 
             const delta_f32x4 sv = *reinterpret_cast<const delta_f32x4*>(&s_s[col][16 * s + 4 * g]);
 #pragma unroll
             for (int j = 0; j < 4; ++j) {
-                x = __builtin_amdgcn_mfma_f32_16x16x4f32(wf[s][j], sv[j], x, 0, 0, 0);
-                y = __builtin_amdgcn_mfma_f32_16x16x4f32(qf[s][j], sv[j], y, 0, 0, 0);
+                x = __builtin_amdgcn_mfma_f32_16x16x4f32(o.wf[s][j], sv[j], x, 0, 0, 0);
+                y = __builtin_amdgcn_mfma_f32_16x16x4f32(o.qf[s][j], sv[j], y, 0, 0, 0);
             }
         }
-        if (blk + 1 < blocks) ask(blk + 1);
+        delta_f32x4 u;
 #pragma unroll
-        for (int i = 0; i < 4; ++i) u[i] -= x[i], y[i] *= expf(gi[i]);
+        for (int i = 0; i < 4; ++i) u[i] = o.u[i] - x[i], y[i] *= expf(o.gi[i]);
         *reinterpret_cast<delta_f32x4*>(&u_s[col][16 * wave + 4 * g]) = u;
         delta_barrier();                                                // the block's writes are in; the state is read
-        const float e_end = expf(g_end);
+        const float e_end = expf(o.g_end);
 #pragma unroll
         for (int b = 0; b < NB; ++b)
 #pragma unroll
@@ -779,20 +812,36 @@ delta_block_scan_kernel(const float* __restrict__ qn, const float* __restrict__ 
             const delta_f32x4 uv = *reinterpret_cast<const delta_f32x4*>(&u_s[col][16 * s + 4 * g]);
 #pragma unroll
             for (int j = 0; j < 4; ++j) {
-                if (s <= wave) y = __builtin_amdgcn_mfma_f32_16x16x4f32(pf[s][j], uv[j], y, 0, 0, 0);
+                if (s <= wave) y = __builtin_amdgcn_mfma_f32_16x16x4f32(o.pf[s][j], uv[j], y, 0, 0, 0);
 #pragma unroll
-                for (int b = 0; b < NB; ++b) S[b] = __builtin_amdgcn_mfma_f32_16x16x4f32(kt[b][s][j], uv[j], S[b], 0, 0, 0);
+                for (int b = 0; b < NB; ++b) S[b] = __builtin_amdgcn_mfma_f32_16x16x4f32(o.kt[b][s][j], uv[j], S[b], 0, 0, 0);
             }
         }
+        // (the state's rows past the head's size stay zero: the products that read them meet anything there)
+#pragma unroll
+        for (int b = 0; b < NB; ++b)
+            if (wave + 4 * b < KB) {
+                delta_f32x4 v = S[b];
+#pragma unroll
+                for (int i = 0; i < 4; ++i) v[i] = 16 * (wave + 4 * b) + 4 * g + i < dim ? v[i] : 0.f;
+                *reinterpret_cast<delta_f32x4*>(&s_s[col][16 * (wave + 4 * b) + 4 * g]) = v;
+            }
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
             const int row = 16 * wave + 4 * g + i;
-            if (live && row < n) o_raw[(first + row) * vv + h * vdim + column] = y[i];
+            if (live && row < o.n) o_raw[(int64_t)(o.first + row) * vv + h * vdim + column] = y[i];
         }
-#pragma unroll
-        for (int b = 0; b < NB; ++b)
-            if (wave + 4 * b < KB) *reinterpret_cast<delta_f32x4*>(&s_s[col][16 * (wave + 4 * b) + 4 * g]) = S[b];
         delta_barrier();                                                // the state is in; the block's writes are read
+    };
+    Operands even, odd;
+    ask(0, even);
+    delta_barrier();
+    for (int blk = 0; blk < blocks; blk += 2) {
+        if (blk + 1 < blocks) ask(blk + 1, odd);
+        run(even);
+        if (blk + 1 >= blocks) break;
+        if (blk + 2 < blocks) ask(blk + 2, even);
+        run(odd);
     }
     if (!live) return;
 #pragma unroll

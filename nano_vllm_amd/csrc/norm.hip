@@ -348,33 +348,35 @@ stream_post_norm_kernel(const T* __restrict__ a, int64_t a_stride, PartialInput 
         return is_f32 ? static_cast<const float*>(v)[i] : to_float(static_cast<const T*>(v)[i]);
     };
     float kept[KEEP], r_k[KEEP], wa_k[KEEP], w_k[KEEP];
+    int at[KEEP];
 #pragma unroll
     for (int n = 0; n < KEEP; ++n) {
-        const int i = tid + n * step;
-        const bool in = i < width;
-        kept[n] = in && !pa.sums ? to_float(ar[i]) : 0.f;
-        r_k[n] = in ? rr[i] : 0.f;
-        wa_k[n] = in ? vec(a_weight, aw_is_f32, i) : 0.f;
-        w_k[n] = in ? vec(weight, w_is_f32, i) : 0.f;
+        at[n] = min(tid + n * step, width - 1);           // (every load unconditional; an entry outside the row counts as zero)
+        kept[n] = 0.f;
+        if (!pa.sums) kept[n] = to_float(ar[at[n]]);
+        r_k[n] = rr[at[n]];
+        wa_k[n] = vec(a_weight, aw_is_f32, at[n]);
+        w_k[n] = vec(weight, w_is_f32, at[n]);
     }
     if (pa.sums) {
         // the splits' sums of all kept entries side by side, each in the order of the splits
-        const float* q = pa.sums + row * width + tid;
-#pragma unroll 4
+        const float* q = pa.sums + row * width;
+#pragma unroll 8
         for (int s = 0; s < pa.splits; ++s)
 #pragma unroll
-            for (int n = 0; n < KEEP; ++n)
-                if (tid + n * step < width) kept[n] += q[s * pa.split_stride + n * step];
+            for (int n = 0; n < KEEP; ++n) kept[n] += q[s * pa.split_stride + at[n]];
 #pragma unroll
         for (int n = 0; n < KEEP; ++n) {
-            const int i = tid + n * step;
-            if (pa.bias && i < width) kept[n] += to_float(static_cast<const T*>(pa.bias)[i]);
+            if (pa.bias) kept[n] += to_float(static_cast<const T*>(pa.bias)[at[n]]);
             kept[n] = round_through<T>(kept[n]);
         }
     }
     float ss = 0.f;
 #pragma unroll
-    for (int n = 0; n < KEEP; ++n) ss += kept[n] * kept[n];
+    for (int n = 0; n < KEEP; ++n) {
+        if (tid + n * step >= width) kept[n] = r_k[n] = 0.f;
+        ss += kept[n] * kept[n];
+    }
     for (int i = tid + KEEP * step; i < width; i += step) {
         const float v = pa.sums ? partial_value<T>(pa, row, width, i) : to_float(ar[i]);
         ss += v * v;
