@@ -721,7 +721,7 @@ __device__ __forceinline__ void delta_barrier() { asm volatile("s_waitcnt lgkmcn
 // portion, 16 columns of S), heads fastest, so that the workgroups of a head meet in one die's L2.  The state's columns lie
 // in accumulators (wave w: the blocks w, w + 4, ... of 16 rows) and, transposed, in LDS for the products that read them.
 template <int KB>
-__global__ void __launch_bounds__(256)
+__global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1)))
 delta_block_scan_kernel(const float* __restrict__ qn, const float* __restrict__ g_cum, const float* __restrict__ w_in,
                         const float* __restrict__ u_in, const float* __restrict__ p_in, const float* __restrict__ kt_in,
                         float* __restrict__ o_raw, float* __restrict__ state, const int32_t* __restrict__ units,
@@ -733,7 +733,7 @@ delta_block_scan_kernel(const float* __restrict__ qn, const float* __restrict__ 
     const int h = blockIdx.x % heads, rest = blockIdx.x / heads;
     const int32_t* ch = chains + 4 * (rest % num_chains);
     const int unit0 = ch[0], blocks = ch[1], seq = ch[2];
-    const int tid = threadIdx.x, wave = tid / NVA_WAVE, lane = tid % NVA_WAVE, col = lane & 15, g = lane >> 4;
+    const int tid = threadIdx.x, wave = __builtin_amdgcn_readfirstlane(tid / NVA_WAVE), lane = tid % NVA_WAVE, col = lane & 15, g = lane >> 4;
     const int column = 16 * (rest / num_chains) + col;
     const bool live = column < vdim;
     const int kvh = h / (heads / kv_heads);
@@ -757,7 +757,10 @@ delta_block_scan_kernel(const float* __restrict__ qn, const float* __restrict__ 
         float g_end;
         int first, n;
     };
+    // (Unconditional, the last block's once more behind the end: a load that may or may not be on its way makes every wait
+    // before its use wait for all of them.)
     auto ask = [&](int blk, Operands& o) __attribute__((always_inline)) {
+        blk = min(blk, blocks - 1);
         const int32_t* un = units + 4 * (unit0 + blk);
         const int64_t ub = (int64_t)(unit0 + blk) * heads + h;
         o.first = un[1], o.n = un[2];
@@ -787,15 +790,19 @@ delta_block_scan_kernel(const float* __restrict__ qn, const float* __restrict__ 
     };
     auto run = [&](const Operands& o) __attribute__((always_inline)) {
         // W S and Q S of this wave's 16 tokens
-        delta_f32x4 x = {0.f, 0.f, 0.f, 0.f}, y = {0.f, 0.f, 0.f, 0.f};
+        delta_f32x4 x = {0.f, 0.f, 0.f, 0.f}, y = {0.f, 0.f, 0.f, 0.f}, sv[2];
+        sv[0] = *reinterpret_cast<const delta_f32x4*>(&s_s[col][4 * g]);
 #pragma unroll
         for (int s = 0; s < KB; ++s) {
-            const delta_f32x4 sv = *reinterpret_cast<const delta_f32x4*>(&s_s[col][16 * s + 4 * g]);
+            // (a step's operand is read from LDS while the step before it multiplies)
+            if (s + 1 < KB) sv[(s + 1) & 1] = *reinterpret_cast<const delta_f32x4*>(&s_s[col][16 * (s + 1) + 4 * g]);
+            __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
             for (int j = 0; j < 4; ++j) {
-                x = __builtin_amdgcn_mfma_f32_16x16x4f32(o.wf[s][j], sv[j], x, 0, 0, 0);
-                y = __builtin_amdgcn_mfma_f32_16x16x4f32(o.qf[s][j], sv[j], y, 0, 0, 0);
+                x = __builtin_amdgcn_mfma_f32_16x16x4f32(o.wf[s][j], sv[s & 1][j], x, 0, 0, 0);
+                y = __builtin_amdgcn_mfma_f32_16x16x4f32(o.qf[s][j], sv[s & 1][j], y, 0, 0, 0);
             }
+            __builtin_amdgcn_sched_barrier(0);
         }
         delta_f32x4 u;
 #pragma unroll
@@ -807,16 +814,21 @@ delta_block_scan_kernel(const float* __restrict__ qn, const float* __restrict__ 
         for (int b = 0; b < NB; ++b)
 #pragma unroll
             for (int i = 0; i < 4; ++i) S[b][i] *= e_end;
+        delta_f32x4 uv[4];
 #pragma unroll
-        for (int s = 0; s < 4; ++s) {
-            const delta_f32x4 uv = *reinterpret_cast<const delta_f32x4*>(&u_s[col][16 * s + 4 * g]);
+        for (int s = 0; s < 4; ++s) uv[s] = *reinterpret_cast<const delta_f32x4*>(&u_s[col][16 * s + 4 * g]);
+        __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
-            for (int j = 0; j < 4; ++j) {
-                if (s <= wave) y = __builtin_amdgcn_mfma_f32_16x16x4f32(o.pf[s][j], uv[j], y, 0, 0, 0);
+        for (int s = 0; s < 4; ++s)
 #pragma unroll
-                for (int b = 0; b < NB; ++b) S[b] = __builtin_amdgcn_mfma_f32_16x16x4f32(o.kt[b][s][j], uv[j], S[b], 0, 0, 0);
-            }
-        }
+            for (int j = 0; j < 4; ++j)
+#pragma unroll
+                for (int b = 0; b < NB; ++b) S[b] = __builtin_amdgcn_mfma_f32_16x16x4f32(o.kt[b][s][j], uv[s][j], S[b], 0, 0, 0);
+#pragma unroll
+        for (int s = 0; s < 4; ++s)
+            if (s <= wave)
+#pragma unroll
+                for (int j = 0; j < 4; ++j) y = __builtin_amdgcn_mfma_f32_16x16x4f32(o.pf[s][j], uv[s][j], y, 0, 0, 0);
         // (the state's rows past the head's size stay zero: the products that read them meet anything there)
 #pragma unroll
         for (int b = 0; b < NB; ++b)
@@ -837,10 +849,10 @@ delta_block_scan_kernel(const float* __restrict__ qn, const float* __restrict__ 
     ask(0, even);
     delta_barrier();
     for (int blk = 0; blk < blocks; blk += 2) {
-        if (blk + 1 < blocks) ask(blk + 1, odd);
+        ask(blk + 1, odd);
         run(even);
         if (blk + 1 >= blocks) break;
-        if (blk + 2 < blocks) ask(blk + 2, even);
+        ask(blk + 2, even);
         run(odd);
     }
     if (!live) return;
