@@ -466,8 +466,11 @@ delta_single_kernel(const T* __restrict__ proj, int64_t stride, DeltaRates rates
 
 // ---------------------------------------------------------------------------- portions in blocks, one decay per head
 // units: int32 [n][4] = (request, the block's first token counted through the step, its tokens, unused); a portion's blocks
-// side by side.  Scratch of block u and head h, each indexed by ub = u * heads + h: g_cum [ub][64], w [ub][64][DP],
-// u [ub][64][DV], p [ub][64][64], k_t [ub][DP][64]; tokens past a block's end are rows of zeros.
+// side by side.  Scratch of block u and head h, each indexed by ub = u * heads + h: g_cum [ub][64], and the operands of the
+// pass over the blocks as its lanes hold them, 64 x 4 floats side by side (one load a wave): w and q [ub][4 x 16 tokens]
+// [KB x 16 channels], p [ub][4 x 16 tokens][4 x 16 tokens], k_t [ub][KB x 16 channels][4 x 16 tokens], all as left operands
+// (row lane % 16, columns 4 (lane / 16) + j), u [ub][DV / 16][4 x 16 tokens] as results (rows 4 (lane / 16) + i, column
+// lane % 16).  Tokens past a block's end are zeros in w, p, k_t and u.
 template <typename T, int TAPS>
 __global__ void __launch_bounds__(DELTA_PREPARE_THREADS)
 delta_block_prepare_kernel(const T* __restrict__ proj, int64_t stride, DeltaRates rates, const T* __restrict__ conv_w,
@@ -571,8 +574,10 @@ template <int KB>
 __global__ void __launch_bounds__(256)
 delta_block_solve_kernel(const float* __restrict__ qn, const float* __restrict__ kn, const float* __restrict__ vf,
                          const float* __restrict__ decay, const float* __restrict__ beta, const int32_t* __restrict__ units,
-                         int heads, int kv_heads, int dim, int vdim, float* __restrict__ g_cum, float* __restrict__ w_out,
-                         float* __restrict__ u_out, float* __restrict__ p_out, float* __restrict__ kt_out) {
+                         int heads, int kv_heads, int dim, int vdim, float* __restrict__ g_cum, delta_f32x4* __restrict__ w_out,
+                         delta_f32x4* __restrict__ q_out, delta_f32x4* __restrict__ u_out, delta_f32x4* __restrict__ p_out,
+                         delta_f32x4* __restrict__ kt_out) {
+    __shared__ __attribute__((aligned(16))) float tile_s[4][16][20];        // a wave's, to turn a result into a left operand
     __shared__ __attribute__((aligned(16))) float a_s[DELTA_BLOCK][DELTA_BLOCK + 4];
     __shared__ __attribute__((aligned(16))) float inv_s[4][16][20];
     __shared__ float g_s[DELTA_BLOCK], b_s[DELTA_BLOCK], bg_s[DELTA_BLOCK], eg_s[DELTA_BLOCK];
@@ -599,6 +604,12 @@ delta_block_solve_kernel(const float* __restrict__ qn, const float* __restrict__
         g_cum[ub * DELTA_BLOCK + lane] = sum;
     }
     __syncthreads();
+    // a wave's 16 x 16 result (rows 4 g + i, column col) as a left operand (row col, columns 4 g + j)
+    auto turned = [&](const delta_f32x4& v) __attribute__((always_inline)) {
+#pragma unroll
+        for (int i = 0; i < 4; ++i) tile_s[wave][4 * g + i][col] = v[i];
+        return *reinterpret_cast<const delta_f32x4*>(&tile_s[wave][col][4 * g]);
+    };
     // the ten blocks of 16 x 16 on and below the diagonal, of k k^T and of q k^T
     for (int task = wave; task < 20; task += 4) {
         const int pair = task >> 1;
@@ -620,13 +631,20 @@ delta_block_solve_kernel(const float* __restrict__ qn, const float* __restrict__
         for (int s = 0; s < KB; ++s)
 #pragma unroll
             for (int j = 0; j < 4; ++j) acc = __builtin_amdgcn_mfma_f32_16x16x4f32(fa[s][j], fb[s][j], acc, 0, 0, 0);
+        delta_f32x4 v;
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
             const int r = 16 * bi + 4 * g + i, c = 16 * bj + col;
             const bool seen = r < n && (of_q ? c <= r : c < r);
-            const float v = seen ? expf(g_s[r] - g_s[c]) * acc[i] : 0.f;
-            if (of_q) p_out[(ub * DELTA_BLOCK + r) * DELTA_BLOCK + c] = v;
-            else a_s[r][c] = b_s[r] * v;
+            v[i] = seen ? expf(g_s[r] - g_s[c]) * acc[i] : 0.f;
+            if (!of_q) a_s[r][c] = b_s[r] * v[i];
+        }
+        if (of_q) {
+            p_out[((ub * 4 + bi) * 4 + bj) * NVA_WAVE + lane] = turned(v);
+            if (bj == 0) {
+#pragma unroll
+                for (int s = 0; s < KB; ++s) q_out[((ub * 4 + bi) * KB + s) * NVA_WAVE + lane] = fa[s];
+            }
         }
     }
     __syncthreads();
@@ -665,11 +683,11 @@ delta_block_solve_kernel(const float* __restrict__ qn, const float* __restrict__
         }
     }
     // forward substitution by blocks of 16 rows: a wave 16 columns at a time, of beta v (the first DV) or of beta exp(G) k
-    const int v_blocks = (vdim + 15) / 16, blocks = v_blocks + (dp + 15) / 16;
+    // (columns past a size repeat the last one: the pass over the blocks meets them with zeros, or writes nothing of them)
+    const int v_blocks = (vdim + 15) / 16, blocks = v_blocks + KB;
     for (int cb = wave; cb < blocks; cb += 4) {
         const bool of_v = cb < v_blocks;
         const int d = 16 * (of_v ? cb : cb - v_blocks) + col, width = of_v ? vdim : dp;
-        const bool live = d < width;
         const float* src = of_v ? vf + first * vv + h * vdim : kn + (first * kv_heads + kvh) * dp;
         const int64_t step = of_v ? vv : (int64_t)kv_heads * dp;
         const float* scale = of_v ? b_s : bg_s;                         // (zero past the block's end)
@@ -678,7 +696,7 @@ delta_block_solve_kernel(const float* __restrict__ qn, const float* __restrict__
         for (int bi = 0; bi < 4; ++bi)
 #pragma unroll
             for (int i = 0; i < 4; ++i) x[bi][i] = src[min(16 * bi + 4 * g + i, n - 1) * step + min(d, width - 1)];
-        if (!of_v && live) {
+        if (!of_v) {
 #pragma unroll
             for (int bi = 0; bi < 4; ++bi) {
                 delta_f32x4 v;
@@ -687,7 +705,7 @@ delta_block_solve_kernel(const float* __restrict__ qn, const float* __restrict__
                     const int t = 16 * bi + 4 * g + i;
                     v[i] = t < n ? x[bi][i] * eg_s[t] : 0.f;
                 }
-                *reinterpret_cast<delta_f32x4*>(kt_out + (ub * dp + d) * DELTA_BLOCK + 16 * bi + 4 * g) = v;
+                kt_out[((ub * KB + cb - v_blocks) * 4 + bi) * NVA_WAVE + lane] = v;
             }
         }
 #pragma unroll
@@ -704,12 +722,10 @@ delta_block_solve_kernel(const float* __restrict__ qn, const float* __restrict__
             for (int j = 0; j < 4; ++j) y = __builtin_amdgcn_mfma_f32_16x16x4f32(inv[bi][j], r[j], y, 0, 0, 0);
             x[bi] = y;
         }
-        float* dst = of_v ? u_out + ub * DELTA_BLOCK * vdim + d : w_out + ub * DELTA_BLOCK * dp + d;
-        if (live) {
 #pragma unroll
-            for (int bi = 0; bi < 4; ++bi)
-#pragma unroll
-                for (int i = 0; i < 4; ++i) dst[(int64_t)(16 * bi + 4 * g + i) * width] = x[bi][i];
+        for (int bi = 0; bi < 4; ++bi) {
+            if (of_v) u_out[((ub * v_blocks + cb) * 4 + bi) * NVA_WAVE + lane] = x[bi];
+            else w_out[((ub * 4 + bi) * KB + cb - v_blocks) * NVA_WAVE + lane] = turned(x[bi]);
         }
     }
 }
@@ -722,11 +738,11 @@ __device__ __forceinline__ void delta_barrier() { asm volatile("s_waitcnt lgkmcn
 // in accumulators (wave w: the blocks w, w + 4, ... of 16 rows) and, transposed, in LDS for the products that read them.
 template <int KB>
 __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1)))
-delta_block_scan_kernel(const float* __restrict__ qn, const float* __restrict__ g_cum, const float* __restrict__ w_in,
-                        const float* __restrict__ u_in, const float* __restrict__ p_in, const float* __restrict__ kt_in,
-                        float* __restrict__ o_raw, float* __restrict__ state, const int32_t* __restrict__ units,
+delta_block_scan_kernel(const float* __restrict__ g_cum, const delta_f32x4* __restrict__ w_in, const delta_f32x4* __restrict__ q_in,
+                        const delta_f32x4* __restrict__ u_in, const delta_f32x4* __restrict__ p_in,
+                        const delta_f32x4* __restrict__ kt_in, float* __restrict__ o_raw, float* __restrict__ state, const int32_t* __restrict__ units,
                         const int32_t* __restrict__ chains, int num_chains, const int32_t* __restrict__ seq_starts,
-                        const int32_t* __restrict__ state_slots, int heads, int kv_heads, int dim, int vdim) {
+                        const int32_t* __restrict__ state_slots, int heads, int dim, int vdim) {
     constexpr int NB = (KB + 3) / 4;
     __shared__ __attribute__((aligned(16))) float s_s[16][16 * KB + 4];     // [column][row]
     __shared__ __attribute__((aligned(16))) float u_s[16][DELTA_BLOCK + 4]; // [column][token]
@@ -736,8 +752,7 @@ delta_block_scan_kernel(const float* __restrict__ qn, const float* __restrict__ 
     const int tid = threadIdx.x, wave = __builtin_amdgcn_readfirstlane(tid / NVA_WAVE), lane = tid % NVA_WAVE, col = lane & 15, g = lane >> 4;
     const int column = 16 * (rest / num_chains) + col;
     const bool live = column < vdim;
-    const int kvh = h / (heads / kv_heads);
-    const int dp = (dim + 3) & ~3, vv = heads * vdim;
+    const int vv = heads * vdim, v_blocks = (vdim + 15) / 16;
     float* S_g = state + ((int64_t)state_slots[seq] * heads + h) * dim * vdim + column;
     const bool has_past = seq_starts[seq] > 0;
     delta_f32x4 S[NB];
@@ -764,27 +779,22 @@ delta_block_scan_kernel(const float* __restrict__ qn, const float* __restrict__ 
         const int32_t* un = units + 4 * (unit0 + blk);
         const int64_t ub = (int64_t)(unit0 + blk) * heads + h;
         o.first = un[1], o.n = un[2];
-        const float* wr = w_in + (ub * DELTA_BLOCK + 16 * wave + col) * dp;
-        const float* qr = qn + ((o.first + min(16 * wave + col, o.n - 1)) * (int64_t)kv_heads + kvh) * dp;
-        const float* pr = p_in + (ub * DELTA_BLOCK + 16 * wave + col) * DELTA_BLOCK + 4 * g;
+        const delta_f32x4* wr = w_in + (ub * 4 + wave) * KB * NVA_WAVE + lane;
+        const delta_f32x4* qr = q_in + (ub * 4 + wave) * KB * NVA_WAVE + lane;
+        const delta_f32x4* pr = p_in + (ub * 4 + wave) * 4 * NVA_WAVE + lane;
         const float* gr = g_cum + ub * DELTA_BLOCK;
-        // (every load unconditional: what lies outside the row reads its first entries, and meets rows of zeros of the state)
 #pragma unroll
         for (int s = 0; s < KB; ++s) {
-            const int at = 16 * s + 4 * g < dp ? 16 * s + 4 * g : 0;
-            o.wf[s] = *reinterpret_cast<const delta_f32x4*>(wr + at);
-            o.qf[s] = *reinterpret_cast<const delta_f32x4*>(qr + at);
+            o.wf[s] = wr[s * NVA_WAVE];
+            o.qf[s] = qr[s * NVA_WAVE];
         }
+        o.u = u_in[((ub * v_blocks + rest / num_chains) * 4 + wave) * NVA_WAVE + lane];
 #pragma unroll
-        for (int i = 0; i < 4; ++i) o.u[i] = u_in[(ub * DELTA_BLOCK + 16 * wave + 4 * g + i) * vdim + (live ? column : 0)];
+        for (int s = 0; s < 4; ++s) o.pf[s] = pr[(s <= wave ? s : 0) * NVA_WAVE];
 #pragma unroll
-        for (int s = 0; s < 4; ++s) o.pf[s] = *reinterpret_cast<const delta_f32x4*>(pr + 16 * (s <= wave ? s : 0));
+        for (int b = 0; b < NB; ++b)
 #pragma unroll
-        for (int b = 0; b < NB; ++b) {
-            const int row = min(16 * (wave + 4 * b) + col, dp - 1);
-#pragma unroll
-            for (int s = 0; s < 4; ++s) o.kt[b][s] = *reinterpret_cast<const delta_f32x4*>(kt_in + (ub * dp + row) * DELTA_BLOCK + 16 * s + 4 * g);
-        }
+            for (int s = 0; s < 4; ++s) o.kt[b][s] = kt_in[((ub * KB + min(wave + 4 * b, KB - 1)) * 4 + s) * NVA_WAVE + lane];
         o.gi = *reinterpret_cast<const delta_f32x4*>(gr + 16 * wave + 4 * g);
         o.g_end = gr[DELTA_BLOCK - 1];
     };
@@ -956,10 +966,12 @@ static int delta_single_groups(int dim, int vdim) {
     return rg >= 1 && (dim + rg - 1) / rg <= 16 ? cg : -1;
 }
 
+// Steps of 16 key channels that the blocks' kernels are built for.
+static int delta_steps(int dim) { return dim <= 32 ? 2 : dim <= 64 ? 4 : dim <= 128 ? 8 : 16; }
+
 // Floats that nva_head_delta's block_scratch holds for n blocks of portions.
 NVA_EXPORT int64_t NVA_NAME(nva_head_delta_block_floats)(int64_t n, int heads, int dim, int vdim) {
-    const int64_t dp = (dim + 3) & ~3;
-    return n * heads * DELTA_BLOCK * (2 * dp + vdim + DELTA_BLOCK + 1);
+    return n * heads * DELTA_BLOCK * (3 * 16 * (int64_t)delta_steps(dim) + (vdim + 15) / 16 * 16 + DELTA_BLOCK + 1);
 }
 
 // One decay per head.  proj: elements [tokens, 2 G D + 2 H DV] = [q | k | v | gate], rows `stride` apart.  rates: float
@@ -1042,21 +1054,23 @@ NVA_EXPORT int NVA_NAME(nva_head_delta)(const void* proj, int64_t stride, const 
                                 blocked_from - first, heads, kv_heads, dim, vdim, stream);
     if (n_units) {
         const int64_t rows = n_units * heads * DELTA_BLOCK;
-        float* w = block_scratch;
-        float* u = w + rows * dp;
-        float* p = u + rows * vdim;
-        float* kt = p + rows * DELTA_BLOCK;
-        float* gc = kt + rows * dp;
         const unsigned slices = (unsigned)((vdim + 15) / 16);
+        const int steps = delta_steps(dim);
+        delta_f32x4* w = (delta_f32x4*)block_scratch;                   // (in units of four floats)
+        delta_f32x4* q = w + rows * 4 * steps;
+        delta_f32x4* kt = q + rows * 4 * steps;
+        delta_f32x4* u = kt + rows * 4 * steps;
+        delta_f32x4* p = u + rows * 4 * slices;
+        float* gc = (float*)(p + rows * (DELTA_BLOCK / 4));
 #define DELTA_BLOCKS(KK)                                                                                                  \
         do {                                                                                                              \
             hipLaunchKernelGGL((delta_block_solve_kernel<KK>), dim3((unsigned)(n_units * heads)), dim3(256), 0, stream, qn, kn, vf, decay, \
-                               beta, units, heads, kv_heads, dim, vdim, gc, w, u, p, kt);                                     \
-            hipLaunchKernelGGL((delta_block_scan_kernel<KK>), dim3((unsigned)(slices * n_chains * heads)), dim3(256), 0, stream, qn, gc, w,  \
-                               u, p, kt, o_raw, s_state, units, chains, (int)n_chains, seq_starts, state_slots, heads, kv_heads, dim,  \
+                               beta, units, heads, kv_heads, dim, vdim, gc, w, q, u, p, kt);                                  \
+            hipLaunchKernelGGL((delta_block_scan_kernel<KK>), dim3((unsigned)(slices * n_chains * heads)), dim3(256), 0, stream, gc, w, q,   \
+                               u, p, kt, o_raw, s_state, units, chains, (int)n_chains, seq_starts, state_slots, heads, dim,           \
                                vdim);                                                                                     \
         } while (0)
-        if (dim <= 32) DELTA_BLOCKS(2); else if (dim <= 64) DELTA_BLOCKS(4); else if (dim <= 128) DELTA_BLOCKS(8); else DELTA_BLOCKS(16);
+        if (steps == 2) DELTA_BLOCKS(2); else if (steps == 4) DELTA_BLOCKS(4); else if (steps == 8) DELTA_BLOCKS(8); else DELTA_BLOCKS(16);
 #undef DELTA_BLOCKS
     }
     hipLaunchKernelGGL((delta_finish_kernel<elem_t, true>), dim3((unsigned)left, (unsigned)heads), dim3(NVA_WAVE), 0, stream, o_raw,
