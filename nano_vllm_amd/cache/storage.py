@@ -56,7 +56,7 @@ def state_bytes_per_slot(needs, state_runs) -> int:
 
 
 def _state_dtype(name: str) -> torch.dtype:
-    return torch.float32 if name == "float32" else torch_dtype(name)
+    return torch.float32 if name == "float32" else torch.int32 if name == "int32" else torch_dtype(name)
 
 
 def allocate(needs, groups, state_runs, num_pages: Sequence[int], page_size: int, num_slots: int,

@@ -1084,3 +1084,218 @@ class BamipelConfig:
         if self.eos_token_id is not None:
             out["eos_token_id"] = list(self.eos_token_id)
         return out
+
+
+# ---------------------------------------------------------------------------- Nemidra
+@dataclass(frozen=True)
+class WindowAttentionConfig:
+    """Grouped causal softmax attention with biases on all four projections and no rotation; values of a size of
+    their own; window None: every earlier position."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    window: Optional[int] = None
+
+
+@dataclass(frozen=True)
+class MatrixMemoryConfig:
+    """A matrix memory with exponential gates: `heads` heads of dim key and vdim value channels; the gates' logits are
+    capped smoothly at +-gate_cap."""
+    heads: int
+    dim: int
+    vdim: int
+    gate_cap: float
+
+
+@dataclass(frozen=True)
+class GatedLinearConfig:
+    """Gated linear attention: a decay sigmoid(z)^(1/tau) per key channel.  The rank of z's two-step projection is read
+    from the tensors' shapes unless the mixer names it (decay_rank: what a folder of random weights is drawn with)."""
+    heads: int
+    dim: int
+    vdim: int
+    tau: float
+    decay_rank: Optional[int] = None
+
+
+@dataclass(frozen=True)
+class PairMixerConfig:
+    """Two mixers of one input: left_scale * left + right_scale * right."""
+    left: WindowAttentionConfig
+    right: MatrixMemoryConfig
+    left_scale: float = 1.0
+    right_scale: float = 1.0
+
+
+@dataclass(frozen=True)
+class SoftmaxScoreExpertsConfig:
+    """A routed feed-forward of gated experts: the `top` of `experts` with the largest softmax scores, weighted by
+    scale times their scores; shared_ff: the inner size of a shared expert behind a sigmoid gate, or None."""
+    experts: int
+    top: int
+    ff: int
+    scale: float = 1.0
+    shared_ff: Optional[int] = None
+
+
+@dataclass(frozen=True)
+class NemidraLayer:
+    kind: str                                    # "parallel" | "gla"
+    mixer: Any                                   # PairMixerConfig | GatedLinearConfig
+    mlp: Any                                     # None | int (a dense layer's inner size) | SoftmaxScoreExpertsConfig
+
+
+@dataclass(frozen=True)
+class BigramConfig:
+    """A second embedding by (token before, token): row (before * mul_prev + token * mul_cur) mod buckets."""
+    buckets: int
+    mul_prev: int
+    mul_cur: int
+
+
+@dataclass(frozen=True)
+class NemidraConfig:
+    """Nemidra: token, bigram and position embeddings; layers with a norm before and after each sublayer on a float32
+    residual stream, then an input of its own from a table of the tokens; the mixer is, layer by layer, a window
+    attention beside a matrix memory or a gated linear attention; the feed-forward dense, a mixture of experts, or
+    absent; layers loop[0] .. loop[1] - 1 run loop[2] times in a row, with the embedding added before every pass but
+    the first.  config.json gives every size and constant, layer by layer."""
+    vocab: int
+    width: int
+    eps: float
+    layers: Tuple[NemidraLayer, ...]
+    max_positions: int
+    side_dim: Optional[int]                      # None: no table of the tokens, no such input
+    bigram: Optional[BigramConfig]
+    loop: Tuple[int, int, int]
+    logit_softcap: Optional[float] = None
+    dtype: str = "bfloat16"
+    eos_token_id: Optional[Tuple[int, ...]] = None
+    architecture: str = "Nemidra"
+
+    @staticmethod
+    def _mixer(kind, m: Mapping[str, Any], ma: str):
+        if kind == "gla":
+            return GatedLinearConfig(
+                heads=_whole(m, "heads", ma), dim=_whole(m, "dim", ma), vdim=_whole(m, "vdim", ma), tau=_require(m, "tau", float, ma),
+                decay_rank=None if m.get("decay_rank") is None else _whole(m, "decay_rank", ma))
+        if kind != "parallel":
+            raise ConfigError(f"{ma}: the layer's type must be 'parallel' or 'gla', got {kind!r}")
+        l, r, la, ra = _section(m, "left", ma), _section(m, "right", ma), ma + ".left", ma + ".right"
+        mask = l.get("mask")
+        left = WindowAttentionConfig(
+            heads=_whole(l, "heads", la), kv_heads=_whole(l, "kv_heads", la), dim=_whole(l, "dim", la), vdim=_whole(l, "vdim", la),
+            scale=_require(l, "scale", float, la), window=None if mask is None else _whole(mask, "size", la + ".mask"))
+        right = MatrixMemoryConfig(heads=_whole(r, "heads", ra), dim=_whole(r, "dim", ra), vdim=_whole(r, "vdim", ra),
+                                   gate_cap=_require(r, "gate_cap", float, ra))
+        scales = {k: 1.0 if m.get(k) is None else _require(m, k, float, ma) for k in ("left_scale", "right_scale")}
+        return PairMixerConfig(left, right, **scales)
+
+    @staticmethod
+    def _mlp(mlp, fa: str):
+        if mlp is None:
+            return None
+        if not isinstance(mlp, Mapping) or mlp.get("kind") not in ("dense", "moe"):
+            raise ConfigError(f"{fa} must be null or an object of kind 'dense' or 'moe', got {mlp!r}")
+        if mlp["kind"] == "dense":
+            return _whole(mlp, "ff", fa)
+        router, shared = _section(mlp, "router", fa), mlp.get("shared")
+        return SoftmaxScoreExpertsConfig(
+            experts=_whole(router, "experts", fa + ".router"), top=_whole(router, "top", fa + ".router"),
+            ff=_whole(_section(mlp, "expert", fa), "ff", fa + ".expert"),
+            scale=1.0 if router.get("scale") is None else _require(router, "scale", float, fa + ".router"),
+            shared_ff=None if shared is None else _whole(shared, "ff", fa + ".shared"))
+
+    @classmethod
+    def from_dict(cls, d: Mapping[str, Any]) -> "NemidraConfig":
+        where = "config.json"
+        entries = d.get("layers")
+        if not isinstance(entries, (list, tuple)) or not entries:
+            raise ConfigError(f"{where}: key 'layers' must be a list of layers")
+        layers = []
+        for i, entry in enumerate(entries):
+            at = f"{where}: layers[{i}]"
+            if not isinstance(entry, Mapping):
+                raise ConfigError(f"{at} must be an object")
+            kind = entry.get("type")
+            layers.append(NemidraLayer(kind, cls._mixer(kind, _section(entry, "mixer", at), at + ".mixer"),
+                                       cls._mlp(entry.get("mlp"), at + ".mlp")))
+        bigram = (d.get("embedding") or {}).get("bigram")
+        if bigram is not None:
+            ba = where + ": embedding.bigram"
+            bigram = BigramConfig(buckets=_whole(bigram, "buckets", ba), mul_prev=_count(bigram, "mul_prev", ba),
+                                  mul_cur=_count(bigram, "mul_cur", ba))
+        loop, side = d.get("loop"), d.get("token_side")
+        turns = (0, len(layers), 1)
+        if loop is not None:
+            turns = (_count(loop, "start", where + ": loop"), _whole(loop, "stop", where + ": loop"),
+                     _whole(loop, "times", where + ": loop"))
+        eos = d.get("eos_token_id")
+        eos = (eos,) if isinstance(eos, int) else tuple(int(x) for x in eos) if isinstance(eos, (list, tuple)) else None
+        cfg = cls(vocab=_whole(d, "vocab", where), width=_whole(d, "width", where),
+                  eps=_require(_section(d, "norm", where), "eps", float, where + ": norm"), layers=tuple(layers),
+                  max_positions=_whole(d, "max_positions", where),
+                  side_dim=None if side is None else _whole(side, "dim", where + ": token_side"), bigram=bigram, loop=turns,
+                  logit_softcap=None if d.get("logit_softcap") is None else _require(d, "logit_softcap", float, where),
+                  dtype=canonical_dtype(d.get("dtype") or d.get("torch_dtype") or "bfloat16"), eos_token_id=eos,
+                  architecture=d.get("architecture") or (d.get("architectures") or ["Nemidra"])[0])
+        cfg.validate()
+        return cfg
+
+    def validate(self) -> None:
+        if not (self.eps > 0):
+            raise ConfigError(f"config.json: norm.eps must be positive, got {self.eps}")
+        start, stop, times = self.loop
+        if not 0 <= start < stop <= len(self.layers) or times < 1:
+            raise ConfigError(f"config.json: a loop over layers {start} .. {stop - 1}, {times} times; there are {len(self.layers)}")
+        if self.logit_softcap is not None and not (self.logit_softcap > 0):
+            raise ConfigError(f"config.json: logit_softcap must be positive, got {self.logit_softcap}")
+        for i, layer in enumerate(self.layers):
+            at = f"config.json: layers[{i}]"
+            m, f = layer.mixer, layer.mlp
+            if layer.kind == "parallel":
+                if m.left.heads % m.left.kv_heads:
+                    raise ConfigError(f"{at}: {m.left.heads} heads do not divide into {m.left.kv_heads} kv_heads")
+                if not (m.left.scale > 0 and m.right.gate_cap > 0):
+                    raise ConfigError(f"{at}: scale and gate_cap must be positive, got {m.left.scale} and {m.right.gate_cap}")
+            elif not (m.tau > 0):
+                raise ConfigError(f"{at}: tau must be positive, got {m.tau}")
+            if isinstance(f, SoftmaxScoreExpertsConfig) and f.top > f.experts:
+                raise ConfigError(f"{at}: {f.top} experts a token out of {f.experts}")
+
+    def to_dict(self) -> dict:
+        """The config.json that describes this configuration."""
+        entries = []
+        for layer in self.layers:
+            m, f = layer.mixer, layer.mlp
+            if layer.kind == "parallel":
+                l, r = m.left, m.right
+                left = {"heads": l.heads, "kv_heads": l.kv_heads, "dim": l.dim, "vdim": l.vdim, "scale": l.scale}
+                if l.window is not None:
+                    left["mask"] = {"size": l.window}
+                mixer = {"left": left, "left_scale": m.left_scale, "right": asdict(r), "right_scale": m.right_scale}
+            else:
+                mixer = {k: v for k, v in asdict(m).items() if v is not None}
+            if f is None:
+                mlp = None
+            elif isinstance(f, int):
+                mlp = {"kind": "dense", "ff": f}
+            else:
+                mlp = {"kind": "moe", "expert": {"ff": f.ff}, "router": {"experts": f.experts, "top": f.top, "scale": f.scale}}
+                if f.shared_ff is not None:
+                    mlp["shared"] = {"ff": f.shared_ff}
+            entries.append({"type": layer.kind, "mixer": mixer, "mlp": mlp})
+        out = {"architecture": self.architecture, "vocab": self.vocab, "width": self.width, "norm": {"eps": self.eps},
+               "max_positions": self.max_positions, "loop": dict(zip(("start", "stop", "times"), self.loop)), "layers": entries,
+               "torch_dtype": self.dtype}
+        if self.bigram is not None:
+            out["embedding"] = {"bigram": asdict(self.bigram)}
+        if self.side_dim is not None:
+            out["token_side"] = {"dim": self.side_dim}
+        if self.logit_softcap is not None:
+            out["logit_softcap"] = self.logit_softcap
+        if self.eos_token_id is not None:
+            out["eos_token_id"] = list(self.eos_token_id)
+        return out

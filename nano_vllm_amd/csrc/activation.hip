@@ -81,7 +81,7 @@ NVA_EXPORT int NVA_NAME(nva_silu_mul)(const void* x, int64_t x_stride, void* out
     return launch_act_mul<NVA_ACT_SILU>(x, x_stride, out, out_stride, rows, inner, stream);
 }
 
-// An activation without a gate: out[t, i] = act(x[t, i]); act by the codes of nva_gate_act (3: relu squared).
+// An activation without a gate: out[t, i] = act(x[t, i]); act by the codes of nva_plain_act.
 // Eight entries a thread where rows and pointers allow.
 template <typename T>
 __global__ void __launch_bounds__(256)
@@ -93,7 +93,7 @@ act8_kernel(const T* __restrict__ x, int64_t x_stride, T* __restrict__ out, int6
     float v[8];
     load8(x + r * x_stride + i, v);
 #pragma unroll
-    for (int e = 0; e < 8; ++e) v[e] = nva_gate_act(act, v[e]);
+    for (int e = 0; e < 8; ++e) v[e] = nva_plain_act(act, v[e]);
     store8(out + r * out_stride + i, v);
 }
 
@@ -104,7 +104,7 @@ act_of_partials_kernel(PartialInput part, T* __restrict__ out, int64_t out_strid
     const int64_t r = blockIdx.y;
     const int i = blockIdx.x * blockDim.x + threadIdx.x;
     if (i >= width) return;
-    out[r * out_stride + i] = from_float<T>(nva_gate_act(act, partial_value<T>(part, r, width, i)));
+    out[r * out_stride + i] = from_float<T>(nva_plain_act(act, partial_value<T>(part, r, width, i)));
 }
 
 template <typename T>
@@ -114,13 +114,13 @@ act_kernel(const T* __restrict__ x, int64_t x_stride, T* __restrict__ out, int64
     if (idx >= rows * width) return;
     const int64_t r = idx / width;
     const int i = (int)(idx % width);
-    out[r * out_stride + i] = from_float<T>(nva_gate_act(act, to_float(x[r * x_stride + i])));
+    out[r * out_stride + i] = from_float<T>(nva_plain_act(act, to_float(x[r * x_stride + i])));
 }
 
 NVA_EXPORT int NVA_NAME(nva_act)(const void* x, int64_t x_stride, void* out, int64_t out_stride, int64_t rows, int width,
                                  int act, hipStream_t stream) {
     if (rows == 0) return 0;
-    if (rows < 0 || width <= 0 || act < 0 || act > 3) return nva_fail("act: bad shape rows=%lld width=%d or activation %d", (long long)rows, width, act);
+    if (rows < 0 || width <= 0 || act < 0 || act > 4) return nva_fail("act: bad shape rows=%lld width=%d or activation %d", (long long)rows, width, act);
     const int64_t total = rows * width;
     if ((total + 255) / 256 > 0x7fffffff) return nva_fail("act: too many entries");
     const size_t vb = 8 * sizeof(elem_t);
@@ -138,13 +138,51 @@ NVA_EXPORT int NVA_NAME(nva_act)(const void* x, int64_t x_stride, void* out, int
 NVA_EXPORT int NVA_NAME(nva_act_of_partials)(const float* sums, int splits, int64_t split_stride, const void* bias, void* out,
                                              int64_t out_stride, int64_t rows, int width, int act, hipStream_t stream) {
     if (rows == 0) return 0;
-    if (rows < 0 || rows > 65535 || width <= 0 || act < 0 || act > 3 || !sums || splits <= 0 || split_stride < rows * (int64_t)width ||
+    if (rows < 0 || rows > 65535 || width <= 0 || act < 0 || act > 4 || !sums || splits <= 0 || split_stride < rows * (int64_t)width ||
         !out || out_stride < width)
         return nva_fail("act_of_partials: bad shape rows=%lld width=%d splits=%d or activation %d", (long long)rows, width, splits, act);
     const PartialInput part{sums, splits, split_stride, bias};
     hipLaunchKernelGGL((act_of_partials_kernel<elem_t>), dim3((width + 255) / 256, (unsigned)rows), dim3(256), 0, stream, part,
                        (elem_t*)out, out_stride, width, act);
     return nva_check_launch("act_of_partials");
+}
+
+// The same times a row of a table: out[t, i] = act(x[t, i]) * table[ids[t], offset + i], in float, rounded once.  x comes as
+// elements or as a product's partial sums.  An id outside the table sets bit 0 of the flag and gives zeros.
+template <typename T>
+__global__ void __launch_bounds__(256)
+act_mul_rows_kernel(const T* __restrict__ x, int64_t x_stride, PartialInput part, const T* __restrict__ table, int64_t table_stride,
+                    int64_t table_rows, int offset, const int32_t* __restrict__ ids, T* __restrict__ out, int64_t out_stride,
+                    int64_t rows, int width, int act, int32_t* error_flag) {
+    const int64_t idx = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
+    if (idx >= rows * width) return;
+    const int64_t r = idx / width;
+    const int i = (int)(idx % width);
+    const int id = ids[r];
+    const bool ok = id >= 0 && id < table_rows;
+    if (!ok && i == 0 && error_flag) atomicOr(error_flag, 1);
+    const float e = ok ? to_float(table[(int64_t)id * table_stride + offset + i]) : 0.f;
+    const float v = part.sums ? partial_value<T>(part, r, width, i) : to_float(x[r * x_stride + i]);
+    out[r * out_stride + i] = from_float<T>(nva_plain_act(act, v) * e);
+}
+
+// x: elements [rows, width], or (sums) partial sums [splits][rows][width] with an optional bias.
+NVA_EXPORT int NVA_NAME(nva_act_mul_rows)(const void* x, int64_t x_stride, const float* sums, int splits, int64_t split_stride,
+                                          const void* bias, const void* table, int64_t table_stride, int64_t table_rows, int offset,
+                                          const int32_t* ids, void* out, int64_t out_stride, int64_t rows, int width, int act,
+                                          int32_t* error_flag, hipStream_t stream) {
+    if (rows == 0) return 0;
+    if (rows < 0 || width <= 0 || act < 0 || act > 4 || (!x && !sums) || !table || !ids || !out || table_rows <= 0 || offset < 0 ||
+        table_stride < (int64_t)offset + width || out_stride < width)
+        return nva_fail("act_mul_rows: bad shape rows=%lld width=%d offset=%d or activation %d", (long long)rows, width, offset, act);
+    if (sums && (splits <= 0 || split_stride < rows * (int64_t)width)) return nva_fail("act_mul_rows: bad partial sums");
+    const int64_t total = rows * width;
+    if ((total + 255) / 256 > 0x7fffffff) return nva_fail("act_mul_rows: too many entries");
+    const PartialInput part{sums, splits, split_stride, bias};
+    hipLaunchKernelGGL((act_mul_rows_kernel<elem_t>), dim3((unsigned)((total + 255) / 256)), dim3(256), 0, stream, (const elem_t*)x,
+                       x_stride, part, (const elem_t*)table, table_stride, table_rows, offset, ids, (elem_t*)out, out_stride, rows,
+                       width, act, error_flag);
+    return nva_check_launch("act_mul_rows");
 }
 
 // A gate on finished outputs: out[t, i] = x[t, i] * sigmoid(g[t, i]), in float, rounded once (out may be x).

@@ -141,6 +141,12 @@ __device__ __forceinline__ float nva_gate_act(int act, float g) {
     return g / (1.f + nva_exp(-g));
 }
 
+// An activation without a gate: the same codes, and 4 gelu in its exact form, g (1 + erf(g / sqrt 2)) / 2.
+__device__ __forceinline__ float nva_plain_act(int act, float g) {
+    if (act == 4) return 0.5f * g * (1.f + erff(g * 0.7071067811865476f));
+    return nva_gate_act(act, g);
+}
+
 // ---------------------------------------------------------------------------- split products
 // A product whose k range was split over workgroups leaves float partial sums
 // [splits][rows][width] (gemm_skinny.hip).  Kernels that consume such a product add the partials

@@ -60,6 +60,113 @@ NVA_EXPORT int NVA_NAME(nva_scale_rows)(float* x, int64_t stride, int64_t rows, 
     return nva_check_launch("scale_rows");
 }
 
+// x <- cap * tanh(x / cap) over a float tensor of rows `stride` apart (logits capped smoothly), four entries a thread where
+// rows and pointer allow.
+__global__ void __launch_bounds__(256) softcap_rows_kernel(float* __restrict__ x, int64_t stride, int64_t rows, int width, float cap,
+                                                           float inv) {
+    const int64_t idx = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
+    if (idx >= rows * width) return;
+    float* p = x + (idx / width) * stride + idx % width;
+    *p = cap * tanhf(*p * inv);
+}
+__global__ void __launch_bounds__(256) softcap_rows4_kernel(float* __restrict__ x, int64_t stride, int64_t rows, int width4, float cap,
+                                                            float inv) {
+    const int64_t idx = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
+    if (idx >= rows * width4) return;
+    float4* p = reinterpret_cast<float4*>(x + (idx / width4) * stride) + idx % width4;
+    float4 v = *p;
+    v.x = cap * tanhf(v.x * inv); v.y = cap * tanhf(v.y * inv);
+    v.z = cap * tanhf(v.z * inv); v.w = cap * tanhf(v.w * inv);
+    *p = v;
+}
+
+NVA_EXPORT int NVA_NAME(nva_softcap_rows)(float* x, int64_t stride, int64_t rows, int width, float cap, hipStream_t stream) {
+    if (rows == 0) return 0;
+    if (rows < 0 || width <= 0 || stride < width || !x || !(cap > 0.f)) return nva_fail("softcap_rows: bad arguments");
+    const bool four = width % 4 == 0 && stride % 4 == 0 && nva_aligned(x, 16);
+    const int64_t total = rows * (four ? width / 4 : width);
+    if ((total + 255) / 256 > 0x7fffffff) return nva_fail("softcap_rows: too many entries");
+    const dim3 grid((unsigned)((total + 255) / 256));
+    if (four) hipLaunchKernelGGL(softcap_rows4_kernel, grid, dim3(256), 0, stream, x, stride, rows, width / 4, cap, 1.f / cap);
+    else hipLaunchKernelGGL(softcap_rows_kernel, grid, dim3(256), 0, stream, x, stride, rows, width, cap, 1.f / cap);
+    return nva_check_launch("softcap_rows");
+}
+
+// A float stream as a sum of learned rows:
+//     out[t] = table[ids[t]] + bigram[row] + positions[p_t]            all sums float; bigram and positions may be absent
+//     row = (before * mul_prev + ids[t] * mul_cur) mod buckets, before = the token before this one in its sequence, or
+//     row = buckets for a sequence's first token.
+// A portion's first token finds the token before it in before_state[slot], where the same workgroup, the only one that
+// looks at that place in this step, then leaves the portion's last token.  One workgroup a token.
+template <typename T>
+__global__ void __launch_bounds__(256)
+summed_embedding_kernel(const T* __restrict__ table, int64_t table_rows, const T* __restrict__ bigram, int64_t buckets, int64_t mul_prev,
+                        int64_t mul_cur, const T* __restrict__ pos_table, int64_t pos_rows, const int32_t* __restrict__ ids,
+                        const int32_t* __restrict__ positions, const int32_t* __restrict__ token_seq,
+                        const int32_t* __restrict__ cu_seqlens_q, const int32_t* __restrict__ seq_starts,
+                        const int32_t* __restrict__ state_slots, int32_t* before_state, float* __restrict__ out, int width,
+                        int32_t* error_flag) {
+    const int64_t t = blockIdx.x;
+    const int id = ids[t], p = positions[t];
+    const bool ok = id >= 0 && id < table_rows && (!pos_table || (p >= 0 && p < pos_rows));
+    if (!ok && threadIdx.x == 0 && error_flag) atomicOr(error_flag, 1);
+    const T* brow = nullptr;
+    if (bigram) {
+        const int s = token_seq[t];
+        const int64_t first = cu_seqlens_q[s];
+        int64_t row = buckets;
+        if (t > first || seq_starts[s] > 0) {
+            const int64_t before = t > first ? ids[t - 1] : before_state[state_slots[s]];
+            row = (max(before, (int64_t)0) * mul_prev + (int64_t)max(id, 0) * mul_cur) % buckets;
+        }
+        if (t == first) {
+            __syncthreads();                             // (every thread has read the token before)
+            if (threadIdx.x == 0) before_state[state_slots[s]] = ids[cu_seqlens_q[s + 1] - 1];
+        }
+        brow = bigram + row * width;
+    }
+    const T* erow = table + (int64_t)(ok ? id : 0) * width;
+    const T* prow = pos_table ? pos_table + (int64_t)(ok ? p : 0) * width : nullptr;
+    for (int i = threadIdx.x; i < width; i += blockDim.x) {
+        float v = to_float(erow[i]);
+        if (brow) v += to_float(brow[i]);
+        if (prow) v += to_float(prow[i]);
+        out[t * width + i] = ok ? v : 0.f;
+    }
+}
+
+NVA_EXPORT int NVA_NAME(nva_summed_embedding)(const void* table, int64_t table_rows, const void* bigram, int64_t buckets,
+                                              int64_t mul_prev, int64_t mul_cur, const void* pos_table, int64_t pos_rows,
+                                              const int32_t* ids, const int32_t* positions, const int32_t* token_seq,
+                                              const int32_t* cu_seqlens_q, const int32_t* seq_starts, const int32_t* state_slots,
+                                              int32_t* before_state, float* out, int64_t tokens, int width, int32_t* error_flag,
+                                              hipStream_t stream) {
+    if (tokens == 0) return 0;
+    if (tokens < 0 || tokens > 0x7fffffff || width <= 0 || table_rows <= 0 || !table || !ids || !out || !positions)
+        return nva_fail("summed_embedding: bad shape tokens=%lld width=%d rows=%lld", (long long)tokens, width, (long long)table_rows);
+    if (bigram && (buckets <= 0 || mul_prev < 0 || mul_cur < 0 || mul_prev > 0x7fffffff || mul_cur > 0x7fffffff || !token_seq ||
+                   !cu_seqlens_q || !seq_starts || !state_slots || !before_state))
+        return nva_fail("summed_embedding: a bigram table needs its constants, the step's requests and their state");
+    if (pos_table && pos_rows <= 0) return nva_fail("summed_embedding: an empty table of positions");
+    const int threads = width >= 1024 ? 256 : (width >= 256 ? 128 : 64);
+    hipLaunchKernelGGL(summed_embedding_kernel<elem_t>, dim3((unsigned)tokens), dim3(threads), 0, stream, (const elem_t*)table,
+                       table_rows, (const elem_t*)bigram, buckets, mul_prev, mul_cur, (const elem_t*)pos_table, pos_rows, ids,
+                       positions, token_seq, cu_seqlens_q, seq_starts, state_slots, before_state, out, width, error_flag);
+    return nva_check_launch("summed_embedding");
+}
+
+// out[r] = x[r] over a float tensor of contiguous rows: a second copy of a stream that is updated in place.
+__global__ void __launch_bounds__(256) copy_rows_kernel(const float* __restrict__ x, float* __restrict__ out, int64_t total) {
+    for (int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x; i < total; i += (int64_t)gridDim.x * blockDim.x) out[i] = x[i];
+}
+NVA_EXPORT int NVA_NAME(nva_copy_rows)(const float* x, float* out, int64_t total, hipStream_t stream) {
+    if (total == 0) return 0;
+    if (total < 0 || !x || !out) return nva_fail("copy_rows: bad arguments");
+    const int64_t blocks = (total + 255) / 256;
+    hipLaunchKernelGGL(copy_rows_kernel, dim3((unsigned)(blocks < 65536 ? blocks : 65536)), dim3(256), 0, stream, x, out, total);
+    return nva_check_launch("copy_rows");
+}
+
 // out[t] = float(table[ids[t]]) * factor: the start of a residual stream kept in float (an embedding with a
 // scale).  An id outside the table sets bit 0 of the flag and gives zeros.
 template <typename T>

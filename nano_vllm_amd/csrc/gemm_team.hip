@@ -159,7 +159,7 @@ linear_team_kernel(const TeamArgs a) {
                 if (a.bias) val += (float)a.bias[n + i];
                 if (a.mode == TM_PLAIN_F32) ((float*)a.y)[(int64_t)m * a.y_stride + n + i] = val;
                 // (an activation works on the rounded product, as a pass of its own would)
-                else if (a.act >= 0) ((__bf16*)a.y)[(int64_t)m * a.y_stride + n + i] = (__bf16)nva_gate_act(a.act, round_through<__bf16>(val));
+                else if (a.act >= 0) ((__bf16*)a.y)[(int64_t)m * a.y_stride + n + i] = (__bf16)nva_plain_act(a.act, round_through<__bf16>(val));
                 else ((__bf16*)a.y)[(int64_t)m * a.y_stride + n + i] = (__bf16)val;
             }
         }
@@ -168,7 +168,7 @@ linear_team_kernel(const TeamArgs a) {
 }
 
 // y = x W^T (+ bias) for 1..16 rows of x.  mode: 0 elements, 1 float, 2 SwiGLU gating of W = [gate
-// rows; up rows] (y [M, N / 2], no bias), 5 to 8 elements through an activation.  teams: the number of workgroups to aim for (the CUs of the
+// rows; up rows] (y [M, N / 2], no bias), 5 to 9 elements through an activation.  teams: the number of workgroups to aim for (the CUs of the
 // GPU); every team takes ceil(blocks / teams) blocks of 16 rows of W.  Returns 1 for shapes this
 // kernel does not take: more than 16 rows, K not a multiple of 32.
 NVA_EXPORT int nva_linear_team_bf16(const void* x, int64_t x_stride, const void* w, int64_t w_stride, const void* bias,
@@ -181,8 +181,8 @@ NVA_EXPORT int nva_linear_team_bf16(const void* x, int64_t x_stride, const void*
     }
     if (teams <= 0 || !x || !w || !y || x_stride % 8 || w_stride % 8 || !nva_aligned(x, 16) || !nva_aligned(w, 16))
         return nva_fail("linear_team: x and W need 16-byte aligned rows, and an output");
-    // modes 2, 3, 4: the gated form with silu, relu, gelu (tanh); 5 to 8: elements, with an activation (nva_gate_act's codes)
-    if (mode < 0 || mode > 8) return nva_fail("linear_team: unknown mode %d", mode);
+    // modes 2, 3, 4: the gated form with silu, relu, gelu (tanh); 5 to 9: elements, with an activation (nva_plain_act's codes)
+    if (mode < 0 || mode > 9) return nva_fail("linear_team: unknown mode %d", mode);
     const int act = mode >= 5 ? mode - 5 : mode >= TM_GATED ? mode - TM_GATED : -1;
     if (mode >= 5) mode = TM_PLAIN;
     else if (mode > TM_GATED) mode = TM_GATED;

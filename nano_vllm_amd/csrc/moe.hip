@@ -13,6 +13,7 @@
 //             expert), a group counts by the largest such choice score in it, only the kept groups' experts can be
 //             chosen (the others do not take part, whatever the sign of the scores); the weights are the chosen
 //             experts' s (without the bias) divided by their sum + 1e-20.
+//             With softmax_scores (mode 3) s = softmax(z) over all experts, chosen by s, weights scale * s, not over their sum.
 //             Experts numbered from `experts` on (the kernels of the products are told how many real ones there are)
 //             are identities: their output is the token's input itself.
 //   plan      the pairs (token, choice) counted and sorted by expert: place[pair] = the pair's row among the
@@ -58,7 +59,7 @@ moe_route_kernel(const float* __restrict__ logits, int64_t stride, int experts, 
     const int64_t t = blockIdx.x;
     const int lane = threadIdx.x;
     const bool all_groups = group_keep == group_count;
-    const bool choice = softmax_top == 2;
+    const bool choice = softmax_top >= 2;            // compared by the softmax over all experts
     if (choice) {
         float m = -INFINITY;
         for (int e = lane; e < experts; e += NVA_WAVE) m = fmaxf(m, logits[t * stride + e]);
@@ -115,18 +116,18 @@ moe_route_kernel(const float* __restrict__ logits, int64_t stride, int experts, 
         if (lane == 0) {
             open_s[best] = 0;
             ids[t * top + k] = best;
-            weights[t * top + k] = choice ? w_s[best] : softmax_top ? v : scale * v;
+            weights[t * top + k] = softmax_top == 2 ? w_s[best] : softmax_top == 1 ? v : scale * v;
         }
         __syncthreads();
     }
-    if (choice) {
+    if (softmax_top == 2) {
         if (lane == 0) {
             float sum = 0.f;
             for (int k = 0; k < top; ++k) sum += weights[t * top + k];
             sum += 1e-20f;
             for (int k = 0; k < top; ++k) weights[t * top + k] /= sum;
         }
-    } else if (softmax_top && lane == 0) {
+    } else if (softmax_top == 1 && lane == 0) {
         // the chosen logits, largest first: their softmax among themselves, summed in the order of the choice
         const float m = weights[t * top];
         float sum = 0.f;
@@ -391,7 +392,7 @@ NVA_EXPORT int NVA_NAME(nva_moe_route)(const float* logits, int64_t stride, int6
     if (tokens < 0 || tokens > 0x7fffffff || experts <= 0 || experts > MOE_MAX_EXPERTS)
         return nva_fail("moe_route: bad counts tokens=%lld experts=%d (up to %d)", (long long)tokens, experts, MOE_MAX_EXPERTS);
     if (group_count <= 0 || experts % group_count || group_keep <= 0 || group_keep > group_count || top <= 0 ||
-        top > group_keep * (experts / group_count) || softmax_top < 0 || softmax_top > 2)
+        top > group_keep * (experts / group_count) || softmax_top < 0 || softmax_top > 3)
         return nva_fail("moe_route: %d of %d experts in %d groups of which %d stay", top, experts, group_count, group_keep);
     if (!logits || !ids || !weights || stride < experts) return nva_fail("moe_route: a tensor is missing");
     hipLaunchKernelGGL(moe_route_kernel, dim3((unsigned)tokens), dim3(NVA_WAVE), 0, stream, logits, stride, experts, top,

@@ -326,51 +326,81 @@ NVA_EXPORT int NVA_NAME(nva_stream_scaled_norm)(const void* a, int64_t a_stride,
 // ---------------------------------------------------------------------------- a normed addend into the float stream
 // A sublayer's output enters the stream through a norm of its own and a constant, and the stream is normed
 // for the next sublayer, all in one pass over the row:
-//     u = a / sqrt(mean(a^2) + eps_a) * wa            a elements, or a split product's partial sums
-//     r <- r + mult * u
-//     y = r / sqrt(mean(r^2) + eps) * w               rounded once, to the element type
+//     u = a / sqrt(mean(a^2) + eps_a) * (off_a + wa)  a elements, or a split product's partial sums; PAIR: sa * a + sb * b
+//     r <- r + mult * u (+ extra)                     extra: float rows, or none
+//     y = r / sqrt(mean(r^2) + eps) * (off + w)       rounded once, to the element type; without w: y = r, rounded
 // All arithmetic in float; r float, in place.  One workgroup a row, which keeps its entries between the sums.
 // A thread keeps KEEP entries of the row between the passes, and everything it needs of them (addend, stream, both weights)
 // is asked for before the first sum; rows of more than KEEP entries a thread read the rest again.
+struct PostNormArgs {
+    const void* a; int64_t a_stride; PartialInput pa; float sa;
+    const void* b; int64_t b_stride; PartialInput pb; float sb;
+    const void* a_weight; int aw_is_f32; float a_off, a_eps, mult;
+    const float* extra; int64_t extra_stride;
+    float* residual; int64_t r_stride;
+    const void* weight; int w_is_f32; float off, eps;
+    void* y; int64_t y_stride; int width;
+};
+
+// KEEP entries of a row (the columns at[]) from elements or from the splits' sums, which are asked for side by side and
+// each added up in the order of the splits.
 template <typename T, int KEEP>
+__device__ __forceinline__ void post_norm_entries(const T* x, int64_t stride, const PartialInput& p, int64_t row, int width,
+                                                  const int (&at)[KEEP], float (&v)[KEEP]) {
+#pragma unroll
+    for (int n = 0; n < KEEP; ++n) v[n] = p.sums ? 0.f : to_float(x[row * stride + at[n]]);
+    if (!p.sums) return;
+    const float* q = p.sums + row * width;
+#pragma unroll 8
+    for (int s = 0; s < p.splits; ++s)
+#pragma unroll
+        for (int n = 0; n < KEEP; ++n) v[n] += q[s * p.split_stride + at[n]];
+#pragma unroll
+    for (int n = 0; n < KEEP; ++n) {
+        if (p.bias) v[n] += to_float(static_cast<const T*>(p.bias)[at[n]]);
+        v[n] = round_through<T>(v[n]);
+    }
+}
+
+template <typename T, int KEEP, bool PAIR>
 __global__ void __launch_bounds__(1024)
-stream_post_norm_kernel(const T* __restrict__ a, int64_t a_stride, PartialInput pa, const void* __restrict__ a_weight,
-                        int aw_is_f32, float a_eps, float mult, float* residual, int64_t r_stride,
-                        const void* __restrict__ weight, int w_is_f32, T* __restrict__ y, int64_t y_stride, int width,
-                        float eps) {
+stream_post_norm_kernel(const PostNormArgs g) {
     __shared__ float scratch[16];
     const int64_t row = blockIdx.x;
-    const T* ar = a ? a + row * a_stride : nullptr;
-    float* rr = residual + row * r_stride;
-    T* yr = y + row * y_stride;
+    const int width = g.width;
+    const T* a = static_cast<const T*>(g.a);
+    const T* b = static_cast<const T*>(g.b);
+    float* rr = g.residual + row * g.r_stride;
+    const float* xr = g.extra ? g.extra + row * g.extra_stride : nullptr;
+    T* yr = static_cast<T*>(g.y) + row * g.y_stride;
     const int step = blockDim.x, tid = threadIdx.x;
     auto vec = [](const void* v, int is_f32, int i) -> float {
         return is_f32 ? static_cast<const float*>(v)[i] : to_float(static_cast<const T*>(v)[i]);
+    };
+    auto addend = [&](int i) -> float {                      // an entry beyond those that are kept
+        float v = g.pa.sums ? partial_value<T>(g.pa, row, width, i) : to_float(a[row * g.a_stride + i]);
+        if (PAIR) v = g.sa * v + g.sb * (g.pb.sums ? partial_value<T>(g.pb, row, width, i) : to_float(b[row * g.b_stride + i]));
+        return v;
     };
     float kept[KEEP], r_k[KEEP], wa_k[KEEP], w_k[KEEP];
     int at[KEEP];
 #pragma unroll
     for (int n = 0; n < KEEP; ++n) {
         at[n] = min(tid + n * step, width - 1);           // (every load unconditional; an entry outside the row counts as zero)
-        kept[n] = 0.f;
-        if (!pa.sums) kept[n] = to_float(ar[at[n]]);
         r_k[n] = rr[at[n]];
-        wa_k[n] = vec(a_weight, aw_is_f32, at[n]);
-        w_k[n] = vec(weight, w_is_f32, at[n]);
+        wa_k[n] = g.a_off + vec(g.a_weight, g.aw_is_f32, at[n]);
+        w_k[n] = g.weight ? g.off + vec(g.weight, g.w_is_f32, at[n]) : 1.f;
     }
-    if (pa.sums) {
-        // the splits' sums of all kept entries side by side, each in the order of the splits
-        const float* q = pa.sums + row * width;
-#pragma unroll 8
-        for (int s = 0; s < pa.splits; ++s)
+    post_norm_entries<T, KEEP>(a, g.a_stride, g.pa, row, width, at, kept);
+    if (PAIR) {
+        float other[KEEP];
+        post_norm_entries<T, KEEP>(b, g.b_stride, g.pb, row, width, at, other);
 #pragma unroll
-            for (int n = 0; n < KEEP; ++n) kept[n] += q[s * pa.split_stride + at[n]];
-#pragma unroll
-        for (int n = 0; n < KEEP; ++n) {
-            if (pa.bias) kept[n] += to_float(static_cast<const T*>(pa.bias)[at[n]]);
-            kept[n] = round_through<T>(kept[n]);
-        }
+        for (int n = 0; n < KEEP; ++n) kept[n] = g.sa * kept[n] + g.sb * other[n];
     }
+    if (xr)
+#pragma unroll
+        for (int n = 0; n < KEEP; ++n) r_k[n] += xr[at[n]];
     float ss = 0.f;
 #pragma unroll
     for (int n = 0; n < KEEP; ++n) {
@@ -378,11 +408,11 @@ stream_post_norm_kernel(const T* __restrict__ a, int64_t a_stride, PartialInput 
         ss += kept[n] * kept[n];
     }
     for (int i = tid + KEEP * step; i < width; i += step) {
-        const float v = pa.sums ? partial_value<T>(pa, row, width, i) : to_float(ar[i]);
+        const float v = addend(i);
         ss += v * v;
     }
     ss = block_sum(ss, scratch);
-    const float a_scale = rsqrtf(ss / (float)width + a_eps) * mult;
+    const float a_scale = rsqrtf(ss / (float)width + g.a_eps) * g.mult;
     float ss2 = 0.f;
 #pragma unroll
     for (int n = 0; n < KEEP; ++n) {
@@ -392,44 +422,83 @@ stream_post_norm_kernel(const T* __restrict__ a, int64_t a_stride, PartialInput 
         ss2 += kept[n] * kept[n];                                     // (entries outside the row are zero)
     }
     for (int i = tid + KEEP * step; i < width; i += step) {
-        const float v = pa.sums ? partial_value<T>(pa, row, width, i) : to_float(ar[i]);
-        const float s = rr[i] + v * a_scale * vec(a_weight, aw_is_f32, i);
+        const float s = rr[i] + (xr ? xr[i] : 0.f) + addend(i) * a_scale * (g.a_off + vec(g.a_weight, g.aw_is_f32, i));
         rr[i] = s;
         ss2 += s * s;
     }
-    ss2 = block_sum(ss2, scratch);
-    const float scale = rsqrtf(ss2 / (float)width + eps);
+    float scale = 1.f;
+    if (g.weight) {
+        ss2 = block_sum(ss2, scratch);
+        scale = rsqrtf(ss2 / (float)width + g.eps);
+    }
 #pragma unroll
     for (int n = 0; n < KEEP; ++n) {
         const int i = tid + n * step;
         if (i < width) yr[i] = from_float<T>(kept[n] * scale * w_k[n]);
     }
-    for (int i = tid + KEEP * step; i < width; i += step) yr[i] = from_float<T>(rr[i] * scale * vec(weight, w_is_f32, i));
+    for (int i = tid + KEEP * step; i < width; i += step)
+        yr[i] = from_float<T>(rr[i] * scale * (g.weight ? g.off + vec(g.weight, g.w_is_f32, i) : 1.f));
 }
 
-// a: elements [rows, width], or (a_sums) partial sums [splits][rows][width] with an optional bias.
+// a: elements [rows, width], or (a_sums) partial sums [splits][rows][width] with an optional bias; b (or b_sums) the same: the
+// addend is then a_scale * a + b_scale * b.  extra: float rows or null.  weight null: y is the stream, rounded.
 NVA_EXPORT int NVA_NAME(nva_stream_post_norm)(const void* a, int64_t a_stride, const float* a_sums, int a_splits,
-                                              int64_t a_split_stride, const void* a_bias, const void* a_weight,
-                                              int aw_is_f32, float a_eps, float mult, float* residual, int64_t r_stride,
-                                              const void* weight, int w_is_f32, void* y, int64_t y_stride, int64_t rows,
-                                              int width, float eps, hipStream_t stream) {
+                                              int64_t a_split_stride, const void* a_bias, float a_scale, const void* b,
+                                              int64_t b_stride, const float* b_sums, int b_splits, int64_t b_split_stride,
+                                              const void* b_bias, float b_scale, const void* a_weight, int aw_is_f32, float a_offset,
+                                              float a_eps, float mult, const float* extra, int64_t extra_stride, float* residual,
+                                              int64_t r_stride, const void* weight, int w_is_f32, float offset, void* y,
+                                              int64_t y_stride, int64_t rows, int width, float eps, hipStream_t stream) {
     if (rows == 0) return 0;
     if (rows < 0 || rows > 0x7fffffff || width <= 0)
         return nva_fail("stream_post_norm: bad shape rows=%lld width=%d", (long long)rows, width);
-    if (!residual || !y || !weight || !a_weight || (!a && !a_sums))
-        return nva_fail("stream_post_norm: the addend, its weight, the stream, the weight and the output are needed");
-    if (a_sums && (a_splits <= 0 || a_split_stride < rows * (int64_t)width)) return nva_fail("stream_post_norm: bad partial sums");
-    const PartialInput pa{a_sums, a_splits, a_split_stride, a_bias};
-    const int threads = a_sums && rows <= 64 && width >= 1024 ? 1024
+    if (!residual || !y || !a_weight || (!a && !a_sums))
+        return nva_fail("stream_post_norm: the addend, its weight, the stream and the output are needed");
+    if ((a_sums && (a_splits <= 0 || a_split_stride < rows * (int64_t)width)) ||
+        (b_sums && (b_splits <= 0 || b_split_stride < rows * (int64_t)width)))
+        return nva_fail("stream_post_norm: bad partial sums");
+    const bool pair = b || b_sums;
+    if (!pair && a_scale != 1.f) return nva_fail("stream_post_norm: a scale goes with a second addend");
+    const PostNormArgs g{a, a_stride, {a_sums, a_splits, a_split_stride, a_bias}, a_scale,
+                         b, b_stride, {b_sums, b_splits, b_split_stride, b_bias}, b_scale,
+                         a_weight, aw_is_f32, a_offset, a_eps, mult, extra, extra_stride, residual, r_stride,
+                         weight, w_is_f32, offset, eps, y, y_stride, width};
+    const int threads = (a_sums || b_sums) && rows <= 64 && width >= 1024 ? 1024
                         : width >= 2048 ? 512 : width >= 1024 ? 256 : width >= 256 ? 128 : 64;
     const int per = (width + threads - 1) / threads;
-#define POST_NORM(KK)                                                                                                  \
-    hipLaunchKernelGGL((stream_post_norm_kernel<elem_t, KK>), dim3((unsigned)rows), dim3(threads), 0, stream,              \
-                       (const elem_t*)a, a_stride, pa, a_weight, aw_is_f32, a_eps, mult, residual, r_stride, weight, w_is_f32, \
-                       (elem_t*)y, y_stride, width, eps)
+#define POST_NORM(KK)                                                                                                               do {                                                                                                                                if (pair) hipLaunchKernelGGL((stream_post_norm_kernel<elem_t, KK, true>), dim3((unsigned)rows), dim3(threads), 0, stream, g);         else hipLaunchKernelGGL((stream_post_norm_kernel<elem_t, KK, false>), dim3((unsigned)rows), dim3(threads), 0, stream, g);        } while (0)
     if (per <= 1) POST_NORM(1); else if (per <= 2) POST_NORM(2); else if (per <= 4) POST_NORM(4); else POST_NORM(8);
 #undef POST_NORM
     return nva_check_launch("stream_post_norm");
+}
+
+// y = sa * a + sb * b, in float, rounded once; a, b elements or partial sums.
+template <typename T>
+__global__ void __launch_bounds__(256)
+pair_scaled_sum_kernel(const T* __restrict__ a, int64_t a_stride, PartialInput pa, float sa, const T* __restrict__ b, int64_t b_stride,
+                       PartialInput pb, float sb, T* __restrict__ y, int64_t y_stride, int64_t rows, int width) {
+    const int64_t idx = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
+    if (idx >= rows * width) return;
+    const int64_t row = idx / width;
+    const int i = (int)(idx % width);
+    const float u = pa.sums ? partial_value<T>(pa, row, width, i) : to_float(a[row * a_stride + i]);
+    const float v = pb.sums ? partial_value<T>(pb, row, width, i) : to_float(b[row * b_stride + i]);
+    y[row * y_stride + i] = from_float<T>(sa * u + sb * v);
+}
+
+NVA_EXPORT int NVA_NAME(nva_pair_scaled_sum)(const void* a, int64_t a_stride, const float* a_sums, int a_splits, int64_t a_split_stride,
+                                             const void* a_bias, float sa, const void* b, int64_t b_stride, const float* b_sums,
+                                             int b_splits, int64_t b_split_stride, const void* b_bias, float sb, void* y,
+                                             int64_t y_stride, int64_t rows, int width, hipStream_t stream) {
+    if (rows == 0) return 0;
+    const int64_t total = rows * width;
+    if (rows < 0 || width <= 0 || (total + 255) / 256 > 0x7fffffff)
+        return nva_fail("pair_scaled_sum: bad shape rows=%lld width=%d", (long long)rows, width);
+    if ((!a && !a_sums) || (!b && !b_sums) || !y) return nva_fail("pair_scaled_sum: both inputs and the output are needed");
+    const PartialInput pa{a_sums, a_splits, a_split_stride, a_bias}, pb{b_sums, b_splits, b_split_stride, b_bias};
+    hipLaunchKernelGGL((pair_scaled_sum_kernel<elem_t>), dim3((unsigned)((total + 255) / 256)), dim3(256), 0, stream, (const elem_t*)a,
+                       a_stride, pa, sa, (const elem_t*)b, b_stride, pb, sb, (elem_t*)y, y_stride, rows, width);
+    return nva_check_launch("pair_scaled_sum");
 }
 
 // ---------------------------------------------------------------------------- Dynamic Tanh on the float stream

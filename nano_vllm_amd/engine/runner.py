@@ -78,7 +78,7 @@ class ModelRunner:
         their first occurrence, and replayed from then on.  Reference: capture_cudagraph and
         the replay branch of run_model (nanovllm/engine/model_runner.py:195-212,222-257),
         which captures every size at start-up."""
-        if any(not self.model.blocks[self.model.order[i].layer].replays_state_steps for i in self.state_runs):
+        if any(not self.model.replays_state_steps(i) for i in self.state_runs):
             return          # a mixer that handles its state on the host cannot be replayed blindly
         if max_len > self.model.spec.max_position:
             raise ValueError(f"decode graphs for {max_len} tokens: the model knows {self.model.spec.max_position} positions")

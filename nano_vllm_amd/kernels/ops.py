@@ -105,7 +105,7 @@ class PendingProduct:
 
 
 def _t(x):
-    return x.tensor() if isinstance(x, (SplitSum, PendingProduct)) else x
+    return x.tensor() if isinstance(x, (SplitSum, PendingProduct)) or hasattr(x, "left_scale") else x
 
 
 def check_positions_fit(table: torch.Tensor, head_dim: int, max_position: Optional[int]) -> None:
@@ -383,6 +383,47 @@ class HipKernels:
                      _p(out), c_i64(width), c_i64(n), c_i32(width), c_f32(float(scale)), _p(self.fault_flag), self._stream())
         return out
 
+    def summed_embedding(self, table: torch.Tensor, ids: torch.Tensor, bigram: Optional[torch.Tensor], constants,
+                         positions: Optional[torch.Tensor], before: Optional[torch.Tensor], batch) -> torch.Tensor:
+        """float32 out[t] = table[ids[t]] + bigram[row_t] + positions[p_t]; constants (buckets, mul_prev, mul_cur): row_t = (the
+        token before * mul_prev + ids[t] * mul_cur) mod buckets, or `buckets` for a sequence's first token; before int32
+        [slots, 1] keeps a request's last token from step to step (read and written here).  bigram and positions may be None."""
+        rows, width, stride = _rows2d(table, "embedding table")
+        n = ids.shape[0]
+        _i32(ids, n, "embedding ids")
+        _i32(batch.positions, n, "positions")
+        for t, need in ((bigram, None if bigram is None else constants[0] + 1), (positions, None)):
+            if t is not None and (t.dim() != 2 or t.shape[1] != width or t.dtype != table.dtype or not t.is_contiguous() or
+                                  (need is not None and t.shape[0] != need)):
+                raise KernelError("summed_embedding: the tables do not fit each other")
+        if stride != width:
+            raise KernelError("summed_embedding: the table must be contiguous")
+        buckets, mul_prev, mul_cur = constants if bigram is not None else (0, 0, 0)
+        if bigram is not None:
+            seqs = batch.num_seqs
+            _i32(batch.token_seq, n, "token_seq")
+            _i32(batch.cu_seqlens_q, seqs + 1, "cu_seqlens_q")
+            _i32(batch.seq_starts, seqs, "seq_starts")
+            _i32(batch.state_slots, seqs, "state_slots")
+            if before is None or before.dtype != torch.int32 or before.dim() != 2 or before.shape[1] != 1 or not before.is_contiguous():
+                raise KernelError("summed_embedding: the tokens before must be contiguous int32 [slots, 1]")
+            if sum(batch.q_lens) != n:
+                raise KernelError("summed_embedding: the batch does not describe the ids")
+        out = torch.empty((n, width), dtype=torch.float32, device=table.device)
+        library.call("embed", _suffix(table), "nva_summed_embedding", _p(table), c_i64(rows), _p(bigram), c_i64(buckets),
+                     c_i64(mul_prev), c_i64(mul_cur), _p(positions), c_i64(0 if positions is None else positions.shape[0]), _p(ids),
+                     _p(batch.positions), _p(batch.token_seq), _p(batch.cu_seqlens_q), _p(batch.seq_starts), _p(batch.state_slots),
+                     _p(before), _p(out), c_i64(n), c_i32(width), _p(self.fault_flag), self._stream())
+        return out
+
+    def copy_rows(self, x: torch.Tensor) -> torch.Tensor:
+        """A second copy of a float32 tensor of contiguous rows."""
+        if x.dtype != torch.float32 or not x.is_contiguous():
+            raise KernelError("copy_rows: the tensor must be contiguous float32")
+        out = torch.empty_like(x)
+        library.call("embed", self.suffix, "nva_copy_rows", _p(x), _p(out), c_i64(x.numel()), self._stream())
+        return out
+
     # ------------------------------------------------------------------ norms
     def _norm_weight(self, weight: torch.Tensor, width: int, x: torch.Tensor):
         if weight.dim() != 1 or weight.shape[0] != width or not weight.is_contiguous():
@@ -455,13 +496,12 @@ class HipKernels:
         """The norm of a residual stream that is kept in float32 whatever the element type:
         residual <- residual + sum(addends) in place (residual None: a new stream that starts as the
         sum of the addends), then y = residual * rsqrt(mean(residual^2) + eps) * (offset + weight),
-        all in float and rounded once.  addends: up to two tensors of the element type [rows, width].
+        all in float and rounded once.  addends: up to two tensors of the element type [rows, width], or one that enters through a
+        norm of its own (NormedAddend), alone or beside a float32 one (StreamAddend).
         Returns (y, residual)."""
         if any(hasattr(a, "mult") for a in addends):
-            if len(addends) != 1 or residual is None or offset != 0.0:
-                raise KernelError("stream_rms_norm: an addend with a norm of its own comes alone, into a stream that exists, "
-                                  "and goes with a plain weight")
-            return self._stream_post_norm(addends[0], residual, weight, eps, out)
+            addend, extra = self._normed_addend(addends, residual)
+            return self._stream_post_norm(addend, residual, weight, eps, out, offset, extra)
         # a product left as partial sums is added up here, while it is read; anything else is a tensor
         addends = [a if isinstance(a, SplitSum) and self.fuse_split_sums else _t(a) for a in addends]
         if len(addends) > 2 or (residual is None and not addends):
@@ -562,11 +602,26 @@ class HipKernels:
                      self._stream())
         return out, (out2 if weight2 is not None else None), residual
 
-    def _stream_post_norm(self, addend, residual: torch.Tensor, weight: torch.Tensor, eps: float,
-                          out: Optional[torch.Tensor] = None):
-        """residual <- residual + mult * a / sqrt(mean(a^2) + eps_a) * w_a, then the stream's own norm, in one pass;
-        `addend` carries a (elements, or a product left as partial sums), w_a, eps_a and mult."""
-        a = addend.x if isinstance(addend.x, SplitSum) and self.fuse_split_sums else _t(addend.x)
+    def _norm_sources(self, x, rows: int, width: int, dtype, what: str) -> list:
+        """The arguments of an input that comes as elements or as a split product's partial sums."""
+        if tuple(x.shape) != (rows, width) or x.dtype != dtype:
+            raise KernelError(f"{what}: the inputs differ in shape or type")
+        if isinstance(x, SplitSum):
+            return [None, c_i64(0), _p(x.sums), c_i32(x.splits), c_i64(rows * width), _p(x.bias)]
+        _, _, xs = _rows2d(x, what)
+        return [_p(x), c_i64(xs), None, c_i32(0), c_i64(0), None]
+
+    def _readable(self, x):
+        return x if isinstance(x, SplitSum) and self.fuse_split_sums else _t(x)
+
+    def _stream_post_norm(self, addend, residual: torch.Tensor, weight: Optional[torch.Tensor], eps: float,
+                          out: Optional[torch.Tensor] = None, offset: float = 0.0, extra: Optional[torch.Tensor] = None):
+        """residual <- residual + mult * a / sqrt(mean(a^2) + eps_a) * (offset_a + w_a) (+ extra), then the stream's own norm
+        with (offset + weight), in one pass; `addend` carries a (elements, a product left as partial sums, or a pair of such
+        with their scales), w_a, offset_a, eps_a and mult; extra float32 [rows, width].  weight None: no norm, the stream
+        rounded to the element type."""
+        pair = hasattr(addend.x, "left_scale")
+        a = self._readable(addend.x.left if pair else addend.x)
         rows, width = a.shape
         rrows, rw, rs = _rows2d(residual, "stream_rms_norm residual")
         if (rrows, rw) != (rows, width) or residual.dtype != torch.float32:
@@ -576,17 +631,49 @@ class HipKernels:
         orows, ow, os_ = _rows2d(out, "stream_rms_norm output")
         if (orows, ow) != (rows, width) or out.dtype != a.dtype:
             raise KernelError("stream_rms_norm: output does not match")
-        wf = self._norm_weight(weight, width, out)
+        wf = 0 if weight is None else self._norm_weight(weight, width, out)
         awf = self._norm_weight(addend.weight, width, out)
-        if isinstance(a, SplitSum):
-            src = [None, c_i64(0), _p(a.sums), c_i32(a.splits), c_i64(rows * width), _p(a.bias)]
+        src = self._norm_sources(a, rows, width, out.dtype, "stream_rms_norm addend")
+        if pair:
+            src += [c_f32(float(addend.x.left_scale)),
+                    *self._norm_sources(self._readable(addend.x.right), rows, width, out.dtype, "stream_rms_norm addend"),
+                    c_f32(float(addend.x.right_scale))]
         else:
-            _, _, as_ = _rows2d(a, "stream_rms_norm addend")
-            src = [_p(a), c_i64(as_), None, c_i32(0), c_i64(0), None]
-        library.call("norm", _suffix(out), "nva_stream_post_norm", *src, _p(addend.weight), c_i32(awf), c_f32(float(addend.eps)),
-                     c_f32(float(addend.mult)), _p(residual), c_i64(rs), _p(weight), c_i32(wf), _p(out), c_i64(os_), c_i64(rows),
-                     c_i32(width), c_f32(eps), self._stream())
+            src += [c_f32(1.0), None, c_i64(0), None, c_i32(0), c_i64(0), None, c_f32(0.0)]
+        xs = 0
+        if extra is not None:
+            xrows, xw, xs = _rows2d(extra, "stream_rms_norm float addend")
+            if (xrows, xw) != (rows, width) or extra.dtype != torch.float32:
+                raise KernelError("stream_rms_norm: a float addend must be float32 of the stream's shape")
+        library.call("norm", _suffix(out), "nva_stream_post_norm", *src, _p(addend.weight), c_i32(awf), c_f32(float(addend.offset)),
+                     c_f32(float(addend.eps)), c_f32(float(addend.mult)), _p(extra), c_i64(xs), _p(residual), c_i64(rs), _p(weight),
+                     c_i32(wf), c_f32(float(offset)), _p(out), c_i64(os_), c_i64(rows), c_i32(width), c_f32(eps), self._stream())
         return out, residual
+
+    def stream_add(self, addends, residual: torch.Tensor):
+        """The addends (as stream_rms_norm takes them where one comes through a norm of its own) into the float32 stream, in
+        place; returns (the stream rounded to the addend's element type, the stream)."""
+        addend, extra = self._normed_addend(addends, residual)
+        return self._stream_post_norm(addend, residual, None, 0.0, extra=extra)
+
+    @staticmethod
+    def _normed_addend(addends, residual):
+        normed = [a for a in addends if hasattr(a, "mult")]
+        extra = [a for a in addends if not hasattr(a, "mult")]
+        if len(normed) != 1 or len(extra) > 1 or residual is None or not all(torch.is_tensor(getattr(a, "x", None)) for a in extra):
+            raise KernelError("stream_rms_norm: an addend with a norm of its own comes alone or with one float addend, into a "
+                              "stream that exists")
+        return normed[0], extra[0].x if extra else None
+
+    def pair_scaled_sum(self, a, sa: float, b, sb: float) -> torch.Tensor:
+        """sa * a + sb * b, in float and rounded once; an input left as partial sums is added up while it is read."""
+        a, b = self._readable(a), self._readable(b)
+        rows, width = a.shape
+        out = torch.empty((rows, width), dtype=a.dtype, device=a.device)
+        library.call("norm", _suffix(out), "nva_pair_scaled_sum", *self._norm_sources(a, rows, width, a.dtype, "pair_scaled_sum"),
+                     c_f32(float(sa)), *self._norm_sources(b, rows, width, a.dtype, "pair_scaled_sum"), c_f32(float(sb)), _p(out),
+                     c_i64(width), c_i64(rows), c_i32(width), self._stream())
+        return out
 
     def stream_dyt(self, addends, residual: Optional[torch.Tensor], weight: torch.Tensor, bias: torch.Tensor,
                    alpha: torch.Tensor, out: Optional[torch.Tensor] = None):
@@ -654,6 +741,14 @@ class HipKernels:
                      c_f32(eps), self._stream())
         return out
 
+    def softcap_(self, x: torch.Tensor, cap: float) -> torch.Tensor:
+        """x <- cap * tanh(x / cap) in place; x float32 [rows, width]."""
+        rows, width, xs = _rows2d(x, "softcap_ input")
+        if x.dtype != torch.float32:
+            raise KernelError("softcap_: the tensor must be float32")
+        library.call("embed", self.suffix, "nva_softcap_rows", _p(x), c_i64(xs), c_i64(rows), c_i32(width), c_f32(cap), self._stream())
+        return x
+
     def scale_(self, x: torch.Tensor, factor: float) -> torch.Tensor:
         """x <- x * factor in place; x float32 [rows, width]."""
         rows, width, xs = _rows2d(x, "scale_ input")
@@ -665,10 +760,10 @@ class HipKernels:
 
     # ------------------------------------------------------------------ feed-forward
     ACTIVATIONS = {"silu": 0, "relu": 1, "gelu_tanh": 2}
-    PLAIN_ACTIVATIONS = {"silu": 0, "relu": 1, "gelu_tanh": 2, "relu2": 3}
+    PLAIN_ACTIVATIONS = {"silu": 0, "relu": 1, "gelu_tanh": 2, "relu2": 3, "gelu": 4}
 
     def act(self, x: torch.Tensor, act: str = "relu2", out: Optional[torch.Tensor] = None) -> torch.Tensor:
-        """act(x), entry by entry: silu, relu, gelu_tanh or relu2 (the square of relu)."""
+        """act(x), entry by entry: silu, relu, gelu_tanh, relu2 (the square of relu) or gelu (the exact form)."""
         if act not in self.PLAIN_ACTIVATIONS:
             raise KernelError(f"act: unknown activation {act!r}; known: {sorted(self.PLAIN_ACTIVATIONS)}")
         x = _t(x)
@@ -704,8 +799,25 @@ class HipKernels:
                      _p(out), c_i64(width), c_i64(rows), c_i32(width), c_i32(self.PLAIN_ACTIVATIONS[act]), self._stream())
         return out
 
+    def act_mul_rows(self, x, table: torch.Tensor, ids: torch.Tensor, offset: int, act: str = "gelu_tanh") -> torch.Tensor:
+        """act(x[t]) * table[ids[t], offset : offset + width], in float and rounded once; x [tokens, width] of the table's type, or
+        a product left as partial sums."""
+        if act not in self.PLAIN_ACTIVATIONS:
+            raise KernelError(f"act_mul_rows: unknown activation {act!r}; known: {sorted(self.PLAIN_ACTIVATIONS)}")
+        x = self._readable(x)
+        tokens, width = x.shape
+        trows, tw, ts = _rows2d(table, "token table")
+        _i32(ids, tokens, "token ids")
+        if table.dtype != x.dtype or offset < 0 or offset + width > tw:
+            raise KernelError("act_mul_rows: the table does not fit the input")
+        out = torch.empty((tokens, width), dtype=table.dtype, device=table.device)
+        library.call("activation", _suffix(table), "nva_act_mul_rows", *self._norm_sources(x, tokens, width, table.dtype, "act_mul_rows"),
+                     _p(table), c_i64(ts), c_i64(trows), c_i32(offset), _p(ids), _p(out), c_i64(width), c_i64(tokens), c_i32(width),
+                     c_i32(self.PLAIN_ACTIVATIONS[act]), _p(self.fault_flag), self._stream())
+        return out
+
     # ------------------------------------------------------------------ routed feed-forward
-    ROUTINGS = {"sigmoid_groups": 0, "softmax_top": 1, "softmax_choice": 2}
+    ROUTINGS = {"sigmoid_groups": 0, "softmax_top": 1, "softmax_choice": 2, "softmax_scores": 3}
 
     def moe_route(self, logits: torch.Tensor, top: int, group_count: int, group_keep: int, scale: float,
                   routing: str = "sigmoid_groups", bias: Optional[torch.Tensor] = None):
@@ -715,7 +827,8 @@ class HipKernels:
         chosen, the `top` with the largest scores.  routing "softmax_top": the `top` largest logits (plus the
         float32 bias [experts], if any) are chosen and weighted by the softmax over the chosen alone.  routing
         "softmax_choice": scores s = softmax(logits) over all experts; chosen by s + bias, within the group_keep groups
-        whose largest s + bias is largest; weights s of the chosen over their sum (+ 1e-20).  logits may be the leading
+        whose largest s + bias is largest; weights s of the chosen over their sum (+ 1e-20).  routing "softmax_scores": the `top`
+        largest s = softmax(logits), weights scale * s.  logits may be the leading
         columns of wider rows."""
         rows, experts, ls = _rows2d(logits, "router logits")
         if logits.dtype != torch.float32:
@@ -739,7 +852,7 @@ class HipKernels:
         [E * 2 ff, k], an expert's gate rows and then its up rows, and the hidden layer act(x Wg_e^T) * (x Wu_e^T).
         An id from num_experts on is an identity: its output is x[t] itself.  add_gate, float32 [tokens] (a column of
         wider rows may be given): add[t] is multiplied by sigmoid(add_gate[t])."""
-        if act not in self.PLAIN_ACTIVATIONS:
+        if act not in self.PLAIN_ACTIVATIONS or act == "gelu":
             raise KernelError(f"moe_experts: unknown activation {act!r}")
         x = _t(x)
         tokens, k, xs = _rows2d(x, "moe input")
@@ -1142,7 +1255,7 @@ class HipKernels:
         return out
 
     def _linear_team(self, x, xs, weight, ws, bias, out, os_, mode, m, n, k):
-        """The kernel for wide weights and at most 16 rows.  mode: 0 elements, 1 float, 2 gated, 5 to 8 an activation."""
+        """The kernel for wide weights and at most 16 rows.  mode: 0 elements, 1 float, 2 gated, 5 to 9 an activation."""
         library.call("gemm_team", "bf16", "nva_linear_team", _p(x), c_i64(xs), _p(weight), c_i64(ws), _p(bias), _p(out),
                      c_i64(os_), c_i32(mode), c_i64(m), c_i64(n), c_i64(k), c_i32(self.teams), self._stream())
         return out

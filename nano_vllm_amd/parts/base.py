@@ -55,6 +55,27 @@ class NormedAddend:
     weight: torch.Tensor              # [width]
     eps: float
     mult: float = 1.0
+    offset: float = 0.0               # the factor is (offset + weight): 1 for a weight that is stored around zero
+
+
+@dataclass
+class ScaledPair:
+    """left_scale * left + right_scale * right, left to the norm that takes it (alone in a NormedAddend) to add up while it
+    reads the two; `tensor()` gives the finished sum."""
+    left: object                      # [rows, width] of the element type (or a product left as partial sums)
+    right: object
+    left_scale: float
+    right_scale: float
+    kernels: object
+
+    def tensor(self) -> torch.Tensor:
+        return self.kernels.pair_scaled_sum(self.left, self.left_scale, self.right, self.right_scale)
+
+
+@dataclass
+class StreamAddend:
+    """A float32 tensor [rows, width] that enters a float32 residual stream as it is, beside a NormedAddend."""
+    x: torch.Tensor
 
 
 @dataclass
@@ -74,6 +95,7 @@ class BuildContext:
     hidden_size: int
     max_position: int
     position_encodings: Dict[str, object] = field(default_factory=dict)
+    tables: Dict[str, object] = field(default_factory=dict)           # the model's shared tables of the tokens
 
 
 class Part:

@@ -30,7 +30,9 @@ The residual stream r is float32 whatever the element type.  The sum is deferred
 sublayer's output leaves the block as a NormedAddend (the output, the post-norm's weight and eps,
 the constant c), and the norm that follows norms it, adds it to the stream and norms the stream in
 one pass.  The first block gets the float32 stream itself from the embedding (an embedding with a
-scale gives one).  A layer may have no feed-forward.
+scale gives one).  A layer may have no feed-forward.  With a part in the role "token_side" every layer ends with a third
+sublayer that reads the stream itself and the step's tokens and enters through a norm of its own:
+    r <- r + side_norm(side(r, tokens))
 
 Interface of a block: forward(h, residual | None, batch, cache) -> (h, residual); h is a tensor,
 or a list of addends for a float32 stream.
@@ -166,8 +168,8 @@ class ParallelResidualBlock(Part):
 
 class SandwichResidualBlock(Part):
     """params: residual_mult (default 1), parts and names by role: mixer_norm, mixer, mixer_post_norm, and,
-    where the layer has a feed-forward, feed_forward_norm, feed_forward, feed_forward_post_norm."""
-    ROLES = ("mixer_norm", "mixer", "mixer_post_norm", "feed_forward_norm", "feed_forward", "feed_forward_post_norm")
+    where the layer has a feed-forward, feed_forward_norm, feed_forward, feed_forward_post_norm; optionally token_side."""
+    ROLES = ("mixer_norm", "mixer", "mixer_post_norm", "feed_forward_norm", "feed_forward", "feed_forward_post_norm", "token_side")
 
     def __init__(self, params: Mapping, build: BuildContext):
         super().__init__(params, build)
@@ -176,7 +178,7 @@ class SandwichResidualBlock(Part):
         self.mult = float(params.get("residual_mult", 1.0))
         self.dtype = build.dtype
         has_ff = bool(parts.get("feed_forward"))
-        missing = [r for r in self.ROLES if r not in parts and (has_ff or not r.startswith("feed_forward"))]
+        missing = [r for r in self.ROLES if r not in parts and r != "token_side" and (has_ff or not r.startswith("feed_forward"))]
         if missing:
             raise ValueError(f"sandwich_residual block: missing parts {missing}")
         self.mixer_norm = make_part("norm", parts["mixer_norm"], build)
@@ -187,6 +189,7 @@ class SandwichResidualBlock(Part):
             self.feed_forward_norm = make_part("norm", parts["feed_forward_norm"], build)
             self.feed_forward = make_part("feed_forward", parts["feed_forward"], build)
             self.feed_forward_post_norm = make_part("norm", parts["feed_forward_post_norm"], build)
+        self.token_side = make_part("token_side", parts["token_side"], build) if parts.get("token_side") else None
         self._children = {names[r]: getattr(self, r) for r in self.ROLES if getattr(self, r) is not None}
 
     def children(self) -> Dict[str, Part]:
@@ -200,7 +203,16 @@ class SandwichResidualBlock(Part):
         return self.mixer.replays_state_steps
 
     def _through(self, post_norm, x) -> NormedAddend:
-        return NormedAddend(x, post_norm.weights["weight"], post_norm.eps, self.mult)
+        return NormedAddend(x, post_norm.weights["weight"], post_norm.eps, self.mult, post_norm.offset)
+
+    def _with_side(self, addend: NormedAddend, residual, batch):
+        """The end of a layer: what is still to be added, and the stream."""
+        if self.token_side is None:
+            return (addend,), residual
+        x, residual = self.kernels.stream_add((addend,), residual)
+        norm = self.token_side.norm
+        y = self.token_side.forward(x, batch.input_ids)
+        return (NormedAddend(y, norm.weights["weight"], norm.eps, self.mult, norm.offset),), residual
 
     def forward(self, h, residual, batch, cache):
         if residual is None:
@@ -213,9 +225,9 @@ class SandwichResidualBlock(Part):
             x, residual = self.mixer_norm.forward_add(tuple(h), residual)
         a = self._through(self.mixer_post_norm, self.mixer.forward(x, batch, cache))
         if self.feed_forward is None:
-            return (a,), residual
+            return self._with_side(a, residual, batch)
         y, residual = self.feed_forward_norm.forward_add((a,), residual)
-        return (self._through(self.feed_forward_post_norm, self.feed_forward.forward(y, batch)),), residual
+        return self._with_side(self._through(self.feed_forward_post_norm, self.feed_forward.forward(y, batch)), residual, batch)
 
 
 register_part("block", "sandwich_residual", SandwichResidualBlock)

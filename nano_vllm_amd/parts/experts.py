@@ -1,6 +1,6 @@
 """Feed-forward parts without a gate, and a mixture of them.
 
-"mlp": m = act(y Wu^T) Wd^T, act one of relu2 (the square of relu), relu, silu, gelu_tanh.
+"mlp": m = act(y Wu^T) Wd^T, act one of relu2 (the square of relu), relu, silu, gelu_tanh, gelu (the exact form, with erf).
 
 "moe": every token runs `top` of `experts` such layers (no biases) and, optionally, a shared one:
     s = sigmoid(y Wr^T)                       router scores, float
@@ -14,6 +14,7 @@ With routing "softmax_top" the router's logits (plus a bias, with router_bias) a
 With routing "softmax_choice" s = softmax(y Wr^T) over all experts; an expert is chosen by s_e + c_e with a learned
 correction c (a float per expert); a group counts by the largest such choice score in it and only the group_keep best
 groups' experts can be chosen; the weights are the chosen experts' s (without the correction) over their sum (+ 1e-20).
+With routing "softmax_scores" the `top` largest s = softmax(y Wr^T) are chosen and weighted by scale * s_e, not over their sum.
 With identity = n the router has n more outputs after the experts', which take part in the softmax, the groups and the
 choice like experts; they have no tensors, and the output of one that is chosen is y itself.
 With shared_gate = True the shared layer's output is multiplied by sigmoid(wg . y), one number per token.
@@ -42,7 +43,7 @@ class PlainMLP(Part):
         self.up_name = params.get("up_name", "up_proj")
         self.down_name = params.get("down_name", "down_proj")
         self.activation = params.get("activation", "relu2")
-        if self.activation not in ACTIVATIONS:
+        if self.activation not in ACTIVATIONS + ("gelu",):
             raise ValueError(f"mlp: unknown activation {self.activation!r}")
 
     def param_decls(self) -> Dict[str, ParamDecl]:
@@ -57,7 +58,7 @@ class PlainMLP(Part):
 class MixtureOfExperts(Part):
     """params: hidden_size, num_experts, top, intermediate_size, scale, group_count, group_keep,
     activation, shared (a PartSpec of a feed-forward, or None), routing ("sigmoid_groups" | "softmax_top" |
-    "softmax_choice"), router_bias (bool), gated (bool), identity (router outputs without an expert), shared_gate (bool),
+    "softmax_choice" | "softmax_scores"), router_bias (bool), gated (bool), identity (router outputs without an expert), shared_gate (bool),
     and names: correction_name, shared_gate_name (below the shared layer's), router_name, shared_name, expert_name (a format with {} for
     the expert's number), gate_name, up_name, down_name."""
 
@@ -77,7 +78,7 @@ class MixtureOfExperts(Part):
         if self.activation not in ACTIVATIONS:
             raise ValueError(f"moe: unknown activation {self.activation!r}")
         self.routing = p.get("routing", "sigmoid_groups")
-        if self.routing not in ("sigmoid_groups", "softmax_top", "softmax_choice"):
+        if self.routing not in ("sigmoid_groups", "softmax_top", "softmax_choice", "softmax_scores"):
             raise ValueError(f"moe: unknown routing {self.routing!r}")
         self.router_bias = bool(p.get("router_bias", False))
         self.gated = bool(p.get("gated", False))
@@ -143,6 +144,8 @@ class MixtureOfExperts(Part):
         elif self.routing == "softmax_top":
             ids, weights = k.moe_route(logits, self.top, 1, 1, 1.0, routing="softmax_top",
                                        bias=w.get(f"{self.router_name}.bias"))
+        elif self.routing == "softmax_scores":
+            ids, weights = k.moe_route(logits, self.top, 1, 1, self.scale, routing="softmax_scores")
         else:
             ids, weights = k.moe_route(logits, self.top, self.group_count, self.group_keep, self.scale)
         shared = self.shared.forward(x, batch) if self.shared is not None else None

@@ -12,7 +12,7 @@ from typing import Dict, List, Optional, Tuple
 
 import torch
 
-from .base import BuildContext, ParamDecl, Part, named_params
+from .base import BuildContext, ParamDecl, Part, StreamAddend, named_params
 from .registry import make_part
 from .spec import LayerRun, ModelSpec, PartSpec
 
@@ -47,6 +47,9 @@ class Model:
         for name, pe in spec.position_encodings.items():
             build.position_encodings[name] = make_part("position_encoding", pe, build)
         self.position_encodings = build.position_encodings
+        for name, table in spec.tables.items():
+            build.tables[name] = make_part("table", table, build)
+        self.tables = build.tables
         sizes = {"vocab_size": spec.vocab_size, "hidden_size": spec.hidden_size}
         self.embedding = make_part("embedding", PartSpec(spec.embedding.kind, {**spec.embedding.params, **sizes}), build)
         self.blocks: List[Part] = []
@@ -62,6 +65,7 @@ class Model:
         roots = [(spec.embedding["name"], self.embedding), (spec.final_norm["name"], self.final_norm),
                  (spec.head["name"], self.head)]
         roots += [(layer.name, block) for layer, block in zip(spec.layers, self.blocks)]
+        roots += [(spec.tables[name]["name"], table) for name, table in self.tables.items()]
         for prefix, part in roots:
             for full, owner, local, decl in named_params(part, prefix):
                 if full in self.param_table:
@@ -88,8 +92,13 @@ class Model:
             for child in part.children().values():
                 told(child)
             part.on_weights_loaded()
-        for part in [*self.position_encodings.values(), self.embedding, *self.blocks, self.final_norm, self.head]:
+        for part in self._roots():
             told(part)
+        for name, (owner, local, _) in self.param_table.items():        # (a part may have put one of its tensors into a larger one)
+            self.params[name] = owner.weights[local]
+
+    def _roots(self) -> List[Part]:
+        return [*self.position_encodings.values(), *self.tables.values(), self.embedding, *self.blocks, self.final_norm, self.head]
 
     BASE_KERNEL_MODULES = ("embed", "norm", "activation", "gemm", "gemm_skinny", "gemm_team", "gemm_tile")
 
@@ -103,7 +112,7 @@ class Model:
                     found.append(m)
             for child in part.children().values():
                 walk(child)
-        for part in [*self.position_encodings.values(), self.embedding, *self.blocks, self.final_norm, self.head]:
+        for part in self._roots():
             walk(part)
         return tuple(found)
 
@@ -113,8 +122,17 @@ class Model:
 
     # ------------------------------------------------------------------ cache
     def cache_needs(self):
-        """Per entry of the order: what its cache must hold, or None when it reads another's."""
-        return [self.blocks[run.layer].cache_need() if run.cache_of is None else None for run in self.order]
+        """Per entry of the order: what its cache must hold, or None when it reads another's; after them,
+        where the embedding keeps state per request, what that must hold."""
+        needs = [self.blocks[run.layer].cache_need() if run.cache_of is None else None for run in self.order]
+        own = getattr(self.embedding, "cache_need", None)
+        if own is not None and own() is not None:
+            needs.append(own())
+        return needs
+
+    def replays_state_steps(self, i: int) -> bool:
+        """Whether the holder of need i (cache_needs) may be captured in a single-token step."""
+        return (self.blocks[self.order[i].layer] if i < len(self.order) else self.embedding).replays_state_steps
 
     def cache_owner(self, i: int) -> int:
         run = self.order[i]
@@ -124,9 +142,18 @@ class Model:
     def forward(self, batch, caches: List[LayerCache]) -> torch.Tensor:
         """Hidden states [T, hidden] of the batch's tokens after the final norm."""
         batch.step_cache = {}        # what kernels share between the layers of one pass (a plan made by the first)
-        h = self.embedding.forward(batch.input_ids)
+        again = any(run.add_embedding for run in self.order)
+        if getattr(self.embedding, "reads_batch", False):
+            own = caches[len(self.order)] if len(caches) > len(self.order) else None
+            h = self.embedding.forward(batch.input_ids, batch, own)
+        else:
+            h = self.embedding.forward(batch.input_ids)
+        # (the stream is updated in place: where the embedding is added again, it is kept beside it)
+        kept = StreamAddend(self.embedding.second_copy(h)) if again else None
         residual = None
         for i, run in enumerate(self.order):
+            if run.add_embedding:
+                h = (*h, kept)
             h, residual = self.blocks[run.layer].forward(h, residual, batch, caches[self.cache_owner(i)])
         if residual is None:
             return self.final_norm.forward(h)

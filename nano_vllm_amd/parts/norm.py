@@ -7,7 +7,8 @@ With weight_offset c the factor is (c + weight): c = 1 is the weight stored arou
 with an offset, and every norm that is handed a list of addends instead of one tensor, works on a
 residual stream kept in float32: the stream takes the sum of the addends, the norm is computed in
 float and rounded once to the element type.  An addend may be a NormedAddend (parts.base): a sublayer's
-output that enters the stream through a norm of its own and a constant factor; the same pass does both norms.
+output that enters the stream through a norm of its own (with an offset of its own) and a constant factor; the same pass does
+both norms, and adds a StreamAddend (a float32 tensor) that comes beside it.
 Or a ScaledAddend: an output that is multiplied, channel by channel, by a learned vector on its way into the stream.
 
 "dynamic_tanh": y = tanh(alpha * x) * weight + bias with one learned number alpha per norm: no mean,
@@ -45,6 +46,9 @@ class RMSNorm(Part):
         """residual <- x + residual; returns (norm(residual), residual).  x may be a list of one or
         two addends: the residual is then a float32 stream (None: it starts as their sum)."""
         if isinstance(x, (tuple, list)):
+            if any(hasattr(a, "mult") for a in x):
+                # (addends that enter through a norm of their own, with or without a float32 one beside them)
+                return self.kernels.stream_rms_norm(tuple(x), residual, self.weights["weight"], self.eps, self.offset, out=out)
             if any(hasattr(a, "scale") for a in x):
                 if self.offset != 0.0:
                     raise ValueError("rms_norm: scaled addends go with a plain weight")

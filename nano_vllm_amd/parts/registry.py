@@ -6,7 +6,8 @@ from __future__ import annotations
 
 from typing import Callable, Dict
 
-ROLES = ("mixer", "feed_forward", "norm", "position_encoding", "block", "embedding", "head")
+ROLES = ("mixer", "feed_forward", "norm", "position_encoding", "block", "embedding", "head", "table",
+         "token_side")
 
 _REGISTRIES: Dict[str, Dict[str, Callable]] = {role: {} for role in ROLES}
 
@@ -35,5 +36,5 @@ def known_parts(role: str):
 
 
 def _load_builtin() -> None:
-    from . import (norm, rotary, attention, latent_attention, retention, state_space, channel_delta, delta, side_by_side, feed_forward, experts, block,  # noqa: F401
-                   embedding)
+    from . import (norm, rotary, attention, latent_attention, retention, state_space, channel_delta, delta, matrix_memory, gated_linear, side_by_side, feed_forward, experts, block,  # noqa: F401
+                   embedding, token_side)

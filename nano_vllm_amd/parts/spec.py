@@ -47,9 +47,12 @@ class LayerRun:
     layer     index into ModelSpec.layers: whose weights run.  A layer may be named twice.
     cache_of  None: the run has a cache of its own.  An index of an earlier entry of the
               order: the run reads that entry's cache and writes none.
+    add_embedding  the embedding's output (as it was before the first entry) is added to the residual
+              stream before the run: the start of a pass over layers that run several times.
     """
     layer: int
     cache_of: Optional[int] = None
+    add_embedding: bool = False
 
 
 @dataclass(frozen=True)
@@ -65,6 +68,7 @@ class ModelSpec:
     final_norm: PartSpec                         # params: name + the norm's own
     head: PartSpec                               # params: name, tied
     position_encodings: Mapping[str, PartSpec]   # shared by name among the mixers
+    tables: Mapping[str, PartSpec] = field(default_factory=dict)     # params: name + the table's own; shared by name among the layers
     eos_token_ids: Tuple[int, ...] = ()
     # How the checkpoint names its tensors where that is not "<part>.<parameter>": pairs (suffix,
     # replacement) tried in turn on every derived name, the first that fits is applied
@@ -78,6 +82,8 @@ class ModelSpec:
         return derived
 
     def validate(self) -> None:
+        if self.order and self.order[0].add_embedding:
+            raise ValueError("order[0] adds the embedding, which is what the stream holds before it")
         for i, run in enumerate(self.order):
             if not 0 <= run.layer < len(self.layers):
                 raise ValueError(f"order[{i}] names layer {run.layer}; there are {len(self.layers)}")

@@ -54,6 +54,38 @@ class TorchKernels:
     def embedding_scaled(self, table, ids, scale):
         return table[ids.long()].float() * scale
 
+    def summed_embedding(self, table, ids, bigram, constants, positions, before, batch):
+        """float32 rows of up to three tables added; the bigram table's row by the token before and this one."""
+        x = table[ids.long()].float()
+        if bigram is not None:
+            buckets, mul_prev, mul_cur = constants
+            toks, t, rows = ids.tolist(), 0, []
+            for slot, start, n in zip(batch.state_slots.tolist(), batch.starts, batch.q_lens):
+                last = int(before[slot, 0]) if start > 0 else None
+                for tok in toks[t:t + n]:
+                    rows.append(buckets if last is None else (last * mul_prev + tok * mul_cur) % buckets)
+                    last = tok
+                before[slot, 0] = last
+                t += n
+            x = x + bigram[torch.tensor(rows, device=bigram.device)].float()
+        if positions is not None:
+            x = x + positions[batch.positions.long()].float()
+        return x
+
+    def copy_rows(self, x):
+        return x.clone()
+
+    def softcap_(self, x, cap):
+        return x.copy_(cap * torch.tanh(x / cap))
+
+    def pair_scaled_sum(self, a, sa, b, sb):
+        return (sa * a.float() + sb * b.float()).to(a.dtype)
+
+    def stream_add(self, addends, residual):
+        dt = next(getattr(a.x, "left", a.x).dtype for a in addends if hasattr(a, "mult"))
+        _, residual = self.stream_rms_norm(addends, residual, torch.ones((), device=residual.device), 1.0)
+        return residual.to(dt), residual
+
     # norms (layernorm.py:16-40)
     def rms_norm(self, x, weight, eps, out=None):
         xf = x.float()
@@ -80,9 +112,12 @@ class TorchKernels:
         dt = out.dtype if out is not None else None
         for a in addends:
             if hasattr(a, "mult"):          # an addend that enters through a norm of its own, times a constant
-                x = a.x.float()
-                dt = dt or a.x.dtype
-                x = a.mult * (x * torch.rsqrt(x.pow(2).mean(-1, keepdim=True) + a.eps) * a.weight.float())
+                pair = hasattr(a.x, "left_scale")            # (the sum of two, each times its constant)
+                x = a.x.left_scale * a.x.left.float() + a.x.right_scale * a.x.right.float() if pair else a.x.float()
+                dt = dt or (a.x.left if pair else a.x).dtype
+                x = a.mult * (x * torch.rsqrt(x.pow(2).mean(-1, keepdim=True) + a.eps) * (a.offset + a.weight.float()))
+            elif hasattr(a, "x"):           # a float32 addend beside it
+                x = a.x
             else:
                 x = a.float()
                 dt = dt or a.dtype
@@ -160,7 +195,12 @@ class TorchKernels:
             return g * torch.sigmoid(g)
         if act == "gelu_tanh":
             return 0.5 * g * (1.0 + torch.tanh(0.7978845608028654 * (g + 0.044715 * g ** 3)))
+        if act == "gelu":
+            return 0.5 * g * (1.0 + torch.erf(g * 0.7071067811865476))
         raise ValueError(act)
+
+    def act_mul_rows(self, x, table, ids, offset, act="gelu_tanh"):
+        return (self._activation(x.float(), act) * table[ids.long(), offset:offset + x.shape[1]].float()).to(table.dtype)
 
     def act(self, x, act="relu2", out=None):
         y = self._activation(x.float(), act).to(x.dtype)
@@ -178,6 +218,9 @@ class TorchKernels:
             z = logits.float() + (bias.float() if bias is not None else 0.0)
             best = z.topk(top, dim=-1)
             return best.indices.to(torch.int32), torch.softmax(best.values, dim=-1)
+        if routing == "softmax_scores":
+            best = torch.softmax(logits.float(), dim=-1).topk(top, dim=-1)
+            return best.indices.to(torch.int32), scale * best.values
         if routing == "softmax_choice":
             s = torch.softmax(logits.float(), dim=-1)
             choice = s + (bias.float() if bias is not None else 0.0)
@@ -293,10 +336,10 @@ class TorchKernels:
             return x.to(dt)
 
         q = prepare(qkv[:, :qd], num_heads, q_weight)
-        qkv[:, :qd] = q.reshape(T, qd)
+        qkv[:, :qd] = q.reshape(T, qd).clone()          # (without norm and rotation q is a view of the row itself)
         if num_kv_heads:
             k = prepare(qkv[:, qd:qd + kd], num_kv_heads, k_weight)
-            qkv[:, qd:qd + kd] = k.reshape(T, kd)
+            qkv[:, qd:qd + kd] = k.reshape(T, kd).clone()
             if k_cache is not None:
                 page_size = k_cache.shape[2]
                 v = qkv[:, qd + kd:].reshape(T, num_kv_heads, D)
@@ -447,6 +490,52 @@ class TorchKernels:
             out.copy_(y)
             return out
         return y
+
+    def gated_linear(self, proj, heads, dim, vdim, a2, a2_bias, tau, norm_w, eps, state, batch):
+        """proj [q | k | v | gate | low]; token by token: S <- diag(a) S + k v^T, o = S^T q, a = sigmoid(low a2^T + b)^(1/tau)."""
+        T, qk, vv = proj.shape[0], heads * dim, heads * vdim
+        p = proj.float()
+        q, k = p[:, :qk].reshape(T, heads, dim) * dim ** -0.5, p[:, qk:2 * qk].reshape(T, heads, dim)
+        v, g = p[:, 2 * qk:2 * qk + vv].reshape(T, heads, vdim), p[:, 2 * qk + vv:2 * qk + 2 * vv]
+        low = p[:, 2 * qk + 2 * vv:2 * qk + 2 * vv + a2.shape[1]]
+        z = low @ a2.float().T + a2_bias
+        a = torch.exp(torch.nn.functional.logsigmoid(z) / tau).reshape(T, heads, dim)
+        o = torch.zeros((T, heads, vdim), device=proj.device)
+        t = 0
+        for slot, start, n in zip(batch.state_slots.tolist(), batch.starts, batch.q_lens):
+            S = state[slot].clone() if start > 0 else torch.zeros_like(state[slot])
+            for i in range(t, t + n):
+                S = a[i][:, :, None] * S + k[i][:, :, None] * v[i][:, None, :]
+                o[i] = torch.einsum("hdv,hd->hv", S, q[i])
+            state[slot] = S
+            t += n
+        o = o * torch.rsqrt(o.pow(2).mean(-1, keepdim=True) + eps) * norm_w.float()
+        return (o.reshape(T, vv) * g * torch.sigmoid(g)).to(proj.dtype)
+
+    def matrix_memory(self, proj, gates, gate_bias, heads, dim, vdim, cap, norm_w, eps, s_state, n_state, m_state, batch):
+        """proj [q | k | v | gate], gates float [i | f]; token by token with the running maximum m."""
+        T, qk, vv = proj.shape[0], heads * dim, heads * vdim
+        p = proj.float()
+        q, k = p[:, :qk].reshape(T, heads, dim) * dim ** -0.5, p[:, qk:2 * qk].reshape(T, heads, dim)
+        v, g = p[:, 2 * qk:2 * qk + vv].reshape(T, heads, vdim), p[:, 2 * qk + vv:2 * qk + 2 * vv]
+        z = cap * torch.tanh((gates.float() + gate_bias) / cap)
+        gi, gf = z[:, :heads], torch.nn.functional.logsigmoid(z[:, heads:])
+        o = torch.zeros((T, heads, vdim), device=proj.device)
+        t = 0
+        for slot, start, n in zip(batch.state_slots.tolist(), batch.starts, batch.q_lens):
+            S, N, M = (x[slot].clone() if start > 0 else torch.zeros_like(x[slot]) for x in (s_state, n_state, m_state))
+            for i in range(t, t + n):
+                m_new = torch.maximum(gf[i] + M, gi[i])
+                keep, write = torch.exp(gf[i] + M - m_new), torch.exp(gi[i] - m_new)
+                S = keep[:, None, None] * S + write[:, None, None] * k[i][:, :, None] * v[i][:, None, :]
+                N = keep[:, None] * N + write[:, None] * k[i]
+                M = m_new
+                den = torch.maximum((N * q[i]).sum(-1).abs(), torch.exp(-M)) + 1e-6
+                o[i] = torch.einsum("hdv,hd->hv", S, q[i]) / den[:, None]
+            s_state[slot], n_state[slot], m_state[slot] = S, N, M
+            t += n
+        o = (o * torch.rsqrt(o.pow(2).mean(-1, keepdim=True) + eps)).reshape(T, vv) * norm_w.float()
+        return (o * torch.sigmoid(g)).to(proj.dtype)
 
     RETENTION_CHUNK = 4
 
