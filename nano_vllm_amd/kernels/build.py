@@ -42,6 +42,7 @@ MODULES: Dict[str, Tuple[str, Tuple[Optional[str], ...]]] = {
     "moe": ("moe.hip", ("bf16", "f32")),
     "delta": ("delta.hip", ("bf16", "f32")),
     "latent": ("latent.hip", ("bf16", "f32")),
+    "memory": ("memory.hip", ("bf16", "f32")),
 }
 
 _HEADERS = ("common.h",)

@@ -26,6 +26,7 @@ _LAST_ERROR_SYMBOL = {
     "qk_rownorm": "nva_qk_rownorm_last_error", "retention": "nva_retention_last_error",
     "ssd": "nva_ssd_last_error", "moe": "nva_moe_last_error",
     "delta": "nva_delta_last_error", "latent": "nva_latent_last_error",
+    "memory": "nva_memory_last_error",
 }
 
 _loaded: Dict[Tuple[str, Optional[str]], ctypes.CDLL] = {}

@@ -170,6 +170,32 @@ def delta_blocks(q_lens, first_seq: int):
     return units, chains
 
 
+MEMORY_CHUNK = 16       # tokens of a chunk of the gated linear attentions' matrix-core form
+
+
+def memory_units(q_lens, first_seq: int, heads: int, cus: int):
+    """The step's portions (the requests from `first_seq` on, which single tokens precede) in units of whole chunks that run side
+    by side: (units, chains), units a flat list of (request, the unit's first token counted through the step, its tokens,
+    kind) with kind 0 for a portion of one unit, 2 for a portion's last, 1 for the others; chains one of (first unit, units,
+    request, 0) for every portion of more than one.  Units of 64 tokens, of more where heads and units then still give
+    every compute unit two workgroups."""
+    total = sum(q_lens[first_seq:])
+    size = 4 * MEMORY_CHUNK
+    while size < 1024 and (total // (2 * size)) * heads >= 2 * cus:
+        size *= 2
+    units, chains = [], []
+    token = sum(q_lens[:first_seq])
+    for s in range(first_seq, len(q_lens)):
+        n = q_lens[s]
+        count = (n + size - 1) // size
+        if count > 1:
+            chains += [len(units) // 4, count, s, 0]
+        for u in range(count):
+            units += [s, token + u * size, min(size, n - u * size), 0 if count == 1 else 2 if u == count - 1 else 1]
+        token += n
+    return units, chains
+
+
 def state_space_blocks(q_lens, first_seq: int):
     """As retention_blocks, for the state-space layer's blocks as products: blocks of 64 tokens, which that kernel takes, as long
     as the step's portions hold at most 16384 tokens (a block's end state is kept until the pass over the blocks);
@@ -329,6 +355,8 @@ class HipKernels:
         self.delta_blocks = True
         self.delta_single_kernel = True
         self.delta_block_min = DELTA_BLOCK
+        # False: the gated linear attention and the matrix memory run portions token by token too
+        self.memory_blocks = True
         # False: the state-space layer runs a portion's tokens one after the other, whatever its length
         self.state_space_blocks_side_by_side = True
         # how the recurrence holds a state of 65 to 128 rows: 0 two lanes a column (what serves), 1 a thread a column
@@ -1895,6 +1923,116 @@ class HipKernels:
         _i32(batch.state_slots, seqs, "state_slots")
         if sum(batch.q_lens) != tokens:
             raise KernelError(f"{what}: the batch does not describe the projections' rows")
+
+    # ------------------------------------------------------------------ gated linear attentions
+    def _memory_plan(self, what, proj, width, heads, dim, vdim, norm_w, norm_n, s_state, batch, with_n):
+        """Checks what both rules share; returns (tokens, row stride, out, (units, their number, chains, their number, the units'
+        states, their decays), whether portions run in blocks)."""
+        tokens, w, stride = _rows2d(proj, f"{what} projections")
+        if w < width:
+            raise KernelError(f"{what}: projections of width {w}, at least {width} are needed")
+        if s_state.dtype != torch.float32 or tuple(s_state.shape[1:]) != (heads, dim, vdim) or not s_state.is_contiguous():
+            raise KernelError(f"{what}: the state must be contiguous float32 [slots, {heads}, {dim}, {vdim}]")
+        if norm_w.dtype != torch.float32 or tuple(norm_w.shape) != (norm_n,) or not norm_w.is_contiguous():
+            raise KernelError(f"{what}: norm_w must be contiguous float32 [{norm_n}]")
+        seqs, first = batch.num_seqs, batch.num_decode
+        _i32(batch.cu_seqlens_q, seqs + 1, "cu_seqlens_q")
+        _i32(batch.seq_starts, seqs, "seq_starts")
+        _i32(batch.state_slots, seqs, "state_slots")
+        if sum(batch.q_lens) != tokens or any(n != 1 for n in batch.q_lens[:first]):
+            raise KernelError(f"{what}: the batch does not describe the projections' rows (single tokens first)")
+        out = torch.empty((tokens, heads * vdim), dtype=proj.dtype, device=proj.device)
+        takes = getattr(library.load("memory", self.suffix), f"nva_memory_takes_blocks_{self.suffix}")
+        if not self.memory_blocks or first == seqs or not takes(c_i32(dim), c_i32(vdim)):
+            return tokens, stride, out, (None, 0, None, 0, None, None), False
+        # the step's portions in units (the same cut for every layer of the step with as many heads)
+        kept = getattr(batch, "step_cache", None)
+        if kept is None:
+            kept = batch.step_cache = {}
+        plan = kept.get(("memory_units", first, heads))
+        if plan is None:
+            flat_units, flat_chains = memory_units(batch.q_lens, first, heads, self.cus)
+            both = torch.tensor(flat_units + flat_chains, dtype=torch.int32).to(proj.device, non_blocking=True)
+            plan = (len(flat_units) // 4, len(flat_chains) // 4, both[: len(flat_units)], both[len(flat_units):])
+            kept[("memory_units", first, heads)] = plan
+        n_units, n_chains, units, chains = plan
+        states = decay = None
+        if n_chains:
+            states = torch.empty(n_units * heads * (dim * vdim + (dim if with_n else 0)), dtype=torch.float32, device=proj.device)
+            decay = torch.empty(n_units * heads * dim, dtype=torch.float32, device=proj.device)
+        return tokens, stride, out, (units, n_units, chains, n_chains, states, decay), True
+
+    @staticmethod
+    def _memory_plan_args(plan) -> list:
+        units, n_units, chains, n_chains, states, decay = plan          # (the caller keeps the tensors until the launch)
+        return [_p(units), c_i64(n_units), _p(chains), c_i64(n_chains), _p(states), _p(decay)]
+
+    def gated_linear(self, proj: torch.Tensor, heads: int, dim: int, vdim: int, a2: torch.Tensor, a2_bias: torch.Tensor, tau: float,
+                     norm_w: torch.Tensor, eps: float, state: torch.Tensor, batch) -> torch.Tensor:
+        """Linear attention with a decay per key channel over the step's tokens: proj [T, 2 H D + 2 H DV + rank (or wider)] = [q |
+        k | v | gate | low].  Per head S <- diag(a) S + k v^T, o = S^T q with q times D^-1/2 and a = sigmoid(low a2^T +
+        a2_bias)^(1/tau), a2 [H D, rank]; then o's RMS norm per head times norm_w [DV] times silu(gate).  state float32 [slots,
+        H, D, DV], a request's row given by batch.state_slots, taken as zero where batch.seq_starts is 0.  Returns [T, H DV]
+        of proj's type.  Single tokens make their decays in the kernel that runs them; portions' come from one product."""
+        proj = _t(proj)
+        hd, vv = heads * dim, heads * vdim
+        rank = a2.shape[1] if a2.dim() == 2 else 0
+        if tuple(a2.shape) != (hd, rank) or a2.dtype != proj.dtype or not a2.is_contiguous() or rank <= 0:
+            raise KernelError(f"gated_linear: the decay's second step must be contiguous [{hd}, rank] of the projections' type")
+        if a2_bias.dtype != torch.float32 or tuple(a2_bias.shape) != (hd,) or not a2_bias.is_contiguous():
+            raise KernelError(f"gated_linear: the decay's bias must be contiguous float32 [{hd}]")
+        if not tau > 0:
+            raise KernelError(f"gated_linear: tau {tau}")
+        at = 2 * hd + 2 * vv
+        tokens, stride, out, plan, blocks = self._memory_plan("gated_linear", proj, at + rank, heads, dim, vdim, norm_w, vdim, state,
+                                                              batch, False)
+        z, first = None, batch.num_decode
+        if blocks:
+            z = self.linear(proj[first:, at:at + rank], a2, out_float32=True)
+            if not z.is_contiguous():
+                z = z.contiguous()
+        library.call("memory", _suffix(proj), "nva_gated_linear", _p(proj), c_i64(stride), _p(z), c_i64(first), _p(a2), c_i32(rank),
+                     _p(a2_bias), _p(norm_w), c_f32(eps), c_f32(1.0 / tau), _p(state), _p(batch.cu_seqlens_q), _p(batch.seq_starts),
+                     _p(batch.state_slots), _p(out), c_i64(vv), c_i64(batch.num_seqs), c_i64(tokens), c_i64(first), c_i32(heads),
+                     c_i32(dim), c_i32(vdim), *self._memory_plan_args(plan), self._stream())
+        return out
+
+    def matrix_memory(self, proj: torch.Tensor, gates, gate_bias: torch.Tensor, heads: int, dim: int, vdim: int, cap: float,
+                      norm_w: torch.Tensor, eps: float, s_state: torch.Tensor, n_state: torch.Tensor, m_state: torch.Tensor,
+                      batch) -> torch.Tensor:
+        """A matrix memory with exponential gates over the step's tokens: proj [T, 2 H D + 2 H DV] = [q | k | v | gate], gates
+        float32 [T, 2 H] = [i | f] (or that product left as partial sums), gate_bias float32 [2 H].  i = cap tanh(i / cap), f =
+        logsigmoid(cap tanh(f / cap)), m' = max(f + m, i), S <- exp(f + m - m') S + exp(i - m') k v^T, n likewise with k, o =
+        S^T q / (max(|n.q|, exp(-m')) + 1e-6) with q times D^-1/2; then o's RMS norm per head times norm_w [H DV] times
+        sigmoid(gate).  s_state float32 [slots, H, D, DV], n_state [slots, H, D], m_state [slots, H].  Returns [T, H DV]."""
+        proj = _t(proj)
+        vv = heads * vdim
+        tokens, stride, out, plan, blocks = self._memory_plan("matrix_memory", proj, 2 * heads * (dim + vdim), heads, dim, vdim, norm_w,
+                                                              vv, s_state, batch, True)
+        if gates.dtype != torch.float32 or tuple(gates.shape) != (tokens, 2 * heads):
+            raise KernelError(f"matrix_memory: the gates must be float32 [{tokens}, {2 * heads}]")
+        if isinstance(gates, SplitSum) and self.fuse_split_sums and gates.bias is None:
+            gate_sums, splits = gates.sums, gates.splits
+        else:
+            gate_sums, splits = _t(gates), 1
+            if not gate_sums.is_contiguous():
+                raise KernelError("matrix_memory: the gates must be contiguous")
+        if gate_bias.dtype != torch.float32 or tuple(gate_bias.shape) != (2 * heads,) or not gate_bias.is_contiguous():
+            raise KernelError(f"matrix_memory: the gates' bias must be contiguous float32 [{2 * heads}]")
+        for t, shape, what in ((n_state, (heads, dim), "n"), (m_state, (heads,), "m")):
+            if t.dtype != torch.float32 or tuple(t.shape) != (s_state.shape[0],) + shape or not t.is_contiguous():
+                raise KernelError(f"matrix_memory: the state {what} must be contiguous float32 [slots, {', '.join(map(str, shape))}]")
+        wide = m = m_start = None
+        if blocks:
+            wide = torch.empty((2, tokens * heads), dtype=torch.float64, device=proj.device)
+            m = torch.empty(tokens * heads, dtype=torch.float32, device=proj.device)
+            m_start = torch.empty(batch.num_seqs * heads, dtype=torch.float32, device=proj.device)
+        library.call("memory", _suffix(proj), "nva_matrix_memory", _p(proj), c_i64(stride), _p(gate_sums), c_i32(splits),
+                     c_i64(tokens * 2 * heads), _p(gate_bias), _p(norm_w), c_f32(eps), c_f32(cap), _p(s_state), _p(n_state), _p(m_state),
+                     _p(batch.cu_seqlens_q), _p(batch.seq_starts), _p(batch.state_slots), _p(out), c_i64(vv), c_i64(batch.num_seqs),
+                     c_i64(tokens), c_i64(batch.num_decode), c_i32(heads), c_i32(dim), c_i32(vdim), *self._memory_plan_args(plan),
+                     _p(None if wide is None else wide[0]), _p(None if wide is None else wide[1]), _p(m), _p(m_start), self._stream())
+        return out
 
     # ------------------------------------------------------------------ state-space layer
     def state_space(self, proj: torch.Tensor, heads: int, vdim: int, n_state: int, groups: int, taps: int,
