@@ -48,6 +48,11 @@ layer sizes.
 does the same for the Bamipel design (layers of a window attention through latents, of the gated delta rule, of a
 grouped attention and of the delta rule again, in turn, each with a dense feed-forward without a gate), beside Kirisun,
 Pemuvik and Qwen3 at equal layer sizes.
+
+    python bench.py --design nemidra [--design-sizes 1024,2048,4096] [--layers 4]
+
+does the same for the Nemidra design (layers of a window attention beside a matrix memory with a routed feed-forward, and of
+a gated linear attention with a dense one, in turn), beside Mafarax, Kirisun and Qwen3 at equal layer sizes.
 """
 import argparse
 import json
@@ -79,7 +84,7 @@ def parse_args():
                     help="context of one more decode point at the default batch (0: none)")
     ap.add_argument("--serve-seqs", type=int, default=256,
                     help="requests of the reference's benchmark workload through LLM.generate (0: not run)")
-    ap.add_argument("--design", default=None, choices=["nozurax", "mafarax", "kirisun", "pemuvik", "bamipel"],
+    ap.add_argument("--design", default=None, choices=["nozurax", "mafarax", "kirisun", "pemuvik", "bamipel", "nemidra"],
                     help="measure this design beside Qwen3 at equal layer sizes instead of the default workload")
     ap.add_argument("--design-sizes", default="1024,2048,4096", help="model widths of the --design measurement")
     ap.add_argument("--design-alone", action="store_true", help="the --design measurement without the models beside it "
@@ -136,11 +141,25 @@ def bamipel_config(width: int, layers: int, dtype: str) -> dict:
     return _bamipel(layers, width, heads, kv, dim, dim, 3 * inner // 2, DESIGN_VOCAB, window=1024, dtype=dtype)
 
 
+def nemidra_config(width: int, layers: int, dtype: str) -> dict:
+    """A Nemidra model of the width's layer sizes: layers of a window attention with the dense model's heads (a window of
+    1024) beside a matrix memory, and of a gated linear attention, in turn (both with as many heads as the dense model has
+    query heads and a state of 128 x 128 a head); 32 gated experts of an eighth of the dense inner size of which a token runs
+    6, beside a shared one of a quarter, in the former, a layer without a gate of 3/2 of it in the latter; 256 entries of a
+    token's row for every layer."""
+    from nano_vllm_amd.models.shapes import _nemidra
+    heads, kv, dim, inner = DESIGN_SIZES[width]
+    return _nemidra(layers, width, heads, kv, dim, dim, inner, DESIGN_VOCAB, window=1024, dtype=dtype)
+
+
 def design_configs(width: int, layers: int, dtype: str, design: str = "nozurax"):
     """config.json of a Nozurax model and of the Qwen3 model with the same layer sizes (and, for the Mafarax
     measurement, of the Mafarax model first)."""
     if design == "mafarax":
         return {"mafarax": mafarax_config(width, layers, dtype), **design_configs(width, layers, dtype)}
+    if design == "nemidra":
+        return {"nemidra": nemidra_config(width, layers, dtype), "mafarax": mafarax_config(width, layers, dtype),
+                "kirisun": kirisun_config(width, layers, dtype), "qwen3": design_configs(width, layers, dtype)["qwen3"]}
     if design == "bamipel":
         return {"bamipel": bamipel_config(width, layers, dtype), "kirisun": kirisun_config(width, layers, dtype),
                 "pemuvik": pemuvik_config(width, layers, dtype), "qwen3": design_configs(width, layers, dtype)["qwen3"]}

@@ -24,7 +24,7 @@
 //     o_t = exp(M_c - M_t) S^T q_t + sum_{s <= t} exp(e_s - M_t) (q_t . k_s) v_s,     M_c the maximum before the chunk
 //     S'  = exp(M_c - M_end) S + sum_s exp(e_s - M_end) k_s v_s^T
 // No exponent of these is positive.  In the linear rule A's factors exp(P_t) and exp(-P_s) are applied to q and k apart as long
-// as no channel of 16 forgets more than exp(-20) in a chunk; where one does, that group of channels is summed pair by pair.
+// as no channel of 16 forgets more than exp(-MEM_APART) in a chunk; where one does, that group of channels is summed pair by pair.
 //
 // A workgroup takes a unit (a run of chunks of one request) and a head; a wave 16 value channels, whose part of S it keeps in
 // accumulators: register r of tile j holds, in lane group g = lane / 16, row 16 j + 4 g + r, which is how the product with q
@@ -34,6 +34,7 @@
 #include "common.h"
 
 enum { MEM_LINEAR = 0, MEM_MATRIX = 1 };
+#define MEM_APART 12.f
 
 typedef __attribute__((ext_vector_type(4))) float mem_f32x4;
 
@@ -52,12 +53,22 @@ struct MemoryArgs {
     // portions
     const int32_t* units; const int32_t* chains;            // [n][4]: request, first token of the step, tokens, kind; [n][4]: first unit, units, request, 0
     float* unit_states; float* unit_decay;                  // [units][H][D DV (+ D)], [units][H][D]
-    double* e; double* M; float* m; float* m_start;         // matrix: [tokens][H] three times, [requests][H]
+    int64_t tokens;
+    double* e; double* M; float* m; float* m_start;         // matrix: [H][tokens] three times, [requests][H]
 };
 enum { MEM_UNIT_ONLY = 0, MEM_UNIT_MORE = 1, MEM_UNIT_LAST = 2 };
 
-__device__ __forceinline__ float mem_log_sigmoid(float x) { return fminf(x, 0.f) - log1pf(expf(-fabsf(x))); }
-__device__ __forceinline__ float mem_sigmoid(float x) { return 1.f / (1.f + expf(-x)); }
+// log sigmoid(x) = min(x, 0) - log(1 + e), e = exp(-|x|).  The bfloat16 build takes the fast exponential and logarithm, and what
+// the rounding of u = 1 + e lost of e back in: log(1 + e) = log u + (e - (u - 1)) / u to first order.
+__device__ __forceinline__ float mem_log_sigmoid(float x) {
+#if defined(NVA_F32)
+    return fminf(x, 0.f) - log1pf(expf(-fabsf(x)));
+#else
+    const float e = __expf(-fabsf(x)), u = 1.f + e;
+    return fminf(x, 0.f) - (__logf(u) + (e - (u - 1.f)) * __frcp_rn(u));
+#endif
+}
+__device__ __forceinline__ float mem_sigmoid(float x) { return 1.f / (1.f + nva_exp(-x)); }
 template <int KIND> __device__ __forceinline__ float mem_gate(float g) { return KIND == MEM_LINEAR ? g * mem_sigmoid(g) : mem_sigmoid(g); }
 
 // The capped gates of a (token, head): i and f = logsigmoid(capped).
@@ -219,8 +230,8 @@ memory_walk_kernel(const MemoryArgs a, int first_seq) {
 }
 
 // ---------------------------------------------------------------------------- the matrix rule's gates of a portion
-// A workgroup per (portion, head): b, e and M of its tokens by scans over 256 tokens at a time, in double.
-#define MEM_SCAN 256
+// A workgroup per (portion, head): b, e and M of its tokens by scans over MEM_SCAN tokens at a time, in double.
+#define MEM_SCAN 1024
 __device__ __forceinline__ double mem_shfl_up(double x, int by) {
     const unsigned long long u = __builtin_bit_cast(unsigned long long, x);
     const int lo = __shfl_up((int)(u & 0xffffffffull), by, NVA_WAVE), hi = __shfl_up((int)(u >> 32), by, NVA_WAVE);
@@ -275,10 +286,11 @@ memory_gates_kernel(const MemoryArgs a, int first_seq) {
         }
         mx = fmax(mx, top);
         if (t < n) {
-            a.e[(tok0 + t) * H + h] = e;
-            a.M[(tok0 + t) * H + h] = mx;
+            const int64_t at = (int64_t)h * a.tokens + tok0 + t;
+            a.e[at] = e;
+            a.M[at] = mx;
             m_last = b + mx;
-            a.m[(tok0 + t) * H + h] = (float)m_last;
+            a.m[at] = (float)m_last;
             if (t == n - 1) a.m_state[slot * H + h] = (float)m_last;
         }
     }
@@ -288,15 +300,18 @@ memory_gates_kernel(const MemoryArgs a, int first_seq) {
 #define MEM_C 16
 #define MEM_TS 20                    // row stride of a transposed key row and of a chunk's scores
 
+// Waves of a workgroup: one for every 16 key channels (a wave prepares one such tile a chunk) and for every 16 value channels.
+__host__ __device__ inline int mem_block_waves(int ndt, int vdim) { return ndt > (vdim + 15) / 16 ? ndt : (vdim + 15) / 16; }
+
 __host__ __device__ inline int mem_block_lds_floats(int ndt, int waves, bool out) {
     const int dp = 16 * ndt;
-    int n = dp * MEM_TS + dp + dp + 2 * MEM_C + 4;                                     // keys, decays, n, weights and factors
-    if (out) n += MEM_C * (dp + 4) + waves * MEM_C * MEM_TS + MEM_C * MEM_TS + 2 * waves * MEM_C + MEM_C;
+    int n = dp * MEM_TS + 3 * dp + 2 * MEM_C + 4;            // keys, decays, n, the unit's logarithms, weights and factors
+    if (out) n += MEM_C * (dp + 4) + waves * MEM_C * MEM_TS + MEM_C * MEM_TS + 2 * waves * MEM_C + 2 * MEM_C;
     return n;
 }
 
-template <typename T, int KIND, int NDT, bool OUT>
-__global__ void __launch_bounds__(1024)
+template <typename T, int KIND, int NDT, bool OUT, int THREADS>
+__global__ void __launch_bounds__(THREADS)
 memory_block_kernel(const MemoryArgs a) {
     extern __shared__ __attribute__((aligned(16))) float lds[];
     __shared__ double e_s[MEM_C], M_s[MEM_C];
@@ -306,7 +321,8 @@ memory_block_kernel(const MemoryArgs a) {
     float* const kT_s = lds;                                 // [DP][20]: keys times their decay to the chunk's end
     float* const dec_s = kT_s + DP * MEM_TS;                 // [DP]: the chunk's decays (linear)
     float* const n_s = dec_s + DP;                           // [DP] (matrix)
-    float* const w_s = n_s + DP;                             // [16]: exp(e_s - M_end)
+    float* const log_s = n_s + DP;                           // [DP]: the unit's log decays so far (linear, without outputs)
+    float* const w_s = log_s + DP;                           // [16]: exp(e_s - M_end)
     float* const inter_s = w_s + MEM_C;                      // [16]: exp(M_c - M_t)
     float* const keep_s = inter_s + MEM_C;                   // [1] (+ 3)
     float* const q_s = keep_s + 4;                           // [16][QS]
@@ -315,6 +331,7 @@ memory_block_kernel(const MemoryArgs a) {
     float* const red_s = a_s + MEM_C * MEM_TS;               // [waves][16]
     float* const qn_s = red_s + waves * MEM_C;               // [waves][16]
     float* const den_s = qn_s + waves * MEM_C;               // [16]
+    float* const floor_s = den_s + MEM_C;                    // [16]: exp(-m_t)
 
     const int h = blockIdx.x;
     const int32_t* u = a.units + 4 * (int64_t)blockIdx.y;
@@ -325,8 +342,10 @@ memory_block_kernel(const MemoryArgs a) {
     const int64_t qk = (int64_t)H * D, vv = (int64_t)H * DV;
     const int64_t q_off = (int64_t)h * D, k_off = qk + q_off, v_off = 2 * qk + (int64_t)h * DV, g_off = v_off + vv;
     const T* const proj = static_cast<const T*>(a.proj);
-    const int c = 16 * wave + i;                             // this lane's value channel
-    const bool has_c = c < DV;
+    const int c = 16 * wave + i, cc = min(c, DV - 1);        // this lane's value channel
+    const bool has_c = c < DV, multiplies = 16 * wave < DV;  // (a wave beyond the value channels only prepares)
+    const int d_own = 16 * wave + i, dc = min(d_own, D - 1); // the key channel it prepares
+    const bool prepares = wave < NDT, has_d = d_own < D;
     const int64_t slot = a.state_slots[seq];
     const bool fresh = a.seq_starts[seq] <= 0;
     const int64_t state_floats = (int64_t)D * DV + (KIND == MEM_MATRIX ? D : 0);
@@ -334,89 +353,95 @@ memory_block_kernel(const MemoryArgs a) {
     float* const s_slot = a.s_state + (slot * H + h) * (int64_t)D * DV;
     float* const n_slot = KIND == MEM_MATRIX ? a.n_state + (slot * H + h) * (int64_t)D : nullptr;
 
-    // the state at the unit's start
+    // ---- a chunk's values, gates, queries, keys and decay logits: asked for a chunk ahead, kept as they were loaded
+    T v_raw[4], g_raw[4], q_raw[4], k_raw[4];
+    float z_raw[4];
+    double e_raw = 0.0, M_raw = 0.0, M_end_raw = 0.0;
+    float m_raw = 0.f;
+    auto ask = [&](int t0) __attribute__((always_inline)) {
+        const int64_t tok = tok0 + t0;
+        const int last = n_tok - t0 - 1;                     // (a token beyond the unit reads the unit's last)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+            const int64_t tt = tok + min(4 * g + r, last);
+            const T* row = proj + tt * a.stride;
+            v_raw[r] = row[v_off + cc];
+            if (OUT) g_raw[r] = row[g_off + cc];
+            if (OUT) q_raw[r] = row[q_off + dc];
+            k_raw[r] = row[k_off + dc];
+            if (KIND == MEM_LINEAR) z_raw[r] = a.z[(tt - a.z_first) * qk + q_off + dc];
+        }
+        if (KIND == MEM_MATRIX) {
+            const int64_t at = (int64_t)h * a.tokens + tok + min(i, last);
+            e_raw = a.e[at];
+            M_raw = a.M[at];
+            M_end_raw = a.M[(int64_t)h * a.tokens + tok + min(MEM_C - 1, last)];
+            if (OUT) m_raw = a.m[at];
+        }
+    };
+    ask(0);
+
+    // ---- the state at the unit's start
     const float* s_from = !OUT ? nullptr : kind != MEM_UNIT_ONLY ? s_unit : fresh ? nullptr : s_slot;
     const float* n_from = KIND == MEM_LINEAR || !s_from ? nullptr : kind != MEM_UNIT_ONLY ? s_unit + (int64_t)D * DV : n_slot;
     mem_f32x4 S[NDT];
+    if (s_from) {
+#pragma unroll
+        for (int j = 0; j < NDT; ++j)
+#pragma unroll
+            for (int r = 0; r < 4; ++r) S[j][r] = s_from[(int64_t)min(16 * j + 4 * g + r, D - 1) * DV + cc];
+    }
 #pragma unroll
     for (int j = 0; j < NDT; ++j)
 #pragma unroll
-        for (int r = 0; r < 4; ++r) {
-            const int d = 16 * j + 4 * g + r;
-            S[j][r] = s_from && has_c && d < D ? s_from[(int64_t)d * DV + c] : 0.f;
-        }
+        for (int r = 0; r < 4; ++r)
+            if (!s_from || !has_c || 16 * j + 4 * g + r >= D) S[j][r] = 0.f;
     for (int d = tid; d < DP; d += blockDim.x) {
         n_s[d] = KIND == MEM_MATRIX && n_from && d < D ? n_from[d] : 0.f;
         dec_s[d] = 1.f;
+        log_s[d] = 0.f;
     }
     double M_before = 0.0;
     if (KIND == MEM_MATRIX)
-        M_before = tok0 == a.cu_seqlens_q[seq] ? (double)a.m_start[(int64_t)seq * H + h] : a.M[(tok0 - 1) * H + h];
+        M_before = tok0 == a.cu_seqlens_q[seq] ? (double)a.m_start[(int64_t)seq * H + h] : a.M[(int64_t)h * a.tokens + tok0 - 1];
     const double M_unit = M_before;
-    constexpr int OWN = NDT;                                 // tiles of channels a wave prepares, at most
-    float log_sum[OWN];                                      // linear, without outputs: the unit's decays of those tiles' channels
-#pragma unroll
-    for (int j = 0; j < OWN; ++j) log_sum[j] = 0.f;
+    const float bias = KIND == MEM_LINEAR ? a.bias[q_off + dc] : 0.f;
+    const float norm_w = OUT ? a.norm_w[KIND == MEM_MATRIX ? h * DV + cc : cc] : 0.f;
     __syncthreads();
 
     for (int t0 = 0; t0 < n_tok; t0 += MEM_C) {
         const int n = min(MEM_C, n_tok - t0);
         const int64_t tok = tok0 + t0;
-        // ---- this lane's values (and output gates) of the chunk
-        float v[4], gate[4];
+        float v[4], gate[4], q[4], k[4], lg[4];
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
-            const int t = 4 * g + r;
-            const T* row = proj + (tok + min(t, n - 1)) * a.stride;
-            const int cc = min(c, DV - 1);
-            v[r] = to_float(row[v_off + cc]);
-            if (OUT) gate[r] = to_float(row[g_off + cc]);
-            if (t >= n || !has_c) v[r] = 0.f;
+            const bool has = has_d && 4 * g + r < n;
+            v[r] = has_c && 4 * g + r < n ? to_float(v_raw[r]) : 0.f;
+            if (OUT) gate[r] = to_float(g_raw[r]);
+            if (OUT) q[r] = has ? to_float(q_raw[r]) * a.scale : 0.f;
+            k[r] = has ? to_float(k_raw[r]) : 0.f;
+            if (KIND == MEM_LINEAR) lg[r] = has ? z_raw[r] + bias : 0.f;
         }
-        double M_end = 0.0;
-        if (KIND == MEM_MATRIX) {
-            M_end = a.M[(tok + n - 1) * H + h];
-            if (tid < MEM_C) {
-                const int64_t at = (tok + min(tid, n - 1)) * H + h;
-                const double e = tid < n ? a.e[at] : -1e300, M = a.M[at];
-                e_s[tid] = e;
-                M_s[tid] = M;
-                w_s[tid] = expf((float)(e - M_end));         // (a token beyond the portion: zero)
-                inter_s[tid] = expf((float)(M_before - M));
-                if (tid == 0) keep_s[0] = expf((float)(M_before - M_end));
-            }
+        const double M_end = M_end_raw, e_now = i < n ? e_raw : -1e300, M_now = M_raw;
+        const float m_now = m_raw;
+        if (t0 + MEM_C < n_tok) ask(t0 + MEM_C);
+        if (KIND == MEM_MATRIX && tid < MEM_C) {
+            e_s[tid] = e_now;
+            M_s[tid] = M_now;
+            w_s[tid] = expf((float)(e_now - M_end));         // (a token beyond the unit: zero)
+            inter_s[tid] = expf((float)(M_before - M_now));
+            if (OUT) floor_s[tid] = expf(-m_now);
+            if (tid == 0) keep_s[0] = expf((float)(M_before - M_end));
         }
-        // ---- q, k and the decays: a wave prepares tiles of 16 key channels; a lane one channel and four tokens
-        mem_f32x4 score = {0.f, 0.f, 0.f, 0.f};
-        float qn[4] = {0.f, 0.f, 0.f, 0.f};
+        // ---- queries, keys and decays: a wave prepares 16 key channels; a lane one channel and four tokens
         float* const mine_s = part_s + wave * MEM_C * MEM_TS;
-        int own = 0;
-#pragma unroll
-        for (int o = 0; o < OWN; ++o) {
-            const int j = wave + o * waves;
-            if (j >= NDT) break;
-            const int d = 16 * j + i;
-            const bool has_d = d < D;
-            const int dc = min(d, D - 1);
-            float q[4], k[4], lg[4];
-#pragma unroll
-            for (int r = 0; r < 4; ++r) {
-                const int t = 4 * g + r;
-                const int64_t tt = tok + min(t, n - 1);
-                const T* row = proj + tt * a.stride;
-                if (OUT) q[r] = to_float(row[q_off + dc]);
-                k[r] = to_float(row[k_off + dc]);
-                if (KIND == MEM_LINEAR) lg[r] = a.z[(tt - a.z_first) * qk + q_off + dc];
-            }
-            const float bias = KIND == MEM_LINEAR ? a.bias[q_off + dc] : 0.f;
-#pragma unroll
-            for (int r = 0; r < 4; ++r) {
-                const bool has = has_d && 4 * g + r < n;
-                if (OUT) q[r] = has ? q[r] * a.scale : 0.f;
-                k[r] = has ? k[r] : 0.f;
-                if (KIND == MEM_LINEAR) lg[r] = has ? mem_log_sigmoid(lg[r] + bias) * a.par : 0.f;
-            }
+        if (prepares) {
+            mem_f32x4 score = {0.f, 0.f, 0.f, 0.f};
+            float qn[4] = {0.f, 0.f, 0.f, 0.f};
+            bool apart = true;
             if (KIND == MEM_LINEAR) {
+#pragma unroll
+                for (int r = 0; r < 4; ++r) lg[r] = has_d && 4 * g + r < n ? mem_log_sigmoid(lg[r]) * a.par : 0.f;
                 // sums up to and including a token, and behind it to the chunk's end
                 const float p0 = lg[0], p1 = p0 + lg[1], p2 = p1 + lg[2], p3 = p2 + lg[3];
                 const float x0 = __shfl(p3, i, NVA_WAVE), x1 = __shfl(p3, i + 16, NVA_WAVE), x2 = __shfl(p3, i + 32, NVA_WAVE),
@@ -426,17 +451,17 @@ memory_block_kernel(const MemoryArgs a) {
                 const float all = x0 + x1 + x2 + x3;
                 const float P[4] = {base + p0, base + p1, base + p2, base + p3};
                 const float B[4] = {after + lg[3] + lg[2] + lg[1], after + lg[3] + lg[2], after + lg[3], after};
-                if (g == 0) dec_s[d] = expf(all);
-                if (!OUT) log_sum[o] += all;
-                *reinterpret_cast<mem_f32x4*>(kT_s + d * MEM_TS + 4 * g) =
-                    mem_f32x4{k[0] * expf(B[0]), k[1] * expf(B[1]), k[2] * expf(B[2]), k[3] * expf(B[3])};
+                if (g == 0) dec_s[d_own] = nva_exp(all);
+                if (!OUT && g == 0) log_s[d_own] += all;
+                *reinterpret_cast<mem_f32x4*>(kT_s + d_own * MEM_TS + 4 * g) =
+                    mem_f32x4{k[0] * nva_exp(B[0]), k[1] * nva_exp(B[1]), k[2] * nva_exp(B[2]), k[3] * nva_exp(B[3])};
                 if (OUT) {
-                    const bool apart = __all(all > -20.f);
+                    apart = __all(all > -MEM_APART);
 #pragma unroll
-                    for (int r = 0; r < 4; ++r) q_s[(4 * g + r) * QS + d] = q[r] * expf(P[r]);
+                    for (int r = 0; r < 4; ++r) q_s[(4 * g + r) * QS + d_own] = q[r] * nva_exp(P[r]);
                     if (apart) {
 #pragma unroll
-                        for (int r = 0; r < 4; ++r) mine_s[(4 * g + r) * MEM_TS + i] = k[r] * expf(-P[r]);
+                        for (int r = 0; r < 4; ++r) mine_s[(4 * g + r) * MEM_TS + i] = k[r] * nva_exp(-P[r]);
                     } else {
                         // a channel that forgets nearly everything within the chunk: pair by pair
                         for (int s = 0; s < n; ++s) {
@@ -449,24 +474,23 @@ memory_block_kernel(const MemoryArgs a) {
                             Ps = __shfl(Ps, from, NVA_WAVE);
 #pragma unroll
                             for (int r = 0; r < 4; ++r) {
-                                float x = 4 * g + r >= s ? q[r] * ks * expf(fminf(P[r] - Ps, 0.f)) : 0.f;
+                                float x = 4 * g + r >= s ? q[r] * ks * nva_exp(fminf(P[r] - Ps, 0.f)) : 0.f;
 #pragma unroll
                                 for (int by = 1; by < 16; by <<= 1) x += __shfl_xor(x, by, NVA_WAVE);
                                 if (i == s) score[r] += x;
                             }
                         }
-                        continue;
                     }
                 }
             } else {
-                *reinterpret_cast<mem_f32x4*>(kT_s + d * MEM_TS + 4 * g) = mem_f32x4{k[0], k[1], k[2], k[3]};
+                *reinterpret_cast<mem_f32x4*>(kT_s + d_own * MEM_TS + 4 * g) = mem_f32x4{k[0], k[1], k[2], k[3]};
                 if (OUT) {
-                    const float nd = n_s[d];
+                    const float nd = n_s[d_own];
 #pragma unroll
                     for (int r = 0; r < 4; ++r) {
-                        q_s[(4 * g + r) * QS + d] = q[r];
+                        q_s[(4 * g + r) * QS + d_own] = q[r];
                         mine_s[(4 * g + r) * MEM_TS + i] = k[r];
-                        qn[r] += q[r] * nd;
+                        qn[r] = q[r] * nd;
                     }
                 }
             }
@@ -474,36 +498,34 @@ memory_block_kernel(const MemoryArgs a) {
                 // the tile's part of the scores (what the wave's lanes wrote, read by its other lanes)
                 __builtin_amdgcn_wave_barrier();
                 asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
-                const mem_f32x4 qa = *reinterpret_cast<const mem_f32x4*>(q_s + i * QS + 16 * j + 4 * g);
-                const mem_f32x4 kb = *reinterpret_cast<const mem_f32x4*>(mine_s + i * MEM_TS + 4 * g);
+                if (apart) {
+                    const mem_f32x4 qa = *reinterpret_cast<const mem_f32x4*>(q_s + i * QS + 16 * wave + 4 * g);
+                    const mem_f32x4 kb = *reinterpret_cast<const mem_f32x4*>(mine_s + i * MEM_TS + 4 * g);
 #pragma unroll
-                for (int r = 0; r < 4; ++r) score = __builtin_amdgcn_mfma_f32_16x16x4f32(qa[r], kb[r], score, 0, 0, 0);
+                    for (int r = 0; r < 4; ++r) score = __builtin_amdgcn_mfma_f32_16x16x4f32(qa[r], kb[r], score, 0, 0, 0);
+                }
                 asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
                 __builtin_amdgcn_wave_barrier();
-            }
-            own = o + 1;
-        }
-        (void)own;
-        if (OUT && wave < NDT) {
 #pragma unroll
-            for (int r = 0; r < 4; ++r) mine_s[(4 * g + r) * 17 + i] = score[r];
-            if (KIND == MEM_MATRIX) {
+                for (int r = 0; r < 4; ++r) mine_s[(4 * g + r) * 17 + i] = score[r];
+                if (KIND == MEM_MATRIX) {
 #pragma unroll
-                for (int r = 0; r < 4; ++r) {
+                    for (int r = 0; r < 4; ++r) {
 #pragma unroll
-                    for (int by = 1; by < 16; by <<= 1) qn[r] += __shfl_xor(qn[r], by, NVA_WAVE);
-                    if (i == 0) qn_s[wave * MEM_C + 4 * g + r] = qn[r];
+                        for (int by = 1; by < 16; by <<= 1) qn[r] += __shfl_xor(qn[r], by, NVA_WAVE);
+                        if (i == 0) qn_s[wave * MEM_C + 4 * g + r] = qn[r];
+                    }
                 }
             }
         }
         __syncthreads();
         // ---- the scores added up over the waves, with their weights; the matrix rule's divisor
         if (OUT) {
-            const int parts = min(waves, NDT);
             for (int idx = tid; idx < MEM_C * MEM_C; idx += blockDim.x) {
                 const int t = idx >> 4, s = idx & 15;
                 float x = 0.f;
-                for (int w = 0; w < parts; ++w) x += part_s[w * MEM_C * MEM_TS + t * 17 + s];
+#pragma unroll
+                for (int w = 0; w < NDT; ++w) x += part_s[w * MEM_C * MEM_TS + t * 17 + s];
                 if (s > t || t >= n) x = 0.f;
                 if (KIND == MEM_MATRIX) {
                     x = s > t || t >= n ? 0.f : x * expf((float)(e_s[s] - M_s[t]));
@@ -512,9 +534,10 @@ memory_block_kernel(const MemoryArgs a) {
                     for (int by = 1; by < 16; by <<= 1) sum += __shfl_xor(sum, by, NVA_WAVE);
                     if (s == 0) {
                         float nq = 0.f;
-                        for (int w = 0; w < parts; ++w) nq += qn_s[w * MEM_C + t];
+#pragma unroll
+                        for (int w = 0; w < NDT; ++w) nq += qn_s[w * MEM_C + t];
                         sum += inter_s[t] * nq;
-                        den_s[t] = t < n ? 1.f / (fmaxf(fabsf(sum), expf(-a.m[(tok + t) * H + h])) + 1e-6f) : 0.f;
+                        den_s[t] = t < n ? 1.f / (fmaxf(fabsf(sum), floor_s[t]) + 1e-6f) : 0.f;
                     }
                 }
                 a_s[t * MEM_TS + s] = x;
@@ -522,28 +545,30 @@ memory_block_kernel(const MemoryArgs a) {
         }
         // ---- what the state gives, and the state behind the chunk
         mem_f32x4 o = {0.f, 0.f, 0.f, 0.f};
-        float vw[4];
-#pragma unroll
-        for (int r = 0; r < 4; ++r) vw[r] = KIND == MEM_MATRIX ? v[r] * w_s[4 * g + r] : v[r];
         const float keep = KIND == MEM_MATRIX ? keep_s[0] : 1.f;
+        if (multiplies) {
+            float vw[4];
 #pragma unroll
-        for (int j = 0; j < NDT; ++j) {
-            if (OUT) {
-                const mem_f32x4 qa = *reinterpret_cast<const mem_f32x4*>(q_s + i * QS + 16 * j + 4 * g);
+            for (int r = 0; r < 4; ++r) vw[r] = KIND == MEM_MATRIX ? v[r] * w_s[4 * g + r] : v[r];
 #pragma unroll
-                for (int r = 0; r < 4; ++r) o = __builtin_amdgcn_mfma_f32_16x16x4f32(qa[r], S[j][r], o, 0, 0, 0);
+            for (int j = 0; j < NDT; ++j) {
+                if (OUT) {
+                    const mem_f32x4 qa = *reinterpret_cast<const mem_f32x4*>(q_s + i * QS + 16 * j + 4 * g);
+#pragma unroll
+                    for (int r = 0; r < 4; ++r) o = __builtin_amdgcn_mfma_f32_16x16x4f32(qa[r], S[j][r], o, 0, 0, 0);
+                }
+                if (KIND == MEM_LINEAR) {
+                    const mem_f32x4 dec = *reinterpret_cast<const mem_f32x4*>(dec_s + 16 * j + 4 * g);
+#pragma unroll
+                    for (int r = 0; r < 4; ++r) S[j][r] *= dec[r];
+                } else {
+#pragma unroll
+                    for (int r = 0; r < 4; ++r) S[j][r] *= keep;
+                }
+                const mem_f32x4 ka = *reinterpret_cast<const mem_f32x4*>(kT_s + (16 * j + i) * MEM_TS + 4 * g);
+#pragma unroll
+                for (int r = 0; r < 4; ++r) S[j] = __builtin_amdgcn_mfma_f32_16x16x4f32(ka[r], vw[r], S[j], 0, 0, 0);
             }
-            if (KIND == MEM_LINEAR) {
-                const mem_f32x4 dec = *reinterpret_cast<const mem_f32x4*>(dec_s + 16 * j + 4 * g);
-#pragma unroll
-                for (int r = 0; r < 4; ++r) S[j][r] *= dec[r];
-            } else {
-#pragma unroll
-                for (int r = 0; r < 4; ++r) S[j][r] *= keep;
-            }
-            const mem_f32x4 ka = *reinterpret_cast<const mem_f32x4*>(kT_s + (16 * j + i) * MEM_TS + 4 * g);
-#pragma unroll
-            for (int r = 0; r < 4; ++r) S[j] = __builtin_amdgcn_mfma_f32_16x16x4f32(ka[r], vw[r], S[j], 0, 0, 0);
         }
         if (KIND == MEM_MATRIX) {
 #pragma unroll
@@ -571,7 +596,6 @@ memory_block_kernel(const MemoryArgs a) {
                 if (i == 0) red_s[wave * MEM_C + 4 * g + r] = x;
             }
             __syncthreads();
-            const float w = a.norm_w[KIND == MEM_MATRIX ? h * DV + min(c, DV - 1) : min(c, DV - 1)];
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
                 const int t = 4 * g + r;
@@ -579,7 +603,7 @@ memory_block_kernel(const MemoryArgs a) {
                 for (int x = 0; x < waves; ++x) ss += red_s[x * MEM_C + t];
                 const float inv = rsqrtf(ss / (float)DV + a.eps);
                 if (t < n && has_c)
-                    static_cast<T*>(a.out)[(tok + t) * a.out_stride + (int64_t)h * DV + c] = from_float<T>(o[r] * inv * w * mem_gate<KIND>(gate[r]));
+                    static_cast<T*>(a.out)[(tok + t) * a.out_stride + (int64_t)h * DV + c] = from_float<T>(o[r] * inv * norm_w * mem_gate<KIND>(gate[r]));
             }
         }
     }
@@ -603,11 +627,8 @@ memory_block_kernel(const MemoryArgs a) {
             const float x = expf((float)(M_unit - M_before));
             for (int d = tid; d < D; d += blockDim.x) dec[d] = x;
         } else {
-#pragma unroll
-            for (int o = 0; o < OWN; ++o) {
-                const int j = wave + o * waves;
-                if (j < NDT && g == 0 && 16 * j + i < D) dec[16 * j + i] = expf(log_sum[o]);
-            }
+            // (the last chunk's barriers lie between the sums and these reads)
+            for (int d = tid; d < D; d += blockDim.x) dec[d] = expf(log_s[d]);
         }
     }
 }
@@ -652,11 +673,10 @@ static int mem_ndt(int dim) { return dim <= 32 ? 2 : dim <= 64 ? 4 : dim <= 128 
 // Whether portions run in chunks on the matrix cores for these sizes.
 NVA_EXPORT int NVA_NAME(nva_memory_takes_blocks)(int dim, int vdim) { return dim <= 256 && vdim <= 256; }
 
-template <int KIND, int NDT, bool OUT>
-static int mem_launch_block(const MemoryArgs& a, int64_t n_units, hipStream_t stream) {
-    const int waves = (a.vdim + 15) / 16;
+template <int KIND, int NDT, bool OUT, int THREADS>
+static int mem_launch_sized(const MemoryArgs& a, int waves, int64_t n_units, hipStream_t stream) {
     const size_t bytes = sizeof(float) * (size_t)mem_block_lds_floats(NDT, waves, OUT);
-    auto kernel = memory_block_kernel<elem_t, KIND, NDT, OUT>;
+    auto kernel = memory_block_kernel<elem_t, KIND, NDT, OUT, THREADS>;
     static bool raised = false;
     if (!raised && bytes > 48 * 1024) {
         if (hipFuncSetAttribute((const void*)kernel, hipFuncAttributeMaxDynamicSharedMemorySize, 128 * 1024) != hipSuccess)
@@ -665,6 +685,13 @@ static int mem_launch_block(const MemoryArgs& a, int64_t n_units, hipStream_t st
     }
     hipLaunchKernelGGL(kernel, dim3((unsigned)a.heads, (unsigned)n_units), dim3(waves * NVA_WAVE), bytes, stream, a);
     return nva_check_launch("memory blocks");
+}
+
+template <int KIND, int NDT, bool OUT>
+static int mem_launch_block(const MemoryArgs& a, int64_t n_units, hipStream_t stream) {
+    const int waves = mem_block_waves(NDT, a.vdim);          // (16 at most)
+    return waves <= 8 ? mem_launch_sized<KIND, NDT, OUT, 512>(a, waves, n_units, stream)
+                      : mem_launch_sized<KIND, NDT, OUT, 1024>(a, waves, n_units, stream);
 }
 
 template <int KIND, bool OUT>
@@ -690,6 +717,7 @@ static int mem_run(MemoryArgs a, int64_t seqs, int64_t tokens, int64_t singles, 
     if (KIND == MEM_MATRIX && (!a.gates || a.splits <= 0 || !a.n_state || !a.m_state)) return nva_fail("memory: the gates or their state are missing");
     if (KIND == MEM_LINEAR && !a.a2 && !a.z) return nva_fail("memory: the decay's logits are missing");
     a.scale = 1.f / sqrtf((float)a.dim);
+    a.tokens = tokens;
     const bool blocks = n_units > 0;
     if (blocks) {
         if (a.dim > 256 || a.vdim > 256 || !a.units || n_units > 65535 || n_chains < 0 || n_chains > 65535 ||
@@ -752,7 +780,7 @@ NVA_EXPORT int NVA_NAME(nva_gated_linear)(const void* proj, int64_t stride, cons
     return mem_run<MEM_LINEAR>(a, seqs, tokens, singles, n_units, n_chains, stream);
 }
 
-// The matrix rule.  gates: float partial sums [splits][tokens][2 H] = [i | f]; e, M: double [tokens, H], m: float [tokens, H],
+// The matrix rule.  gates: float partial sums [splits][tokens][2 H] = [i | f]; e, M: double [H, tokens], m: float [H, tokens],
 // m_start: float [requests, H], scratch of the portions' gates.
 NVA_EXPORT int NVA_NAME(nva_matrix_memory)(const void* proj, int64_t stride, const float* gates, int splits, int64_t split_stride,
                                            const float* bias, const float* norm_w, float eps, float cap, float* s_state, float* n_state,

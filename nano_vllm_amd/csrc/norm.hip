@@ -463,7 +463,8 @@ NVA_EXPORT int NVA_NAME(nva_stream_post_norm)(const void* a, int64_t a_stride, c
                          b, b_stride, {b_sums, b_splits, b_split_stride, b_bias}, b_scale,
                          a_weight, aw_is_f32, a_offset, a_eps, mult, extra, extra_stride, residual, r_stride,
                          weight, w_is_f32, offset, eps, y, y_stride, width};
-    const int threads = (a_sums || b_sums) && rows <= 64 && width >= 1024 ? 1024
+    // (few rows: two entries a thread, so that a row is asked for at once)
+    const int threads = rows <= 64 && width >= 1024 ? 1024
                         : width >= 2048 ? 512 : width >= 1024 ? 256 : width >= 256 ? 128 : 64;
     const int per = (width + threads - 1) / threads;
 #define POST_NORM(KK)                                                                                                               do {                                                                                                                                if (pair) hipLaunchKernelGGL((stream_post_norm_kernel<elem_t, KK, true>), dim3((unsigned)rows), dim3(threads), 0, stream, g);         else hipLaunchKernelGGL((stream_post_norm_kernel<elem_t, KK, false>), dim3((unsigned)rows), dim3(threads), 0, stream, g);        } while (0)

@@ -1,7 +1,7 @@
 """Named config.json contents for runs with random weights (there is no checkpoint to read
 them from): two tiny test shapes and the Qwen3 dense sizes that the benchmarks use, three
 Nozurax shapes (a tiny one, and layers of the Qwen3 1.7B and 8B sizes), two Mafarax shapes (a tiny
-one, and layers of the Qwen3 1.7B sizes) and two Kirisun, two Pemuvik and two Bamipel shapes of the same kind.  These are
+one, and layers of the Qwen3 1.7B sizes) and two Kirisun, two Pemuvik, two Bamipel and two Nemidra shapes of the same kind.  These are
 inputs, as a model folder's config.json is; nothing in the model code reads them.
 
     python -m nano_vllm_amd.cli random-model --shape qwen3-8b --config-only --out DIR
@@ -137,7 +137,41 @@ def _bamipel(layers, width, heads, kv_heads, dim, vdim, inner, vocab, window, ep
     return {"architecture": "Bamipel", "vocab": vocab, "width": width, "norm": {"eps": eps}, "layers": out, "torch_dtype": dtype}
 
 
+def _nemidra(layers, width, heads, kv_heads, dim, vdim, inner, vocab, window, eps=1e-6, dtype="bfloat16", memory_heads=None,
+             memory_dim=None, memory_vdim=None, gate_cap=15.0, gla_heads=None, gla_dim=None, gla_vdim=None, tau=16.0, rank=16,
+             experts=32, top=6, buckets=32749, side_dim=256, max_positions=65536, loop=None,
+             pattern=(("parallel", "moe"), ("gla", "dense"))) -> dict:
+    """Layers that follow `pattern` in turn: the window attention beside the matrix memory (as many heads of the same sizes
+    unless named) and the gated linear attention (the same), each with a dense layer of 3/2 `inner` without a gate or with
+    `top` of `experts` gated experts of inner / 8 each beside a shared expert of inner / 4 (a token runs the dense layer's
+    inner size)."""
+    mixers = {
+        "parallel": {"left": {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "scale": dim ** -0.5,
+                              "mask": {"size": window}},
+                     "right": {"heads": memory_heads or heads, "dim": memory_dim or dim, "vdim": memory_vdim or vdim, "gate_cap": gate_cap},
+                     "left_scale": 0.75, "right_scale": 0.5},
+        "gla": {"heads": gla_heads or heads, "dim": gla_dim or dim, "vdim": gla_vdim or vdim, "tau": tau, "decay_rank": rank},
+    }
+    mlps = {
+        "dense": {"kind": "dense", "ff": 3 * inner // 2},
+        "moe": {"kind": "moe", "expert": {"ff": max(1, inner // 8)}, "shared": {"ff": max(1, inner // 4)},
+                "router": {"experts": experts, "top": top, "scale": 1.5}},
+        None: None,
+    }
+    entries = [{"type": kind, "mixer": mixers[kind], "mlp": mlps[mlp]} for kind, mlp in (pattern[i % len(pattern)] for i in range(layers))]
+    out = {"architecture": "Nemidra", "vocab": vocab, "width": width, "norm": {"eps": eps}, "max_positions": max_positions,
+           "embedding": {"bigram": {"buckets": buckets, "mul_prev": 40503, "mul_cur": 31}}, "token_side": {"dim": side_dim},
+           "logit_softcap": 25.0, "layers": entries, "torch_dtype": dtype}
+    if loop is not None:
+        out["loop"] = dict(zip(("start", "stop", "times"), loop))
+    return out
+
+
 SHAPES: Dict[str, dict] = {
+    "nemidra-tiny": _nemidra(4, 64, 4, 2, 16, 24, 96, 256, window=12, eps=1e-5, dtype="float32", memory_heads=2, memory_dim=12,
+                             memory_vdim=20, gate_cap=6.0, gla_heads=3, gla_dim=10, gla_vdim=14, tau=4.0, rank=5, experts=6, top=2,
+                             buckets=97, side_dim=12, max_positions=256, loop=(1, 3, 2)),
+    "nemidra-1b": _nemidra(16, 2048, 16, 8, 128, 128, 6144, 32768, window=1024),
     "bamipel-tiny": _bamipel(5, 64, 4, 2, 16, 24, 96, 256, window=12, eps=1e-5, dtype="float32", rot=8, latent_heads=2, latent_dim=12,
                              latent_rot=4, latent_vdim=8, q_rank=28, kv_rank=20, delta_heads=4, delta_kv_heads=2, delta_dim=12,
                              delta_vdim=8, conv=3, scaling={"factor": 4.0, "low": 1.0, "high": 4.0, "original": 64}, again={4: 0}),

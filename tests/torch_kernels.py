@@ -83,7 +83,7 @@ class TorchKernels:
 
     def stream_add(self, addends, residual):
         dt = next(getattr(a.x, "left", a.x).dtype for a in addends if hasattr(a, "mult"))
-        _, residual = self.stream_rms_norm(addends, residual, torch.ones((), device=residual.device), 1.0)
+        _, residual = TorchKernels.stream_rms_norm(self, addends, residual, torch.ones((), device=residual.device), 1.0)
         return residual.to(dt), residual
 
     # norms (layernorm.py:16-40)
