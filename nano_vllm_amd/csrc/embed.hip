@@ -105,7 +105,7 @@ summed_embedding_kernel(const T* __restrict__ table, int64_t table_rows, const T
                         const int32_t* __restrict__ positions, const int32_t* __restrict__ token_seq,
                         const int32_t* __restrict__ cu_seqlens_q, const int32_t* __restrict__ seq_starts,
                         const int32_t* __restrict__ state_slots, int32_t* before_state, float* __restrict__ out, int width,
-                        int32_t* error_flag) {
+                        int vec, int32_t* error_flag) {
     const int64_t t = blockIdx.x;
     const int id = ids[t], p = positions[t];
     const bool ok = id >= 0 && id < table_rows && (!pos_table || (p >= 0 && p < pos_rows));
@@ -113,20 +113,37 @@ summed_embedding_kernel(const T* __restrict__ table, int64_t table_rows, const T
     const T* brow = nullptr;
     if (bigram) {
         const int s = token_seq[t];
-        const int64_t first = cu_seqlens_q[s];
+        const int64_t first = cu_seqlens_q[s], next = cu_seqlens_q[s + 1];
+        const int start = seq_starts[s], slot = state_slots[s];
         int64_t row = buckets;
-        if (t > first || seq_starts[s] > 0) {
-            const int64_t before = t > first ? ids[t - 1] : before_state[state_slots[s]];
+        if (t > first || start > 0) {
+            const int64_t before = t > first ? ids[t - 1] : before_state[slot];
             row = (max(before, (int64_t)0) * mul_prev + (int64_t)max(id, 0) * mul_cur) % buckets;
         }
         if (t == first) {
             __syncthreads();                             // (every thread has read the token before)
-            if (threadIdx.x == 0) before_state[state_slots[s]] = ids[cu_seqlens_q[s + 1] - 1];
+            if (threadIdx.x == 0) before_state[slot] = ids[next - 1];
         }
         brow = bigram + row * width;
     }
     const T* erow = table + (int64_t)(ok ? id : 0) * width;
     const T* prow = pos_table ? pos_table + (int64_t)(ok ? p : 0) * width : nullptr;
+    if (vec) {
+        for (int i = 8 * threadIdx.x; i < width; i += 8 * blockDim.x) {
+            float v[8], b[8], q[8];
+            load8(erow + i, v);
+            if (brow) load8(brow + i, b);
+            if (prow) load8(prow + i, q);
+#pragma unroll
+            for (int e = 0; e < 8; ++e) {
+                if (brow) v[e] += b[e];
+                if (prow) v[e] += q[e];
+                if (!ok) v[e] = 0.f;
+            }
+            store8(out + t * width + i, v);
+        }
+        return;
+    }
     for (int i = threadIdx.x; i < width; i += blockDim.x) {
         float v = to_float(erow[i]);
         if (brow) v += to_float(brow[i]);
@@ -149,9 +166,12 @@ NVA_EXPORT int NVA_NAME(nva_summed_embedding)(const void* table, int64_t table_r
         return nva_fail("summed_embedding: a bigram table needs its constants, the step's requests and their state");
     if (pos_table && pos_rows <= 0) return nva_fail("summed_embedding: an empty table of positions");
     const int threads = width >= 1024 ? 256 : (width >= 256 ? 128 : 64);
+    const size_t vb = 8 * sizeof(elem_t);
+    const int vec = width % 8 == 0 && nva_aligned(table, vb) && (!bigram || nva_aligned(bigram, vb)) &&
+                    (!pos_table || nva_aligned(pos_table, vb)) && nva_aligned(out, 32);
     hipLaunchKernelGGL(summed_embedding_kernel<elem_t>, dim3((unsigned)tokens), dim3(threads), 0, stream, (const elem_t*)table,
                        table_rows, (const elem_t*)bigram, buckets, mul_prev, mul_cur, (const elem_t*)pos_table, pos_rows, ids,
-                       positions, token_seq, cu_seqlens_q, seq_starts, state_slots, before_state, out, width, error_flag);
+                       positions, token_seq, cu_seqlens_q, seq_starts, state_slots, before_state, out, width, vec, error_flag);
     return nva_check_launch("summed_embedding");
 }
 

@@ -385,6 +385,39 @@ moe_combine_kernel(const T* __restrict__ o, int64_t o_stride, const int32_t* __r
     y[t * y_stride + i] = from_float<T>(sum);
 }
 
+// The same eight entries a thread, where rows and pointers allow: the rows of all choices are asked for side by side.
+template <typename T>
+__global__ void __launch_bounds__(256)
+moe_combine8_kernel(const T* __restrict__ o, int64_t o_stride, const int32_t* __restrict__ place,
+                    const float* __restrict__ weights, int top, const T* __restrict__ add, int64_t add_stride,
+                    const float* __restrict__ add_gate, int64_t gate_stride, const T* __restrict__ x, int64_t x_stride,
+                    T* __restrict__ y, int64_t y_stride, int64_t tokens, int width8) {
+    const int64_t idx = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
+    if (idx >= tokens * width8) return;
+    const int64_t t = idx / width8;
+    const int i = (int)(idx % width8) * 8;
+    float sum[8];
+#pragma unroll
+    for (int e = 0; e < 8; ++e) sum[e] = 0.f;
+#pragma unroll 4
+    for (int c = 0; c < top; ++c) {
+        const int at = place[t * top + c];
+        const float w = weights[t * top + c];
+        float v[8];
+        load8(at < 0 ? x + t * x_stride + i : o + (int64_t)at * o_stride + i, v);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) sum[e] += w * v[e];
+    }
+    if (add) {
+        float v[8];
+        load8(add + t * add_stride + i, v);
+        const float s = add_gate ? 1.f + expf(-add_gate[t * gate_stride]) : 1.f;
+#pragma unroll
+        for (int e = 0; e < 8; ++e) sum[e] += v[e] / s;
+    }
+    store8(y + t * y_stride + i, sum);
+}
+
 NVA_EXPORT int NVA_NAME(nva_moe_route)(const float* logits, int64_t stride, int64_t tokens, int experts, int top,
                                        int group_count, int group_keep, float scale, int softmax_top, const float* bias,
                                        int32_t* ids, float* weights, hipStream_t stream) {
@@ -474,6 +507,14 @@ NVA_EXPORT int NVA_NAME(nva_moe_experts)(const void* x, int64_t x_stride, const 
     hipLaunchKernelGGL((moe_tile_kernel<elem_t, false>), dim3((unsigned)max_tiles, (k + MOE_BN - 1) / MOE_BN), dim3(256), 0,
                        stream, (const elem_t*)hidden, (int64_t)ff, (const elem_t*)down, k, ff, rows, top, tile_expert,
                        tile_row0, tile_rows, num_tiles, act, (elem_t*)outs, (int64_t)k);
+    }
+    const size_t vb = 8 * sizeof(elem_t);
+    if (k % 8 == 0 && x_stride % 8 == 0 && y_stride % 8 == 0 && (!add || add_stride % 8 == 0) && nva_aligned(x, vb) && nva_aligned(y, vb) &&
+        nva_aligned(outs, vb) && (!add || nva_aligned(add, vb)) && (tokens * (k / 8) + 255) / 256 <= 0x7fffffff) {
+        hipLaunchKernelGGL((moe_combine8_kernel<elem_t>), dim3((unsigned)((tokens * (k / 8) + 255) / 256)), dim3(256), 0, stream,
+                           (const elem_t*)outs, (int64_t)k, place, weights, top, (const elem_t*)add, add_stride, add_gate, gate_stride,
+                           (const elem_t*)x, x_stride, (elem_t*)y, y_stride, tokens, k / 8);
+        return nva_check_launch("moe_experts");
     }
     for (int64_t t0 = 0; t0 < tokens; t0 += 65535) {
         const unsigned nt = (unsigned)((tokens - t0) < 65535 ? (tokens - t0) : 65535);

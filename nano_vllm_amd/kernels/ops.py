@@ -173,15 +173,16 @@ def delta_blocks(q_lens, first_seq: int):
 MEMORY_CHUNK = 16       # tokens of a chunk of the gated linear attentions' matrix-core form
 
 
-def memory_units(q_lens, first_seq: int, heads: int, cus: int):
+def memory_units(q_lens, first_seq: int, heads: int, cus: int, tokens: int = 0):
     """The step's portions (the requests from `first_seq` on, which single tokens precede) in units of whole chunks that run side
     by side: (units, chains), units a flat list of (request, the unit's first token counted through the step, its tokens,
     kind) with kind 0 for a portion of one unit, 2 for a portion's last, 1 for the others; chains one of (first unit, units,
-    request, 0) for every portion of more than one.  Units of 64 tokens, of more where heads and units then still give
-    every compute unit two workgroups."""
+    request, 0) for every portion of more than one.  Units of 32 tokens, of more where heads and units then still give
+    every compute unit a workgroup (tokens: that many, a multiple of a chunk): a unit's start and end states travel through
+    memory, and a step of few tokens has few units."""
     total = sum(q_lens[first_seq:])
-    size = 4 * MEMORY_CHUNK
-    while size < 1024 and (total // (2 * size)) * heads >= 2 * cus:
+    size = tokens or 2 * MEMORY_CHUNK
+    while not tokens and size < 1024 and (total // (2 * size)) * heads >= cus:
         size *= 2
     units, chains = [], []
     token = sum(q_lens[:first_seq])
@@ -357,6 +358,7 @@ class HipKernels:
         self.delta_block_min = DELTA_BLOCK
         # False: the gated linear attention and the matrix memory run portions token by token too
         self.memory_blocks = True
+        self.memory_unit_tokens = 0         # tokens of a unit of their portions, a multiple of MEMORY_CHUNK; 0: the rule
         # False: the state-space layer runs a portion's tokens one after the other, whatever its length
         self.state_space_blocks_side_by_side = True
         # how the recurrence holds a state of 65 to 128 rows: 0 two lanes a column (what serves), 1 a thread a column
@@ -1951,7 +1953,7 @@ class HipKernels:
             kept = batch.step_cache = {}
         plan = kept.get(("memory_units", first, heads))
         if plan is None:
-            flat_units, flat_chains = memory_units(batch.q_lens, first, heads, self.cus)
+            flat_units, flat_chains = memory_units(batch.q_lens, first, heads, self.cus, self.memory_unit_tokens)
             both = torch.tensor(flat_units + flat_chains, dtype=torch.int32).to(proj.device, non_blocking=True)
             plan = (len(flat_units) // 4, len(flat_chains) // 4, both[: len(flat_units)], both[len(flat_units):])
             kept[("memory_units", first, heads)] = plan

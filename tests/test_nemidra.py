@@ -477,19 +477,19 @@ def test_long_portions_beside_single_tokens(backend, dtype, kind, shape):
         pytest.skip("the stand-ins run one way only")
     eps = 1e-5
     r = K.rule(kind, shape, 41, dtype)
-    lens = {"a": 9, "b": 130, "c": 67, "d": 200, "e": 68}
+    lens = {"a": 9, "b": 130, "c": 67, "d": 200, "e": 68, "f": 33, "g": 32}
     inputs = {q: r.inputs(n, 50 + i) for i, (q, n) in enumerate(lens.items())}
     want = {q: r.plain(inputs[q], eps) for q in lens}
-    slot = {"a": 2, "b": 0, "c": 4, "d": 1, "e": 3}
-    steps = [[("a", 0, 8), ("b", 0, 64), ("c", 0, 65), ("d", 0, 3)],
+    slot = {"a": 2, "b": 0, "c": 4, "d": 1, "e": 3, "f": 6, "g": 7}
+    steps = [[("a", 0, 8), ("b", 0, 64), ("c", 0, 65), ("d", 0, 3), ("f", 0, 33), ("g", 0, 32)],
              [("a", 8, 1), ("b", 64, 1), ("d", 3, 131), ("c", 65, 2), ("e", 0, 67)],
              [("e", 67, 1), ("b", 65, 65), ("d", 134, 66)]]
     found = {}
-    for blocks in (True, False) if backend == "hip" else (True,):
+    for blocks in (True, 64, False) if backend == "hip" else (True,):            # (64: units of that many tokens)
         if backend == "hip":
-            k.memory_blocks = blocks
+            k.memory_blocks, k.memory_unit_tokens = bool(blocks), 64 if blocks == 64 else 0
         try:
-            states, got = r.states(dev, 6), {q: [] for q in lens}
+            states, got = r.states(dev, 8), {q: [] for q in lens}
             for step in steps:
                 part = tuple(torch.cat([inputs[q][i][s:s + n] for q, s, n in step]) for i in range(len(inputs["a"])))
                 out = r.run(k, dev, part, eps, states, [n for _, _, n in step], [s for _, s, _ in step], [slot[q] for q, _, _ in step])
@@ -503,11 +503,13 @@ def test_long_portions_beside_single_tokens(backend, dtype, kind, shape):
             found[blocks] = states
         finally:
             if backend == "hip":
-                k.memory_blocks = True
+                k.memory_blocks, k.memory_unit_tokens = True, 0
     if backend == "hip":
         # the states agree far below what bfloat16's outputs show (linear: the portions' decay logits come from another product)
-        for a, b in zip(found[True], found[False]):
-            _close(a[:5], b[:5].cpu(), torch.float32, "states", 1e-4)
+        held = [s for s in range(8) if s != 5]
+        for other in (True, 64):
+            for a, b in zip(found[other], found[False]):
+                _close(a[held], b[held].cpu(), torch.float32, "states", 1e-4)
 
 
 @pytest.mark.parametrize("backend", BACKENDS)
@@ -579,13 +581,16 @@ def test_a_far_write_is_read_out(backend, kind, shape):
 def test_portions_are_cut_into_units():
     from nano_vllm_amd.kernels.ops import memory_units
     units, chains = memory_units([1, 1, 130, 2, 64], 2, 4, 256)
-    assert units == [2, 2, 64, 1, 2, 66, 64, 1, 2, 130, 2, 2, 3, 132, 2, 0, 4, 134, 64, 0] and chains == [0, 3, 2, 0]
+    assert units == [2, 2, 32, 1, 2, 34, 32, 1, 2, 66, 32, 1, 2, 98, 32, 1, 2, 130, 2, 2, 3, 132, 2, 0, 4, 134, 32, 1, 4, 166, 32, 2]
+    assert chains == [0, 5, 2, 0, 6, 2, 4, 0]
+    units, chains = memory_units([130, 2], 0, 4, 256, tokens=64)
+    assert units == [0, 0, 64, 1, 0, 64, 64, 1, 0, 128, 2, 2, 1, 130, 2, 0] and chains == [0, 3, 0, 0]
     for n, heads in ((20000, 16), (100000, 32), (300, 2)):
         units, chains = memory_units([n], 0, heads, 256)
         sizes = units[2::4]
         assert sum(sizes) == n and all(s % 16 == 0 and s == sizes[0] for s in sizes[:-1]) and 0 < sizes[-1] <= sizes[0]
         assert units[1::4] == [i * sizes[0] for i in range(len(sizes))] and units[3::4] == [1] * (len(sizes) - 1) + [2]
-        assert sizes[0] == 64 or len(sizes) * heads >= 512
+        assert sizes[0] == 32 or len(sizes) * heads >= 256
 
 
 # ------------------------------------------------------------------------------ the model through the step function
