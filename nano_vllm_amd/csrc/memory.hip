@@ -596,12 +596,12 @@ memory_block_kernel(const MemoryArgs a) {
                 if (i == 0) red_s[wave * MEM_C + 4 * g + r] = x;
             }
             __syncthreads();
+            mem_f32x4 ss = {0.f, 0.f, 0.f, 0.f};
+            for (int x = 0; x < waves; ++x) ss += *reinterpret_cast<const mem_f32x4*>(red_s + x * MEM_C + 4 * g);
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
                 const int t = 4 * g + r;
-                float ss = 0.f;
-                for (int x = 0; x < waves; ++x) ss += red_s[x * MEM_C + t];
-                const float inv = rsqrtf(ss / (float)DV + a.eps);
+                const float inv = rsqrtf(ss[r] / (float)DV + a.eps);
                 if (t < n && has_c)
                     static_cast<T*>(a.out)[(tok + t) * a.out_stride + (int64_t)h * DV + c] = from_float<T>(o[r] * inv * norm_w * mem_gate<KIND>(gate[r]));
             }
