@@ -139,7 +139,7 @@ def _embed_batch(dev, q_lens, starts, slots):
 
 @pytest.mark.parametrize("backend", BACKENDS)
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("buckets,mul_prev,mul_cur,vocab,width", [(89, 7, 3, 60, 48), (1, 5, 2, 30, 20), (1021, 40503, 0, 3000, 130),
+@pytest.mark.parametrize("buckets,mul_prev,mul_cur,vocab,width", [(89, 7, 3, 60, 48), (1, 5, 2, 30, 20), (1013, 40503, 0, 3000, 130),
                                                                   (997, 2000000011, 1999999973, 5000, 24)])
 def test_three_embeddings_and_the_token_before(backend, dtype, buckets, mul_prev, mul_cur, vocab, width):
     """Whole, token by token, in portions, unequal requests in one batch, a slot that another request left: a first token
@@ -291,12 +291,12 @@ def test_the_exact_gelu_after_a_product(backend, dtype, tokens, width, inner):
 
 
 @pytest.mark.parametrize("backend", BACKENDS)
-@pytest.mark.parametrize("width", [97, 576, 4096])
+@pytest.mark.parametrize("width", [97, 580, 4096])
 def test_capped_logits(backend, width):
     k, dev = _kernels(backend)
     x = torch.linspace(-200.0, 200.0, 5 * width).view(5, width)
-    got = k.softcap_(x.clone().to(dev), 30.0)
-    _close(got, 30.0 * torch.tanh(x.double() / 30.0), torch.float32, tol=1e-6)
+    got = k.softcap_(x.clone().to(dev), 25.0)
+    _close(got, 25.0 * torch.tanh(x.double() / 25.0), torch.float32, tol=1e-6)
 
 
 # ------------------------------------------------------------------------------ experts
@@ -371,7 +371,7 @@ def _window_run(k, dev, dtype, hq, hkv, D, DV, page, lens, q_lens, window, scale
     (4, 2, 12, 16, 8, 10, [30, 9, 41], [1, 1, 41]),
     (3, 1, 6, 10, 4, 1, [13, 6], [1, 6]),
     (6, 3, 24, 24, 16, 33, [50, 33], [17, 33]),
-    (4, 2, 48, 48, 64, 70, [200, 3, 130], [1, 2, 130]),            # a head size that the matrix cores' kernels leave to the general one
+    (6, 2, 40, 40, 64, 70, [200, 3, 130], [1, 2, 130]),            # a head size that the matrix cores' kernels leave to the general one
     (8, 2, 64, 64, 32, 48, [130, 70, 100], [1, 2, 64]),
 ])
 def test_window_attention_over_pages(backend, dtype, hq, hkv, D, DV, page, window, lens, q_lens):
@@ -387,7 +387,7 @@ def test_window_attention_over_pages(backend, dtype, hq, hkv, D, DV, page, windo
 
 @pytest.mark.parametrize("backend", BACKENDS)
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("D,DV,page,window", [(12, 8, 8, 23), (48, 48, 32, 64), (48, 48, 64, 65), (64, 64, 32, 23)])
+@pytest.mark.parametrize("D,DV,page,window", [(12, 8, 8, 23), (40, 40, 32, 64), (40, 56, 64, 65), (64, 64, 32, 23)])
 def test_a_key_just_inside_and_just_outside_the_window(backend, dtype, D, DV, page, window):
     """One key takes nearly all the weight of the queries whose window holds it: the last query of a portion, of a whole
     prompt, and a single token follow it at the window's oldest place, and take nothing of it one place further."""
